@@ -57,10 +57,16 @@ class ModelSpec:
     head: PartSpec
     eos_token_ids: Tuple[int, ...] = ()
     injections: Tuple[PartSpec, ...] = ()
+    # 0: one residual stream.  n > 0: n streams side by side, all equal to the embedding output at the start, mixed by
+    # the blocks (which must be of the arrangement that knows streams); the final norm reads their sum.
+    streams: int = 0
 
     def validate(self) -> None:
         if not self.layers:
             raise ValueError("model spec: no layers")
+        if self.streams < 0 or (self.streams and self.injections):
+            raise ValueError("model spec: the number of streams must not be negative, and nothing is injected between "
+                             "layers where there are several")
         if not self.order:
             raise ValueError("model spec: empty execution order")
         for i, e in enumerate(self.order):

@@ -19,15 +19,30 @@ __device__ __forceinline__ void wave_lds_sync() {
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
-// What a (token, head)'s sums of values are multiplied by at the end: one over the sum of the weights, to which a
-// softmax with a SINK adds exp(sink[head] - maximum) (a term of the denominator that has no key and no value), and,
-// where the heads have gates, times sigmoid(gate[token, head]).
-__device__ __forceinline__ float finish_factor(float l, float m, const float* __restrict__ sink, const float* __restrict__ gate,
-                                               long gate_stride, int t, int head) {
-    if (sink && l != 0.f) l += expf(sink[head] - m);
+// What some mixers add to the plain rule (null: not there).  `sink`: a number a head; the softmax's denominator also
+// holds exp(sink[head]), a term without key or value.  `gate`: float32 rows behind a sigmoid that multiply the outputs,
+// one number a head (gate[token, head]) or, with per_column, one a head and value column (gate[token, head * dv + d]).
+// `slopes`: a number a head; the score of a key loses slopes[head] times its distance from the query.
+struct MaExtras { const float* sink; const float* gate; long gate_stride; int per_column; const float* slopes; };
+
+// What a (token, head)'s sums of values are multiplied by at the end: one over the sum of the weights (with the sink's
+// term, counted once), and the head's gate where heads have one.
+__device__ __forceinline__ float finish_factor(float l, float m, const MaExtras& ex, int t, int head) {
+    if (ex.sink && l != 0.f) l += expf(ex.sink[head] - m);
     float f = l != 0.f ? 1.0f / l : 0.f;
-    if (gate) f *= 1.0f / (1.0f + expf(-gate[(size_t)t * gate_stride + head]));
+    if (ex.gate && !ex.per_column) f *= 1.0f / (1.0f + expf(-ex.gate[(size_t)t * ex.gate_stride + head]));
     return f;
+}
+
+// The gate of one value column (1 where the columns have none of their own), and of four neighbouring ones at once.
+__device__ __forceinline__ float column_gate(const MaExtras& ex, int t, int head, int dv, int d) {
+    if (!ex.gate || !ex.per_column) return 1.0f;
+    return 1.0f / (1.0f + expf(-ex.gate[(size_t)t * ex.gate_stride + (size_t)head * dv + d]));
+}
+__device__ __forceinline__ float4 column_gate4(const MaExtras& ex, int t, int head, int dv, int d) {
+    if (!ex.gate || !ex.per_column) return float4{1.f, 1.f, 1.f, 1.f};
+    const float4 g = *reinterpret_cast<const float4*>(ex.gate + (size_t)t * ex.gate_stride + (size_t)head * dv + d);
+    return float4{1.0f / (1.0f + expf(-g.x)), 1.0f / (1.0f + expf(-g.y)), 1.0f / (1.0f + expf(-g.z)), 1.0f / (1.0f + expf(-g.w))};
 }
 
 // The general kernel (any sizes, both dtypes): a block of NW waves per (token, query head); wave w takes the
@@ -41,7 +56,7 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_wave_kernel(
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_list,
     const int* __restrict__ seg_of_token,
     const int* __restrict__ q_start, const int* __restrict__ q_len, const int* __restrict__ ctx_len,
-    int nh, int nkv, int dk, int dv, int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* __restrict__ sink, const float* __restrict__ gate, long gate_stride) {
+    int nh, int nkv, int dk, int dv, int page_size, int num_pages, int window, int keep_first, float softcap, float scale, MaExtras ex) {
     extern __shared__ float smem[];
     float* qs = smem;                                        // [dk]
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -98,6 +113,7 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_wave_kernel(
                 }
                 sc = dot * scale;
                 if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+                if (ex.slopes) sc -= ex.slopes[h] * (float)(p - key);
             }
         }
         const float m_new = fmaxf(m, wave_max(sc));
@@ -125,11 +141,11 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_wave_kernel(
     }
     TO* orow = out + ((size_t)t * nh + h) * dv;
     if constexpr (NW == 1) {
-        const float fin = finish_factor(l, m, sink, gate, gate_stride, t, h);
+        const float fin = finish_factor(l, m, ex, t, h);
 #pragma unroll
         for (int c = 0; c < NC; ++c) {
             const int d = lane + c * LI_WAVE;
-            if (d < dv) store_from_float(orow + d, acc[c] * fin);
+            if (d < dv) store_from_float(orow + d, acc[c] * fin * column_gate(ex, t, h, dv, d));
         }
     } else {
         float* mine = join + (size_t)w * (dv + 2);
@@ -150,12 +166,12 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_wave_kernel(
             f[x] = (lx == 0.f) ? 0.f : expf(mx - mm);
             ll += lx * f[x];
         }
-        const float fin = finish_factor(ll, mm, sink, gate, gate_stride, t, h);
+        const float fin = finish_factor(ll, mm, ex, t, h);
         for (int d = threadIdx.x; d < dv; d += 64 * NW) {
             float a = 0.f;
 #pragma unroll
             for (int x = 0; x < NW; ++x) a += join[(size_t)x * (dv + 2) + d] * f[x];
-            store_from_float(orow + d, a * fin);
+            store_from_float(orow + d, a * fin * column_gate(ex, t, h, dv, d));
         }
     }
 }
@@ -165,14 +181,14 @@ static int launch_masked(const float* q, int qts, int qhs, void* out, const void
                          const int* block_table, int max_blocks, const int* token_list, int n_tokens, const int* seg_of_token,
                          const int* q_start, const int* q_len,
                          const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size, int num_pages, int window,
-                         int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int waves, hipStream_t stream) {
+                         int keep_first, float softcap, float scale, MaExtras ex, int waves, hipStream_t stream) {
     const dim3 grid(n_tokens, nh);
     constexpr int E = 16 / sizeof(T);
     const bool vec = dk % E == 0 && k_row % E == 0 && ((uintptr_t)kc % 16) == 0;
 #define MA_GO(V, NW)                                                                                                         \
     masked_attention_wave_kernel<T, TO, NC, V, NW><<<grid, 64 * NW, (size_t)(dk + NW * 128 + NW * (dv + 2)) * 4, stream>>>(  \
         q, qts, qhs, (TO*)out, (const T*)kc, (const T*)vc, k_row, v_row, block_table, max_blocks, token_list, seg_of_token,  \
-        q_start, q_len, ctx_len, nh, nkv, dk, dv, page_size, num_pages, window, keep_first, softcap, scale, sink, gate, gate_stride)
+        q_start, q_len, ctx_len, nh, nkv, dk, dv, page_size, num_pages, window, keep_first, softcap, scale, ex)
     if (waves >= 8) { if (vec) MA_GO(true, 8); else MA_GO(false, 8); }
     else if (waves >= 4) { if (vec) MA_GO(true, 4); else MA_GO(false, 4); }
     else { if (vec) MA_GO(true, 1); else MA_GO(false, 1); }
@@ -190,15 +206,16 @@ extern "C" int li_masked_attention(const float* q, int q_token_stride, int q_hea
                                    const int* block_table, int max_blocks, const int* token_list, int n_tokens,
                                    const int* seg_of_token, const int* q_start,
                                    const int* q_len, const int* ctx_len, int nh, int nkv, int dk, int dv,
-                                   int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride,
+                                   int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes,
                                    int waves, hipStream_t stream) {
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
     if (n_tokens <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || dk <= 0 || dv <= 0 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || nh > 65535 || dk > 4096 || dv > 64 * MA_MAX_CHUNKS)
         return LI_ERR_SIZE;
     const int nc = (dv + 63) / 64;
 #define MA_ARGS q, q_token_stride, q_head_stride, out, kc, vc, k_row, v_row, block_table, max_blocks, token_list, n_tokens,  \
                 seg_of_token, q_start, q_len, ctx_len, nh, nkv, dk, dv, page_size, num_pages, window, keep_first, softcap,   \
-                scale, sink, gate, gate_stride, waves, stream
+                scale, ex, waves, stream
 #define MA_PICK(T, TO)                                                                  \
     {                                                                                   \
         if (nc <= 1) return launch_masked<T, TO, 1>(MA_ARGS);                           \
@@ -246,7 +263,7 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
     const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc, int k_row, int v_row,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ tiles,
     const int* __restrict__ q_start, const int* __restrict__ q_len, const int* __restrict__ ctx_len,
-    int nh, int nkv, int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* __restrict__ sink, const float* __restrict__ gate, long gate_stride,
+    int nh, int nkv, int page_size, int num_pages, int window, int keep_first, float softcap, float scale, MaExtras ex,
     int nsplit, float* __restrict__ parts) {
     constexpr int DK = KS * 16, DV = DT * 32, KROW = DK + 8;
     constexpr int NT = NW * 64;
@@ -267,6 +284,7 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
     const int hh = (blockIdx.z / nsplit) * NW + w;                             // this wave's head within the group
     const bool active = hh < rep;
     const int head = kvh * rep + (active ? hh : 0);
+    const float slope = ex.slopes ? ex.slopes[head] : 0.f;
     const int pq = p0 + ql;                                               // this lane's query (ql >= ntok: none)
     const int lq = (window > 0) ? pq - window + 1 : 0;
     const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
@@ -382,6 +400,11 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
                 if (softcap > 0.f) sc = softcap * fast_tanh(sc * inv_cap);
                 sv[r] = sc;
             }
+            if (ex.slopes) {
+#pragma unroll
+                for (int r = 0; r < 16; ++r)
+                    sv[r] -= slope * (float)(pq - visible_key(i0 + 8 * (r >> 2) + 4 * h + (r & 3), n_first, lo_min));
+            }
             if (!whole) {
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
@@ -450,21 +473,21 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
         if (h == 0) { part[DV] = m; part[DV + 1] = l; }
         return;
     }
-    const float inv = finish_factor(l, m, sink, gate, gate_stride, t0 + ql, head);
+    const float inv = finish_factor(l, m, ex, t0 + ql, head);
     bf16_t* orow = out + ((size_t)(t0 + ql) * nh + head) * DV;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
         for (int rg = 0; rg < 4; ++rg) {           // registers 4 rg .. 4 rg + 3: value columns 32 dt + 8 rg + 4 h ..
             uint32_t* dst = reinterpret_cast<uint32_t*>(orow + 32 * dt + 8 * rg + 4 * h);
-            dst[0] = pack2_bf16(acc[dt][4 * rg] * inv, acc[dt][4 * rg + 1] * inv);
-            dst[1] = pack2_bf16(acc[dt][4 * rg + 2] * inv, acc[dt][4 * rg + 3] * inv);
+            const float4 cg = column_gate4(ex, t0 + ql, head, DV, 32 * dt + 8 * rg + 4 * h);
+            dst[0] = pack2_bf16(acc[dt][4 * rg] * inv * cg.x, acc[dt][4 * rg + 1] * inv * cg.y);
+            dst[1] = pack2_bf16(acc[dt][4 * rg + 2] * inv * cg.z, acc[dt][4 * rg + 3] * inv * cg.w);
         }
 }
 
 __global__ void masked_attention_join_kernel(const float* __restrict__ parts, bf16_t* __restrict__ out,
-                                             const int* __restrict__ token_list, int nh, int dv, int nsplit, const float* __restrict__ sink,
-                                             const float* __restrict__ gate, long gate_stride, int by_token = 0);
+                                             const int* __restrict__ token_list, int nh, int dv, int nsplit, MaExtras ex, int by_token = 0);
 
 // ------------------------------------------------------------------------------------------- single tokens, MFMA
 // Decoding where a kv head serves many query heads (a compressed cache serves ALL of them): the same transposed
@@ -477,7 +500,7 @@ __global__ __launch_bounds__(64) void masked_attention_heads_kernel(
     const bf16_t* __restrict__ kc, const bf16_t* __restrict__ vc, int k_row, int v_row,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_list,
     const int* __restrict__ seg_of_token, const int* __restrict__ q_start, const int* __restrict__ q_len, const int* __restrict__ ctx_len,
-    int nh, int nkv, int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* __restrict__ sink, const float* __restrict__ gate, long gate_stride,
+    int nh, int nkv, int page_size, int num_pages, int window, int keep_first, float softcap, float scale, MaExtras ex,
     int nsplit, float* __restrict__ parts) {
     constexpr int DK = KS * 16, DV = DT * 32, KROW = DK + 8;
     constexpr int NT = 64;
@@ -500,6 +523,7 @@ __global__ __launch_bounds__(64) void masked_attention_heads_kernel(
     const bool has = hq < rep;
     const bool active = true;
     const int head = kvh * rep + (has ? hq : 0);
+    const float slope = ex.slopes ? ex.slopes[head] : 0.f;
     (void)w;
     const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
 
@@ -603,6 +627,11 @@ __global__ __launch_bounds__(64) void masked_attention_heads_kernel(
                 if (softcap > 0.f) sc = softcap * fast_tanh(sc * inv_cap);
                 sv[r] = sc;
             }
+            if (ex.slopes) {
+#pragma unroll
+                for (int r = 0; r < 16; ++r)
+                    sv[r] -= slope * (float)(p0 - visible_key(i0 + 8 * (r >> 2) + 4 * h + (r & 3), n_first, lo_min));
+            }
             if (!whole) {
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
@@ -653,15 +682,16 @@ __global__ __launch_bounds__(64) void masked_attention_heads_kernel(
     l += __shfl_xor(l, 32, LI_WAVE);
     if (!has) return;
     if (nsplit == 1) {
-        const float inv = finish_factor(l, m, sink, gate, gate_stride, t, head);
+        const float inv = finish_factor(l, m, ex, t, head);
         bf16_t* orow = out + ((size_t)t * nh + head) * DV;
 #pragma unroll
         for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
             for (int rg = 0; rg < 4; ++rg) {       // registers 4 rg .. 4 rg + 3: value columns 32 dt + 8 rg + 4 h ..
                 uint32_t* dst = reinterpret_cast<uint32_t*>(orow + 32 * dt + 8 * rg + 4 * h);
-                dst[0] = pack2_bf16(acc[dt][4 * rg] * inv, acc[dt][4 * rg + 1] * inv);
-                dst[1] = pack2_bf16(acc[dt][4 * rg + 2] * inv, acc[dt][4 * rg + 3] * inv);
+                const float4 cg = column_gate4(ex, t, head, DV, 32 * dt + 8 * rg + 4 * h);
+                dst[0] = pack2_bf16(acc[dt][4 * rg] * inv * cg.x, acc[dt][4 * rg + 1] * inv * cg.y);
+                dst[1] = pack2_bf16(acc[dt][4 * rg + 2] * inv * cg.z, acc[dt][4 * rg + 3] * inv * cg.w);
             }
     } else {                                       // this split's sums, maximum and sum of weights, for the join kernel
         float* part = parts + (((size_t)blockIdx.x * nh + head) * nsplit + sp) * (DV + 2);
@@ -688,15 +718,17 @@ extern "C" int li_masked_attention_tiles(const float* q, int q_token_stride, int
                                          const void* vc, int k_row, int v_row, const int* block_table, int max_blocks,
                                          const int* tiles, int num_tiles, const int* q_start, const int* q_len,
                                          const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size, int num_pages,
-                                         int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int nsplit, float* parts,
+                                         int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int nsplit, float* parts,
                                          long parts_floats, const int* multi_tokens, int num_multi, int num_tokens,
                                          hipStream_t stream) {
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
     if (num_tiles <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || nkv > 65535 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || k_row % 8 || v_row % 8 || q_token_stride % 4 || q_head_stride % 4 ||
         ((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) % 16 || (uintptr_t)out % 8 || !li_masked_attention_tiles_takes(dk, dv) ||
         nsplit < 1 || nsplit > 16 || num_multi <= 0 ||
         (nsplit > 1 && (!parts || (uintptr_t)parts % 8 || parts_floats < (long)num_tokens * nh * nsplit * (dv + 2))))
         return LI_ERR_SIZE;
+    if (gate && gate_per_column && ((uintptr_t)gate % 16 || gate_stride % 4)) return LI_ERR_SIZE;
     const int rep = nh / nkv;
     // five to eight heads a kv head: one block of eight waves (one staging of every block of keys for all of them)
     // rather than blocks of four and of one to four; more heads: whichever leaves fewer waves idle
@@ -707,15 +739,15 @@ extern "C" int li_masked_attention_tiles(const float* q, int q_token_stride, int
         if (nw == 8)                                                                                                       \
             masked_attention_tile_kernel<K / 16, V / 32, 8><<<grid, 512, 0, stream>>>(                                     \
                 q, q_token_stride, q_head_stride, (bf16_t*)out, (const bf16_t*)kc, (const bf16_t*)vc, k_row, v_row, block_table, \
-                max_blocks, tiles, q_start, q_len, ctx_len, nh, nkv, page_size, num_pages, window, keep_first, softcap, scale, sink, gate, gate_stride, \
+                max_blocks, tiles, q_start, q_len, ctx_len, nh, nkv, page_size, num_pages, window, keep_first, softcap, scale, ex, \
                 nsplit, parts);                                                                                            \
         else                                                                                                               \
             masked_attention_tile_kernel<K / 16, V / 32, 4><<<grid, 256, 0, stream>>>(                                     \
                 q, q_token_stride, q_head_stride, (bf16_t*)out, (const bf16_t*)kc, (const bf16_t*)vc, k_row, v_row, block_table, \
-                max_blocks, tiles, q_start, q_len, ctx_len, nh, nkv, page_size, num_pages, window, keep_first, softcap, scale, sink, gate, gate_stride, \
+                max_blocks, tiles, q_start, q_len, ctx_len, nh, nkv, page_size, num_pages, window, keep_first, softcap, scale, ex, \
                 nsplit, parts);                                                                                            \
         if (nsplit > 1)                                                                                                    \
-            masked_attention_join_kernel<<<dim3(num_multi, nh), dv >= 256 ? 256 : 128, 0, stream>>>(parts, (bf16_t*)out, multi_tokens, nh, dv, nsplit, sink, gate, gate_stride, 1); \
+            masked_attention_join_kernel<<<dim3(num_multi, nh), dv >= 256 ? 256 : 128, 0, stream>>>(parts, (bf16_t*)out, multi_tokens, nh, dv, nsplit, ex, 1); \
         return li_launch_status();                                                                                         \
     }
     MT_GO(64, 64) MT_GO(128, 128) MT_GO(128, 64) MT_GO(64, 128) MT_GO(96, 64) MT_GO(160, 128) MT_GO(192, 128)
@@ -729,13 +761,15 @@ extern "C" int li_masked_attention_heads(const float* q, int q_token_stride, int
                                          const void* vc, int k_row, int v_row, const int* block_table, int max_blocks,
                                          const int* token_list, int n_tokens, const int* seg_of_token, const int* q_start,
                                          const int* q_len, const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size,
-                                         int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int nsplit,
+                                         int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int nsplit,
                                          float* parts, long parts_floats, hipStream_t stream) {
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
     if (n_tokens <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || nkv > 65535 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || k_row % 8 || v_row % 8 || q_token_stride % 4 || q_head_stride % 4 ||
         ((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) % 16 || (uintptr_t)out % 8 || !li_masked_attention_tiles_takes(dk, dv) ||
         nsplit < 1 || nsplit > 64 || (nsplit > 1 && (!parts || parts_floats < (long)n_tokens * nh * nsplit * (dv + 2))))
         return LI_ERR_SIZE;
+    if (gate && gate_per_column && ((uintptr_t)gate % 16 || gate_stride % 4)) return LI_ERR_SIZE;
     const int rep = nh / nkv;
     const dim3 grid(n_tokens, nkv, ((rep + 31) / 32) * nsplit);
 #define MH_GO(K, V)                                                                                                        \
@@ -743,9 +777,9 @@ extern "C" int li_masked_attention_heads(const float* q, int q_token_stride, int
         masked_attention_heads_kernel<K / 16, V / 32><<<grid, 64, 0, stream>>>(                                            \
             q, q_token_stride, q_head_stride, (bf16_t*)out, (const bf16_t*)kc, (const bf16_t*)vc, k_row, v_row, block_table, \
             max_blocks, token_list, seg_of_token, q_start, q_len, ctx_len, nh, nkv, page_size, num_pages, window, keep_first, \
-            softcap, scale, sink, gate, gate_stride, nsplit, parts);                                                                                \
+            softcap, scale, ex, nsplit, parts);                                                                                \
         if (nsplit > 1)                                                                                                    \
-            masked_attention_join_kernel<<<dim3(n_tokens, nh), dv >= 256 ? 256 : 128, 0, stream>>>(parts, (bf16_t*)out, token_list, nh, dv, nsplit, sink, gate, gate_stride); \
+            masked_attention_join_kernel<<<dim3(n_tokens, nh), dv >= 256 ? 256 : 128, 0, stream>>>(parts, (bf16_t*)out, token_list, nh, dv, nsplit, ex); \
         return li_launch_status();                                                                                         \
     }
     MH_GO(64, 64) MH_GO(128, 128) MH_GO(128, 64) MH_GO(64, 128) MH_GO(96, 64) MH_GO(160, 128) MH_GO(192, 128)
@@ -789,7 +823,7 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ token_list,
     const int* __restrict__ seg_of_token, const int* __restrict__ q_start, const int* __restrict__ q_len,
     const int* __restrict__ ctx_len, int nh, int nkv, int dk, int dv, int page_size, int num_pages, int window,
-    int keep_first, float softcap, float scale, const float* __restrict__ sink, const float* __restrict__ gate, long gate_stride, int tab_cap, int pshift, int nsplit, float* __restrict__ parts) {
+    int keep_first, float softcap, float scale, MaExtras ex, int tab_cap, int pshift, int nsplit, float* __restrict__ parts) {
     extern __shared__ float join[];                 // [4 waves][RH][dv + 2], then tab_cap table entries
     int* tab = (int*)(join + (size_t)4 * RH * (dv + 2));
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, g = lane >> 3, j = lane & 7;
@@ -845,13 +879,18 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
     // later use wait for all loads)
     size_t ro[U];
     bool ok[U];
+    int kpos[U];                                    // the keys' positions
     uint4 kp[U][NPK], vp[U][NPV];
-#define MS_ROWS(I0, RO, OK)                                                                                          \
+    float slope[RH];
+#pragma unroll
+    for (int hh = 0; hh < RH; ++hh) slope[hh] = (ex.slopes && hh < nheads) ? ex.slopes[kvh * rep + hfirst + hh] : 0.f;
+#define MS_ROWS(I0, RO, OK, KPOS)                                                                                          \
     _Pragma("unroll") for (int u = 0; u < U; ++u) {                                                                  \
         const int i = (I0) + 32 * u + 8 * w + g;                                                                     \
         OK[u] = i < n_keys;                                                                                          \
         const int ii = OK[u] ? i : 0;                                                                                \
         const int key = visible_key(ii, n_first, lo);                                                                \
+        KPOS[u] = key;                                                                                               \
         const int blk = pshift >= 0 ? key >> pshift : key / page_size;                                               \
         const int page = in_lds ? tab[ii < n_first ? nb_w + blk : blk - b_lo] : table[blk];                          \
         OK[u] = OK[u] && page >= 0 && page < num_pages;                                                              \
@@ -868,13 +907,14 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
             VP[u][c] = *reinterpret_cast<const uint4*>(vc + RO[u] * v_row + (d0 < dv ? d0 : 0));                     \
         }                                                                                                            \
     }
-    MS_ROWS(i_begin, ro, ok)
+    MS_ROWS(i_begin, ro, ok, kpos)
     MS_FETCH(ro, kp, vp)
     for (int i0 = i_begin; i0 < n_keys; i0 += 32 * U) {
         size_t ro2[U];
         bool ok2[U];
+        int kpos2[U];
         uint4 kp2[U][NPK], vp2[U][NPV];
-        MS_ROWS(i0 + 32 * U, ro2, ok2)
+        MS_ROWS(i0 + 32 * U, ro2, ok2, kpos2)
         MS_FETCH(ro2, kp2, vp2)
         float sc[U][RH];
 #pragma unroll
@@ -891,6 +931,7 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
                     for (int e = 0; e < 8; ++e) d = fmaf(qr[hh][c][e], kf[c][e], d);      // (pieces past dk meet zeros of q)
                 d = sum_over_8_lanes(d) * scale;
                 if (softcap > 0.f) d = softcap * fast_tanh(d * inv_cap);
+                if (ex.slopes) d -= slope[hh] * (float)(p - kpos[u]);
                 sc[u][hh] = ok[u] ? d : -INFINITY;
             }
         }
@@ -926,6 +967,7 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             ok[u] = ok2[u];
+            kpos[u] = kpos2[u];
 #pragma unroll
             for (int c = 0; c < NPK; ++c) kp[u][c] = kp2[u][c];
 #pragma unroll
@@ -981,7 +1023,7 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
         }
         const int head = kvh * rep + hfirst + hh;
         if (nsplit == 1) {
-            out[((size_t)t * nh + head) * dv + d].bits = float_to_bf16(a * finish_factor(ll, mm, sink, gate, gate_stride, t, head));
+            out[((size_t)t * nh + head) * dv + d].bits = float_to_bf16(a * finish_factor(ll, mm, ex, t, head) * column_gate(ex, t, head, dv, d));
         } else {                                    // this split's sums, maximum and sum of weights: joined by the kernel behind
             float* part = parts + (((size_t)blockIdx.x * nh + head) * nsplit + sp) * (dv + 2);
             part[d] = a;
@@ -993,8 +1035,7 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
 // joins the splits of every (token, head) in split order: a block a (token, head)
 // (the parts of a token lie at its place in the list, or, with by_token, at its own number)
 __global__ void masked_attention_join_kernel(const float* __restrict__ parts, bf16_t* __restrict__ out,
-                                             const int* __restrict__ token_list, int nh, int dv, int nsplit, const float* __restrict__ sink,
-                                             const float* __restrict__ gate, long gate_stride, int by_token) {
+                                             const int* __restrict__ token_list, int nh, int dv, int nsplit, MaExtras ex, int by_token) {
     const int t = token_list ? token_list[blockIdx.x] : blockIdx.x, head = blockIdx.y;
     const float* base = parts + ((size_t)(by_token ? t : (int)blockIdx.x) * nh + head) * nsplit * (dv + 2);
     float mm = -INFINITY;
@@ -1007,7 +1048,7 @@ __global__ void masked_attention_join_kernel(const float* __restrict__ parts, bf
             a += r[d] * f;
             ll += r[dv + 1] * f;
         }
-        out[((size_t)t * nh + head) * dv + d].bits = float_to_bf16(a * finish_factor(ll, mm, sink, gate, gate_stride, t, head));
+        out[((size_t)t * nh + head) * dv + d].bits = float_to_bf16(a * finish_factor(ll, mm, ex, t, head) * column_gate(ex, t, head, dv, d));
     }
 }
 
@@ -1029,8 +1070,9 @@ extern "C" int li_masked_attention_single(const float* q, int q_token_stride, in
                                           const void* vc, int k_row, int v_row, const int* block_table, int max_blocks,
                                           const int* token_list, int n_tokens, const int* seg_of_token, const int* q_start,
                                           const int* q_len, const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size,
-                                          int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride,
+                                          int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes,
                                           int nsplit, float* parts, long parts_floats, hipStream_t stream) {
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
     if (n_tokens <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || nkv > 65535 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || num_pages <= 0 || k_row % 8 || v_row % 8 || q_token_stride % 4 ||
         q_head_stride % 4 || ((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) % 16 || !li_masked_attention_single_takes(dk, dv))
@@ -1050,10 +1092,10 @@ extern "C" int li_masked_attention_single(const float* q, int q_token_stride, in
     masked_attention_single_kernel<K, V, R, UU><<<grid, 256, lds, stream>>>(                                                \
         q, q_token_stride, q_head_stride, (bf16_t*)out, (const bf16_t*)kc, (const bf16_t*)vc, k_row, v_row, block_table,    \
         max_blocks, token_list, seg_of_token, q_start, q_len, ctx_len, nh, nkv, dk, dv, page_size, num_pages, window,       \
-        keep_first, softcap, scale, sink, gate, gate_stride, tab_cap, pshift, nsplit, parts)
+        keep_first, softcap, scale, ex, tab_cap, pshift, nsplit, parts)
 #define MS_JOIN                                                                                                             \
     if (nsplit > 1)                                                                                                         \
-        masked_attention_join_kernel<<<dim3(n_tokens, nh), dv >= 256 ? 256 : 128, 0, stream>>>(parts, (bf16_t*)out, token_list, nh, dv, nsplit, sink, gate, gate_stride);
+        masked_attention_join_kernel<<<dim3(n_tokens, nh), dv >= 256 ? 256 : 128, 0, stream>>>(parts, (bf16_t*)out, token_list, nh, dv, nsplit, ex);
 #define MS_SMALL(K, V)                                                                                                      \
     if (npk == K && npv == V) {                                                                                             \
         if (rh == 4) MS_GO(K, V, 4, 4); else if (rh == 2) MS_GO(K, V, 2, 4); else MS_GO(K, V, 1, 4);                        \
@@ -1078,7 +1120,8 @@ extern "C" int li_masked_attention_single(const float* q, int q_token_stride, in
 // ------------------------------------------------------------------------------------------- per-head products
 // out[t, h, j] = sum_k m[h, j, k] * x[t, h, k]: every head has a matrix of its own, [n_out, n_in], stored one after
 // the other.  x and out are addressed by a token stride and a head stride, so that a head's columns may lie inside
-// a wider row.  With `gate`, head h's outputs of token t are multiplied by sigmoid(gate[t * gate_stride + h]).
+// a wider row.  With `gate`, head h's outputs of token t are multiplied by sigmoid(gate[t * gate_stride + h]), or, with
+// gate_per_column, output j of head h by sigmoid(gate[t * gate_stride + h * n_out + j]).
 // A block takes one head, HL_TOK tokens and 256 outputs: the tokens' inputs lie in LDS as float32, a
 // thread owns an output and reads its matrix row once for all the tokens.  Sums are float32, in the order of k.
 #define HL_TOK 8
@@ -1101,7 +1144,7 @@ template <typename TX, typename TM, typename TO, bool VEC>
 __global__ __launch_bounds__(256) void headwise_linear_kernel(
     const TX* __restrict__ x, long x_token_stride, int x_head_stride, const TM* __restrict__ m, TO* __restrict__ out,
     long o_token_stride, int o_head_stride, int T_, int n_out, int n_in, const float* __restrict__ gate, long gate_stride,
-    HeadTail tail) {
+    int gate_per_column, HeadTail tail) {
     extern __shared__ float xs[];                    // [HL_TOK][n_in]
     const int h = blockIdx.y, t0 = blockIdx.x * HL_TOK;
     const int nt = (T_ - t0 < HL_TOK) ? T_ - t0 : HL_TOK;
@@ -1118,7 +1161,7 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(
     // the heads' gates are asked for before the products, so that they have arrived when the outputs are ready
     float gf[HL_TOK];
 #pragma unroll
-    for (int tt = 0; tt < HL_TOK; ++tt) gf[tt] = gate ? gate[(size_t)(t0 + (tt < nt ? tt : 0)) * gate_stride + h] : 0.f;
+    for (int tt = 0; tt < HL_TOK; ++tt) gf[tt] = gate && !gate_per_column ? gate[(size_t)(t0 + (tt < nt ? tt : 0)) * gate_stride + h] : 0.f;
     __syncthreads();
     // four neighbouring threads share an output: each takes every fourth piece of the matrix row
     constexpr int E = VEC ? 16 / (int)sizeof(TM) : 1;
@@ -1159,7 +1202,8 @@ __global__ __launch_bounds__(256) void headwise_linear_kernel(
         }
         if (on && part == 0)
             for (int tt = 0; tt < nt; ++tt) {
-                const float f = gate ? 1.0f / (1.0f + expf(-gf[tt])) : 1.0f;
+                const float gv = gate_per_column ? gate[(size_t)(t0 + tt) * gate_stride + (size_t)h * n_out + j] : gf[tt];
+                const float f = gate ? 1.0f / (1.0f + expf(-gv)) : 1.0f;
                 store_from_float(out + (size_t)(t0 + tt) * o_token_stride + (size_t)h * o_head_stride + j, acc[tt] * f);
             }
     }
@@ -1173,7 +1217,7 @@ template <typename TX, typename TO>
 __global__ __launch_bounds__(256) void headwise_linear_mfma_kernel(
     const TX* __restrict__ x, long x_token_stride, int x_head_stride, const bf16_t* __restrict__ m, TO* __restrict__ out,
     long o_token_stride, int o_head_stride, int T_, int n_out, int n_in, const float* __restrict__ gate, long gate_stride,
-    HeadTail tail) {
+    int gate_per_column, HeadTail tail) {
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, ql = lane & 31, h2 = lane >> 5;
     const int head = blockIdx.y, t0 = blockIdx.x * 32;
     if (tail.n > 0 && blockIdx.z == 0) {
@@ -1206,7 +1250,17 @@ __global__ __launch_bounds__(256) void headwise_linear_mfma_kernel(
         acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a.v, b.v, acc, 0, 0, 0);
     }
     if (t0 + ql >= T_) return;
-    if (gate) {
+    if (gate && gate_per_column) {                 // (a lane's outputs come in fours: 16-byte pieces of the gates' row)
+        const float* grow = gate + (size_t)(t0 + ql) * gate_stride + (size_t)head * n_out + j0 + 4 * h2;
+#pragma unroll
+        for (int rg = 0; rg < 4; ++rg) {
+            const float4 g = *reinterpret_cast<const float4*>(grow + 8 * rg);
+            acc[4 * rg] *= 1.0f / (1.0f + expf(-g.x));
+            acc[4 * rg + 1] *= 1.0f / (1.0f + expf(-g.y));
+            acc[4 * rg + 2] *= 1.0f / (1.0f + expf(-g.z));
+            acc[4 * rg + 3] *= 1.0f / (1.0f + expf(-g.w));
+        }
+    } else if (gate) {
         const float f = 1.0f / (1.0f + expf(-gate[(size_t)(t0 + ql) * gate_stride + head]));
 #pragma unroll
         for (int r = 0; r < 16; ++r) acc[r] *= f;
@@ -1227,31 +1281,33 @@ __global__ __launch_bounds__(256) void headwise_linear_mfma_kernel(
 
 template <typename TX, typename TO>
 static bool headwise_mfma(const void* x, long xts, int xhs, const void* m, void* out, long ots, int ohs, int T_, int nh,
-                          int n_out, int n_in, const float* gate, long gate_stride, HeadTail tail, hipStream_t stream) {
+                          int n_out, int n_in, const float* gate, long gate_stride, int gate_per_column, HeadTail tail, hipStream_t stream) {
     const int ex = 16 / (int)sizeof(TX) / 2 * 2, eo = 4;       // elements that the 16-byte (32-byte) loads and the stores must start on
     if (T_ < 16 || n_in % 16 || n_out % 32 || xts % ex || xhs % ex || ots % eo || ohs % eo ||
-        (uintptr_t)x % 16 || (uintptr_t)m % 16 || (uintptr_t)out % 16)
+        (uintptr_t)x % 16 || (uintptr_t)m % 16 || (uintptr_t)out % 16 ||
+        (gate && gate_per_column && (gate_stride % 4 || (uintptr_t)gate % 16)))
         return false;
     const dim3 grid((T_ + 31) / 32, nh, (n_out + 127) / 128);
     headwise_linear_mfma_kernel<TX, TO><<<grid, 256, 0, stream>>>((const TX*)x, xts, xhs, (const bf16_t*)m, (TO*)out, ots, ohs,
-                                                                  T_, n_out, n_in, gate, gate_stride, tail);
+                                                                  T_, n_out, n_in, gate, gate_stride, gate_per_column, tail);
     return true;
 }
 
 extern "C" int li_headwise_linear(const void* x, int x_dtype, long x_token_stride, int x_head_stride, const void* m, int m_dtype,
                                   void* out, int out_dtype, long o_token_stride, int o_head_stride, int T_, int nh, int n_out,
-                                  int n_in, const float* gate, long gate_stride, int tail_n, int tail_split, const float* cosv,
+                                  int n_in, const float* gate, long gate_stride, int gate_per_column, int tail_n, int tail_split, const float* cosv,
                                   const float* sinv, hipStream_t stream) {
-    if (T_ <= 0 || nh <= 0 || nh > 65535 || n_out <= 0 || n_in <= 0 || n_in > 2048 || (gate && gate_stride < nh)) return LI_ERR_SIZE;
+    if (T_ <= 0 || nh <= 0 || nh > 65535 || n_out <= 0 || n_in <= 0 || n_in > 2048 || (gate && gate_stride < (gate_per_column ? (long)nh * n_out : nh))) return LI_ERR_SIZE;
     if (tail_n < 0 || (tail_n & 1) || (tail_n > 0 && (!cosv || !sinv || o_head_stride < n_out + tail_n))) return LI_ERR_SIZE;
+    if (!gate) gate_per_column = 0;
     const HeadTail tail{tail_n, tail_split, cosv, sinv};
     // many tokens against bfloat16 matrices of even sizes: the matrix cores
     if (m_dtype == LI_BF16) {
         bool took = false;
-        if (x_dtype == LI_F32 && out_dtype == LI_F32) took = headwise_mfma<float, float>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, tail, stream);
-        else if (x_dtype == LI_F32 && out_dtype == LI_BF16) took = headwise_mfma<float, bf16_t>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, tail, stream);
-        else if (x_dtype == LI_BF16 && out_dtype == LI_BF16) took = headwise_mfma<bf16_t, bf16_t>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, tail, stream);
-        else if (x_dtype == LI_BF16 && out_dtype == LI_F32) took = headwise_mfma<bf16_t, float>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, tail, stream);
+        if (x_dtype == LI_F32 && out_dtype == LI_F32) took = headwise_mfma<float, float>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, gate_per_column, tail, stream);
+        else if (x_dtype == LI_F32 && out_dtype == LI_BF16) took = headwise_mfma<float, bf16_t>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, gate_per_column, tail, stream);
+        else if (x_dtype == LI_BF16 && out_dtype == LI_BF16) took = headwise_mfma<bf16_t, bf16_t>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, gate_per_column, tail, stream);
+        else if (x_dtype == LI_BF16 && out_dtype == LI_F32) took = headwise_mfma<bf16_t, float>(x, x_token_stride, x_head_stride, m, out, o_token_stride, o_head_stride, T_, nh, n_out, n_in, gate, gate_stride, gate_per_column, tail, stream);
         if (took) return li_launch_status();
     }
     const int zs = (n_out + 63) / 64;
@@ -1262,10 +1318,10 @@ extern "C" int li_headwise_linear(const void* x, int x_dtype, long x_token_strid
         constexpr int E = 16 / sizeof(TM);                                                                                 \
         if (n_in % E == 0 && ((uintptr_t)m % 16) == 0)                                                                     \
             headwise_linear_kernel<TX, TM, TO, true><<<grid, 256, lds, stream>>>(                                          \
-                (const TX*)x, x_token_stride, x_head_stride, (const TM*)m, (TO*)out, o_token_stride, o_head_stride, T_, n_out, n_in, gate, gate_stride, tail); \
+                (const TX*)x, x_token_stride, x_head_stride, (const TM*)m, (TO*)out, o_token_stride, o_head_stride, T_, n_out, n_in, gate, gate_stride, gate_per_column, tail); \
         else                                                                                                               \
             headwise_linear_kernel<TX, TM, TO, false><<<grid, 256, lds, stream>>>(                                         \
-                (const TX*)x, x_token_stride, x_head_stride, (const TM*)m, (TO*)out, o_token_stride, o_head_stride, T_, n_out, n_in, gate, gate_stride, tail); \
+                (const TX*)x, x_token_stride, x_head_stride, (const TM*)m, (TO*)out, o_token_stride, o_head_stride, T_, n_out, n_in, gate, gate_stride, gate_per_column, tail); \
         return li_launch_status();                                                                                         \
     }
     if (x_dtype == LI_F32 && m_dtype == LI_F32 && out_dtype == LI_F32) HL_GO(float, float, float)

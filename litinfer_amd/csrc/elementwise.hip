@@ -5,13 +5,13 @@
 #include "common.h"
 
 // ---------------------------------------------------------------- embedding
-// out[t, :] = float(table[id(t), :])  (row copy, no scaling), with id(t) = ids[t], or, where
+// out[t, :] = scale * float(table[id(t), :])  (scale 1: a row copy), with id(t) = ids[t], or, where
 // id_src is given and id_src[t] >= 0, feedback[id_src[t]]: a token that an earlier kernel on the
 // stream chose and the host has not seen yet.
 template <typename T>
 __global__ void embedding_kernel(const int* __restrict__ ids, const int* __restrict__ id_src,
                                  const int* __restrict__ feedback, const T* __restrict__ table,
-                                 float* __restrict__ out, int H, int V) {
+                                 float* __restrict__ out, int H, int V, float scale) {
     const int t = blockIdx.x;
     int id = ids[t];
     if (id_src) {
@@ -24,16 +24,16 @@ __global__ void embedding_kernel(const int* __restrict__ ids, const int* __restr
         return;
     }
     const T* row = table + (size_t)id * H;
-    for (int j = threadIdx.x; j < H; j += blockDim.x) o[j] = load_as_float(row + j);
+    for (int j = threadIdx.x; j < H; j += blockDim.x) o[j] = scale * load_as_float(row + j);
 }
 
 extern "C" int li_embedding(const int* ids, const int* id_src, const int* feedback, const void* table,
-                            int table_dtype, float* out, int T, int H, int V, hipStream_t stream) {
+                            int table_dtype, float* out, int T, int H, int V, float scale, hipStream_t stream) {
     if (T <= 0 || H <= 0 || (id_src && !feedback)) return LI_ERR_SIZE;
     if (table_dtype == LI_F32)
-        embedding_kernel<float><<<T, 256, 0, stream>>>(ids, id_src, feedback, (const float*)table, out, H, V);
+        embedding_kernel<float><<<T, 256, 0, stream>>>(ids, id_src, feedback, (const float*)table, out, H, V, scale);
     else if (table_dtype == LI_BF16)
-        embedding_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, id_src, feedback, (const bf16_t*)table, out, H, V);
+        embedding_kernel<bf16_t><<<T, 256, 0, stream>>>(ids, id_src, feedback, (const bf16_t*)table, out, H, V, scale);
     else return LI_ERR_DTYPE;
     return li_launch_status();
 }
@@ -697,13 +697,82 @@ extern "C" int li_qk_norm_pairs_store(float* qkv, int row_stride, int nh, int nk
     return li_launch_status();
 }
 
+// The same step for a mixer that norms every query head and every key head BY ITSELF, with one weight vector of dk
+// values for all query heads (wq) and one for all key heads (wk): rows [q | k | v], or, with keys_are_values, rows
+// [q | k], where the value of a token is its key as projected, before the norm.  A wave a (token, head).
+template <typename T>
+__global__ __launch_bounds__(256) void qk_head_norm_store_kernel(
+    float* __restrict__ qkv, long row_stride, int nh, int nkv, int dk, int dv, int rotary_dim,
+    const float* __restrict__ wq, const float* __restrict__ wk, float eps,
+    const float* __restrict__ cosv, const float* __restrict__ sinv, const int* __restrict__ slot_map,
+    T* __restrict__ kc, T* __restrict__ vc, int page_size, int store, int half_split, int keys_are_values) {
+    const int t = blockIdx.x, lane = threadIdx.x & 63, unit = blockIdx.y * 4 + (threadIdx.x >> 6);
+    const int units = nh + (store ? (keys_are_values ? nkv : 2 * nkv) : 0);
+    if (unit >= units) return;
+    float* row = qkv + (size_t)t * row_stride;
+    const bool is_q = unit < nh;
+    const int head = is_q ? unit : (unit - nh) % nkv;
+    const int slot = is_q ? 0 : slot_map[t], page = slot / page_size, off = slot % page_size;
+    const size_t crow = (size_t)(page * nkv + head) * page_size + off;
+    if (unit >= nh + nkv) {                                // a head of separate values
+        const float* v = row + (size_t)(nh + nkv) * dk + (size_t)head * dv;
+        for (int d = lane; d < dv; d += LI_WAVE) store_from_float(vc + crow * dv + d, v[d]);
+        return;
+    }
+    float* x = row + (size_t)unit * dk;                    // (the key heads lie behind the query heads)
+    const float* w = is_q ? wq : wk;
+    float ss = 0.f;
+    for (int d = lane; d < dk; d += LI_WAVE) {
+        const float v = x[d];
+        ss += v * v;
+        if (!is_q && keys_are_values) store_from_float(vc + crow * dv + d, v);
+    }
+    ss = wave_sum(ss);
+    const float inv = 1.0f / sqrtf(ss / (float)dk + eps);
+    const int half = rotary_dim / 2, pieces = half + (dk - rotary_dim);      // the pairs, then the columns that are not rotated
+    for (int i = lane; i < pieces; i += LI_WAVE) {
+        if (i < half) {
+            const int d1 = half_split ? i : 2 * i, d2 = half_split ? i + half : 2 * i + 1;
+            float ra, rb;
+            rotate_pair(x[d1] * inv * w[d1], x[d2] * inv * w[d2], cosv[(size_t)t * half + i], sinv[(size_t)t * half + i], ra, rb);
+            if (is_q) { x[d1] = ra; x[d2] = rb; }
+            else { store_from_float(kc + crow * dk + d1, ra); store_from_float(kc + crow * dk + d2, rb); }
+        } else {
+            const int d = rotary_dim + (i - half);
+            const float v = x[d] * inv * w[d];
+            if (is_q) x[d] = v; else store_from_float(kc + crow * dk + d, v);
+        }
+    }
+}
+
+extern "C" int li_qk_head_norm_store(float* qkv, long row_stride, int nh, int nkv, int dk, int dv, int rotary_dim,
+                                     const float* wq, const float* wk, float eps, const float* cosv, const float* sinv,
+                                     const int* slot_map, void* kc, void* vc, int cache_dtype, int page_size, int store,
+                                     int half_split, int keys_are_values, int T, hipStream_t stream) {
+    if (T <= 0 || nh <= 0 || nkv <= 0 || dk <= 0 || dv <= 0 || rotary_dim < 0 || (rotary_dim & 1) || rotary_dim > dk || !wq || !wk ||
+        (keys_are_values && dv != dk) || row_stride < (long)nh * dk + (long)nkv * (keys_are_values ? dk : dk + dv) || page_size <= 0 ||
+        (rotary_dim > 0 && (!cosv || !sinv)) || (store && (!slot_map || !kc || !vc)))
+        return LI_ERR_SIZE;
+    const int units = nh + (store ? (keys_are_values ? nkv : 2 * nkv) : 0);
+    if ((units + 3) / 4 > 65535) return LI_ERR_SIZE;
+    const dim3 grid(T, (units + 3) / 4);
+    if (cache_dtype == LI_F32)
+        qk_head_norm_store_kernel<float><<<grid, 256, 0, stream>>>(qkv, row_stride, nh, nkv, dk, dv, rotary_dim, wq, wk, eps, cosv, sinv,
+                                                                   slot_map, (float*)kc, (float*)vc, page_size, store, half_split, keys_are_values);
+    else if (cache_dtype == LI_BF16)
+        qk_head_norm_store_kernel<bf16_t><<<grid, 256, 0, stream>>>(qkv, row_stride, nh, nkv, dk, dv, rotary_dim, wq, wk, eps, cosv, sinv,
+                                                                    slot_map, (bf16_t*)kc, (bf16_t*)vc, page_size, store, half_split, keys_are_values);
+    else return LI_ERR_DTYPE;
+    return li_launch_status();
+}
+
 // The same step for attention over a compressed cache.  `q` (float32 rows, may be absent: nh = 0) holds nh heads of
 // (dn + dr) columns, the last dr of each rotated; `down` (float32 rows, which may lie inside the same buffer) holds
 // `rank` latent columns and dr columns of one rotated key part that all heads share.  The latent is RMS-normed
 // (weights wc) and written to columns 0..rank-1 of the token's page row, the rotated shared part behind it; the
 // rotated part of every query head goes to columns rank.. of that head's row in `qfull` (float32 rows of
 // nh x (rank + dr): the first `rank` columns are filled by the product with the keys' expansion matrix afterwards).
-// `split`: 0 pairs neighbouring columns (2i, 2i + 1), 1 pairs column i with column i + dr/2.
+// `split`: 0 pairs neighbouring columns (2i, 2i + 1), 1 pairs column i with column i + dr/2.  dr may be 0: no positions.
 // Where the queries go through a latent of their own, `ql` holds its q_rank columns before the norm and `cq` takes
 // the RMS norm with weights wq (in the dtype of the product that follows).
 template <typename T, typename TQ, int NT>
@@ -759,7 +828,7 @@ extern "C" int li_latent_norm_pairs_store(const float* q, long q_stride, int nh,
                                           const float* sinv, const int* slot_map, void* cache, int cache_dtype, float* qfull,
                                           int store, int split, const float* ql, long ql_stride, int q_rank, const float* wq,
                                           void* cq, int cq_dtype, int T, hipStream_t stream) {
-    if (T <= 0 || nh < 0 || dn < 0 || dr <= 0 || (dr & 1) || rank <= 0 || q_rank < 0) return LI_ERR_SIZE;
+    if (T <= 0 || nh < 0 || dn < 0 || dr < 0 || (dr & 1) || rank <= 0 || q_rank < 0 || (dr > 0 && (!cosv || !sinv))) return LI_ERR_SIZE;
     if ((nh > 0 && (!q || !qfull || q_stride < (long)nh * (dn + dr))) || (store && (!down || !cache || !slot_map || down_stride < rank + dr)) ||
         (q_rank > 0 && (!ql || !wq || !cq || ql_stride < q_rank)))
         return LI_ERR_SIZE;
@@ -1032,6 +1101,230 @@ extern "C" int li_concat_rows(const float* a, const float* b, void* out, int out
     if (T <= 0 || H <= 0) return LI_ERR_SIZE;
     if (out_dtype == LI_F32) concat_rows_kernel<float><<<T, 256, 0, stream>>>(a, b, (float*)out, H);
     else if (out_dtype == LI_BF16) concat_rows_kernel<bf16_t><<<T, 256, 0, stream>>>(a, b, (bf16_t*)out, H);
+    else return LI_ERR_DTYPE;
+    return li_launch_status();
+}
+
+// ============================================================================================
+// Several residual streams with learned mixing (hyper-connections), and element-wise steps: xIELU, tanh.
+// ============================================================================================
+
+// A token's residual is `n` streams x_0 .. x_{n-1}, rows of H float32 values one behind the other ([T, n, H]).  One
+// kernel takes what a sublayer put out and prepares the next sublayer's input:
+//   write:  b = a1 y (+ a2 y2),  x_t <- sum_s mix[s, t] x_s + out[t] b   (every stream from the old ones);
+//   read:   u = sum_s win[s] x_s of the (new) streams, xn = w * u / sqrt(mean(u^2) + eps).
+// Either may be absent.  src_streams 1: all streams are equal to the one row of `src` (the start of a step).  A block a
+// token; pieces of V values (16 bytes where the rows allow it); u stays in registers, up to PER pieces a thread.
+template <int V> struct hyper_piece { float v[V]; };
+template <int V> __device__ __forceinline__ hyper_piece<V> hyper_load(const float* p) {
+    hyper_piece<V> r;
+    if constexpr (V == 4) {
+        const float4 f = *reinterpret_cast<const float4*>(p);
+        r.v[0] = f.x; r.v[1] = f.y; r.v[2] = f.z; r.v[3] = f.w;
+    } else r.v[0] = p[0];
+    return r;
+}
+template <int V> __device__ __forceinline__ void hyper_store(float* p, const hyper_piece<V>& r) {
+    if constexpr (V == 4) *reinterpret_cast<float4*>(p) = float4{r.v[0], r.v[1], r.v[2], r.v[3]};
+    else p[0] = r.v[0];
+}
+
+template <typename TO, int S, int V, int NT, int PER>
+__global__ __launch_bounds__(NT) void hyper_step_kernel(
+    const float* src, int src_streams, float* dst, const float* __restrict__ y, const float* __restrict__ y2, float a1, float a2,
+    const float* __restrict__ mix, const float* __restrict__ outw, const float* __restrict__ win, const float* __restrict__ w,
+    float eps, TO* __restrict__ xn, int n, int H) {
+    __shared__ float red[NT / LI_WAVE];
+    const size_t t = blockIdx.x;
+    const float* xr = src + t * (size_t)src_streams * H;
+    const long xs = src_streams > 1 ? H : 0;               // from one stream's row to the next
+    float* xo = dst + t * (size_t)n * H;
+    const float* yr = y + t * (size_t)H;
+    const float* yr2 = y2 ? y2 + t * (size_t)H : nullptr;
+    const int np = H / V;
+    hyper_piece<V> u[PER];
+    float ss = 0.f;
+    // the piece at column j: read the old streams, write the new ones, and return the next reader's sum
+    auto piece = [&](int j) {
+        hyper_piece<V> x[S];
+#pragma unroll
+        for (int s = 0; s < S; ++s)
+            if (s < n) x[s] = hyper_load<V>(xr + s * xs + j);
+        hyper_piece<V> uu;
+#pragma unroll
+        for (int e = 0; e < V; ++e) uu.v[e] = 0.f;
+        if (mix) {
+            hyper_piece<V> b = hyper_load<V>(yr + j);
+#pragma unroll
+            for (int e = 0; e < V; ++e) b.v[e] *= a1;
+            if (yr2) {
+                const hyper_piece<V> b2 = hyper_load<V>(yr2 + j);
+#pragma unroll
+                for (int e = 0; e < V; ++e) b.v[e] = fmaf(a2, b2.v[e], b.v[e]);
+            }
+#pragma unroll
+            for (int to = 0; to < S; ++to)
+                if (to < n) {
+                    hyper_piece<V> z;
+#pragma unroll
+                    for (int e = 0; e < V; ++e) z.v[e] = outw[to] * b.v[e];
+#pragma unroll
+                    for (int s = 0; s < S; ++s)
+                        if (s < n) {
+                            const float m = mix[s * n + to];
+#pragma unroll
+                            for (int e = 0; e < V; ++e) z.v[e] = fmaf(m, x[s].v[e], z.v[e]);
+                        }
+                    hyper_store<V>(xo + (size_t)to * H + j, z);
+                    if (win) {
+#pragma unroll
+                        for (int e = 0; e < V; ++e) uu.v[e] = fmaf(win[to], z.v[e], uu.v[e]);
+                    }
+                }
+        } else {
+#pragma unroll
+            for (int s = 0; s < S; ++s)
+                if (s < n) {
+#pragma unroll
+                    for (int e = 0; e < V; ++e) uu.v[e] = fmaf(win[s], x[s].v[e], uu.v[e]);
+                }
+        }
+        return uu;
+    };
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int p = threadIdx.x + i * NT;
+        if (p < np) {
+            u[i] = piece(p * V);
+#pragma unroll
+            for (int e = 0; e < V; ++e) ss = fmaf(u[i].v[e], u[i].v[e], ss);
+        }
+    }
+    for (int p = threadIdx.x + PER * NT; p < np; p += NT) {
+        const hyper_piece<V> r = piece(p * V);
+#pragma unroll
+        for (int e = 0; e < V; ++e) ss = fmaf(r.v[e], r.v[e], ss);
+    }
+    if (!win) return;
+    ss = block_sum<NT>(ss, red);
+    const float inv = 1.0f / sqrtf(ss / (float)H + eps);
+    TO* o = xn + t * (size_t)H;
+    auto finish = [&](int j, const hyper_piece<V>& r) {
+        if constexpr (V == 4) {
+            const float4 g = *reinterpret_cast<const float4*>(w + j);
+            const float o0 = g.x * r.v[0] * inv, o1 = g.y * r.v[1] * inv, o2 = g.z * r.v[2] * inv, o3 = g.w * r.v[3] * inv;
+            if constexpr (sizeof(TO) == 2) *reinterpret_cast<uint2*>(o + j) = uint2{pack2_bf16(o0, o1), pack2_bf16(o2, o3)};
+            else *reinterpret_cast<float4*>(o + j) = float4{o0, o1, o2, o3};
+        } else {
+            store_from_float(o + j, w[j] * r.v[0] * inv);
+        }
+    };
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int p = threadIdx.x + i * NT;
+        if (p < np) finish(p * V, u[i]);
+    }
+    for (int p = threadIdx.x + PER * NT; p < np; p += NT) {          // long rows: the sum once more, from what this thread left
+        const int j = p * V;
+        hyper_piece<V> r;
+#pragma unroll
+        for (int e = 0; e < V; ++e) r.v[e] = 0.f;
+        for (int s = 0; s < n; ++s) {
+            const hyper_piece<V> x = hyper_load<V>(mix ? xo + (size_t)s * H + j : xr + s * xs + j);
+#pragma unroll
+            for (int e = 0; e < V; ++e) r.v[e] = fmaf(win[s], x.v[e], r.v[e]);
+        }
+        finish(j, r);
+    }
+}
+
+extern "C" int li_hyper_step(const float* src, int src_streams, float* dst, const float* y, const float* y2, float a1, float a2,
+                             const float* mix, const float* outw, const float* win, const float* w, float eps, void* xn,
+                             int xn_dtype, int n, int T, int H, hipStream_t stream) {
+    if (T <= 0 || H <= 0 || n <= 0 || n > 16 || !src || (src_streams != 1 && src_streams != n) || (!mix && !win) ||
+        (mix && (!dst || !y || !outw)) || (win && (!w || !xn)))
+        return LI_ERR_SIZE;
+    const uintptr_t all = (uintptr_t)src | (uintptr_t)dst | (uintptr_t)y | (uintptr_t)y2 | (uintptr_t)w | (uintptr_t)xn;
+    const bool vec = H % 4 == 0 && all % 16 == 0;
+    const bool wide = T < 256 && H > 1024;                  // few rows (a decoding step): one piece a thread
+#define HY_GO(TO, S_, V_, NT_, PER_)                                                                                           hyper_step_kernel<TO, S_, V_, NT_, PER_><<<T, NT_, 0, stream>>>(src, src_streams, dst, y, y2, a1, a2, mix, outw, win, w, eps, (TO*)xn, n, H)
+#define HY_S(TO, S_)                                                                                                           {                                                                                                                              if (vec) { if (wide) HY_GO(TO, S_, 4, 1024, 2); else HY_GO(TO, S_, 4, 256, 4); }                                           else HY_GO(TO, S_, 1, 256, 4);                                                                                             return li_launch_status();                                                                                             }
+#define HY_T(TO)                                                                                                               {                                                                                                                              if (n == 1) HY_S(TO, 1) if (n == 2) HY_S(TO, 2) if (n == 3) HY_S(TO, 3) if (n == 4) HY_S(TO, 4)                            if (n <= 8) HY_S(TO, 8) HY_S(TO, 16)                                                                                   }
+    if (!win || xn_dtype == LI_F32) HY_T(float)
+    if (xn_dtype == LI_BF16) HY_T(bf16_t)
+#undef HY_T
+#undef HY_S
+#undef HY_GO
+    return LI_ERR_DTYPE;
+}
+
+// out[i, :] = the sum of the n streams of token rows[i] (rows null: of token i)
+__global__ void stream_sum_kernel(const float* __restrict__ x, const int* __restrict__ rows, float* __restrict__ out, int n, int H) {
+    const int i = blockIdx.x;
+    const float* xr = x + (size_t)(rows ? rows[i] : i) * n * H;
+    for (int j = threadIdx.x; j < H; j += blockDim.x) {
+        float s = 0.f;
+        for (int k = 0; k < n; ++k) s += xr[(size_t)k * H + j];
+        out[(size_t)i * H + j] = s;
+    }
+}
+
+extern "C" int li_stream_sum(const float* x, const int* rows, float* out, int num, int n, int H, hipStream_t stream) {
+    if (num <= 0 || n <= 0 || H <= 0) return LI_ERR_SIZE;
+    stream_sum_kernel<<<num, 256, 0, stream>>>(x, rows, out, n, H);
+    return li_launch_status();
+}
+
+// xIELU with two numbers worked out by the caller, sp = softplus(p) and sq = 1/2 + softplus(q):
+// z > 0: sp z^2 + z / 2;  z <= 0: sq (exp(z) - 1 - z) + z / 2
+__device__ __forceinline__ float xielu(float z, float sp, float sq) {
+    return (z > 0.f ? sp * z * z : sq * (expm1f(z) - z)) + 0.5f * z;
+}
+template <typename TI, typename TO>
+__global__ void xielu_kernel(const TI* __restrict__ x, TO* __restrict__ out, long n, float sp, float sq) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) store_from_float(out + i, xielu(load_as_float(x + i), sp, sq));
+}
+// four float32 values a thread
+template <typename TO>
+__global__ void xielu_vec_kernel(const float* __restrict__ x, TO* __restrict__ out, long n4, float sp, float sq) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i >= n4) return;
+    const float4 v = reinterpret_cast<const float4*>(x)[i];
+    const float a = xielu(v.x, sp, sq), b = xielu(v.y, sp, sq), c = xielu(v.z, sp, sq), d = xielu(v.w, sp, sq);
+    if constexpr (sizeof(TO) == 2) reinterpret_cast<uint2*>(out)[i] = uint2{pack2_bf16(a, b), pack2_bf16(c, d)};
+    else reinterpret_cast<float4*>(out)[i] = float4{a, b, c, d};
+}
+
+extern "C" int li_xielu(const void* x, int x_dtype, void* out, int out_dtype, long n, float sp, float sq, hipStream_t stream) {
+    if (n <= 0) return LI_ERR_SIZE;
+    if (x_dtype == LI_F32 && n % 4 == 0 && ((uintptr_t)x | (uintptr_t)out) % 16 == 0) {
+        const unsigned blocks = (unsigned)((n / 4 + 255) / 256);
+        if (out_dtype == LI_F32) xielu_vec_kernel<float><<<blocks, 256, 0, stream>>>((const float*)x, (float*)out, n / 4, sp, sq);
+        else if (out_dtype == LI_BF16) xielu_vec_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const float*)x, (bf16_t*)out, n / 4, sp, sq);
+        else return LI_ERR_DTYPE;
+        return li_launch_status();
+    }
+    const unsigned blocks = (unsigned)((n + 255) / 256);
+    if (x_dtype == LI_F32 && out_dtype == LI_F32) xielu_kernel<float, float><<<blocks, 256, 0, stream>>>((const float*)x, (float*)out, n, sp, sq);
+    else if (x_dtype == LI_F32 && out_dtype == LI_BF16) xielu_kernel<float, bf16_t><<<blocks, 256, 0, stream>>>((const float*)x, (bf16_t*)out, n, sp, sq);
+    else if (x_dtype == LI_BF16 && out_dtype == LI_BF16) xielu_kernel<bf16_t, bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, n, sp, sq);
+    else return LI_ERR_DTYPE;
+    return li_launch_status();
+}
+
+// out[t, j] = tanh(x[t, j]) for n columns of float32 rows that lie inside wider ones
+template <typename TO>
+__global__ void tanh_rows_kernel(const float* __restrict__ x, long stride, TO* __restrict__ out, int T, int n) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < (long)T * n) store_from_float(out + i, tanhf(x[(i / n) * stride + i % n]));
+}
+
+extern "C" int li_tanh_rows(const float* x, long stride, void* out, int out_dtype, int T, int n, hipStream_t stream) {
+    if (T <= 0 || n <= 0 || stride < n) return LI_ERR_SIZE;
+    const unsigned blocks = (unsigned)(((long)T * n + 255) / 256);
+    if (out_dtype == LI_F32) tanh_rows_kernel<float><<<blocks, 256, 0, stream>>>(x, stride, (float*)out, T, n);
+    else if (out_dtype == LI_BF16) tanh_rows_kernel<bf16_t><<<blocks, 256, 0, stream>>>(x, stride, (bf16_t*)out, T, n);
     else return LI_ERR_DTYPE;
     return li_launch_status();
 }

@@ -2,7 +2,7 @@
 // per channel with its tail of past inputs, the selective state-space recurrence
 //   S_t = a_t S_{t-1} + dt_t B_t x_t^T,  y_t = S_t^T C_t + D x_t,  a_t = exp(-exp(A_log) dt_t),
 // (with `fixed_a`: a_t = fixed_a[head] and dt_t = fixed_dt for every token, a retention with a decay a head),
-// the gated delta rule, and the gated RMS norm in groups of columns behind them.  Everything here is float32: inputs, decays,
+// the gated delta rule, the delta rule with a decay and a removal rate a channel, and the gated RMS norm in groups of columns behind them.  Everything here is float32: inputs, decays,
 // step sizes, the state and the sums; only the normed output is rounded to the activations' type.
 #include "common.h"
 
@@ -920,10 +920,267 @@ extern "C" int li_delta_scan(const float* xkq, long x_stride, const float* ba, l
     return LI_ERR_SIZE;
 }
 
+// ------------------------------------------------------------------------------------ delta rule, channel by channel
+// Per head, with a state S of N x vdim values and the unit key u_t = k_t / sqrt(sum k_t^2 + 1e-6):
+//   S <- diag(w_t) S - (a_t * u_t) (u_t^T S) + k_t v_t^T      (both terms read the old S),      o_t = S^T r_t,
+// with w_t = exp(-exp(-1/2) sigmoid(low_t)) and a_t = sigmoid(araw_t), one number a head and key channel each.  With
+// k = |k| u the step of a state value is  S[n] <- w[n] S[n] + u[n] (|k| v - a[n] (u^T S)):  u, a, w and r are all a token
+// needs beside its |k| v.  A token's step is again S <- A_t S + k_t v_t^T with a matrix A_t = diag(w_t) - (a_t * u_t) u_t^T,
+// so a portion runs as chunks side by side exactly as the gated delta rule's does (same modes, same carry kernel), and
+// the layout is the same: a lane owns CW neighbouring columns x NR state values, NS neighbouring lanes share a column.
+// No heads share keys here: the waves of a block are columns of ONE head (as many waves as the head has units, up to
+// four) and share u, a, w and r, which are worked out when a block of TB tokens is staged in LDS.
+// Rows of x: [r: heads x N | k: heads x N | v: heads x vdim | a: heads x N]; rows of low: heads x N.
+#define CD_DECAY 0.6065306597126334f               // exp(-1/2)
+
+template <int NR, int NS, int CW, int MODE>
+__global__ __launch_bounds__(256) void channel_delta_kernel(
+    const float* __restrict__ x, long x_stride, const float* __restrict__ low, long low_stride, float* __restrict__ state,
+    const int* __restrict__ slots, const int* __restrict__ q_start, const int* __restrict__ q_len,
+    const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, float* __restrict__ pmat,
+    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int Q) {
+    constexpr int NP = NR * NS, PW = 64 * CW / NS, TB = NP > 128 ? 8 : 16;
+    extern __shared__ __align__(16) float lds[];
+    const int nthreads = blockDim.x, nw = nthreads >> 6;
+    float* sU = lds;                                   // [TB][NP] each
+    float* sA = sU + TB * NP;
+    float* sW = sA + TB * NP;
+    float* sR = sW + TB * NP;
+    float* sN = sR + TB * NP;                          // [TB]: |k|
+    float* sX = sN + TB;                               // [nw][TB][PW]
+    const int bx = blockIdx.x;
+    const int seg = chunk_seg ? chunk_seg[bx] : bx;
+    if (seg < 0) return;
+    const int c = chunk_seg ? chunk_idx[bx] : 0;
+    const int L = q_len[seg], first = c * Q;
+    if (first >= L) return;
+    const int ntok = chunk_seg ? ((L - first < Q) ? L - first : Q) : L;
+    const bool last = first + ntok >= L;
+    if (MODE == 1 && last) return;                      // nobody needs the last chunk's own state
+    const int t0 = q_start[seg] + first;
+    // units of a head: blocks of PW value columns, and in MODE 1 behind them blocks of PW columns of P
+    const int PSV = (vdim + PW - 1) / PW, PS = PSV + (MODE == 1 ? (N + PW - 1) / PW : 0);
+    const int ublocks = (PS + nw - 1) / nw;
+    const int head = blockIdx.y / ublocks, ub = blockIdx.y % ublocks;
+    const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int unit = ub * nw + w;
+    const bool active = unit < PS;
+    const int sub = active ? unit : 0;
+    const bool is_p = MODE == 1 && sub >= PSV;
+    const int pbase = (is_p ? sub - PSV : sub) * PW;
+    const int pq = lane / NS, s = lane % NS, p = pbase + CW * pq;       // the first of the lane's columns
+    const long n_key = (long)heads * N;
+    const float* xr0 = x + (size_t)head * N;
+    const float* xv0 = x + 2 * n_key + (size_t)head * vdim;
+    const float* xa0 = x + 2 * n_key + (long)heads * vdim + (size_t)head * N;
+    const float* lw0 = low + (size_t)head * N;
+    float* st = state + ((size_t)slots[seg] * heads + head) * N * vdim;
+    const float* src = chunk_seg ? carry + ((size_t)bx * heads + head) * N * vdim : st;
+    float S[NR][CW];
+#pragma unroll
+    for (int r = 0; r < NR; ++r) {
+        const int n = s * NR + r;
+        if (MODE == 1) {
+#pragma unroll
+            for (int cc = 0; cc < CW; ++cc) S[r][cc] = (is_p && n == p + cc) ? 1.f : 0.f;
+        } else if constexpr (CW == 4) {
+            const float4 v4 = (active && n < N && p < vdim) ? *reinterpret_cast<const float4*>(src + (size_t)n * vdim + p)
+                                                            : float4{0.f, 0.f, 0.f, 0.f};
+            S[r][0] = v4.x; S[r][1] = v4.y; S[r][2] = v4.z; S[r][3] = v4.w;
+        } else {
+#pragma unroll
+            for (int cc = 0; cc < CW; ++cc) S[r][cc] = (active && n < N && p + cc < vdim) ? src[(size_t)n * vdim + p + cc] : 0.f;
+        }
+    }
+    for (int b0 = 0; b0 < ntok; b0 += TB) {
+        __syncthreads();
+        for (int i = threadIdx.x; i < TB * NP; i += nthreads) {
+            const int tt = i / NP, n = i % NP;
+            const bool ok = b0 + tt < ntok && n < N;
+            const size_t row = (size_t)(t0 + b0 + (b0 + tt < ntok ? tt : 0));
+            const int nn = n < N ? n : 0;
+            const float kv = xr0[row * x_stride + n_key + nn], av = xa0[row * x_stride + nn], lv = lw0[row * low_stride + nn];
+            sU[i] = ok ? kv : 0.f;
+            sA[i] = ok ? 1.0f / (1.0f + expf(-av)) : 0.f;
+            sW[i] = ok ? expf(-CD_DECAY / (1.0f + expf(-lv))) : 1.f;
+            if (MODE == 0) sR[i] = ok ? xr0[row * x_stride + nn] : 0.f;
+        }
+        if (active) {
+            for (int i = lane; i < TB * PW; i += 64) {
+                const int tt = i / PW, pp = pbase + i % PW;
+                const bool ok = !is_p && b0 + tt < ntok && pp < vdim;
+                sX[w * TB * PW + i] = ok ? xv0[(size_t)(t0 + b0 + tt) * x_stride + pp] : 0.f;
+            }
+        }
+        __syncthreads();
+        // unit keys: sixteen neighbouring lanes share a token's N values
+        for (int tt = threadIdx.x >> 4; tt < TB; tt += nthreads >> 4) {
+            const int part = threadIdx.x & 15;
+            float sk = 0.f;
+            for (int n = part; n < NP; n += 16) sk = fmaf(sU[tt * NP + n], sU[tt * NP + n], sk);
+#pragma unroll
+            for (int o = 1; o < 16; o <<= 1) sk += __shfl_xor(sk, o, LI_WAVE);
+            const float len = sqrtf(sk + 1e-6f), inv = 1.0f / len;
+            for (int n = part; n < NP; n += 16) sU[tt * NP + n] *= inv;
+            if (part == 0) sN[tt] = len;
+        }
+        __syncthreads();
+        if (!active) continue;
+        const int nt = (ntok - b0 < TB) ? ntok - b0 : TB;
+        for (int tt = 0; tt < nt; ++tt) {
+            const float len = sN[tt];
+            float vn[CW], ks[CW], ov[CW];
+#pragma unroll
+            for (int cc = 0; cc < CW; ++cc) { vn[cc] = len * sX[(w * TB + tt) * PW + CW * pq + cc]; ks[cc] = 0.f; ov[cc] = 0.f; }
+            const float4* Up = reinterpret_cast<const float4*>(sU + tt * NP + s * NR);
+            const float4* Ap = reinterpret_cast<const float4*>(sA + tt * NP + s * NR);
+            const float4* Wp = reinterpret_cast<const float4*>(sW + tt * NP + s * NR);
+            const float4* Rp = reinterpret_cast<const float4*>(sR + tt * NP + s * NR);
+#pragma unroll
+            for (int r4 = 0; r4 < NR / 4; ++r4) {
+                const float4 uv = Up[r4];
+                const float uu[4] = {uv.x, uv.y, uv.z, uv.w};
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int cc = 0; cc < CW; ++cc) ks[cc] = fmaf(S[4 * r4 + j][cc], uu[j], ks[cc]);
+            }
+#pragma unroll
+            for (int o = 1; o < NS; o <<= 1)
+#pragma unroll
+                for (int cc = 0; cc < CW; ++cc) ks[cc] += __shfl_xor(ks[cc], o, LI_WAVE);
+#pragma unroll
+            for (int r4 = 0; r4 < NR / 4; ++r4) {
+                const float4 uv = Up[r4], av = Ap[r4], wv = Wp[r4];
+                const float uu[4] = {uv.x, uv.y, uv.z, uv.w}, aa[4] = {av.x, av.y, av.z, av.w}, ww[4] = {wv.x, wv.y, wv.z, wv.w};
+                float rr[4] = {0.f, 0.f, 0.f, 0.f};
+                if (MODE == 0) { const float4 rv = Rp[r4]; rr[0] = rv.x; rr[1] = rv.y; rr[2] = rv.z; rr[3] = rv.w; }
+#pragma unroll
+                for (int j = 0; j < 4; ++j)
+#pragma unroll
+                    for (int cc = 0; cc < CW; ++cc) {
+                        const float nv = fmaf(ww[j], S[4 * r4 + j][cc], uu[j] * fmaf(-aa[j], ks[cc], vn[cc]));
+                        S[4 * r4 + j][cc] = nv;
+                        if (MODE == 0) ov[cc] = fmaf(nv, rr[j], ov[cc]);
+                    }
+            }
+            if (MODE == 0) {
+#pragma unroll
+                for (int o = 1; o < NS; o <<= 1)
+#pragma unroll
+                    for (int cc = 0; cc < CW; ++cc) ov[cc] += __shfl_xor(ov[cc], o, LI_WAVE);
+                if (s == 0) {
+                    float* yr = y + (size_t)(t0 + b0 + tt) * y_stride + (size_t)head * vdim + p;
+                    if constexpr (CW == 4) {
+                        if (p < vdim) *reinterpret_cast<float4*>(yr) = float4{ov[0], ov[1], ov[2], ov[3]};
+                    } else {
+#pragma unroll
+                        for (int cc = 0; cc < CW; ++cc) if (p + cc < vdim) yr[cc] = ov[cc];
+                    }
+                }
+            }
+        }
+    }
+    if (!active) return;
+    if (MODE == 1 && is_p) {                            // PT[j][n]: the lane's columns j, its n values side by side
+        float* pt = pmat + ((size_t)bx * heads + head) * N * N;
+#pragma unroll
+        for (int cc = 0; cc < CW; ++cc)
+#pragma unroll
+            for (int r = 0; r < NR; ++r) {
+                const int n = s * NR + r;
+                if (n < N && p + cc < N) pt[(size_t)(p + cc) * N + n] = S[r][cc];
+            }
+        return;
+    }
+    float* dst = MODE == 1 ? carry + ((size_t)bx * heads + head) * N * vdim : (last ? st : nullptr);
+    if (!dst) return;
+#pragma unroll
+    for (int r = 0; r < NR; ++r) {
+        const int n = s * NR + r;
+        if (n >= N) continue;
+        if constexpr (CW == 4) {
+            if (p < vdim) *reinterpret_cast<float4*>(dst + (size_t)n * vdim + p) = float4{S[r][0], S[r][1], S[r][2], S[r][3]};
+        } else {
+#pragma unroll
+            for (int cc = 0; cc < CW; ++cc) if (p + cc < vdim) dst[(size_t)n * vdim + p + cc] = S[r][cc];
+        }
+    }
+}
+
+template <int NR, int NS, int CW>
+static int channel_delta_launch(const float* x, long x_stride, const float* low, long low_stride, float* state, const int* slots,
+                                const int* q_start, const int* q_len, int* chunk_tab, float* carry, float* pmat, float* y,
+                                long y_stride, int heads, int vdim, int N, int Q, int segs, int max_chunks, bool chunked,
+                                hipStream_t stream) {
+    constexpr int NP = NR * NS, PW = 64 * CW / NS, TB = NP > 128 ? 8 : 16;
+    const int PSV = (vdim + PW - 1) / PW, PSP = (N + PW - 1) / PW;
+    auto waves = [](int units) { return units < 4 ? units : 4; };
+    auto lds = [](int nw) { return (size_t)(4 * TB * NP + TB + nw * TB * PW) * sizeof(float); };
+    const int w0 = waves(PSV), w1 = waves(PSV + PSP);
+    const int ub0 = (PSV + w0 - 1) / w0, ub1 = (PSV + PSP + w1 - 1) / w1;
+    if (!chunked) {
+        channel_delta_kernel<NR, NS, CW, 0><<<dim3(segs, heads * ub0), 64 * w0, lds(w0), stream>>>(
+            x, x_stride, low, low_stride, state, slots, q_start, q_len, nullptr, nullptr, nullptr, nullptr, y, y_stride, heads, vdim, N, Q);
+        return li_launch_status();
+    }
+    int* chunk_seg = chunk_tab;
+    int* chunk_idx = chunk_tab + max_chunks;
+    int* chunk_first = chunk_tab + 2 * max_chunks;
+    ssm_chunk_index_kernel<<<1, 256, 0, stream>>>(q_len, segs, Q, max_chunks, chunk_seg, chunk_idx, chunk_first);
+    channel_delta_kernel<NR, NS, CW, 1><<<dim3(max_chunks, heads * ub1), 64 * w1, lds(w1), stream>>>(
+        x, x_stride, low, low_stride, state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, pmat, y, y_stride, heads, vdim, N, Q);
+    delta_carry_launch(carry, pmat, state, slots, q_len, chunk_first, heads, vdim, N, Q, segs, stream);
+    channel_delta_kernel<NR, NS, CW, 0><<<dim3(max_chunks, heads * ub0), 64 * w0, lds(w0), stream>>>(
+        x, x_stride, low, low_stride, state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, pmat, y, y_stride, heads, vdim, N, Q);
+    return li_launch_status();
+}
+
+extern "C" int li_channel_delta(const float* x, long x_stride, const float* low, long low_stride, float* state, const int* slots,
+                                const int* q_start, const int* q_len, float* y, long y_stride, int heads, int vdim, int N, int Q,
+                                int T, int segs, int max_q_len, void* work, long work_bytes, hipStream_t stream) {
+    if (T <= 0 || segs <= 0 || heads <= 0 || vdim <= 0 || N <= 0 || N > 256 || Q <= 0 || max_q_len <= 0 ||
+        x_stride < 3L * heads * N + (long)heads * vdim || low_stride < (long)heads * N || y_stride < (long)heads * vdim)
+        return LI_ERR_SIZE;
+    const bool chunked = max_q_len > Q;
+    int max_chunks = 0;
+    int* chunk_tab = nullptr;
+    float *carry = nullptr, *pmat = nullptr;
+    if (chunked) {
+        const long need = li_delta_scan_work_bytes(T, segs, heads, vdim, N, Q, &max_chunks);
+        if (!work || work_bytes < need || ((uintptr_t)work % 16)) return LI_ERR_SIZE;
+        chunk_tab = (int*)work;
+        const long ints = ((3L * max_chunks + segs + 1 + 3) / 4) * 4;
+        carry = (float*)work + ints;
+        pmat = carry + (size_t)max_chunks * heads * N * vdim;
+    }
+#define CD_ARGS x, x_stride, low, low_stride, state, slots, q_start, q_len, chunk_tab, carry, pmat, y, y_stride, heads, vdim, N, Q,                 segs, max_chunks, chunked, stream
+    const bool aligned = ((uintptr_t)state | (uintptr_t)y | (uintptr_t)carry) % 16 == 0 && y_stride % 4 == 0;
+    int qs = 0, qr = 0;
+    if (aligned && ssm_quad_layout(N, vdim, &qs, &qr)) {
+#define CD_QUAD(NR_, NS_) if (qr == NR_ && qs == NS_) return channel_delta_launch<NR_, NS_, 4>(CD_ARGS);
+        CD_QUAD(4, 2) CD_QUAD(8, 2) CD_QUAD(16, 2) CD_QUAD(32, 2)
+        CD_QUAD(4, 4) CD_QUAD(8, 4) CD_QUAD(16, 4) CD_QUAD(32, 4)
+        CD_QUAD(4, 8) CD_QUAD(8, 8) CD_QUAD(16, 8) CD_QUAD(32, 8)
+        CD_QUAD(4, 16) CD_QUAD(8, 16) CD_QUAD(16, 16)
+#undef CD_QUAD
+    }
+    int ns = 0, nr = 0;
+    if (!li_ssm_scan_layout(N, vdim, &ns, &nr)) return LI_ERR_SIZE;
+#define CD_GO(NR_, NS_) if (nr == NR_ && ns == NS_) return channel_delta_launch<NR_, NS_, 1>(CD_ARGS);
+    CD_GO(16, 1) CD_GO(32, 1) CD_GO(64, 1) CD_GO(128, 1)
+    CD_GO(16, 2) CD_GO(32, 2) CD_GO(64, 2) CD_GO(128, 2)
+    CD_GO(16, 4) CD_GO(32, 4) CD_GO(64, 4)
+#undef CD_GO
+#undef CD_ARGS
+    return LI_ERR_SIZE;
+}
+
 // ------------------------------------------------------------------------------------ gated norm in groups
 // Every group of `gs` neighbouring columns has its own root mean square.  gate_after 0: out[t, c] = w[c] * v /
 // sqrt(mean of v^2 over c's group + eps) with v = y[t, c] * silu(z[t, c]): the gate comes before the norm.
-// gate_after 1: out[t, c] = w[c] * y / sqrt(mean of y^2 + eps) * silu(z[t, c]): the norm sees y alone.  w null: ones.
+// gate_after 1: out[t, c] = w[c] * y / sqrt(mean of y^2 + eps) * silu(z[t, c]): the norm sees y alone.  gate_after 2: the
+// same with sigmoid(z) for silu(z).  w null: ones.
 // A block a (token, group).
 template <typename TO, int PER>
 __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __restrict__ y, long y_stride,
@@ -940,13 +1197,13 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     for (int i = 0; i < PER; ++i) {
         const int j = threadIdx.x + i * 256;
         float g = 0.f, sg = 0.f;
-        if (j < gs) { const float zz = zr[j]; sg = zz / (1.0f + expf(-zz)); g = gate_after ? yr[j] : yr[j] * sg; }
+        if (j < gs) { const float zz = zr[j]; sg = (gate_after == 2 ? 1.0f : zz) / (1.0f + expf(-zz)); g = gate_after ? yr[j] : yr[j] * sg; }
         v[i] = g;
         gt[i] = gate_after ? sg : 1.f;
         ss += g * g;
     }
     for (int j = threadIdx.x + PER * 256; j < gs; j += 256) {
-        const float zz = zr[j], sg = zz / (1.0f + expf(-zz)), g = gate_after ? yr[j] : yr[j] * sg;
+        const float zz = zr[j], sg = (gate_after == 2 ? 1.0f : zz) / (1.0f + expf(-zz)), g = gate_after ? yr[j] : yr[j] * sg;
         ss += g * g;
     }
     ss = block_sum<256>(ss, red);
@@ -958,7 +1215,7 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
         if (j < gs) store_from_float(o + j, (w ? w[c0 + j] : 1.f) * v[i] * inv * gt[i]);
     }
     for (int j = threadIdx.x + PER * 256; j < gs; j += 256) {
-        const float zz = zr[j], sg = zz / (1.0f + expf(-zz)), g = gate_after ? yr[j] : yr[j] * sg;
+        const float zz = zr[j], sg = (gate_after == 2 ? 1.0f : zz) / (1.0f + expf(-zz)), g = gate_after ? yr[j] : yr[j] * sg;
         store_from_float(o + j, (w ? w[c0 + j] : 1.f) * g * inv * (gate_after ? sg : 1.f));
     }
 }

@@ -9,7 +9,7 @@ import torch
 from ..config.spec import ModelSpec, PartSpec
 from ..kernels import ops
 from ..parts.base import Runtime, build_part
-from ..parts.stream import ResidualStream
+from ..parts.stream import HyperStream, ResidualStream
 from ..weights.loader import ParamSpec
 
 
@@ -98,7 +98,7 @@ class Model:
             # an injection reads the embedding output again later: a copy beside the stream
             ctx.embedding_out = ctx.ws.buffer("model.embedding_out", (ctx.num_tokens, h), torch.float32)
             ops.cast(x, ctx.embedding_out)
-        stream = ResidualStream(x, ctx.ws)
+        stream = HyperStream(x, ctx.ws, self.spec.streams) if self.spec.streams else ResidualStream(x, ctx.ws)
         stream.ws_dtype = self.rt.dtype
         for i, e in enumerate(self.order):
             if e.inject is not None:
@@ -110,12 +110,11 @@ class Model:
             stream.next_plain = follower is not None and bool(getattr(follower, "reads_stream_itself", False))
             self.layers[e.layer].forward(stream, ctx, cache.view(i))
             if self.tap is not None:
-                self.tap(i, stream.x)
-        x = stream.tensor()
+                self.tap(i, stream.total())
         if ctx.num_want == 0:
             return None
         rows = ctx.ws.buffer("model.rows", (ctx.num_want, h), torch.float32)
-        ops.gather_rows(x, ctx.want_rows, rows)
+        stream.gather(ctx.want_rows, rows)
         xn = ctx.ws.buffer("model.rows_normed", (ctx.num_want, h), self.rt.dtype)
         self.final_norm.forward(rows, xn)
         logits = torch.empty((ctx.num_want, self.spec.vocab_size), dtype=torch.float32,

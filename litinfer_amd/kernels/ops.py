@@ -27,7 +27,7 @@ MAX_HEAD_DIM = 256
 P, I, F, L = c_void_p, c_int, c_float, c_long
 _SIGNATURES = {
     "elementwise": {
-        "li_embedding": [P, P, P, P, I, P, I, I, I],
+        "li_embedding": [P, P, P, P, I, P, I, I, I, F],
         "li_rmsnorm": [P, I, P, F, P, I, I, I],
         "li_gather_rows": [P, P, P, I, I],
         "li_cast": [P, I, P, I, L],
@@ -44,6 +44,11 @@ _SIGNATURES = {
         "li_rope_freq_table": [P, P, I, F, P, P, I],
         "li_rope_pairs_apply": [P, I, I, I, I, I, P, P, I],
         "li_qk_norm_pairs_store": [P, I, I, I, I, I, I, P, P, F, P, P, P, P, P, I, I, I, I, I],
+        "li_qk_head_norm_store": [P, L, I, I, I, I, I, P, P, F, P, P, P, P, P, I, I, I, I, I, I],
+        "li_hyper_step": [P, I, P, P, P, F, F, P, P, P, P, F, P, I, I, I, I],
+        "li_stream_sum": [P, P, P, I, I, I],
+        "li_xielu": [P, I, P, I, L, F, F],
+        "li_tanh_rows": [P, L, P, I, I, I],
         "li_latent_norm_pairs_store": [P, L, I, I, I, P, L, I, P, F, P, P, P, P, I, P, I, I, P, L, I, P, P, I, I],
         "li_pair_embedding": [P, P, P, P, P, P, P, P, P, P, P, I, P, I, I, I, I, L, L],
         "li_layernorm": [P, P, P, F, P, I, I, I],
@@ -58,6 +63,7 @@ _SIGNATURES = {
         "li_causal_conv_silu": [P, L, I, I, P, P, P, P, P, P, P, P, L, I, I, I],
         "li_ssm_scan": [P, L, P, L, P, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, I, P, L, P, F],
         "li_delta_scan": [P, L, P, L, P, P, P, P, P, P, P, L, I, I, I, I, F, I, I, I, I, P, L],
+        "li_channel_delta": [P, L, P, L, P, P, P, P, P, L, I, I, I, I, I, I, I, P, L],
         "li_gated_group_norm": [P, L, P, L, P, F, P, I, L, I, I, I, I],
     },
     "moe": {
@@ -67,11 +73,11 @@ _SIGNATURES = {
         "li_moe_combine": [P, L, P, L, P, P, P, P, L, I, I, I, P, I, P, I, L],
     },
     "attention_masked": {
-        "li_masked_attention": [P, I, I, P, I, P, P, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I],
-        "li_masked_attention_single": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, L],
-        "li_masked_attention_heads": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, L],
-        "li_masked_attention_tiles": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, L, P, I, I],
-        "li_headwise_linear": [P, I, L, I, P, I, P, I, L, I, I, I, I, I, P, L, I, I, P, P],
+        "li_masked_attention": [P, I, I, P, I, P, P, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I],
+        "li_masked_attention_single": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, P, L],
+        "li_masked_attention_heads": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, P, L],
+        "li_masked_attention_tiles": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, P, L, P, I, I],
+        "li_headwise_linear": [P, I, L, I, P, I, P, I, L, I, I, I, I, I, P, L, I, I, I, P, P],
     },
     "gemm": {
         "li_linear": [P, P, P, P, I, I, I, I, I, I, P, L],
@@ -208,8 +214,8 @@ def check_attention_sizes(num_heads: int, num_kv_heads: int, head_dim: int) -> N
 
 # ---------------------------------------------------------------- elementwise
 def embedding(ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor,
-              id_src: Optional[torch.Tensor] = None, feedback: Optional[torch.Tensor] = None) -> None:
-    """out[t, :] = table[id(t), :] as float32 with id(t) = ids[t], or
+              id_src: Optional[torch.Tensor] = None, feedback: Optional[torch.Tensor] = None, scale: float = 1.0) -> None:
+    """out[t, :] = scale * table[id(t), :] as float32 with id(t) = ids[t], or
     feedback[id_src[t]] where id_src is given and id_src[t] >= 0 (a token chosen
     on the device that the host has not seen yet).  Ids given by the host must
     already be inside the table (the step checks them); an id outside it (one
@@ -226,7 +232,7 @@ def embedding(ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor,
     if t:
         _run("elementwise", "li_embedding", ids.data_ptr(), 0 if id_src is None else id_src.data_ptr(),
              0 if id_src is None else feedback.data_ptr(), table.data_ptr(), _DT[table.dtype],
-             out.data_ptr(), t, h, table.shape[0])
+             out.data_ptr(), t, h, table.shape[0], float(scale))
 
 
 def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor) -> None:
@@ -497,8 +503,101 @@ def qk_norm_pairs_store(qkv: torch.Tensor, nh: int, nkv: int, dk: int, dv: int, 
              int(bool(half_split)), t)
 
 
+def qk_head_norm_store(qkv: torch.Tensor, nh: int, nkv: int, dk: int, dv: int, rotary_dim: int, wq: torch.Tensor,
+                       wk: torch.Tensor, eps: float, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor],
+                       slot_map: Optional[torch.Tensor], k: Optional[torch.Tensor], v: Optional[torch.Tensor], page_size: int,
+                       half_split: bool = False, keys_are_values: bool = False) -> None:
+    """qkv float32 rows [q (nh*dk) | k (nkv*dk) | v (nkv*dv)], or [q | k] with `keys_are_values` (the value is the key as
+    it stands in the row, before its norm).  Every query head and every key head is RMS-normed by itself (weights wq, wk
+    [dk], the same for all heads) and its first `rotary_dim` columns rotated (0: none); q stays in place, k and v go to
+    their page slots (k None: only q is prepared)."""
+    _gpu(qkv, wq, wk, cos, sin, slot_map, k, v)
+    t = qkv.shape[0]
+    need = nh * dk + nkv * (dk if keys_are_values else dk + dv)
+    _chk(_rows_ok(qkv) and qkv.dtype is torch.float32 and qkv.shape[1] >= need, "qk_head_norm_store: qkv must be float32 rows of q, k and v")
+    _chk(rotary_dim % 2 == 0 and 0 <= rotary_dim <= dk and (not keys_are_values or dk == dv), "qk_head_norm_store: sizes")
+    if rotary_dim:
+        _check_tables("qk_head_norm_store", t, rotary_dim, cos, sin, None)
+    _chk(all(w.dtype is torch.float32 and w.numel() == dk and w.is_contiguous() for w in (wq, wk)), "qk_head_norm_store: norm weights [dk]")
+    if k is not None:
+        _chk(k.dim() == 4 and v.dim() == 4 and k.shape[1:] == (nkv, page_size, dk) and v.shape[1:] == (nkv, page_size, dv)
+             and k.shape[0] == v.shape[0] and k.is_contiguous() and v.is_contiguous() and k.dtype is v.dtype
+             and k.dtype in _DT and slot_map is not None and slot_map.dtype is torch.int32 and slot_map.numel() == t
+             and slot_map.is_contiguous(), "qk_head_norm_store: cache")
+    if t:
+        _run("elementwise", "li_qk_head_norm_store", qkv.data_ptr(), qkv.stride(0), nh, nkv, dk, dv, rotary_dim, wq.data_ptr(),
+             wk.data_ptr(), float(eps), cos.data_ptr() if rotary_dim else 0, sin.data_ptr() if rotary_dim else 0,
+             0 if k is None else slot_map.data_ptr(), 0 if k is None else k.data_ptr(), 0 if k is None else v.data_ptr(),
+             _DT[k.dtype] if k is not None else 0, page_size, int(k is not None), int(bool(half_split)), int(bool(keys_are_values)), t)
+
+
+MAX_STREAMS = 16
+
+
+def hyper_step(src: torch.Tensor, dst: Optional[torch.Tensor], streams: int, y: Optional[torch.Tensor] = None,
+               y2: Optional[torch.Tensor] = None, factors=(1.0, 1.0), mix: Optional[torch.Tensor] = None,
+               out: Optional[torch.Tensor] = None, read: Optional[torch.Tensor] = None, weight: Optional[torch.Tensor] = None,
+               eps: float = 0.0, xn: Optional[torch.Tensor] = None) -> None:
+    """One token's `streams` residual streams x_s, float32 [T, streams, H] (`src` [T, H]: all streams are that row).
+    With `mix` [streams, streams] and `out` [streams]: dst gets x_t <- sum_s mix[s, t] x_s + out[t] b for
+    b = factors[0] y (+ factors[1] y2), every stream from the old ones (dst may be src).  With `read` [streams]: xn gets the
+    RMS norm (weights `weight`, `eps`) of sum_s read[s] x_s over the new streams (the old ones where nothing is written)."""
+    _gpu(src, dst, y, y2, mix, out, read, weight, xn)
+    n, h = int(streams), src.shape[-1]
+    t = src.shape[0]
+    _chk(src.dtype is torch.float32 and src.is_contiguous() and src.shape in ((t, h), (t, n, h)) and 1 <= n <= MAX_STREAMS, "hyper_step: src")
+    _chk((mix is None) == (y is None) and (mix is None) == (out is None) and (mix is not None or read is not None), "hyper_step: nothing to do")
+    if mix is not None:
+        _chk(dst is not None and dst.shape == (t, n, h) and dst.is_contiguous() and dst.dtype is torch.float32, "hyper_step: dst")
+        for b in (y, y2):
+            _chk(b is None or (b.shape == (t, h) and b.is_contiguous() and b.dtype is torch.float32), "hyper_step: the sublayer's output")
+        _chk(mix.shape == (n, n) and out.numel() == n and mix.dtype is torch.float32 and out.dtype is torch.float32
+             and mix.is_contiguous() and out.is_contiguous(), "hyper_step: mix, out")
+    if read is not None:
+        _chk(read.numel() == n and read.dtype is torch.float32 and read.is_contiguous() and weight is not None and weight.numel() == h
+             and weight.dtype is torch.float32 and weight.is_contiguous() and xn is not None and xn.shape == (t, h)
+             and xn.is_contiguous() and xn.dtype in _DT, "hyper_step: read, weight, xn")
+
+    def ptr(v):
+        return 0 if v is None else v.data_ptr()
+    if t:
+        _run("elementwise", "li_hyper_step", src.data_ptr(), n if src.dim() == 3 else 1, ptr(dst) if mix is not None else 0, ptr(y), ptr(y2),
+             float(factors[0]), float(factors[1]), ptr(mix), ptr(out), ptr(read), ptr(weight) if read is not None else 0, float(eps),
+             ptr(xn) if read is not None else 0, _DT[xn.dtype] if read is not None else 0, n, t, h)
+
+
+def stream_sum(x: torch.Tensor, out: torch.Tensor, rows: Optional[torch.Tensor] = None) -> None:
+    """out[i] = the sum over the streams of token rows[i] (every token, without `rows`); x float32 [T, streams, H]."""
+    _gpu(x, out, rows)
+    _chk(x.dim() == 3 and x.is_contiguous() and x.dtype is torch.float32 and out.dim() == 2 and out.shape[1] == x.shape[2]
+         and out.is_contiguous() and out.dtype is torch.float32, "stream_sum: x [T, streams, H], out [n, H]")
+    _chk((rows is None and out.shape[0] == x.shape[0]) or (rows is not None and rows.dtype is torch.int32 and rows.numel() == out.shape[0]
+                                                           and rows.is_contiguous()), "stream_sum: rows")
+    if out.shape[0]:
+        _run("elementwise", "li_stream_sum", x.data_ptr(), 0 if rows is None else rows.data_ptr(), out.data_ptr(), out.shape[0],
+             x.shape[1], x.shape[2])
+
+
+def xielu(x: torch.Tensor, out: torch.Tensor, sp: float, sq: float) -> None:
+    """z > 0: sp z^2 + z / 2; z <= 0: sq (exp(z) - 1 - z) + z / 2 (sp = softplus(p), sq = 1/2 + softplus(q))."""
+    _gpu(x, out)
+    _chk(x.shape == out.shape and x.is_contiguous() and out.is_contiguous() and x.dtype in _DT and out.dtype in _DT
+         and (x.dtype is torch.float32 or out.dtype is x.dtype), "xielu: x, out")
+    if x.numel():
+        _run("elementwise", "li_xielu", x.data_ptr(), _DT[x.dtype], out.data_ptr(), _DT[out.dtype], x.numel(), float(sp), float(sq))
+
+
+def tanh_rows(x: torch.Tensor, out: torch.Tensor) -> None:
+    """out = tanh(x) for float32 rows that may lie inside wider ones."""
+    _gpu(x, out)
+    t, n = out.shape
+    _chk(x.dtype is torch.float32 and _rows_ok(x) and x.shape == (t, n) and out.is_contiguous() and out.dtype in _DT, "tanh_rows: x, out")
+    if t:
+        _run("elementwise", "li_tanh_rows", x.data_ptr(), x.stride(0), out.data_ptr(), _DT[out.dtype], t, n)
+
+
 def latent_norm_pairs_store(qd: Optional[torch.Tensor], nh: int, dn: int, dr: int, rank: int, wc: torch.Tensor, eps: float,
-                            cos: torch.Tensor, sin: torch.Tensor, slot_map: Optional[torch.Tensor],
+                            cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], slot_map: Optional[torch.Tensor],
                             cache: Optional[torch.Tensor], qfull: Optional[torch.Tensor], down: Optional[torch.Tensor] = None,
                             half_split: bool = False, q_latent: Optional[torch.Tensor] = None,
                             wq: Optional[torch.Tensor] = None, cq: Optional[torch.Tensor] = None) -> None:
@@ -507,11 +606,14 @@ def latent_norm_pairs_store(qd: Optional[torch.Tensor], nh: int, dn: int, dr: in
     be None: then no query is touched.  The latent is RMS-normed and written with the rotated shared part to the
     token's page row [rank + dr]; every query head's rotated part goes to columns rank.. of its row in qfull
     [T, nh, rank + dr] (float32).  Pairs are neighbouring columns, or column i with column i + dr/2 (`half_split`).
-    With `q_latent` (float32 rows, a view is fine) also cq = the RMS norm of those rows with weights wq."""
+    With `q_latent` (float32 rows, a view is fine) also cq = the RMS norm of those rows with weights wq.  dr 0: nothing
+    is rotated (cos and sin are not read, the queries are not touched)."""
     _gpu(qd, wc, cos, sin, slot_map, cache, qfull, down, q_latent, wq, cq)
-    t = cos.shape[0]
+    t = (down if down is not None else qd).shape[0]
     if qd is None:
         nh = 0
+    if not dr:                                   # no rotated part: nothing of the queries is touched here
+        nh, cos, sin = 0, None, None
     if nh:
         need = nh * (dn + dr) + (0 if down is not None else rank + dr)
         _chk(_rows_ok(qd) and qd.dtype is torch.float32 and qd.shape[0] == t and qd.shape[1] >= need, "latent_norm_pairs_store: qd")
@@ -519,8 +621,12 @@ def latent_norm_pairs_store(qd: Optional[torch.Tensor], nh: int, dn: int, dr: in
              "latent_norm_pairs_store: qfull")
     if down is None and nh:
         down = qd[:, nh * (dn + dr):]
-    _chk(dr % 2 == 0 and dr > 0, "latent_norm_pairs_store: the rotated size must be even")
-    _check_tables("latent_norm_pairs_store", t, dr, cos, sin, slot_map if cache is not None else None)
+    _chk(dr % 2 == 0 and dr >= 0, "latent_norm_pairs_store: the rotated size must be even")
+    if dr:
+        _check_tables("latent_norm_pairs_store", t, dr, cos, sin, slot_map if cache is not None else None)
+    else:
+        _chk(cache is None or (slot_map is not None and slot_map.dtype is torch.int32 and slot_map.numel() == t
+                               and slot_map.is_contiguous()), "latent_norm_pairs_store: slot_map")
     _chk(wc.dtype is torch.float32 and wc.numel() == rank and wc.is_contiguous(), "latent_norm_pairs_store: norm weight")
     if cache is not None:
         _chk(down is not None and _rows_ok(down) and down.dtype is torch.float32 and down.shape == (t, rank + dr),
@@ -537,7 +643,7 @@ def latent_norm_pairs_store(qd: Optional[torch.Tensor], nh: int, dn: int, dr: in
     if t and (nh or cache is not None or q_rank):
         _run("elementwise", "li_latent_norm_pairs_store", qd.data_ptr() if nh else 0, qd.stride(0) if nh else 0, nh, dn, dr,
              down.data_ptr() if cache is not None else 0, down.stride(0) if cache is not None else 0, rank, wc.data_ptr(),
-             float(eps), cos.data_ptr(), sin.data_ptr(), 0 if cache is None else slot_map.data_ptr(),
+             float(eps), cos.data_ptr() if dr else 0, sin.data_ptr() if dr else 0, 0 if cache is None else slot_map.data_ptr(),
              0 if cache is None else cache.data_ptr(), _DT[cache.dtype] if cache is not None else 0,
              qfull.data_ptr() if nh else 0, int(cache is not None), int(bool(half_split)),
              q_latent.data_ptr() if q_rank else 0, q_latent.stride(0) if q_rank else 0, q_rank,
@@ -624,7 +730,8 @@ def _single_blocks(n: int, nh: int, nkv: int, dk: int, dv: int) -> int:
 def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, out: torch.Tensor, k: torch.Tensor,
                      v: torch.Tensor, meta, nh: int, nkv: int, dk: int, dv: int, page_size: int, window: int,
                      keep_first: int, softcap: float, scale: float, ws=None, sink: Optional[torch.Tensor] = None,
-                     head_gate: Optional[torch.Tensor] = None) -> None:
+                     head_gate: Optional[torch.Tensor] = None, column_gate: Optional[torch.Tensor] = None,
+                     slopes: Optional[torch.Tensor] = None) -> None:
     """Attention of every token of the step over its request's cached keys: position p sees j <= p with
     p - j < window (0: all) or j < keep_first; scores (q . k) * scale, then softcap * tanh(score / softcap)
     where softcap > 0; softmax and sums in float32.  q: a float32 tensor in which head h of token t starts at
@@ -632,8 +739,9 @@ def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, o
     may be one tensor: then the value is the first dv columns of the key's row); out [T, nh * dv].
     `sink` (float32 [nh]): the softmax's denominator also holds exp(sink[head]), a term without key or value.
     `head_gate` (float32 rows [T, nh], a view of columns is fine): head h's output of token t is multiplied by
-    sigmoid(head_gate[t, h])."""
-    _gpu(q, out, k, v, meta.block_table, sink, head_gate)
+    sigmoid(head_gate[t, h]).  `column_gate` (float32 rows [T, nh * dv], a view is fine) does that with a number for every
+    head and value column.  `slopes` (float32 [nh]): a key's score loses slopes[head] * (p - j)."""
+    _gpu(q, out, k, v, meta.block_table, sink, head_gate, column_gate, slopes)
     t = out.shape[0]
     _chk(q.dtype is torch.float32 and q.is_contiguous() and q.numel() >= (t - 1) * q_token_stride + (nh - 1) * q_head_stride + dk,
          "masked_attention: q")
@@ -646,8 +754,12 @@ def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, o
     _chk(sink is None or (sink.dtype is torch.float32 and sink.numel() == nh and sink.is_contiguous()), "masked_attention: sink")
     _chk(head_gate is None or (head_gate.dtype is torch.float32 and _rows_ok(head_gate) and head_gate.shape == (t, nh)),
          "masked_attention: head_gate")
-    fin = (0 if sink is None else sink.data_ptr(), 0 if head_gate is None else head_gate.data_ptr(),
-           0 if head_gate is None else head_gate.stride(0))
+    _chk(column_gate is None or (head_gate is None and column_gate.dtype is torch.float32 and _rows_ok(column_gate)
+                                 and column_gate.shape == (t, nh * dv)), "masked_attention: column_gate")
+    _chk(slopes is None or (slopes.dtype is torch.float32 and slopes.numel() == nh and slopes.is_contiguous()), "masked_attention: slopes")
+    gate = head_gate if column_gate is None else column_gate
+    fin = (0 if sink is None else sink.data_ptr(), 0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0),
+           int(column_gate is not None), 0 if slopes is None else slopes.data_ptr())
     if not t:
         return
     # keys that one query may see, as far as the host knows without looking at the contexts (a recorded step
@@ -663,7 +775,8 @@ def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, o
              nh, nkv, dk, dv, page_size, k.shape[0], int(window), int(keep_first), float(softcap or 0.0), float(scale), *fin, waves)
 
     fast = (k.dtype is torch.bfloat16 and out.dtype is torch.bfloat16 and k.shape[3] % 8 == 0 and v.shape[3] % 8 == 0
-            and q_token_stride % 4 == 0 and q_head_stride % 4 == 0 and q.data_ptr() % 16 == 0)
+            and q_token_stride % 4 == 0 and q_head_stride % 4 == 0 and q.data_ptr() % 16 == 0
+            and (column_gate is None or (column_gate.data_ptr() % 16 == 0 and column_gate.stride(0) % 4 == 0)))
 
     def singles(token_list, n):
         # single tokens in bfloat16, at the sizes it has: rows spread over lanes, a row read once for a group's heads
@@ -773,10 +886,11 @@ def masked_tiles_take(dk: int, dv: int) -> bool:
 
 def headwise_linear(x: torch.Tensor, x_token_stride: int, x_head_stride: int, m: torch.Tensor, out: torch.Tensor,
                     o_token_stride: int, o_head_stride: int, tokens: int, gate: Optional[torch.Tensor] = None,
-                    rotate_tail=None) -> None:
+                    rotate_tail=None, gate_columns: bool = False) -> None:
     """out[t, h, j] = sum_k m[h, j, k] * x[t, h, k] for m [heads, n_out, n_in]; head h of token t starts at
     t * token_stride + h * head_stride in x (n_in values) and in out (n_out values).  With `gate` (float32 rows
-    [tokens, heads], a view of columns is fine) head h's outputs of token t are multiplied by sigmoid(gate[t, h]).
+    [tokens, heads], a view of columns is fine) head h's outputs of token t are multiplied by sigmoid(gate[t, h]); with
+    `gate_columns` the rows are [tokens, heads * n_out] and every output has a gate of its own.
     With `rotate_tail` = (n, cos, sin, half_split) the n columns behind a head's inputs are rotated by the token's
     angles (cos, sin [tokens, n / 2]) and written behind the head's outputs."""
     _gpu(x, m, out, gate)
@@ -788,7 +902,8 @@ def headwise_linear(x: torch.Tensor, x_token_stride: int, x_head_stride: int, m:
         _chk(tn % 2 == 0 and x_head_stride >= n_in + tn and o_head_stride >= n_out + tn
              and x.numel() >= (tokens - 1) * x_token_stride + (nh - 1) * x_head_stride + n_in + tn
              and out.numel() >= (tokens - 1) * o_token_stride + (nh - 1) * o_head_stride + n_out + tn, "headwise_linear: the rotated tail")
-    _chk(gate is None or (_rows_ok(gate) and gate.dtype is torch.float32 and gate.shape == (tokens, nh)), "headwise_linear: gate")
+    _chk(gate is None or (_rows_ok(gate) and gate.dtype is torch.float32 and gate.shape == (tokens, nh * (n_out if gate_columns else 1))),
+         "headwise_linear: gate")
     _chk(m.is_contiguous() and m.dtype in _DT and x.dtype in _DT and out.dtype in _DT and x.is_contiguous()
          and out.is_contiguous(), "headwise_linear: operands")
     _chk(x.numel() >= (tokens - 1) * x_token_stride + (nh - 1) * x_head_stride + n_in
@@ -800,7 +915,7 @@ def headwise_linear(x: torch.Tensor, x_token_stride: int, x_head_stride: int, m:
         _run("attention_masked", "li_headwise_linear", x.data_ptr(), _DT[x.dtype], int(x_token_stride), int(x_head_stride),
              m.data_ptr(), _DT[m.dtype], out.data_ptr(), _DT[out.dtype], int(o_token_stride), int(o_head_stride),
              tokens, nh, n_out, n_in, 0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0),
-             int(tn), int(bool(tsplit)), tcos.data_ptr() if tn else 0, tsin.data_ptr() if tn else 0)
+             int(bool(gate_columns)), int(tn), int(bool(tsplit)), tcos.data_ptr() if tn else 0, tsin.data_ptr() if tn else 0)
 
 
 # ---------------------------------------------------------------------- gemm
@@ -1599,20 +1714,54 @@ def delta_scan(xkq: torch.Tensor, ba: torch.Tensor, dt_bias: torch.Tensor, a_log
          work, work_bytes)
 
 
+def channel_delta(x: torch.Tensor, low: torch.Tensor, state: torch.Tensor, ctx, y: torch.Tensor, heads: int, vdim: int,
+                  n_state: int, ws=None) -> None:
+    """The delta rule with a decay and a removal rate for every key channel, over each request's tokens of the step, from
+    and into `state` [slots, heads, n_state, vdim] (float32):  S <- diag(w) S - (a * u) (u^T S) + k v^T (the old S in both
+    terms),  y = S^T r,  with u = k / sqrt(sum k^2 + 1e-6), w = exp(-exp(-1/2) sigmoid(low)) and a = sigmoid(a_raw).
+    x: float32 rows [r: heads * n_state | k: heads * n_state | v: heads * vdim | a_raw: heads * n_state]; low: float32 rows
+    [heads * n_state]; y: float32 rows [heads * vdim].  With a workspace, portions longer than SSM_CHUNK tokens run as
+    chunks side by side, as the gated delta rule's do; without one, token after token."""
+    _gpu(x, low, state, y)
+    t = y.shape[0]
+    _chk(all(v.dtype is torch.float32 for v in (x, low, state, y)), "channel_delta: everything is float32")
+    _chk(_rows_ok(x) and x.shape == (t, heads * (3 * n_state + vdim)) and _rows_ok(low) and low.shape == (t, heads * n_state)
+         and _rows_ok(y) and y.shape == (t, heads * vdim), "channel_delta: rows")
+    _chk(state.is_contiguous() and state.shape[1:] == (heads, n_state, vdim), "channel_delta: state [slots, heads, N, vdim]")
+    _chk(ctx.num_tokens == t and int(ctx.host_state_slots.max(initial=0)) < state.shape[0], "channel_delta: batch")
+    _chk(delta_scan_takes(n_state, vdim), f"channel_delta: no kernel for a state of {n_state} values a column (at most 256)")
+    if not t:
+        return
+    work, work_bytes, q = 0, 0, SSM_CHUNK
+    if not DELTA_CHUNKED:
+        ws = None
+    if ctx.max_q_len > SSM_CHUNK and ws is not None:
+        need = _lib_fn("recurrent", "li_delta_scan_work_bytes", [c_int] * 6 + [c_void_p], c_long)(
+            t, ctx.num_segments, heads, vdim, n_state, SSM_CHUNK, None)
+        buf = ws.buffer("delta_scan.work", ((int(need) + 3) // 4,), torch.float32)
+        work, work_bytes = buf.data_ptr(), buf.numel() * 4
+    elif ctx.max_q_len > SSM_CHUNK:
+        q = int(ctx.max_q_len)                       # one chunk a request: the recurrence token after token
+    _run("recurrent", "li_channel_delta", x.data_ptr(), x.stride(0), low.data_ptr(), low.stride(0), state.data_ptr(),
+         ctx.state_slots.data_ptr(), ctx.q_start.data_ptr(), ctx.q_len.data_ptr(), y.data_ptr(), y.stride(0), heads, vdim, n_state,
+         q, t, ctx.num_segments, int(ctx.max_q_len), work, work_bytes)
+
+
 def gated_group_norm(y: torch.Tensor, z: torch.Tensor, weight: Optional[torch.Tensor], eps: float, groups: int, out: torch.Tensor,
-                     gate_after: bool = False) -> None:
+                     gate_after: bool = False, gate: str = "silu") -> None:
     """out = weight * v / sqrt(mean over the group of v^2 + eps), v = y * silu(z), every one of `groups` equal runs of
-    columns by its own mean; with `gate_after` the norm sees y alone and its result is multiplied by silu(z).
-    weight None: ones.  y, z float32 rows; out in either dtype."""
+    columns by its own mean; with `gate_after` the norm sees y alone and its result is multiplied by silu(z),
+    or, with `gate` "sigmoid", by sigmoid(z).  weight None: ones.  y, z float32 rows; out in either dtype."""
     _gpu(y, z, weight, out)
     t, n = out.shape
+    _chk(gate == "silu" or (gate == "sigmoid" and gate_after), "gated_group_norm: gate")
     _chk(y.dtype is torch.float32 and z.dtype is torch.float32 and _rows_ok(y) and _rows_ok(z) and y.shape == (t, n) and z.shape == (t, n)
          and _rows_ok(out) and out.dtype in _DT and (weight is None or (weight.dtype is torch.float32 and weight.numel() == n and weight.is_contiguous()))
          and groups > 0 and n % groups == 0, "gated_group_norm: y, z [T, n] float32, weight [n], out [T, n]")
     if t:
         _run("recurrent", "li_gated_group_norm", y.data_ptr(), y.stride(0), z.data_ptr(), z.stride(0),
              0 if weight is None else weight.data_ptr(), float(eps), out.data_ptr(), _DT[out.dtype], out.stride(0), t, n, int(groups),
-             int(bool(gate_after)))
+             (2 if gate == "sigmoid" else 1) if gate_after else 0)
 
 
 # --------------------------------------------------------------------------------------- routed feed-forward

@@ -7,7 +7,8 @@ float32; when tied, Wout is the embedding table itself (one buffer), and so it
 is when the configuration says untied but the checkpoint holds no head matrix
 (python/llaisys/models/qwen2.py:196-199).
 
-Options that other designs use: the embedding may add a sinusoidal position vector
+Options that other designs use: the embedding may multiply its rows by a number (`scale`; a tied head still uses the
+table as it is); it may add a sinusoidal position vector
 (`sinusoid_base` b: column 2i gets sin(p b^(-2i/H)), column 2i+1 the cosine of the same
 angle; the frequencies are worked out once in float64 and rounded to float32, the angle is
 float(p) * f in float32); the head may scale its logits (`logit_scale`) and cap them
@@ -36,6 +37,7 @@ class TokenEmbedding(Part):
         self.sinusoid_base = float(spec.args.get("sinusoid_base") or 0.0)
         if self.sinusoid_base < 0:
             raise ValueError("embedding: the base of the position vector must be positive")
+        self.scale = float(spec.args["scale"]) if spec.args.get("scale") is not None else 1.0
         self.table = None
         self.freq = None
 
@@ -53,7 +55,7 @@ class TokenEmbedding(Part):
         return None
 
     def forward(self, ids, out, id_src=None, feedback=None, positions=None, ctx=None, cache=None):
-        ops.embedding(ids, self.table, out, id_src, feedback)
+        ops.embedding(ids, self.table, out, id_src, feedback, scale=self.scale)
         if self.freq is not None:
             if positions is None:
                 raise ValueError("embedding: the position vector needs the tokens' positions")
@@ -75,6 +77,8 @@ class PairHashEmbedding(TokenEmbedding):
             raise ValueError("pair embedding: buckets must be positive and the multipliers not negative")
         if (self.vocab - 1) * (self.mul_prev + self.mul_cur) >= 1 << 62:
             raise ValueError("pair embedding: the multipliers are too large for 64-bit sums")
+        if self.scale != 1.0:
+            raise ValueError("pair embedding: the rows' scale is not supported here")
         self.pair_param = self.prefix + str(a.get("pair_param", "bigram"))
         self.pair = None
 

@@ -105,8 +105,11 @@ class ReluSquaredMLP(FeedForward):
         u = ctx.ws.buffer("mlp.up32", (t, self.inter), torch.float32)
         self.up(xn, u, ws=ctx.ws)
         h = ctx.ws.buffer("mlp.h", (t, self.inter), self.rt.dtype)
-        ops.relu_squared(u, h)
+        self.activate(u, h)
         residual.add_linear(self.down, h)
+
+    def activate(self, u, h):
+        ops.relu_squared(u, h)
 
 
 register_part("feed_forward", "relu2_mlp", ReluSquaredMLP)
@@ -152,3 +155,28 @@ class GeluMLP(FeedForward):
 
 
 register_part("feed_forward", "gelu_mlp", GeluMLP)
+
+
+class XieluMLP(ReluSquaredMLP):
+    """Dense feed-forward with xIELU, whose two numbers p, q are the tensor `act`: y = xielu(xn Wu^T) Wd^T, no biases;
+    z > 0: softplus(p) z^2 + z / 2; z <= 0: (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2.  The two softplus values are
+    worked out once, on the host; the first product is left in float32 and the activation rounds once."""
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        self.names.setdefault("act", "act")
+        self.sp = self.sq = None
+
+    def expected_params(self):
+        return {**super().expected_params(), self.prefix + self.names["act"]: ParamSpec((2,))}
+
+    def load_params(self, get):
+        super().load_params(get)
+        p, q = torch.nn.functional.softplus(get(self.prefix + self.names["act"]).to(torch.float64)).tolist()
+        self.sp, self.sq = p, 0.5 + q
+
+    def activate(self, u, h):
+        ops.xielu(u, h, self.sp, self.sq)
+
+
+register_part("feed_forward", "xielu_mlp", XieluMLP)

@@ -44,6 +44,15 @@ class ResidualStream:
         self._scaled = self._normed = None
         return self.x
 
+    def total(self) -> torch.Tensor:
+        """The sum so far, to be read only."""
+        return self.x
+
+    def gather(self, rows: torch.Tensor, out: torch.Tensor) -> None:
+        """The sum so far at the given tokens."""
+        from ..kernels import ops
+        ops.gather_rows(self.x, rows, out)
+
     def add_linear(self, linear, h: torch.Tensor) -> None:
         """x += h W^T + b."""
         norm, self._scaled, self._normed = self.next_norm, None, None
@@ -150,3 +159,74 @@ class BranchStream(ResidualStream):
 
     def result(self) -> torch.Tensor:
         return self.tensor()
+
+
+class StreamReader:
+    """How a sublayer reads several streams: the norm (an RMS norm) of sum_s weights[s] x_s."""
+
+    def __init__(self, norm):
+        self.norm = norm
+        self.weights = None                  # float32 [streams], bound with the tensors
+
+    def args(self) -> dict:
+        scaling = self.norm.as_scaling()
+        if scaling is None:
+            raise NotImplementedError("streams are read through RMS norms with weights")
+        return {"read": self.weights, "weight": scaling.weight, "eps": scaling.eps}
+
+
+class HyperStream:
+    """Several residual streams side by side (hyper-connections), float32 [T, streams, H].  All are equal to the
+    embedding output at the start, which is kept as ONE row a token until the first write.  `read(reader, out)` hands
+    out the norm of a reader's weighted sum; `write(branch, ...)` replaces all streams at once by their mixture and a
+    share of a sublayer's output, and, where the caller says who reads next, the same kernel leaves that reader's rows."""
+
+    def __init__(self, x: torch.Tensor, ws, streams: int):
+        self.ws = ws
+        self.streams = int(streams)
+        self.shape = x.shape
+        self.state = x
+        self.next_norm = None                # the StreamReader of whoever reads after this block, if known
+        self.next_plain = False
+        self.ws_dtype = torch.bfloat16
+        self._left = None                    # (reader, its rows) left by the last write
+
+    def tensor(self) -> torch.Tensor:
+        raise NotImplementedError("several residual streams have no one tensor to add into")
+
+    def read(self, reader: StreamReader, out: torch.Tensor) -> torch.Tensor:
+        if self._left is not None and self._left[0] is reader:
+            return self._left[1]
+        from ..kernels import ops
+        ops.hyper_step(self.state, None, self.streams, xn=out, **reader.args())
+        return out
+
+    def write(self, branch: BranchStream, mix: torch.Tensor, out: torch.Tensor, next_reader: Optional[StreamReader] = None) -> None:
+        """x_t <- sum_s mix[s, t] x_s + out[t] y for the branch's output y (or the weighted sum of its two)."""
+        from ..kernels import ops
+        y, y2, factors = branch.outputs()
+        dst = self.ws.buffer("stream.several", (self.shape[0], self.streams, self.shape[1]), torch.float32)
+        rows, args = None, {}
+        if next_reader is not None:
+            rows = self.ws.buffer("stream.normed_rows", self.shape, self.ws_dtype)
+            args = {"xn": rows, **next_reader.args()}
+        ops.hyper_step(self.state, dst, self.streams, y, y2, factors, mix, out, **args)
+        self.state = dst
+        self._left = (next_reader, rows) if next_reader is not None else None
+
+    def total(self) -> torch.Tensor:
+        """The sum of the streams."""
+        from ..kernels import ops
+        out = self.ws.buffer("stream.total", self.shape, torch.float32)
+        ops.stream_sum(self._all(), out)
+        return out
+
+    def gather(self, rows: torch.Tensor, out: torch.Tensor) -> None:
+        """The sum of the streams at the given tokens."""
+        from ..kernels import ops
+        ops.stream_sum(self._all(), out, rows)
+
+    def _all(self) -> torch.Tensor:
+        if self.state.dim() == 2:            # nothing has been written: all streams are this row
+            raise NotImplementedError("a model of several streams needs a layer")
+        return self.state

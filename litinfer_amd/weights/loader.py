@@ -34,11 +34,19 @@ INIT_KINDS = ("normal", "one_plus_normal", "zeros", "ones")
 @dataclass(frozen=True)
 class ParamSpec:
     """A tensor a part expects.  `init` says how random weights draw it: "normal" is
-    N(0, 0.02), "one_plus_normal" 1 + N(0, 0.02) (the weights of a norm), "zeros", "ones"."""
+    N(0, 0.02), "one_plus_normal" 1 + N(0, 0.02) (the weights of a norm), "zeros", "ones".
+    `free_dims`: dimensions whose size no configuration gives and the stored tensor decides (the rank of a pair of
+    low-rank matrices); `shape` then holds the size that random weights have there."""
     shape: Tuple[int, ...]
     required: bool = True
     integer: bool = False
     init: str = "normal"
+    free_dims: Tuple[int, ...] = ()
+
+    def matches(self, shape) -> bool:
+        shape = tuple(shape)
+        return len(shape) == len(self.shape) and all(
+            got == want or (i in self.free_dims and got > 0) for i, (got, want) in enumerate(zip(shape, self.shape)))
 
     def __post_init__(self):
         if self.init not in INIT_KINDS:
@@ -88,7 +96,7 @@ def check_entries(expected: Dict[str, ParamSpec], found: Dict[str, Tuple[str, Tu
     for n, (dt, shape) in found.items():
         if n not in expected:
             continue
-        if tuple(shape) != tuple(expected[n].shape):
+        if not expected[n].matches(shape):
             wrong_shape.append((n, expected[n].shape, shape))
         if expected[n].integer and dt not in _INT_ST:
             wrong_dtype.append((n, f"expected an integer table, found {dt}"))

@@ -15,11 +15,11 @@ def require_gpu(device):
     return None
 
 
-def embedding(ids, table, out, id_src=None, feedback=None):
+def embedding(ids, table, out, id_src=None, feedback=None, scale=1.0):
     ids = ids.long()
     if id_src is not None:
         ids = torch.where(id_src >= 0, feedback.long()[id_src.clamp(min=0).long()], ids)
-    out.copy_(table[ids].float())
+    out.copy_(scale * table[ids].float())
 
 
 def rmsnorm(x, weight, eps, out):
