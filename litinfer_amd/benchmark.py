@@ -819,9 +819,49 @@ def kufolorn_config(size: str, layers: int, vocab: int = 32000) -> Dict[str, obj
                         "mlp": dense if i % 2 == 0 else moe} for i in range(layers)]}
 
 
+DIMELIX_SIZES = {         # delta heads, key and value size of a delta head; streams
+    "1.5b": (24, 64, 4),
+    "7b": (28, 128, 4),
+}
+
+
+def dimelix_config(size: str, layers: int, vocab: int = 32000) -> Dict[str, object]:
+    """A Dimelix model at the layer sizes of a Qwen2 family member: latent attention without positions, windowed attention
+    with a distance bias beside a channel-wise delta rule, and rotary attention with a sink in turn, layers 1..2 passed twice."""
+    width, heads, kv, dim, ff, rank, _, _ = DESIGN_SIZES[size]
+    dheads, ddim, streams = DIMELIX_SIZES[size]
+    mlp = {"kind": "dense", "ff": ff}
+    latent = {"type": "latent_attention", "mlp": mlp,
+              "mixer": {"heads": heads, "dim": dim, "vdim": dim, "kv_rank": rank, "scale": dim ** -0.5}}
+    par = {"type": "parallel", "mlp": mlp,
+           "mixer": {"left": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": DESIGN_WINDOW}},
+                     "right": {"heads": dheads, "dim": ddim}, "left_scale": 0.8, "right_scale": 0.6}}
+    attn = {"type": "attention", "mlp": mlp,
+            "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "rot": {"base": 10000.0, "dims": dim // 2}}}
+    return {"architecture": "Dimelix", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "streams": streams,
+            "embedding": {"scale": 2.0}, "logit_softcap": 30.0, "layers": [(latent, par, attn)[i % 3] for i in range(layers)],
+            "loop": {"start": 1, "stop": 3, "times": 2} if layers >= 4 else None}
+
+
+def tovasun_beside_dimelix_config(size: str, layers: int, vocab: int = 32000) -> Dict[str, object]:
+    """The closest existing model to Dimelix: a Tovasun model with the same order of latent (no window), windowed and
+    full attention layers, the same loop and feed-forwards of the same two matrices; no delta rule, one residual stream."""
+    width, heads, kv, dim, ff, rank, rot, _ = DESIGN_SIZES[size]
+    mlp = {"kind": "dense", "ff": ff}
+    latent = {"type": "latent_attention", "mlp": mlp,
+              "mixer": {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": dim, "kv_rank": rank, "scale": (dim + rot) ** -0.5,
+                        "rot": {"base": 10000.0, "dims": rot}}}
+    full = {"type": "attention", "mlp": mlp,
+            "mixer": {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "rot": {"base": 10000.0, "dims": dim // 2}}}
+    windowed = {**full, "mixer": {**full["mixer"], "mask": {"size": DESIGN_WINDOW}}}
+    return {"architecture": "Tovasun", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+            "layers": [(latent, windowed, full)[i % 3] for i in range(layers)],
+            "loop": {"start": 1, "stop": 3, "times": 2} if layers >= 4 else None}
+
+
 def compare_designs(a) -> Dict[str, object]:
-    """Prefill and decode throughput of a second design (`--design`: Tovasun, Sogenex or Nusuvik) beside Qwen2 (Nusuvik:
-    beside its closest relative, an all-latent Tovasun model) at the same width, heads, (active) feed-forward width,
+    """Prefill and decode throughput of a second design (`--design`) beside Qwen2 or, where another model is closer
+    (Nusuvik, Kufolorn, Dimelix), beside that one, at the same width, heads, (active) feed-forward width,
     window and number of layer runs (random weights, random cache content)."""
     import numpy as np
     import torch
@@ -833,11 +873,13 @@ def compare_designs(a) -> Dict[str, object]:
     for size in sizes:
         layers = a.layers or 6
         design = getattr(a, "design", None) or "tovasun"
-        tcfg = {"sogenex": sogenex_config, "nusuvik": nusuvik_config, "kufolorn": kufolorn_config}.get(design, tovasun_config)(size, layers)
+        tcfg = {"sogenex": sogenex_config, "nusuvik": nusuvik_config, "kufolorn": kufolorn_config, "dimelix": dimelix_config}.get(design, tovasun_config)(size, layers)
         runs = layers + (2 if tcfg.get("loop") else 0)
         width, heads, kv, dim, ff = DESIGN_SIZES[size][:5]
         if design == "nusuvik":
             beside, qcfg = "tovasun", tovasun_latent_config(size, layers)
+        elif design == "dimelix":
+            beside, qcfg = "tovasun", tovasun_beside_dimelix_config(size, layers)
         elif design == "kufolorn":                   # its closest relative: recurrent layers, every third one attention, routed feed-forwards
             beside, qcfg = "sogenex", sogenex_config(size, layers)
         else:
@@ -849,7 +891,7 @@ def compare_designs(a) -> Dict[str, object]:
             if a.only and name != a.only:
                 continue
             eng = Engine.from_random(cfg, seed=0, dtype=ENGINE_DTYPE[a.dtype], device=dev, page_size=PAGE,
-                                     num_pages=(64 * ((2 if design in ("nusuvik", "kufolorn") else 1) * DESIGN_WINDOW + 64) + 2 * PREFILL_TOKENS) // PAGE,
+                                     num_pages=(64 * ((2 if design in ("nusuvik", "kufolorn", "dimelix") else 1) * DESIGN_WINDOW + 64) + 2 * PREFILL_TOKENS) // PAGE,
                                      max_seqs=65)
             for g in eng.cache.groups:
                 for data in g.data.values():
@@ -903,7 +945,7 @@ def compare_designs(a) -> Dict[str, object]:
     first = out[sizes[0]]
     title = design.capitalize()
     return {"metric": f"decode tok/s ({title} at the Qwen2-{sizes[0]} layer sizes, batch {a.batch}, "
-                      + ("no window)" if design in ("nusuvik", "kufolorn") else f"window {DESIGN_WINDOW})"),
+                      + ("no window)" if design in ("nusuvik", "kufolorn") else f"window {DESIGN_WINDOW} in every third layer)" if design == "dimelix" else f"window {DESIGN_WINDOW})"),
             "value": first[a.only or design][f"decode_b{a.batch}_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": a.steps,
             "warmup": a.warmup, "ms_per_step": first[a.only or design][f"decode_b{a.batch}_ms"], "higher_is_better": True,
             "scaling": "weak", "vs_baseline": None, "dtype": a.dtype,
@@ -925,8 +967,8 @@ def main(argv: Optional[List[str]] = None) -> int:
     ap.add_argument("--mode", default="headline", choices=["headline", "serving", "long", "sweep", "designs"])
     ap.add_argument("--shape", default=None, choices=sorted(SHAPES),
                     help="sweep: the member of the family whose layer sizes are taken (7b); designs: 1.5b or 7b (both)")
-    ap.add_argument("--design", default="tovasun", choices=["tovasun", "sogenex", "nusuvik", "kufolorn"],
-                    help="designs: the design that is set beside Qwen2 (Nusuvik: beside an all-latent Tovasun; Kufolorn: beside Sogenex)")
+    ap.add_argument("--design", default="tovasun", choices=["tovasun", "sogenex", "nusuvik", "kufolorn", "dimelix"],
+                    help="designs: the design that is set beside Qwen2 (Nusuvik: beside an all-latent Tovasun; Kufolorn: beside Sogenex; Dimelix: beside a Tovasun of the same layer order)")
     ap.add_argument("--only", default=None, help="designs: run one of the two models only (its name)")
     ap.add_argument("--page-order-seed", type=int, default=0,
                     help="headline: the cache's pages are handed out in a shuffled order, as a pool that has served requests "

@@ -555,6 +555,20 @@ extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_ra
 // in LDS DR_TB tokens at a time (normed there: sixteen lanes a token add the squares in a fixed order).
 // Rows of xkq: [v: heads x vdim | k: G x N | q: G x N]; rows of ba: [b: heads | a: heads].
 #define DR_TB 16
+
+// The sum over NS neighbouring lanes (NS = 1, 2, 4, 8, 16), in every lane of the group, by lane moves inside the vector
+// ALU: quad_perm [1,0,3,2] and [2,3,0,1], then row_half_mirror and row_mirror (whose partners hold the other half's sum).
+template <int CTRL> __device__ __forceinline__ float lane_move(float v) {
+    return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xF, 0xF, true));
+}
+template <int NS> __device__ __forceinline__ float lanes_sum(float v) {
+    if constexpr (NS >= 2) v += lane_move<0xB1>(v);
+    if constexpr (NS >= 4) v += lane_move<0x4E>(v);
+    if constexpr (NS >= 8) v += lane_move<0x141>(v);
+    if constexpr (NS >= 16) v += lane_move<0x140>(v);
+    return v;
+}
+
 //
 // A step's portion of a request is cut into chunks of Q tokens that run side by side, as the state-space recurrence's
 // are.  Here a token's step is S <- A_t S + beta_t k_t v_t^T with the MATRIX A_t = g_t (I - beta_t k_t k_t^T), so what a
@@ -685,9 +699,7 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void delta_scan_kernel(
                     for (int cc = 0; cc < CW; ++cc) ks[cc] = fmaf(S[4 * r4 + j][cc], kk[j], ks[cc]);
             }
 #pragma unroll
-            for (int o = 1; o < NS; o <<= 1)
-#pragma unroll
-                for (int cc = 0; cc < CW; ++cc) ks[cc] += __shfl_xor(ks[cc], o, LI_WAVE);
+            for (int cc = 0; cc < CW; ++cc) ks[cc] = lanes_sum<NS>(ks[cc]);
             float u[CW], ov[CW];
 #pragma unroll
             for (int cc = 0; cc < CW; ++cc) { u[cc] = beta * (xv[cc] - gd * ks[cc]); ov[cc] = 0.f; }
@@ -708,9 +720,7 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void delta_scan_kernel(
             }
             if (MODE == 0) {
 #pragma unroll
-                for (int o = 1; o < NS; o <<= 1)
-#pragma unroll
-                    for (int cc = 0; cc < CW; ++cc) ov[cc] += __shfl_xor(ov[cc], o, LI_WAVE);
+                for (int cc = 0; cc < CW; ++cc) ov[cc] = lanes_sum<NS>(ov[cc]);
                 if (s == 0) {
                     float* yr = y + (size_t)(t0 + b0 + tt) * y_stride + (size_t)head * vdim + p;
                     if constexpr (CW == 4) {
@@ -752,88 +762,111 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void delta_scan_kernel(
 }
 
 // carry[chunk] holds what the chunk alone built up from zero, pmat[chunk] its matrix (transposed); afterwards carry[chunk]
-// holds the state with which the chunk begins.  A block takes a request, a head and DC_COLS columns of the state, chunk
-// after chunk; the state's columns lie in LDS, thread (slice, column) owns PER consecutive values of the column
-// (DC_SLICES * PER >= N).  A chunk's step is a product P x (state's columns): the thread walks P's rows j, which hold its
-// PER values side by side, DC_AHEAD rows at a time: their loads are issued
-// together and without conditions (a value past N reads the row's last one and is never stored), so that a trip to memory
-// serves DC_AHEAD rows and not one.
-#define DC_COLS 16
-#define DC_SLICES 16
-#define DC_ROUND 16                 // the state's rows in LDS are rounded up to this: the most rows a trip takes
-template <int PER, int DC_AHEAD, bool VEC>      // VEC: N and PER multiples of 4, P on 16 bytes: a row's values in 16-byte pieces
-__global__ __launch_bounds__(DC_COLS * DC_SLICES) void delta_carry_kernel(
+// holds the state with which the chunk begins.  A block takes a request, a head and 16 columns of the state, which lie in
+// LDS, chunk after chunk: S_in(c + 1) = P_c S_in(c) + S_own(c), on the float32 matrix cores (v_mfma_f32_16x16x4_f32: row
+// operand P, one value a lane (row lane % 16, k lane / 16), which lie side by side in a row of the stored transpose; column
+// operand the state from LDS; the accumulator starts as S_own and holds rows 4 (lane / 16) + r of column lane % 16).  A
+// wave owns RT tiles of 16 rows; P comes in groups of 64 k's, and a group is on its way while the one before it is used,
+// across the chunks' borders too (P and S_own do not depend on the state).  Rows and k's past N: loads are clamped, the
+// state's rows past N are zeros in LDS, and results past N are never stored.
+#define DC_GROUP 16                 // matrix instructions (4 k's each) of a group
+typedef float dc_f32x4 __attribute__((ext_vector_type(4)));
+template <int RT>
+__global__ __launch_bounds__(256) void delta_carry_kernel(
     float* __restrict__ carry, const float* __restrict__ pmat, const float* __restrict__ state, const int* __restrict__ slots,
     const int* __restrict__ q_len, const int* __restrict__ chunk_first, int heads, int vdim, int N, int Q) {
-    extern __shared__ float run[];                      // [N rounded up to DC_ROUND][DC_COLS + 1]
-    const int seg = blockIdx.x, head = blockIdx.y, cl = threadIdx.x % DC_COLS, sl = threadIdx.x / DC_COLS;
-    const int col = blockIdx.z * DC_COLS + cl;
+    extern __shared__ float run[];                      // [N rounded up to 64][16]
+    const int seg = blockIdx.x, head = blockIdx.y, lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+    const int cl = lane & 15, kq = lane >> 4, col = blockIdx.z * 16 + cl;
     const int nch = (q_len[seg] + Q - 1) / Q, base = chunk_first[seg];
-    const int n0 = sl * PER;
     const bool on = col < vdim;
-    const int NA = (N + DC_ROUND - 1) / DC_ROUND * DC_ROUND;
+    const int groups = (N + 4 * DC_GROUP - 1) / (4 * DC_GROUP);
     const float* stp = state + ((size_t)slots[seg] * heads + head) * N * vdim;
-    int off[PER];                                       // the thread's values within a row of P (clamped: loads carry no conditions)
-#pragma unroll
-    for (int i = 0; i < PER; ++i) off[i] = n0 + i < N ? n0 + i : N - 1;
-#pragma unroll
-    for (int i = 0; i < PER; ++i)
-        if (n0 + i < NA) run[(n0 + i) * (DC_COLS + 1) + cl] = (on && n0 + i < N) ? stp[(size_t)(n0 + i) * vdim + col] : 0.f;
-    __syncthreads();
-    for (int k = 0; k < nch; ++k) {
-        float* at = carry + ((size_t)(base + k) * heads + head) * N * vdim;
-        const float* pt = pmat + ((size_t)(base + k) * heads + head) * N * N;
-        float acc[PER];
-        const bool more = k + 1 < nch;
-#pragma unroll
-        for (int i = 0; i < PER; ++i) acc[i] = (more && on && n0 + i < N) ? at[(size_t)(n0 + i) * vdim + col] : 0.f;
-        if (more) {
-            for (int j0 = 0; j0 < N; j0 += DC_AHEAD) {
-                float pv[DC_AHEAD][PER], cv[DC_AHEAD];
-#pragma unroll
-                for (int u = 0; u < DC_AHEAD; ++u) {
-                    const float* prow = pt + (size_t)(j0 + u < N ? j0 + u : N - 1) * N;
-                    if constexpr (VEC) {
-#pragma unroll
-                        for (int v = 0; v < PER / 4; ++v) {
-                            const float4 t4 = *reinterpret_cast<const float4*>(prow + (n0 + 4 * v < N ? n0 + 4 * v : N - 4));
-                            pv[u][4 * v] = t4.x; pv[u][4 * v + 1] = t4.y; pv[u][4 * v + 2] = t4.z; pv[u][4 * v + 3] = t4.w;
-                        }
-                    } else {
-#pragma unroll
-                        for (int i = 0; i < PER; ++i) pv[u][i] = prow[off[i]];
-                    }
-                    cv[u] = run[(j0 + u) * (DC_COLS + 1) + cl];             // (rows N .. NA - 1 of the state are zeros)
-                }
-#pragma unroll
-                for (int u = 0; u < DC_AHEAD; ++u)
-#pragma unroll
-                    for (int i = 0; i < PER; ++i) acc[i] = fmaf(pv[u][i], cv[u], acc[i]);
-            }
-        }
-        // the chunk begins with `run`; the next one with what has just been added up
-#pragma unroll
-        for (int i = 0; i < PER; ++i)
-            if (on && n0 + i < N) at[(size_t)(n0 + i) * vdim + col] = run[(n0 + i) * (DC_COLS + 1) + cl];
-        __syncthreads();
-#pragma unroll
-        for (int i = 0; i < PER; ++i)
-            if (n0 + i < N) run[(n0 + i) * (DC_COLS + 1) + cl] = acc[i];
-        __syncthreads();
+    for (int i = threadIdx.x; i < groups * 4 * DC_GROUP * 16; i += 256) {
+        const int n = i / 16, cc = blockIdx.z * 16 + i % 16;
+        run[i] = (n < N && cc < vdim) ? stp[(size_t)n * vdim + cc] : 0.f;
     }
+    int arow[RT], crow[RT];                             // this lane's row of P (operand) and its first row of the result
+#pragma unroll
+    for (int rt = 0; rt < RT; ++rt) {
+        const int r = 16 * (w * RT + rt);
+        arow[rt] = r + cl < N ? r + cl : N - 1;
+        crow[rt] = r + 4 * kq;
+    }
+    float pa[RT][DC_GROUP], pb[RT][DC_GROUP], own[RT][4];
+    dc_f32x4 acc[RT];
+    const int steps = (nch - 1) * groups;               // a request's last chunk only takes the state it begins with
+    auto fetch = [&](int st, float (&p)[RT][DC_GROUP]) {
+        if (st >= steps) return;
+        const float* pt = pmat + ((size_t)(base + st / groups) * heads + head) * N * N;
+        const int k0 = (st % groups) * 4 * DC_GROUP + kq;
+#pragma unroll
+        for (int x = 0; x < DC_GROUP; ++x) {
+            const int k = k0 + 4 * x < N ? k0 + 4 * x : N - 1;
+#pragma unroll
+            for (int rt = 0; rt < RT; ++rt) p[rt][x] = pt[(size_t)k * N + arow[rt]];
+        }
+    };
+    auto own_of = [&](int k) {
+        if (k + 1 >= nch) return;
+        const float* at = carry + ((size_t)(base + k) * heads + head) * N * vdim + (on ? col : 0);
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) own[rt][r] = at[(size_t)(crow[rt] + r < N ? crow[rt] + r : N - 1) * vdim];
+    };
+    auto leave = [&](int k) {                           // the state with which chunk k begins
+        float* at = carry + ((size_t)(base + k) * heads + head) * N * vdim + col;
+#pragma unroll
+        for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r)
+                if (on && crow[rt] + r < N) at[(size_t)(crow[rt] + r) * vdim] = run[(crow[rt] + r) * 16 + cl];
+    };
+    auto step = [&](int st, const float (&p)[RT][DC_GROUP]) {
+        const int k = st / groups, g = st % groups;
+        if (g == 0) {
+#pragma unroll
+            for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) acc[rt][r] = own[rt][r];
+            own_of(k + 1);
+            leave(k);
+        }
+#pragma unroll
+        for (int x = 0; x < DC_GROUP; ++x) {
+            const float b = run[(g * 4 * DC_GROUP + 4 * x + kq) * 16 + cl];
+#pragma unroll
+            for (int rt = 0; rt < RT; ++rt) acc[rt] = __builtin_amdgcn_mfma_f32_16x16x4f32(p[rt][x], b, acc[rt], 0, 0, 0);
+        }
+        if (g == groups - 1) {
+            __syncthreads();
+#pragma unroll
+            for (int rt = 0; rt < RT; ++rt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r)
+                    if (crow[rt] + r < N) run[(crow[rt] + r) * 16 + cl] = acc[rt][r];
+            __syncthreads();
+        }
+    };
+    fetch(0, pa);
+    own_of(0);
+    __syncthreads();
+    for (int st = 0; st < steps; st += 2) {
+        fetch(st + 1, pb);
+        step(st, pa);
+        fetch(st + 2, pa);
+        if (st + 1 < steps) step(st + 1, pb);
+    }
+    leave(nch - 1);
 }
 
 static void delta_carry_launch(float* carry, const float* pmat, const float* state, const int* slots, const int* q_len,
                                const int* chunk_first, int heads, int vdim, int N, int Q, int segs, hipStream_t stream) {
-    const dim3 grid(segs, heads, (vdim + DC_COLS - 1) / DC_COLS);
-    const size_t lds = (size_t)((N + DC_ROUND - 1) / DC_ROUND * DC_ROUND) * (DC_COLS + 1) * sizeof(float);
-    const int per = (N + DC_SLICES - 1) / DC_SLICES;
-#define DC_GO(P_, V_) delta_carry_kernel<P_, 8, V_><<<grid, DC_COLS * DC_SLICES, lds, stream>>>(carry, pmat, state, slots, q_len, chunk_first, heads, vdim, N, Q)
-    const bool vec = N % 4 == 0 && ((uintptr_t)pmat % 16) == 0;
-    if (per <= 1) DC_GO(1, false); else if (per <= 2) DC_GO(2, false);
-    else if (per <= 4) { if (vec) DC_GO(4, true); else DC_GO(4, false); }
-    else if (per <= 8) { if (vec) DC_GO(8, true); else DC_GO(8, false); }
-    else { if (vec) DC_GO(16, true); else DC_GO(16, false); }
+    const dim3 grid(segs, heads, (vdim + 15) / 16);
+    const size_t lds = (size_t)((N + 4 * DC_GROUP - 1) / (4 * DC_GROUP) * 4 * DC_GROUP) * 16 * sizeof(float);
+#define DC_GO(R_) delta_carry_kernel<R_><<<grid, 256, lds, stream>>>(carry, pmat, state, slots, q_len, chunk_first, heads, vdim, N, Q)
+    if (N <= 64) DC_GO(1); else if (N <= 128) DC_GO(2); else DC_GO(4);
 #undef DC_GO
 }
 
@@ -929,25 +962,26 @@ extern "C" int li_delta_scan(const float* xkq, long x_stride, const float* ba, l
 // so a portion runs as chunks side by side exactly as the gated delta rule's does (same modes, same carry kernel), and
 // the layout is the same: a lane owns CW neighbouring columns x NR state values, NS neighbouring lanes share a column.
 // No heads share keys here: the waves of a block are columns of ONE head (as many waves as the head has units, up to
-// four) and share u, a, w and r, which are worked out when a block of TB tokens is staged in LDS.
+// four) and share u, a, w and r, which are worked out when a block of CD_TB tokens is staged in LDS; the next block's raw
+// values are on their way in registers meanwhile.
 // Rows of x: [r: heads x N | k: heads x N | v: heads x vdim | a: heads x N]; rows of low: heads x N.
 #define CD_DECAY 0.6065306597126334f               // exp(-1/2)
+#define CD_TB 8                                    // tokens staged at a time
 
-template <int NR, int NS, int CW, int MODE>
-__global__ __launch_bounds__(256) void channel_delta_kernel(
+template <int NR, int NS, int CW, int NW, int MODE>
+__global__ __launch_bounds__(64 * NW) void channel_delta_kernel(
     const float* __restrict__ x, long x_stride, const float* __restrict__ low, long low_stride, float* __restrict__ state,
     const int* __restrict__ slots, const int* __restrict__ q_start, const int* __restrict__ q_len,
     const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, float* __restrict__ pmat,
     float* __restrict__ y, long y_stride, int heads, int vdim, int N, int Q) {
-    constexpr int NP = NR * NS, PW = 64 * CW / NS, TB = NP > 128 ? 8 : 16;
-    extern __shared__ __align__(16) float lds[];
-    const int nthreads = blockDim.x, nw = nthreads >> 6;
-    float* sU = lds;                                   // [TB][NP] each
-    float* sA = sU + TB * NP;
-    float* sW = sA + TB * NP;
-    float* sR = sW + TB * NP;
-    float* sN = sR + TB * NP;                          // [TB]: |k|
-    float* sX = sN + TB;                               // [nw][TB][PW]
+    constexpr int NP = NR * NS, PW = 64 * CW / NS, TB = CD_TB, NT = 64 * NW;
+    constexpr int IT = (TB * NP + NT - 1) / NT, IV = (TB * PW + 63) / 64;      // staged values a thread (keys' vectors; a wave's v)
+    __shared__ __attribute__((aligned(16))) float sU[TB * NP];
+    __shared__ __attribute__((aligned(16))) float sA[TB * NP];
+    __shared__ __attribute__((aligned(16))) float sW[TB * NP];
+    __shared__ __attribute__((aligned(16))) float sR[MODE == 0 ? TB * NP : 4];
+    __shared__ __attribute__((aligned(16))) float sX[NW * TB * PW];
+    __shared__ float sN[TB];                            // |k|
     const int bx = blockIdx.x;
     const int seg = chunk_seg ? chunk_seg[bx] : bx;
     if (seg < 0) return;
@@ -960,10 +994,10 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
     const int t0 = q_start[seg] + first;
     // units of a head: blocks of PW value columns, and in MODE 1 behind them blocks of PW columns of P
     const int PSV = (vdim + PW - 1) / PW, PS = PSV + (MODE == 1 ? (N + PW - 1) / PW : 0);
-    const int ublocks = (PS + nw - 1) / nw;
+    const int ublocks = (PS + NW - 1) / NW;
     const int head = blockIdx.y / ublocks, ub = blockIdx.y % ublocks;
     const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    const int unit = ub * nw + w;
+    const int unit = ub * NW + w;
     const bool active = unit < PS;
     const int sub = active ? unit : 0;
     const bool is_p = MODE == 1 && sub >= PSV;
@@ -976,6 +1010,27 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
     const float* lw0 = low + (size_t)head * N;
     float* st = state + ((size_t)slots[seg] * heads + head) * N * vdim;
     const float* src = chunk_seg ? carry + ((size_t)bx * heads + head) * N * vdim : st;
+    // a block of tokens on its way: raw values in registers (a place past the end reads a valid one and is blanked below)
+    float gk[IT], ga[IT], gl[IT], gr[IT], gv[IV];
+    auto fetch = [&](int b0) {
+#pragma unroll
+        for (int it = 0; it < IT; ++it) {
+            const int i = threadIdx.x + NT * it, tt = i / NP, n = i % NP;
+            const size_t row = (size_t)(t0 + (tt < TB && b0 + tt < ntok ? b0 + tt : 0));
+            const int nn = n < N ? n : 0;
+            gk[it] = xr0[row * x_stride + n_key + nn];
+            ga[it] = xa0[row * x_stride + nn];
+            gl[it] = lw0[row * low_stride + nn];
+            if (MODE == 0) gr[it] = xr0[row * x_stride + nn];
+        }
+#pragma unroll
+        for (int it = 0; it < IV; ++it) {
+            const int i = lane + 64 * it, tt = i / PW, pp = pbase + i % PW;
+            const size_t row = (size_t)(t0 + (tt < TB && b0 + tt < ntok ? b0 + tt : 0));
+            gv[it] = xv0[row * x_stride + (!is_p && pp < vdim ? pp : 0)];
+        }
+    };
+    fetch(0);
     float S[NR][CW];
 #pragma unroll
     for (int r = 0; r < NR; ++r) {
@@ -994,37 +1049,35 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
     }
     for (int b0 = 0; b0 < ntok; b0 += TB) {
         __syncthreads();
-        for (int i = threadIdx.x; i < TB * NP; i += nthreads) {
-            const int tt = i / NP, n = i % NP;
+#pragma unroll
+        for (int it = 0; it < IT; ++it) {
+            const int i = threadIdx.x + NT * it, tt = i / NP, n = i % NP;
             const bool ok = b0 + tt < ntok && n < N;
-            const size_t row = (size_t)(t0 + b0 + (b0 + tt < ntok ? tt : 0));
-            const int nn = n < N ? n : 0;
-            const float kv = xr0[row * x_stride + n_key + nn], av = xa0[row * x_stride + nn], lv = lw0[row * low_stride + nn];
-            sU[i] = ok ? kv : 0.f;
-            sA[i] = ok ? 1.0f / (1.0f + expf(-av)) : 0.f;
-            sW[i] = ok ? expf(-CD_DECAY / (1.0f + expf(-lv))) : 1.f;
-            if (MODE == 0) sR[i] = ok ? xr0[row * x_stride + nn] : 0.f;
-        }
-        if (active) {
-            for (int i = lane; i < TB * PW; i += 64) {
-                const int tt = i / PW, pp = pbase + i % PW;
-                const bool ok = !is_p && b0 + tt < ntok && pp < vdim;
-                sX[w * TB * PW + i] = ok ? xv0[(size_t)(t0 + b0 + tt) * x_stride + pp] : 0.f;
+            if (TB * NP % NT == 0 || i < TB * NP) {
+                sU[i] = ok ? gk[it] : 0.f;
+                sA[i] = ok ? 1.0f / (1.0f + expf(-ga[it])) : 0.f;
+                sW[i] = ok ? expf(-CD_DECAY / (1.0f + expf(-gl[it]))) : 1.f;
+                if (MODE == 0) sR[i] = ok ? gr[it] : 0.f;
             }
+        }
+#pragma unroll
+        for (int it = 0; it < IV; ++it) {
+            const int i = lane + 64 * it, tt = i / PW, pp = pbase + i % PW;
+            if (TB * PW % 64 == 0 || i < TB * PW) sX[w * TB * PW + i] = (!is_p && b0 + tt < ntok && pp < vdim) ? gv[it] : 0.f;
         }
         __syncthreads();
         // unit keys: sixteen neighbouring lanes share a token's N values
-        for (int tt = threadIdx.x >> 4; tt < TB; tt += nthreads >> 4) {
+        for (int tt = threadIdx.x >> 4; tt < TB; tt += NT / 16) {
             const int part = threadIdx.x & 15;
             float sk = 0.f;
             for (int n = part; n < NP; n += 16) sk = fmaf(sU[tt * NP + n], sU[tt * NP + n], sk);
-#pragma unroll
-            for (int o = 1; o < 16; o <<= 1) sk += __shfl_xor(sk, o, LI_WAVE);
+            sk = lanes_sum<16>(sk);
             const float len = sqrtf(sk + 1e-6f), inv = 1.0f / len;
             for (int n = part; n < NP; n += 16) sU[tt * NP + n] *= inv;
             if (part == 0) sN[tt] = len;
         }
         __syncthreads();
+        if (b0 + TB < ntok) fetch(b0 + TB);              // (on its way while this block is worked on)
         if (!active) continue;
         const int nt = (ntok - b0 < TB) ? ntok - b0 : TB;
         for (int tt = 0; tt < nt; ++tt) {
@@ -1035,7 +1088,7 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
             const float4* Up = reinterpret_cast<const float4*>(sU + tt * NP + s * NR);
             const float4* Ap = reinterpret_cast<const float4*>(sA + tt * NP + s * NR);
             const float4* Wp = reinterpret_cast<const float4*>(sW + tt * NP + s * NR);
-            const float4* Rp = reinterpret_cast<const float4*>(sR + tt * NP + s * NR);
+            const float4* Rp = reinterpret_cast<const float4*>(sR + (MODE == 0 ? tt * NP + s * NR : 0));
 #pragma unroll
             for (int r4 = 0; r4 < NR / 4; ++r4) {
                 const float4 uv = Up[r4];
@@ -1046,9 +1099,7 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
                     for (int cc = 0; cc < CW; ++cc) ks[cc] = fmaf(S[4 * r4 + j][cc], uu[j], ks[cc]);
             }
 #pragma unroll
-            for (int o = 1; o < NS; o <<= 1)
-#pragma unroll
-                for (int cc = 0; cc < CW; ++cc) ks[cc] += __shfl_xor(ks[cc], o, LI_WAVE);
+            for (int cc = 0; cc < CW; ++cc) ks[cc] = lanes_sum<NS>(ks[cc]);
 #pragma unroll
             for (int r4 = 0; r4 < NR / 4; ++r4) {
                 const float4 uv = Up[r4], av = Ap[r4], wv = Wp[r4];
@@ -1066,9 +1117,7 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
             }
             if (MODE == 0) {
 #pragma unroll
-                for (int o = 1; o < NS; o <<= 1)
-#pragma unroll
-                    for (int cc = 0; cc < CW; ++cc) ov[cc] += __shfl_xor(ov[cc], o, LI_WAVE);
+                for (int cc = 0; cc < CW; ++cc) ov[cc] = lanes_sum<NS>(ov[cc]);
                 if (s == 0) {
                     float* yr = y + (size_t)(t0 + b0 + tt) * y_stride + (size_t)head * vdim + p;
                     if constexpr (CW == 4) {
@@ -1108,19 +1157,17 @@ __global__ __launch_bounds__(256) void channel_delta_kernel(
     }
 }
 
-template <int NR, int NS, int CW>
+// W0, W1: waves a block without and with P's columns (as many as a head of as many columns as rows has units, up to four)
+template <int NR, int NS, int CW, int W0, int W1>
 static int channel_delta_launch(const float* x, long x_stride, const float* low, long low_stride, float* state, const int* slots,
                                 const int* q_start, const int* q_len, int* chunk_tab, float* carry, float* pmat, float* y,
                                 long y_stride, int heads, int vdim, int N, int Q, int segs, int max_chunks, bool chunked,
                                 hipStream_t stream) {
-    constexpr int NP = NR * NS, PW = 64 * CW / NS, TB = NP > 128 ? 8 : 16;
+    constexpr int PW = 64 * CW / NS;
     const int PSV = (vdim + PW - 1) / PW, PSP = (N + PW - 1) / PW;
-    auto waves = [](int units) { return units < 4 ? units : 4; };
-    auto lds = [](int nw) { return (size_t)(4 * TB * NP + TB + nw * TB * PW) * sizeof(float); };
-    const int w0 = waves(PSV), w1 = waves(PSV + PSP);
-    const int ub0 = (PSV + w0 - 1) / w0, ub1 = (PSV + PSP + w1 - 1) / w1;
+    const int ub0 = (PSV + W0 - 1) / W0, ub1 = (PSV + PSP + W1 - 1) / W1;
     if (!chunked) {
-        channel_delta_kernel<NR, NS, CW, 0><<<dim3(segs, heads * ub0), 64 * w0, lds(w0), stream>>>(
+        channel_delta_kernel<NR, NS, CW, W0, 0><<<dim3(segs, heads * ub0), 64 * W0, 0, stream>>>(
             x, x_stride, low, low_stride, state, slots, q_start, q_len, nullptr, nullptr, nullptr, nullptr, y, y_stride, heads, vdim, N, Q);
         return li_launch_status();
     }
@@ -1128,10 +1175,10 @@ static int channel_delta_launch(const float* x, long x_stride, const float* low,
     int* chunk_idx = chunk_tab + max_chunks;
     int* chunk_first = chunk_tab + 2 * max_chunks;
     ssm_chunk_index_kernel<<<1, 256, 0, stream>>>(q_len, segs, Q, max_chunks, chunk_seg, chunk_idx, chunk_first);
-    channel_delta_kernel<NR, NS, CW, 1><<<dim3(max_chunks, heads * ub1), 64 * w1, lds(w1), stream>>>(
+    channel_delta_kernel<NR, NS, CW, W1, 1><<<dim3(max_chunks, heads * ub1), 64 * W1, 0, stream>>>(
         x, x_stride, low, low_stride, state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, pmat, y, y_stride, heads, vdim, N, Q);
     delta_carry_launch(carry, pmat, state, slots, q_len, chunk_first, heads, vdim, N, Q, segs, stream);
-    channel_delta_kernel<NR, NS, CW, 0><<<dim3(max_chunks, heads * ub0), 64 * w0, lds(w0), stream>>>(
+    channel_delta_kernel<NR, NS, CW, W0, 0><<<dim3(max_chunks, heads * ub0), 64 * W0, 0, stream>>>(
         x, x_stride, low, low_stride, state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, pmat, y, y_stride, heads, vdim, N, Q);
     return li_launch_status();
 }
@@ -1155,25 +1202,19 @@ extern "C" int li_channel_delta(const float* x, long x_stride, const float* low,
         pmat = carry + (size_t)max_chunks * heads * N * vdim;
     }
 #define CD_ARGS x, x_stride, low, low_stride, state, slots, q_start, q_len, chunk_tab, carry, pmat, y, y_stride, heads, vdim, N, Q,                 segs, max_chunks, chunked, stream
-    const bool aligned = ((uintptr_t)state | (uintptr_t)y | (uintptr_t)carry) % 16 == 0 && y_stride % 4 == 0;
-    int qs = 0, qr = 0;
-    if (aligned && ssm_quad_layout(N, vdim, &qs, &qr)) {
-#define CD_QUAD(NR_, NS_) if (qr == NR_ && qs == NS_) return channel_delta_launch<NR_, NS_, 4>(CD_ARGS);
-        CD_QUAD(4, 2) CD_QUAD(8, 2) CD_QUAD(16, 2) CD_QUAD(32, 2)
-        CD_QUAD(4, 4) CD_QUAD(8, 4) CD_QUAD(16, 4) CD_QUAD(32, 4)
-        CD_QUAD(4, 8) CD_QUAD(8, 8) CD_QUAD(16, 8) CD_QUAD(32, 8)
-        CD_QUAD(4, 16) CD_QUAD(8, 16) CD_QUAD(16, 16)
-#undef CD_QUAD
+    // four columns a lane and rows of the state in 16-byte pieces, or (sizes that are no multiple of four) one column a lane
+    const bool quad = vdim % 4 == 0 && ((uintptr_t)state | (uintptr_t)y | (uintptr_t)carry) % 16 == 0 && y_stride % 4 == 0;
+#define CD_GO(NR_, NS_, W0_, W1_)                                                   \
+    {                                                                               \
+        if (quad) return channel_delta_launch<NR_, NS_, 4, W0_, W1_>(CD_ARGS);      \
+        return channel_delta_launch<NR_, NS_, 1, 4, 4>(CD_ARGS);                    \
     }
-    int ns = 0, nr = 0;
-    if (!li_ssm_scan_layout(N, vdim, &ns, &nr)) return LI_ERR_SIZE;
-#define CD_GO(NR_, NS_) if (nr == NR_ && ns == NS_) return channel_delta_launch<NR_, NS_, 1>(CD_ARGS);
-    CD_GO(16, 1) CD_GO(32, 1) CD_GO(64, 1) CD_GO(128, 1)
-    CD_GO(16, 2) CD_GO(32, 2) CD_GO(64, 2) CD_GO(128, 2)
-    CD_GO(16, 4) CD_GO(32, 4) CD_GO(64, 4)
+    if (N <= 32) CD_GO(4, 8, 1, 2)
+    if (N <= 64) CD_GO(8, 8, 2, 4)
+    if (N <= 128) CD_GO(16, 8, 4, 4)
+    CD_GO(16, 16, 4, 4)
 #undef CD_GO
 #undef CD_ARGS
-    return LI_ERR_SIZE;
 }
 
 // ------------------------------------------------------------------------------------ gated norm in groups
@@ -1220,11 +1261,56 @@ __global__ __launch_bounds__(256) void gated_group_norm_kernel(const float* __re
     }
 }
 
+// The same for narrow groups (up to 256 columns): a wave a (token, group), four of them a block.
+template <typename TO>
+__global__ __launch_bounds__(256) void gated_group_norm_wave_kernel(const float* __restrict__ y, long y_stride,
+                                                                    const float* __restrict__ z, long z_stride,
+                                                                    const float* __restrict__ w, float eps, TO* __restrict__ out,
+                                                                    long out_stride, long units, int groups, int gs, int gate_after) {
+    const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
+    if (unit >= units) return;
+    const long t = unit / groups;
+    const int c0 = (int)(unit % groups) * gs;
+    const float* yr = y + t * y_stride + c0;
+    const float* zr = z + t * z_stride + c0;
+    float v[4], gt[4];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int j = lane + 64 * i;
+        v[i] = 0.f; gt[i] = 1.f;
+        if (j < gs) {
+            const float zz = zr[j], sg = (gate_after == 2 ? 1.0f : zz) / (1.0f + expf(-zz));
+            v[i] = gate_after ? yr[j] : yr[j] * sg;
+            if (gate_after) gt[i] = sg;
+        }
+        ss = fmaf(v[i], v[i], ss);
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)gs + eps);
+    TO* o = out + t * out_stride + c0;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int j = lane + 64 * i;
+        if (j < gs) store_from_float(o + j, (w ? w[c0 + j] : 1.f) * v[i] * inv * gt[i]);
+    }
+}
+
 extern "C" int li_gated_group_norm(const float* y, long y_stride, const float* z, long z_stride, const float* w, float eps,
                                    void* out, int out_dtype, long out_stride, int T, int n, int groups, int gate_after,
                                    hipStream_t stream) {
     if (T <= 0 || n <= 0 || groups <= 0 || n % groups || groups > 65535 || y_stride < n || z_stride < n || out_stride < n)
         return LI_ERR_SIZE;
+    if (n / groups <= 256) {
+        const long units = (long)T * groups;
+        const unsigned blocks = (unsigned)((units + 3) / 4);
+        if (out_dtype == LI_F32)
+            gated_group_norm_wave_kernel<float><<<blocks, 256, 0, stream>>>(y, y_stride, z, z_stride, w, eps, (float*)out, out_stride, units, groups, n / groups, gate_after);
+        else if (out_dtype == LI_BF16)
+            gated_group_norm_wave_kernel<bf16_t><<<blocks, 256, 0, stream>>>(y, y_stride, z, z_stride, w, eps, (bf16_t*)out, out_stride, units, groups, n / groups, gate_after);
+        else return LI_ERR_DTYPE;
+        return li_launch_status();
+    }
     const dim3 grid(T, groups);
     if (out_dtype == LI_F32)
         gated_group_norm_kernel<float, 8><<<grid, 256, 0, stream>>>(y, y_stride, z, z_stride, w, eps, (float*)out, out_stride, n / groups, gate_after);
