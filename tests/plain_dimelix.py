@@ -171,8 +171,9 @@ def order(cfg):
     return list(range(loop["start"])) + loop["times"] * list(range(loop["start"], loop["stop"])) + list(range(loop["stop"], n))
 
 
-def forward(cfg, w, ids, taps=None):
-    """Logits [T, vocab] of a whole sequence.  `taps`, a list, receives the sum of the streams after every layer run."""
+def forward(cfg, w, ids, taps=None, rounding=None):
+    """Logits [T, vocab] of a whole sequence.  `taps`, a list, receives the sum of the streams after every layer run.
+    `rounding`, a function, is applied to every sublayer's normed input (to see how far a rounding there is carried)."""
     eps = cfg["norm"]["eps"]
     x = w["embed"][np.asarray(ids)] * cfg["embedding"]["scale"]
     xs = [x.copy() for _ in range(cfg["streams"])]
@@ -180,9 +181,11 @@ def forward(cfg, w, ids, taps=None):
     for i in order(cfg):
         L, p = cfg["layers"][i], f"l{i}."
         u = offset_norm(read_streams(xs, w, p + "hc1."), w[p + "norm1"], eps)
+        u = rounding(u) if rounding else u
         xs = write_streams(xs, mixer(L, u, w, p + "mix.", eps, positions), w, p + "hc1.")
         if L.get("mlp") is not None:
             u = offset_norm(read_streams(xs, w, p + "hc2."), w[p + "norm2"], eps)
+            u = rounding(u) if rounding else u
             xs = write_streams(xs, dense_ff(u, w, p + "mlp."), w, p + "hc2.")
         if taps is not None:
             taps.append(sum(xs))
