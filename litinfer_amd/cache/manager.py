@@ -3,11 +3,12 @@ and slots for per-request state of fixed size.
 
 Entries of the model's execution order that need a cache are put into GROUPS
 by what they need: the named tensors they keep per token (keys and values of
-some head layout, a compressed latent, keys alone ...) and the window.  A
+some head layout, a compressed latent, keys alone ...) and what later queries still
+see of them (a window, a chunk).  A
 group has one page pool and, for each of its tensors, one device tensor
 [entries, pages, *leading sizes, page_size, last size]; a page id is valid in
 every entry and every tensor of its group, and each request has one block table
-per group.  A windowed group gives a page back as soon as no later query
+per group.  A windowed or chunked group gives a page back as soon as no later query
 can see any of its positions; its table entry becomes -1 and is never
 addressed again.  All pages of a request go back when it is released.
 
@@ -157,6 +158,8 @@ class CacheManager:
             self._book = None
             raise ValueError(err)
         for gi, g in enumerate(self.groups):
+            if g.need.chunk and self._lib.li_book_set_chunk(self._book, gi, int(g.need.chunk)) < 0:
+                raise ValueError(self._error())
             if g.need.keep_first and self._lib.li_book_set_keep_first(self._book, gi, int(g.need.keep_first)) < 0:
                 raise ValueError(self._error())
         self._ints = (ctypes.c_int * max(ng, 1))()

@@ -28,6 +28,10 @@ from .dimelix import DimelixConfig, dimelix_model_spec
 
 register_architecture("Dimelix", DimelixConfig.from_dict, dimelix_model_spec, aliases=("dimelix",))
 
-__all__ = ["DimelixConfig", "dimelix_model_spec", "KufolornConfig", "kufolorn_model_spec", "NusuvikConfig", "nusuvik_model_spec", "TovasunConfig", "tovasun_model_spec", "SogenexConfig", "sogenex_model_spec", "ExecEntry", "LayerSpec", "ModelSpec", "PartSpec", "Architecture", "architecture_name",
+from .besorax import BesoraxConfig, besorax_model_spec
+
+register_architecture("Besorax", BesoraxConfig.from_dict, besorax_model_spec, aliases=("besorax",))
+
+__all__ = ["BesoraxConfig", "besorax_model_spec", "DimelixConfig", "dimelix_model_spec", "KufolornConfig", "kufolorn_model_spec", "NusuvikConfig", "nusuvik_model_spec", "TovasunConfig", "tovasun_model_spec", "SogenexConfig", "sogenex_model_spec", "ExecEntry", "LayerSpec", "ModelSpec", "PartSpec", "Architecture", "architecture_name",
            "load_config", "lookup", "read_config_json", "register_architecture",
            "registered_architectures", "ConfigError", "Qwen2Config", "qwen2_model_spec"]

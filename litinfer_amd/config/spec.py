@@ -60,6 +60,8 @@ class ModelSpec:
     # 0: one residual stream.  n > 0: n streams side by side, all equal to the embedding output at the start, mixed by
     # the blocks (which must be of the arrangement that knows streams); the final norm reads their sum.
     streams: int = 0
+    # what every sublayer's output is multiplied by when it joins the residual stream (one stream only)
+    residual_scale: float = 1.0
 
     def validate(self) -> None:
         if not self.layers:
@@ -67,6 +69,8 @@ class ModelSpec:
         if self.streams < 0 or (self.streams and self.injections):
             raise ValueError("model spec: the number of streams must not be negative, and nothing is injected between "
                              "layers where there are several")
+        if self.residual_scale != 1.0 and self.streams:
+            raise ValueError("model spec: a factor on the sublayers' outputs goes with one residual stream")
         if not self.order:
             raise ValueError("model spec: empty execution order")
         for i, e in enumerate(self.order):

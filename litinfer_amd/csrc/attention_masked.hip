@@ -1,5 +1,5 @@
 // Attention over the paged cache for mixers that the plain kernels do not cover: a window with a number of
-// first positions that stay visible, scores capped by a tanh, keys and values of unequal sizes, and keys and
+// first positions that stay visible, or chunks of positions (a query sees only its own chunk), scores capped by a tanh, keys and values of unequal sizes, and keys and
 // values that are two column ranges of ONE cached row (a compressed cache: every query head reads the same
 // row, the values are its first columns).  Queries are float32; scores, softmax and sums are float32.
 // Beside it the per-head products that a compressed cache needs on both sides of the attention.
@@ -22,8 +22,16 @@ __device__ __forceinline__ void wave_lds_sync() {
 // What some mixers add to the plain rule (null: not there).  `sink`: a number a head; the softmax's denominator also
 // holds exp(sink[head]), a term without key or value.  `gate`: float32 rows behind a sigmoid that multiply the outputs,
 // one number a head (gate[token, head]) or, with per_column, one a head and value column (gate[token, head * dv + d]).
-// `slopes`: a number a head; the score of a key loses slopes[head] times its distance from the query.
-struct MaExtras { const float* sink; const float* gate; long gate_stride; int per_column; const float* slopes; };
+// `slopes`: a number a head; the score of a key loses slopes[head] times its distance from the query.  `chunk` > 0: a
+// query sees only keys of its own run of `chunk` positions, counted from the request's position 0.
+struct MaExtras { const float* sink; const float* gate; long gate_stride; int per_column; const float* slopes; int chunk; };
+
+// The lowest position that the query at p sees beside the kept first ones (it never falls as p grows).
+__device__ __forceinline__ int lower_edge(int p, int window, int chunk) {
+    const int w = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int c = chunk > 0 ? p / chunk * chunk : 0;
+    return w > c ? w : c;
+}
 
 // What a (token, head)'s sums of values are multiplied by at the end: one over the sum of the weights (with the sink's
 // term, counted once), and the head's gate where heads have one.
@@ -66,7 +74,7 @@ __global__ __launch_bounds__(64 * NW) void masked_attention_wave_kernel(
     const int t = token_list ? token_list[blockIdx.x] : blockIdx.x, h = blockIdx.y;
     const int s = seg_of_token[t];
     const int p = ctx_len[s] - q_len[s] + (t - q_start[s]);
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = lower_edge(p, window, ex.chunk);
     const int n_first = keep_first < lo ? keep_first : lo;
     const int n_keys = n_first + (p - lo + 1);
     const int kvh = h / (nh / nkv);
@@ -206,9 +214,10 @@ extern "C" int li_masked_attention(const float* q, int q_token_stride, int q_hea
                                    const int* block_table, int max_blocks, const int* token_list, int n_tokens,
                                    const int* seg_of_token, const int* q_start,
                                    const int* q_len, const int* ctx_len, int nh, int nkv, int dk, int dv,
-                                   int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes,
+                                   int page_size, int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int chunk,
                                    int waves, hipStream_t stream) {
-    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
+    if (chunk < 0 || (chunk > 0 && keep_first > 0)) return LI_ERR_SIZE;
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes, chunk};
     if (n_tokens <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || dk <= 0 || dv <= 0 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || nh > 65535 || dk > 4096 || dv > 64 * MA_MAX_CHUNKS)
         return LI_ERR_SIZE;
@@ -274,7 +283,7 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
     const int s = tiles[4 * tile], t0 = tiles[4 * tile + 1], ntok = tiles[4 * tile + 2];
     const int p0 = ctx_len[s] - q_len[s] + (t0 - q_start[s]);             // position of the tile's first query
     const int p_last = p0 + ntok - 1;
-    const int lo_min = (window > 0 && p0 - window + 1 > 0) ? p0 - window + 1 : 0;
+    const int lo_min = lower_edge(p0, window, ex.chunk);
     const int n_first = keep_first < lo_min ? keep_first : lo_min;
     const int n_keys = n_first + (p_last - lo_min + 1);
     const int* table = block_table + (size_t)s * max_blocks;
@@ -286,7 +295,7 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
     const int head = kvh * rep + (active ? hh : 0);
     const float slope = ex.slopes ? ex.slopes[head] : 0.f;
     const int pq = p0 + ql;                                               // this lane's query (ql >= ntok: none)
-    const int lq = (window > 0) ? pq - window + 1 : 0;
+    const int lq = lower_edge(pq, window, ex.chunk);
     const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
 
     ma_frag8 qf[KS];
@@ -306,7 +315,7 @@ __global__ __launch_bounds__(NW * 64) void masked_attention_tile_kernel(
 #pragma unroll
         for (int r = 0; r < 16; ++r) acc[dt][r] = 0.f;
     float m = -INFINITY, l = 0.f;
-    const int lq_last = (window > 0) ? p_last - window + 1 : 0;           // the highest lower edge among the tile's queries
+    const int lq_last = lower_edge(p_last, window, ex.chunk);           // the highest lower edge among the tile's queries
 
     // The cache row of key place tid of the block of keys that starts at list index i0 (threads 0..31).
     auto row_of = [&](int i0) -> int {
@@ -511,7 +520,7 @@ __global__ __launch_bounds__(64) void masked_attention_heads_kernel(
     const int s = seg_of_token[t];
     const int p0 = ctx_len[s] - q_len[s] + (t - q_start[s]);              // the token's position
     const int p_last = p0;
-    const int lo_min = (window > 0 && p0 - window + 1 > 0) ? p0 - window + 1 : 0;
+    const int lo_min = lower_edge(p0, window, ex.chunk);
     const int n_first = keep_first < lo_min ? keep_first : lo_min;
     const int n_all = n_first + (p_last - lo_min + 1);
     const int hc = blockIdx.z / nsplit, sp = blockIdx.z % nsplit;         // the chunk of 32 heads and the split of the keys
@@ -718,10 +727,11 @@ extern "C" int li_masked_attention_tiles(const float* q, int q_token_stride, int
                                          const void* vc, int k_row, int v_row, const int* block_table, int max_blocks,
                                          const int* tiles, int num_tiles, const int* q_start, const int* q_len,
                                          const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size, int num_pages,
-                                         int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int nsplit, float* parts,
+                                         int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int chunk, int nsplit, float* parts,
                                          long parts_floats, const int* multi_tokens, int num_multi, int num_tokens,
                                          hipStream_t stream) {
-    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
+    if (chunk < 0 || (chunk > 0 && keep_first > 0)) return LI_ERR_SIZE;
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes, chunk};
     if (num_tiles <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || nkv > 65535 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || k_row % 8 || v_row % 8 || q_token_stride % 4 || q_head_stride % 4 ||
         ((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) % 16 || (uintptr_t)out % 8 || !li_masked_attention_tiles_takes(dk, dv) ||
@@ -761,9 +771,10 @@ extern "C" int li_masked_attention_heads(const float* q, int q_token_stride, int
                                          const void* vc, int k_row, int v_row, const int* block_table, int max_blocks,
                                          const int* token_list, int n_tokens, const int* seg_of_token, const int* q_start,
                                          const int* q_len, const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size,
-                                         int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int nsplit,
+                                         int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int chunk, int nsplit,
                                          float* parts, long parts_floats, hipStream_t stream) {
-    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
+    if (chunk < 0 || (chunk > 0 && keep_first > 0)) return LI_ERR_SIZE;
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes, chunk};
     if (n_tokens <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || nkv > 65535 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || k_row % 8 || v_row % 8 || q_token_stride % 4 || q_head_stride % 4 ||
         ((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) % 16 || (uintptr_t)out % 8 || !li_masked_attention_tiles_takes(dk, dv) ||
@@ -832,7 +843,7 @@ __global__ __launch_bounds__(256) void masked_attention_single_kernel(
     const int nheads = rep - hfirst < RH ? rep - hfirst : RH;
     const int s = seg_of_token[t];
     const int p = ctx_len[s] - q_len[s] + (t - q_start[s]);
-    const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+    const int lo = lower_edge(p, window, ex.chunk);
     const int n_first = keep_first < lo ? keep_first : lo;
     const int n_all = n_first + (p - lo + 1);
     // this block's share of the visible keys (split sp of nsplit)
@@ -1070,9 +1081,10 @@ extern "C" int li_masked_attention_single(const float* q, int q_token_stride, in
                                           const void* vc, int k_row, int v_row, const int* block_table, int max_blocks,
                                           const int* token_list, int n_tokens, const int* seg_of_token, const int* q_start,
                                           const int* q_len, const int* ctx_len, int nh, int nkv, int dk, int dv, int page_size,
-                                          int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes,
+                                          int num_pages, int window, int keep_first, float softcap, float scale, const float* sink, const float* gate, long gate_stride, int gate_per_column, const float* slopes, int chunk,
                                           int nsplit, float* parts, long parts_floats, hipStream_t stream) {
-    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes};
+    if (chunk < 0 || (chunk > 0 && keep_first > 0)) return LI_ERR_SIZE;
+    const MaExtras ex{sink, gate, gate_stride, gate_per_column, slopes, chunk};
     if (n_tokens <= 0 || nh <= 0 || nkv <= 0 || nh % nkv || nkv > 65535 || dk > k_row || dv > v_row || page_size <= 0 ||
         window < 0 || keep_first < 0 || max_blocks <= 0 || num_pages <= 0 || k_row % 8 || v_row % 8 || q_token_stride % 4 ||
         q_head_stride % 4 || ((uintptr_t)q | (uintptr_t)kc | (uintptr_t)vc) % 16 || !li_masked_attention_single_takes(dk, dv))
@@ -1082,7 +1094,8 @@ extern "C" int li_masked_attention_single(const float* q, int q_token_stride, in
     if (nsplit < 1 || nsplit > 64 || (nsplit > 1 && (!parts || parts_floats < (long)n_tokens * nh * nsplit * (dv + 2)))) return LI_ERR_SIZE;
     const dim3 grid(n_tokens, nkv, ((rep + rh - 1) / rh) * nsplit);
     // room for the pages of one query's visible keys: the window's and the kept ones, or the whole table's width
-    long cap = window > 0 ? (long)window / page_size + 3 + (keep_first + page_size - 1) / page_size : (long)max_blocks;
+    const long reach = window > 0 && (chunk <= 0 || window < chunk) ? window : chunk;      // (0: no bound)
+    long cap = reach > 0 ? reach / page_size + 3 + (keep_first + page_size - 1) / page_size : (long)max_blocks;
     if (cap > 12288) cap = 0;                       // (longer tables are read where they lie)
     const int tab_cap = (int)cap;
     int pshift = -1;

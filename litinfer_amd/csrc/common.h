@@ -37,6 +37,9 @@ __device__ __forceinline__ float load_as_float(const bf16_t* p) { return bf16_to
 __device__ __forceinline__ void store_from_float(float* p, float v) { *p = v; }
 __device__ __forceinline__ void store_from_float(bf16_t* p, float v) { p->bits = float_to_bf16(v); }
 
+// GELU with the error function
+__device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
     for (int o = LI_WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, LI_WAVE);

@@ -189,31 +189,38 @@ extern "C" int li_swiglu(const void* gu, void* out, int dtype, int T, int I, hip
 }
 
 // out[t, i] = act(gate) * up with gate = gu[t, i], up = gu[t, I + i]; act 0: z / (1 + exp(-z)),
-// act 1: the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).  Arithmetic in float32.
+// act 1: the tanh form of GELU, 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))); act 2: the clamped form
+// out = g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit).  Arithmetic in float32.
 template <typename TI, typename TO>
-__global__ void gated_act_kernel(const TI* __restrict__ gu, TO* __restrict__ out, int I, int act) {
+__global__ void gated_act_kernel(const TI* __restrict__ gu, TO* __restrict__ out, int I, int act, float limit) {
     const TI* g = gu + (size_t)blockIdx.y * 2 * I;
     TO* o = out + (size_t)blockIdx.y * I;
     const int i = blockIdx.x * blockDim.x + threadIdx.x;
     if (i < I) {
-        const float gv = load_as_float(g + i), uv = load_as_float(g + I + i);
+        float gv = load_as_float(g + i), uv = load_as_float(g + I + i);
+        if (act == 2) {
+            gv = fminf(gv, limit);
+            uv = fminf(fmaxf(uv, -limit), limit);
+            store_from_float(o + i, (uv + 1.0f) * (gv / (1.0f + expf(-1.702f * gv))));
+            return;
+        }
         const float a = act == 1 ? 0.5f * gv * (1.0f + tanhf(0.7978845608028654f * (gv + 0.044715f * gv * gv * gv)))
                                  : gv / (1.0f + expf(-gv));
         store_from_float(o + i, a * uv);
     }
 }
 
-extern "C" int li_gated_act(const void* gu, int in_dtype, void* out, int out_dtype, int T, int I, int act, hipStream_t stream) {
-    if (T <= 0 || I <= 0 || T > 65535 * 32 || act < 0 || act > 1) return LI_ERR_SIZE;
+extern "C" int li_gated_act(const void* gu, int in_dtype, void* out, int out_dtype, int T, int I, int act, float limit, hipStream_t stream) {
+    if (T <= 0 || I <= 0 || T > 65535 * 32 || act < 0 || act > 2 || (act == 2 && !(limit > 0.f))) return LI_ERR_SIZE;
     for (int t0 = 0; t0 < T; t0 += 65535) {
         const int rows = (T - t0 < 65535) ? T - t0 : 65535;
         dim3 grid((I + 255) / 256, rows);
         if (in_dtype == LI_F32 && out_dtype == LI_F32)
-            gated_act_kernel<float, float><<<grid, 256, 0, stream>>>((const float*)gu + (size_t)t0 * 2 * I, (float*)out + (size_t)t0 * I, I, act);
+            gated_act_kernel<float, float><<<grid, 256, 0, stream>>>((const float*)gu + (size_t)t0 * 2 * I, (float*)out + (size_t)t0 * I, I, act, limit);
         else if (in_dtype == LI_F32 && out_dtype == LI_BF16)
-            gated_act_kernel<float, bf16_t><<<grid, 256, 0, stream>>>((const float*)gu + (size_t)t0 * 2 * I, (bf16_t*)out + (size_t)t0 * I, I, act);
+            gated_act_kernel<float, bf16_t><<<grid, 256, 0, stream>>>((const float*)gu + (size_t)t0 * 2 * I, (bf16_t*)out + (size_t)t0 * I, I, act, limit);
         else if (in_dtype == LI_BF16 && out_dtype == LI_BF16)
-            gated_act_kernel<bf16_t, bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gu + (size_t)t0 * 2 * I, (bf16_t*)out + (size_t)t0 * I, I, act);
+            gated_act_kernel<bf16_t, bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)gu + (size_t)t0 * 2 * I, (bf16_t*)out + (size_t)t0 * I, I, act, limit);
         else return LI_ERR_DTYPE;
     }
     return li_launch_status();
@@ -679,7 +686,7 @@ extern "C" int li_qk_norm_pairs_store(float* qkv, int row_stride, int nh, int nk
                                       const int* slot_map, void* kc, void* vc, int cache_dtype, int page_size, int store,
                                       int half_split, int T, hipStream_t stream) {
     if (T <= 0 || nh <= 0 || nkv <= 0 || dk <= 0 || dv <= 0 || rotary_dim < 0 || (rotary_dim & 1) || rotary_dim > dk ||
-        row_stride < nh * dk + nkv * (dk + dv) || page_size <= 0)
+        row_stride < nh * dk + (store ? nkv * (dk + dv) : 0) || page_size <= 0)
         return LI_ERR_SIZE;
     // few rows (a decoding step): 1024 threads a row, so that the one row is gone through with the least latency
     const bool wide = T < 256 && nh * dk > 1024;
@@ -1066,6 +1073,61 @@ extern "C" int li_layernorm(const float* x, const float* w, const float* b, floa
     else if (out_dtype == LI_BF16) LI_LNORM(bf16_t)
     else return LI_ERR_DTYPE;
 #undef LI_LNORM
+    return li_launch_status();
+}
+
+// A norm without statistics: y = tanh(alpha * x) * w + b, element by element, in float32.  Four neighbouring columns a
+// thread where the rows allow it (VEC), else one.
+template <typename TO, bool VEC>
+__global__ __launch_bounds__(256) void tanh_norm_kernel(const float* __restrict__ x, float alpha, const float* __restrict__ w,
+                                                        const float* __restrict__ b, TO* __restrict__ out, long n, int H) {
+    constexpr int E = VEC ? 4 : 1;
+    const long i = ((long)blockIdx.x * 256 + threadIdx.x) * E;
+    if (i >= n) return;
+    const int j = (int)(i % H);
+    if constexpr (VEC) {
+        const float4 v = *reinterpret_cast<const float4*>(x + i), g = *reinterpret_cast<const float4*>(w + j), c = *reinterpret_cast<const float4*>(b + j);
+        const float4 r = float4{fmaf(tanhf(alpha * v.x), g.x, c.x), fmaf(tanhf(alpha * v.y), g.y, c.y),
+                                fmaf(tanhf(alpha * v.z), g.z, c.z), fmaf(tanhf(alpha * v.w), g.w, c.w)};
+        if constexpr (sizeof(TO) == 2) *reinterpret_cast<uint2*>(out + i) = uint2{pack2_bf16(r.x, r.y), pack2_bf16(r.z, r.w)};
+        else *reinterpret_cast<float4*>(out + i) = r;
+    } else {
+        store_from_float(out + i, fmaf(tanhf(alpha * x[i]), w[j], b[j]));
+    }
+}
+
+extern "C" int li_tanh_norm(const float* x, float alpha, const float* w, const float* b, void* out, int out_dtype, int T, int H,
+                            hipStream_t stream) {
+    if (T <= 0 || H <= 0) return LI_ERR_SIZE;
+    const long n = (long)T * H;
+    const bool vec = H % 4 == 0 && ((uintptr_t)x | (uintptr_t)w | (uintptr_t)b | (uintptr_t)out) % 16 == 0;
+    const unsigned blocks = (unsigned)((n / (vec ? 4 : 1) + 255) / 256);
+#define LI_TN(TO)                                                                                            \
+    {                                                                                                        \
+        if (vec) tanh_norm_kernel<TO, true><<<blocks, 256, 0, stream>>>(x, alpha, w, b, (TO*)out, n, H);     \
+        else tanh_norm_kernel<TO, false><<<blocks, 256, 0, stream>>>(x, alpha, w, b, (TO*)out, n, H);        \
+    }
+    if (out_dtype == LI_F32) LI_TN(float)
+    else if (out_dtype == LI_BF16) LI_TN(bf16_t)
+    else return LI_ERR_DTYPE;
+#undef LI_TN
+    return li_launch_status();
+}
+
+// out = gelu(x) with the error function, 0.5 x (1 + erf(x / sqrt(2))), element by element
+template <typename TI, typename TO>
+__global__ void gelu_erf_kernel(const TI* __restrict__ x, TO* __restrict__ out, long n) {
+    const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+    if (i < n) store_from_float(out + i, gelu_erf(load_as_float(x + i)));
+}
+
+extern "C" int li_gelu_erf(const void* x, int x_dtype, void* out, int out_dtype, long n, hipStream_t stream) {
+    if (n <= 0) return LI_ERR_SIZE;
+    const unsigned blocks = (unsigned)((n + 255) / 256);
+    if (x_dtype == LI_F32 && out_dtype == LI_F32) gelu_erf_kernel<float, float><<<blocks, 256, 0, stream>>>((const float*)x, (float*)out, n);
+    else if (x_dtype == LI_F32 && out_dtype == LI_BF16) gelu_erf_kernel<float, bf16_t><<<blocks, 256, 0, stream>>>((const float*)x, (bf16_t*)out, n);
+    else if (x_dtype == LI_BF16 && out_dtype == LI_BF16) gelu_erf_kernel<bf16_t, bf16_t><<<blocks, 256, 0, stream>>>((const bf16_t*)x, (bf16_t*)out, n);
+    else return LI_ERR_DTYPE;
     return li_launch_status();
 }
 

@@ -1,4 +1,5 @@
-// out[M, N] = x[M, K] w[N, K]^T (+ bias[N]) (+ out), float32 accumulation.
+// out[M, N] = x[M, K] w[N, K]^T (+ bias[N]), or out += accumulate * (x w^T + bias) where the number `accumulate`
+// is not 0 (1 for a plain sum), float32 accumulation.
 //
 // float32 operands: an LDS-tiled FMA kernel (true 32-bit, no reduced-precision
 // matrix mode).  bfloat16 operands: MFMA tiles for 64-wide waves.  For each
@@ -16,9 +17,9 @@ typedef float floatx4 __attribute__((ext_vector_type(4)));
 
 template <typename TO>
 __device__ __forceinline__ void epilogue_store(TO* out, size_t idx, float acc, const float* bias,
-                                               int col, bool accumulate) {
+                                               int col, float accumulate) {
     if (bias) acc += bias[col];
-    if (accumulate) acc += load_as_float(out + idx);
+    if (accumulate != 0.f) acc = fmaf(accumulate, acc, load_as_float(out + idx));
     store_from_float(out + idx, acc);
 }
 
@@ -32,7 +33,7 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const float* __restrict__
                                                         const float* __restrict__ w,
                                                         const float* __restrict__ bias,
                                                         float* __restrict__ out, int M, int N, int K,
-                                                        int accumulate) {
+                                                        float accumulate) {
     __shared__ float As[F32_BK][F32_BM + 4];
     __shared__ float Bs[F32_BK][F32_BN + 4];
     const int tid = threadIdx.x;
@@ -87,7 +88,7 @@ __global__ __launch_bounds__(256) void gemm_f32_big_kernel(const float* __restri
                                                             const float* __restrict__ w,
                                                             const float* __restrict__ bias,
                                                             float* __restrict__ out, int M, int N, int K,
-                                                            int accumulate) {
+                                                            float accumulate) {
     __shared__ __attribute__((aligned(16))) float As[2][F32B_BK][F32B_BM + 4];
     __shared__ __attribute__((aligned(16))) float Bs[2][F32B_BK][F32B_BN + 4];
     const int tid = threadIdx.x;
@@ -175,7 +176,7 @@ __global__ __launch_bounds__(256) void gemm_f32_big_kernel(const float* __restri
 #define F32M_LD (F32M_BM + 4)
 __global__ __launch_bounds__(256) void gemm_f32_mfma_kernel(const float* __restrict__ x, const float* __restrict__ w,
                                                              const float* __restrict__ bias, float* __restrict__ out,
-                                                             int M, int N, int K, int accumulate) {
+                                                             int M, int N, int K, float accumulate) {
     __shared__ float As[2][F32M_BK * F32M_LD];
     __shared__ float Bs[2][F32M_BK * F32M_LD];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -269,7 +270,7 @@ __global__ __launch_bounds__(256) void gemm_f32_mfma_kernel(const float* __restr
 #pragma unroll
             for (int r = 0; r < 16; ++r) {
                 const int row = m0 + wm + 32 * i + 8 * (r >> 2) + 4 * fk + (r & 3);
-                if (row < M && col < N) epilogue_store(out, (size_t)row * N + col, acc[i][j][r], bias, col, accumulate != 0);
+                if (row < M && col < N) epilogue_store(out, (size_t)row * N + col, acc[i][j][r], bias, col, accumulate);
             }
         }
 }
@@ -290,7 +291,7 @@ __global__ __launch_bounds__(F32RM_WAVES * 64) void gemm_f32_rows_mfma_kernel(co
                                                                               const float* __restrict__ w,
                                                                               const float* __restrict__ bias,
                                                                               float* __restrict__ out, int M, int N, int K,
-                                                                              int accumulate, int cols) {
+                                                                              float accumulate, int cols, float limit) {
     // TILES: MFMA tiles of 16 columns side by side in a block (`cols` <= 16 TILES): they share the block's
     // loads of x, which come through the same path as w (a matrix of many columns has blocks enough).
     // RT: tiles of 16 rows one above the other (M <= 16 RT): they share the block's loads of w, which is
@@ -403,9 +404,15 @@ __global__ __launch_bounds__(F32RM_WAVES * 64) void gemm_f32_rows_mfma_kernel(co
             float up = part[0][at + 256];
 #pragma unroll
             for (int v2 = 1; v2 < F32RM_WAVES; ++v2) up += part[v2][at + 256];
-            out[(size_t)row * N + n0 + j] = up * (v / (1.0f + expf(-v)));
+            if (limit > 0.f) {                                  // the clamped form (see gated_bf16)
+                v = fminf(v, limit);
+                up = fminf(fmaxf(up, -limit), limit);
+                out[(size_t)row * N + n0 + j] = (up + 1.0f) * (v / (1.0f + expf(-1.702f * v)));
+            } else {
+                out[(size_t)row * N + n0 + j] = up * (v / (1.0f + expf(-v)));
+            }
         } else {
-            epilogue_store(out, (size_t)row * N + n0 + j, v, bias, n0 + j, accumulate != 0);
+            epilogue_store(out, (size_t)row * N + n0 + j, v, bias, n0 + j, accumulate);
         }
     }
 }
@@ -416,7 +423,7 @@ static int compute_units();
 
 // swiglu: w is [gate; up] of N rows each and out [M, N] gets the activation (no bias, no accumulation)
 static int launch_f32_rows(const float* x, const float* w, const float* bias, float* out, int M, int N, int K,
-                           int accumulate, hipStream_t stream, bool swiglu = false) {
+                           float accumulate, hipStream_t stream, bool swiglu = false, float limit = 0.f) {
     // as many blocks as a whole number of rounds over the compute units, each with the same share of the columns;
     // two MFMA tiles side by side where 16 columns a block would not fit one round (they share the loads of x:
     // the 7B's gate/up matrix at 8 rows 136 -> 130 us)
@@ -435,7 +442,7 @@ static int launch_f32_rows(const float* x, const float* w, const float* bias, fl
     // pieces a trip: a long K keeps four a wave in flight, a short one two (measured: 3,584 columns 136 against
     // 156 us for the 7B's gate/up matrix, 18,944 columns 68.6 against 74.0 us for its way back), a tiny one, and
     // many rows (whose registers hold the rows' pieces too), one
-#define LI_F32RM(AH, TL, RTV, SW) gemm_f32_rows_mfma_kernel<AH, TL, RTV, SW><<<grid, F32RM_WAVES * 64, 0, stream>>>(x, w, bias, out, M, N, K, accumulate, cols)
+#define LI_F32RM(AH, TL, RTV, SW) gemm_f32_rows_mfma_kernel<AH, TL, RTV, SW><<<grid, F32RM_WAVES * 64, 0, stream>>>(x, w, bias, out, M, N, K, accumulate, cols, limit)
     const int ahead = rt == 4 ? 1 : K >= 8192 && rt == 1 ? 4 : K >= 32 * F32RM_WAVES * 4 ? 2 : 1;
     if (swiglu) {
         if (rt == 1) { if (ahead == 4) LI_F32RM(4, 2, 1, true); else if (ahead == 2) LI_F32RM(2, 2, 1, true); else LI_F32RM(1, 2, 1, true); }
@@ -492,7 +499,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
                                                          const bf16_t* __restrict__ w,
                                                          const float* __restrict__ bias,
                                                          TO* __restrict__ out, int M, int N, int K,
-                                                         int accumulate) {
+                                                         float accumulate) {
     __shared__ __attribute__((aligned(16))) uint16_t As[BF_BM * BF_LDS_STRIDE];
     __shared__ __attribute__((aligned(16))) uint16_t Bs[BF_BN * BF_LDS_STRIDE];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -624,7 +631,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_big_kernel(const bf16_t* __rest
                                                              const bf16_t* __restrict__ w,
                                                              const float* __restrict__ bias,
                                                              TO* __restrict__ out, int M, int N, int K,
-                                                             int accumulate) {
+                                                             float accumulate) {
     constexpr int WM = BM / 2, WN = BN / 2, TM = WM / 32, TN = WN / 32;
     constexpr int CPR = BK / 8;                                   // 16-byte chunks in a row of a stage
     constexpr int WRAP = 128 / BK;                                // rows that fill all 64 banks once
@@ -756,10 +763,10 @@ __global__ __launch_bounds__(256) void gemm_bf16_big_kernel(const bf16_t* __rest
                     }
                     if constexpr (sizeof(TO) == 4) {
                         float4* o = reinterpret_cast<float4*>(reinterpret_cast<float*>(out) + idx);
-                        if (accumulate) {
+                        if (accumulate != 0.f) {
                             const float4 a0 = o[0], a1 = o[1];
-                            v[0] += a0.x; v[1] += a0.y; v[2] += a0.z; v[3] += a0.w;
-                            v[4] += a1.x; v[5] += a1.y; v[6] += a1.z; v[7] += a1.w;
+                            v[0] = fmaf(accumulate, v[0], a0.x); v[1] = fmaf(accumulate, v[1], a0.y); v[2] = fmaf(accumulate, v[2], a0.z); v[3] = fmaf(accumulate, v[3], a0.w);
+                            v[4] = fmaf(accumulate, v[4], a1.x); v[5] = fmaf(accumulate, v[5], a1.y); v[6] = fmaf(accumulate, v[6], a1.z); v[7] = fmaf(accumulate, v[7], a1.w);
                         }
                         o[0] = float4{v[0], v[1], v[2], v[3]};
                         o[1] = float4{v[4], v[5], v[6], v[7]};
@@ -807,6 +814,14 @@ __device__ __forceinline__ float swiglu_bf16(float gate, float up) {
     return up * (gate * __builtin_amdgcn_rcpf(1.0f + e));
 }
 
+// With limit > 0 the clamped form: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+__device__ __forceinline__ float gated_bf16(float gate, float up, float limit) {
+    if (!(limit > 0.f)) return swiglu_bf16(gate, up);
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    const float e = __builtin_amdgcn_exp2f(-1.702f * 1.44269504088896341f * g);
+    return (u + 1.0f) * (g * __builtin_amdgcn_rcpf(1.0f + e));
+}
+
 // f(std::integral_constant<int, 0>) ... f(std::integral_constant<int, N - 1>)
 template <typename F, int... I>
 __device__ __forceinline__ void static_for_impl(F&& f, std::integer_sequence<int, I...>) {
@@ -828,8 +843,10 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
                                                              const bf16_t* __restrict__ w,
                                                              const float* __restrict__ bias,
                                                              TO* __restrict__ out, int M, int N, int K,
-                                                             int accumulate, int nsplit,
-                                                             const float* __restrict__ row_parts, int nparts, float eps) {
+                                                             float accumulate, int nsplit,
+                                                             const float* __restrict__ row_parts, int nparts, float eps,
+                                                             float limit) {
+    // limit: see gated_bf16 (SwiGLU tiles).
     // row_parts (SwiGLU tiles of 64 rows, up to 32 rows of x): x is the xg of li_linear_residual_norm and these
     // are its sq_parts; every row's sums are scaled by 1 / sqrt(sum of the row's parts / K + eps) before the
     // activation, which makes the result that of the RMS norm (the factor of a row does not depend on k).
@@ -1090,7 +1107,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
                 float f = 1.0f;
                 if constexpr (ROWSCALE) f = row_parts ? row_inv[row & 31] : 1.0f;      // (row_parts: M <= 32, so row < 32 here)
 #pragma unroll
-                for (int e = 0; e < 8; ++e) v[e] = swiglu_bf16(gs[e] * f, us[e] * f);
+                for (int e = 0; e < 8; ++e) v[e] = gated_bf16(gs[e] * f, us[e] * f, limit);
                 const size_t o_idx = (size_t)row * NO + col;
                 if (col + 8 <= NO && (NO % 8) == 0) {
                     chunk16 o;
@@ -1131,7 +1148,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
                             uv *= f;
                         }
                     }
-                    band[(8 * (r >> 2) + crow + (r & 3)) * ESTRIDE + 16 * j + ccol] = swiglu_bf16(gv, uv);
+                    band[(8 * (r >> 2) + crow + (r & 3)) * ESTRIDE + 16 * j + ccol] = gated_bf16(gv, uv, limit);
                 }
         } else {
 #pragma unroll
@@ -1157,10 +1174,10 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
                 }
                 if constexpr (sizeof(TO) == 4) {
                     float4* o = reinterpret_cast<float4*>(reinterpret_cast<float*>(out) + o_idx);
-                    if (accumulate) {
+                    if (accumulate != 0.f) {
                         const float4 a0 = o[0], a1 = o[1];
-                        v[0] += a0.x; v[1] += a0.y; v[2] += a0.z; v[3] += a0.w;
-                        v[4] += a1.x; v[5] += a1.y; v[6] += a1.z; v[7] += a1.w;
+                        v[0] = fmaf(accumulate, v[0], a0.x); v[1] = fmaf(accumulate, v[1], a0.y); v[2] = fmaf(accumulate, v[2], a0.z); v[3] = fmaf(accumulate, v[3], a0.w);
+                        v[4] = fmaf(accumulate, v[4], a1.x); v[5] = fmaf(accumulate, v[5], a1.y); v[6] = fmaf(accumulate, v[6], a1.z); v[7] = fmaf(accumulate, v[7], a1.w);
                     }
                     o[0] = float4{v[0], v[1], v[2], v[3]};
                     o[1] = float4{v[4], v[5], v[6], v[7]};
@@ -1182,8 +1199,8 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
 
 template <int BM, int BN, int BK, int NSTAGE, bool SWIGLU, typename TO, int WLM = 2>
 static int launch_dma(const bf16_t* x, const bf16_t* w, const float* bias, TO* out, int M, int N, int K,
-                      int accumulate, hipStream_t stream, int nsplit = 1, const float* row_parts = nullptr,
-                      int nparts = 0, float eps = 0.f) {
+                      float accumulate, hipStream_t stream, int nsplit = 1, const float* row_parts = nullptr,
+                      int nparts = 0, float eps = 0.f, float limit = 0.f) {
     if (row_parts && !(SWIGLU && BM == 64 && M <= 32 && nparts > 0)) return LI_ERR_SIZE;
     const long mtiles = (M + BM - 1) / BM, ntiles = (N + BN - 1) / BN;
     if (nsplit < 1 || nsplit > 65535 || nsplit > K / BK) return LI_ERR_SIZE;
@@ -1201,14 +1218,14 @@ static int launch_dma(const bf16_t* x, const bf16_t* w, const float* bias, TO* o
             return LI_ERR_LAUNCH;
         configured = true;
     }
-    gemm_bf16_dma_kernel<BM, BN, BK, NSTAGE, SWIGLU, TO, WLM><<<(unsigned)blocks, 256, lds_bytes, stream>>>(x, w, bias, out, M, N, K, accumulate, nsplit, row_parts, nparts, eps);
+    gemm_bf16_dma_kernel<BM, BN, BK, NSTAGE, SWIGLU, TO, WLM><<<(unsigned)blocks, 256, lds_bytes, stream>>>(x, w, bias, out, M, N, K, accumulate, nsplit, row_parts, nparts, eps, limit);
     return li_launch_status();
 }
 
 // out (+)= sum over the parts, in the order of the parts, + bias
 template <typename TO>
 __global__ void splitk_reduce_kernel(const float* __restrict__ part, int nsplit, size_t mn, int N,
-                                     const float* __restrict__ bias, TO* __restrict__ out, int accumulate) {
+                                     const float* __restrict__ bias, TO* __restrict__ out, float accumulate) {
     const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
     if (i >= mn) return;
     float v = part[i];
@@ -1217,12 +1234,12 @@ __global__ void splitk_reduce_kernel(const float* __restrict__ part, int nsplit,
 }
 
 // The same for the residual sum, one block a row, with the RMS norm of the new sum as a second
-// result: out[m, :] += sum of the parts + bias (float32), xn[m, :] = gamma * out[m, :] /
+// result: out[m, :] += factor * (sum of the parts + bias) (float32), xn[m, :] = gamma * out[m, :] /
 // sqrt(mean(out[m, :]^2) + eps).  A row is kept in registers (N <= NT * PER).
 template <typename TN, int NT, int PER>
 __global__ __launch_bounds__(NT) void splitk_reduce_norm_kernel(const float* __restrict__ part, int nsplit, size_t mn, int N,
                                                                  const float* __restrict__ bias, float* __restrict__ out,
-                                                                 const float* __restrict__ gamma, float eps,
+                                                                 float factor, const float* __restrict__ gamma, float eps,
                                                                  TN* __restrict__ xn) {
     __shared__ float red[NT / LI_WAVE];
     const size_t row = (size_t)blockIdx.x * N;
@@ -1243,7 +1260,7 @@ __global__ __launch_bounds__(NT) void splitk_reduce_norm_kernel(const float* __r
 #pragma unroll
             for (int sp = 1; sp < 8; ++sp) t += sp < nsplit ? a[sp] : 0.f;
             if (bias) t += bias[n];
-            t += o;
+            t = fmaf(factor, t, o);
             out[row + n] = t;
             v[i] = t;
         }
@@ -1257,12 +1274,35 @@ __global__ __launch_bounds__(NT) void splitk_reduce_norm_kernel(const float* __r
         if (n < N) store_from_float(xn + row + n, gamma[n] * v[i] * inv);
     }
 }
+
+// The same with a tanh norm, which takes no statistics of a row: out += factor * (sum of the parts + bias) (float32),
+// xn = tanh(alpha * out) * gamma + beta, element by element.
+template <typename TN>
+__global__ __launch_bounds__(256) void splitk_reduce_tanh_kernel(const float* __restrict__ part, int nsplit, size_t mn, int N,
+                                                                 const float* __restrict__ bias, float* __restrict__ out,
+                                                                 float factor, float alpha, const float* __restrict__ gamma,
+                                                                 const float* __restrict__ beta, TN* __restrict__ xn) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= mn) return;
+    const int n = (int)(i % N);
+    float a[8];
+#pragma unroll
+    for (int sp = 0; sp < 8; ++sp) a[sp] = part[(size_t)(sp < nsplit ? sp : 0) * mn + i];      // (all loads at once, as above)
+    const float o = out[i], g = gamma[n], b = beta[n];
+    float t = a[0];
+#pragma unroll
+    for (int sp = 1; sp < 8; ++sp) t += sp < nsplit ? a[sp] : 0.f;
+    if (bias) t += bias[n];
+    t = fmaf(factor, t, o);
+    out[i] = t;
+    store_from_float(xn + i, fmaf(tanhf(alpha * t), g, b));
+}
 #define REDUCE_NORM_NT 1024
 #define REDUCE_NORM_PER 8
 
 template <int BM, int BN, int BK, typename TO>
 static int launch_big(const bf16_t* x, const bf16_t* w, const float* bias, TO* out, int M, int N, int K,
-                      int accumulate, hipStream_t stream) {
+                      float accumulate, hipStream_t stream) {
     const long mtiles = (M + BM - 1) / BM, ntiles = (N + BN - 1) / BN;
     const long per_xcd = TileOrder::blocks(mtiles, ntiles) / 8;
     if (per_xcd * 8 > 0x7fffffffL) return LI_ERR_SIZE;
@@ -1310,7 +1350,8 @@ struct SkinnyArgs {
     const bf16_t* w;        // [N, K], or [2 N, K] with SWIGLU
     const float* bias;      // [N] or null
     void* out;              // [M, N]
-    int M, N, K, accumulate;
+    int M, N, K;
+    float accumulate;       // 0: out is written; else out += accumulate * (product + bias)
     // ROPE (the packed q/k/v projection of a decoding step): rotary tables [M, dh / 2], the page
     // slot of each row, the cache layer's keys and values [pages, nkv, page_size, dh]
     const float* cos;
@@ -1334,6 +1375,12 @@ struct SkinnyArgs {
     // Columns a block takes (with ROPE: rotation pairs a block takes); 0: as many as its tiles hold.
     // Fewer than the tiles hold where that spreads a matrix of few columns evenly over the compute units.
     int cols;
+    // A tanh norm behind the sum (beta given): xg[m, n] = bf16(tanh(alpha * out[m, n]) * gamma[n] + beta[n]).  It takes
+    // no statistics of a row, so it is done here and sq_parts stays as it is.
+    const float* beta;
+    float alpha;
+    // SWIGLU with limit > 0: g = min(gate, limit), u = clamp(up, -limit, limit), out = g sigmoid(1.702 g) (u + 1)
+    float limit;
 };
 #define SK_MAX_PARTS 512            // blocks of a producing product whose sums one consumer adds up
 
@@ -1392,7 +1439,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
     // that will write the results: the answers arrive with the first chunk, and the epilogue
     // waits for no memory.  Never conditional per lane: a place past the end reads the last one.
     constexpr bool PRE = MT <= 2 && !SWIGLU;        // (wave mt writes row tile mt: thread t of the epilogue is lane t % 64 of wave t / 64)
-    float pre_bias[NT][4], pre_res[NT][4], pre_gamma[NT][4], pre_cos[NT][4], pre_sin[NT][4];
+    float pre_bias[NT][4], pre_res[NT][4], pre_gamma[NT][4], pre_beta[NT][4], pre_cos[NT][4], pre_sin[NT][4];
     int pre_slot = 0;
     if constexpr (PRE) {
         if (wave < MT) {
@@ -1420,8 +1467,9 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                         const int nc = n < nend ? n : nend - 1;
                         pre_bias[nt][r] = a.bias ? a.bias[nc] : 0.f;
                         pre_gamma[nt][r] = a.gamma ? a.gamma[nc] : 0.f;
+                        pre_beta[nt][r] = a.beta ? a.beta[nc] : 0.f;
                         if constexpr (sizeof(TO) == 4)
-                            pre_res[nt][r] = a.accumulate ? reinterpret_cast<const float*>(a.out)[(size_t)m * N + nc] : 0.f;
+                            pre_res[nt][r] = a.accumulate != 0.f ? reinterpret_cast<const float*>(a.out)[(size_t)m * N + nc] : 0.f;
                         else pre_res[nt][r] = 0.f;
                     }
             }
@@ -1615,10 +1663,11 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                 const int n = n0 + 4 * (l >> 4) + r;
                 if (n < nend) {
                     const float gv = s[0][r], uv = s[NT - 1][r];
-                    store_from_float(out + (size_t)m * N + n, swiglu_bf16(gv, uv));
+                    store_from_float(out + (size_t)m * N + n, gated_bf16(gv, uv, a.limit));
                 }
             }
         } else {
+            [[maybe_unused]] const float factor = a.accumulate != 0.f ? a.accumulate : 1.0f;
             if constexpr (sizeof(TO) == 4 && MT <= 2) {
                 if (a.xg) {                          // the sum goes out three ways (see SkinnyArgs)
                     float sq = 0.f;
@@ -1629,12 +1678,14 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                             const int n = n0 + 16 * nt + 4 * (l >> 4) + r;
                             if (n < nend) {
                                 const size_t idx = (size_t)m * N + n;
-                                const float v = (s[nt][r] + pre_bias[nt][r]) + pre_res[nt][r];
+                                const float v = fmaf(factor, s[nt][r] + pre_bias[nt][r], pre_res[nt][r]);
                                 reinterpret_cast<float*>(out)[idx] = v;
-                                a.xg[idx].bits = float_to_bf16(pre_gamma[nt][r] * v);
+                                a.xg[idx].bits = float_to_bf16(a.beta ? fmaf(tanhf(a.alpha * v), pre_gamma[nt][r], pre_beta[nt][r])
+                                                                      : pre_gamma[nt][r] * v);
                                 sq += v * v;
                             }
                         }
+                    if (a.beta) continue;            // (nobody asks for sums of squares)
                     // the four lanes of a row (l, l ^ 16, l ^ 32, l ^ 48: all of them are here, or none)
                     sq += __shfl_xor(sq, 16, 64);
                     sq += __shfl_xor(sq, 32, 64);
@@ -1648,7 +1699,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                 for (int r = 0; r < 4; ++r) {
                     const int n = n0 + 16 * nt + 4 * (l >> 4) + r;
                     if (n >= nend) continue;
-                    if constexpr (PRE) store_from_float(out + (size_t)m * N + n, (s[nt][r] + pre_bias[nt][r]) + pre_res[nt][r]);
+                    if constexpr (PRE) store_from_float(out + (size_t)m * N + n, fmaf(factor, s[nt][r] + pre_bias[nt][r], pre_res[nt][r]));
                     else epilogue_store(out, (size_t)m * N + n, s[nt][r], a.bias, n, a.accumulate);
                 }
         }
@@ -1722,7 +1773,7 @@ static void launch_skinny(SkinnyArgs a, hipStream_t stream) {
 
 // Few rows (M <= 64), bfloat16, K a multiple of 8.  swiglu: w has 2 N rows ([gate; up]).
 extern "C" int li_linear_skinny(const void* x, const void* w, const float* bias, void* out, int M, int N,
-                                int K, int out_dtype, int accumulate, int swiglu, hipStream_t stream) {
+                                int K, int out_dtype, float accumulate, int swiglu, hipStream_t stream) {
     if (M <= 0 || M > 64 || N <= 0 || K <= 0 || (K % 8)) return LI_ERR_SIZE;
     if (accumulate && out_dtype != LI_F32) return LI_ERR_DTYPE;
     if (swiglu && (bias || accumulate || out_dtype != LI_BF16)) return LI_ERR_DTYPE;
@@ -1735,7 +1786,7 @@ extern "C" int li_linear_skinny(const void* x, const void* w, const float* bias,
     return li_launch_status();
 }
 
-// The product before an RMS norm that is fused into its neighbours (see SkinnyArgs): out += x w^T + bias
+// The product before an RMS norm that is fused into its neighbours (see SkinnyArgs): out += factor * (x w^T + bias)
 // in float32, xg = bf16(gamma * out), sq_parts[block * R + m] = the block's share of row m's sum of
 // squares (R = 16 up to 16 rows, 32 above).  Up to 32 rows.  li_residual_norm_parts(N) is the number of
 // blocks, i.e. of parts.
@@ -1746,10 +1797,10 @@ extern "C" int li_residual_norm_parts(int N) {
 }
 
 extern "C" int li_linear_residual_norm(const void* x, const void* w, const float* bias, float* out, int M, int N,
-                                       int K, const float* gamma, void* xg, float* sq_parts, hipStream_t stream) {
-    if (M <= 0 || M > 32 || N <= 0 || K <= 0 || (K % 8) || !gamma || !xg || !sq_parts) return LI_ERR_SIZE;
+                                       int K, float factor, const float* gamma, void* xg, float* sq_parts, hipStream_t stream) {
+    if (M <= 0 || M > 32 || N <= 0 || K <= 0 || (K % 8) || factor == 0.f || !gamma || !xg || !sq_parts) return LI_ERR_SIZE;
     if (li_residual_norm_parts(N) > SK_MAX_PARTS) return LI_ERR_SIZE;
-    SkinnyArgs a{(const bf16_t*)x, (const bf16_t*)w, bias, out, M, N, K, 1,
+    SkinnyArgs a{(const bf16_t*)x, (const bf16_t*)w, bias, out, M, N, K, factor,
                  nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, gamma, (bf16_t*)xg, sq_parts, nullptr, 0, 0.f};
     launch_skinny<false, float>(a, stream);
     return li_launch_status();
@@ -1795,7 +1846,7 @@ static bool mid_rows_take(int M, int N, int K) {
 }
 
 static int linear_mid_rows(const bf16_t* x, const bf16_t* w, const float* bias, void* out, int M, int N,
-                           int K, int out_dtype, int accumulate, void* work, long work_bytes,
+                           int K, int out_dtype, float accumulate, void* work, long work_bytes,
                            hipStream_t stream) {
     if (!mid_rows_take(M, N, K) || K % 64 || (out_dtype != LI_F32 && out_dtype != LI_BF16)) return -1;
 #define LI_MID(BN, NS, TO, dst, b, acc, split) launch_dma<64, BN, 64, NS, false, TO>(x, w, b, (TO*)(dst), M, N, K, acc, stream, split)
@@ -1930,12 +1981,12 @@ extern "C" long li_linear_work_bytes(int M, int N, int K, int in_dtype) {
     return nsplit < 2 ? 0 : (long)nsplit * M * N * (long)sizeof(float);
 }
 
-// out += x w^T + bias (float32 out: the residual sum) and xn = the RMS norm of the new out with weights
+// out += factor * (x w^T + bias) (float32 out: the residual sum) and xn = the RMS norm of the new out with weights
 // gamma, where li_linear would cut K into parts anyway: the kernel that adds the parts up then has
 // whole rows in its hands.  xn is bfloat16 (xn_dtype LI_BF16) or float32.  Returns -1, having done
 // nothing, where the product is not cut (the caller then multiplies and norms in two calls).
 extern "C" int li_linear_then_norm(const void* x, const void* w, const float* bias, float* out, int M, int N, int K,
-                                   void* work, long work_bytes, const float* gamma, float eps, void* xn,
+                                   void* work, long work_bytes, float factor, const float* gamma, float eps, void* xn,
                                    int xn_dtype, hipStream_t stream) {
     if (N <= 0 || K <= 0 || (K % 64) || li_few_rows_preferred(M, N, K) || !gamma || !xn || eps < 0.f) return -1;
     if (N > REDUCE_NORM_NT * REDUCE_NORM_PER || (xn_dtype != LI_BF16 && xn_dtype != LI_F32)) return -1;
@@ -1950,10 +2001,43 @@ extern "C" int li_linear_then_norm(const void* x, const void* w, const float* bi
     if (rc != LI_OK) return rc;
     if (xn_dtype == LI_BF16)
         splitk_reduce_norm_kernel<bf16_t, REDUCE_NORM_NT, REDUCE_NORM_PER><<<M, REDUCE_NORM_NT, 0, stream>>>(
-            (const float*)work, nsplit, mn, N, bias, out, gamma, eps, (bf16_t*)xn);
+            (const float*)work, nsplit, mn, N, bias, out, factor, gamma, eps, (bf16_t*)xn);
     else
         splitk_reduce_norm_kernel<float, REDUCE_NORM_NT, REDUCE_NORM_PER><<<M, REDUCE_NORM_NT, 0, stream>>>(
-            (const float*)work, nsplit, mn, N, bias, out, gamma, eps, (float*)xn);
+            (const float*)work, nsplit, mn, N, bias, out, factor, gamma, eps, (float*)xn);
+    return li_launch_status();
+}
+
+// out += factor * (x w^T + bias) (float32: the residual sum) and xn = tanh(alpha * out) * gamma + beta in one go: in the
+// epilogue of the few-row kernel (up to 32 rows, bfloat16 xn), or, where li_linear would cut K into parts, in the kernel
+// that adds the parts up.  Returns -1, having done nothing, where neither is the case.
+extern "C" int li_linear_tanh_norm(const void* x, const void* w, const float* bias, float* out, int M, int N, int K,
+                                   void* work, long work_bytes, float factor, float alpha, const float* gamma,
+                                   const float* beta, void* xn, int xn_dtype, hipStream_t stream) {
+    if (M <= 0 || N <= 0 || K <= 0 || K % 8 || factor == 0.f || !gamma || !beta || !xn || (xn_dtype != LI_BF16 && xn_dtype != LI_F32)) return -1;
+    if (M <= 32 && li_few_rows_preferred(M, N, K)) {
+        if (xn_dtype != LI_BF16) return -1;
+        SkinnyArgs a{(const bf16_t*)x, (const bf16_t*)w, bias, out, M, N, K, factor,
+                     nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, gamma, (bf16_t*)xn, nullptr, nullptr, 0, 0.f};
+        a.beta = beta;
+        a.alpha = alpha;
+        launch_skinny<false, float>(a, stream);
+        return li_launch_status();
+    }
+    const long need = li_linear_work_bytes(M, N, K, LI_BF16);
+    if (need <= 0 || !work || work_bytes < need) return -1;
+    const size_t mn = (size_t)M * N;
+    const int nsplit = (int)(need / (long)(mn * sizeof(float)));
+    if (nsplit > 8) return -1;                      // (the adding-up kernel takes up to 8 parts)
+    const int rc = M <= 64
+        ? launch_dma<64, 128, 64, 4, false, float>((const bf16_t*)x, (const bf16_t*)w, nullptr, (float*)work, M, N, K, 0.f, stream, nsplit)
+        : launch_dma<128, 128, 64, 4, false, float>((const bf16_t*)x, (const bf16_t*)w, nullptr, (float*)work, M, N, K, 0.f, stream, nsplit);
+    if (rc != LI_OK) return rc;
+    const unsigned blocks = (unsigned)((mn + 255) / 256);
+    if (xn_dtype == LI_BF16)
+        splitk_reduce_tanh_kernel<bf16_t><<<blocks, 256, 0, stream>>>((const float*)work, nsplit, mn, N, bias, out, factor, alpha, gamma, beta, (bf16_t*)xn);
+    else
+        splitk_reduce_tanh_kernel<float><<<blocks, 256, 0, stream>>>((const float*)work, nsplit, mn, N, bias, out, factor, alpha, gamma, beta, (float*)xn);
     return li_launch_status();
 }
 
@@ -1964,7 +2048,7 @@ extern "C" int li_linear_then_norm(const void* x, const void* w, const float* bi
 extern "C" int li_linear_row_tile(int in_dtype) { return in_dtype == LI_F32 ? F32_BM : BF_BM; }
 
 extern "C" int li_linear(const void* x, const void* w, const float* bias, void* out, int M, int N,
-                         int K, int in_dtype, int out_dtype, int accumulate, void* work, long work_bytes,
+                         int K, int in_dtype, int out_dtype, float accumulate, void* work, long work_bytes,
                          hipStream_t stream) {
     if (M <= 0 || N <= 0 || K <= 0) return LI_ERR_SIZE;
     if (accumulate && out_dtype != LI_F32) return LI_ERR_DTYPE;
@@ -2054,19 +2138,19 @@ extern "C" int li_linear(const void* x, const void* w, const float* bias, void* 
 
 // The same in float32 for up to 64 rows (K a multiple of 4): the few-row product on the float32 matrix cores with
 // the activation in its epilogue.
-extern "C" int li_linear_swiglu_f32(const float* x, const float* w, float* out, int M, int I, int K, hipStream_t stream) {
+extern "C" int li_linear_swiglu_f32(const float* x, const float* w, float* out, int M, int I, int K, float limit, hipStream_t stream) {
     if (M <= 0 || M > F32_ROWS_MAX || I <= 0 || K <= 0 || K % 4 || I > 0x3fffffff) return LI_ERR_SIZE;
     if ((((uintptr_t)x | (uintptr_t)w) & 15) != 0) return LI_ERR_SIZE;
-    return launch_f32_rows(x, w, nullptr, out, M, I, K, 0, stream, true);
+    return launch_f32_rows(x, w, nullptr, out, M, I, K, 0.f, stream, true, limit);
 }
 
 // out[m, n] = up * gate / (1 + exp(-gate)) with [gate, up] = x w^T, w = [gate; up] of I rows each:
 // the activation as the product's epilogue, so the 2 I columns never go to memory.  bfloat16;
-// K a multiple of 8 for up to 64 rows, a multiple of 64 above.
+// K a multiple of 8 for up to 64 rows, a multiple of 64 above.  limit > 0: the clamped form (see gated_bf16).
 // row_parts (may be null): x is the xg of li_linear_residual_norm and these are its sq_parts, nparts of
 // them; every row's result is that of the RMS norm with eps (up to 16 rows).
 extern "C" int li_linear_swiglu(const void* x, const void* w, void* out, int M, int I, int K,
-                                const float* row_parts, int nparts, float eps, hipStream_t stream) {
+                                const float* row_parts, int nparts, float eps, float limit, hipStream_t stream) {
     if (M <= 0 || I <= 0 || K <= 0 || I > 0x3fffffff) return LI_ERR_SIZE;
     const int N = 2 * I;
     if (row_parts && (M > 32 || (K % 8) || nparts <= 0 || nparts > SK_MAX_PARTS || eps < 0.f)) return LI_ERR_SIZE;
@@ -2103,21 +2187,23 @@ extern "C" int li_linear_swiglu(const void* x, const void* w, void* out, int M, 
             const double c = tile_cost(64, widths[i], 1.0, M, N, K);
             if (pick < 0 || c < best) { best = c; pick = i; }
         }
-#define LI_SW64(BN, NS) launch_dma<64, BN, 64, NS, true, bf16_t>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0, stream, 1, row_parts, nparts, eps)
+#define LI_SW64(BN, NS) launch_dma<64, BN, 64, NS, true, bf16_t>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, row_parts, nparts, eps, limit)
         if (pick == 0) return LI_SW64(256, 3);
         if (pick == 1) return LI_SW64(192, 4);
         if (pick == 2) return LI_SW64(128, 4);
 #undef LI_SW64
     }
-    if (row_parts) {
-        SkinnyArgs a{(const bf16_t*)x, (const bf16_t*)w, nullptr, out, M, I, K, 0,
+    if (row_parts || (M <= 64 && limit > 0.f)) {
+        if (K % 8) return LI_ERR_SIZE;
+        SkinnyArgs a{(const bf16_t*)x, (const bf16_t*)w, nullptr, out, M, I, K, 0.f,
                      nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, nullptr, nullptr, nullptr, row_parts, nparts, eps};
+        a.limit = limit;
         launch_skinny<true, bf16_t>(a, stream);
         return li_launch_status();
     }
     if (M <= 64) return li_linear_skinny(x, w, nullptr, out, M, I, K, LI_BF16, 0, 1, stream);
     if (K % 64) return LI_ERR_SIZE;
-#define LI_DMA(BM, BN, BK, NS, WLM) launch_dma<BM, BN, BK, NS, true, bf16_t, WLM>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0, stream)
+#define LI_DMA(BM, BN, BK, NS, WLM) launch_dma<BM, BN, BK, NS, true, bf16_t, WLM>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, nullptr, 0, 0.f, limit)
     // (a tile's columns are gate and up columns in turn, 32 of each: its width is a multiple of 64)
     // (128 x 320: 160 gate columns in one wave, their ups in the wave beside it; for portions of a few hundred rows,
     // where no other width comes near whole rounds of the compute units: 512 rows against the 1.5B's 17,920

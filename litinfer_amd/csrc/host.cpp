@@ -86,6 +86,7 @@ struct Request {
 struct Book {
     int page_size = 0, max_seqs = 0;
     std::vector<int> windows;                  // per group, 0 = all keys
+    std::vector<int> chunks;                   // per group: a query sees only its own run of so many positions (0: no chunks)
     std::vector<int> keep_first;               // per group: a windowed group never gives back the pages of its first so many positions
     std::vector<Pool> pools;
     std::vector<int> free_slots;
@@ -98,10 +99,11 @@ struct Book {
         return it == requests.end() ? nullptr : &it->second;
     }
     int first_needed_block(int g, int first_query_pos) const {      // first block a query at that position or later sees
-        if (windows[g] <= 0) return 0;
-        const int lo = first_query_pos - windows[g] + 1;
-        return (lo > 0 ? lo : 0) / page_size;
+        int lo = windows[g] > 0 ? std::max(first_query_pos - windows[g] + 1, 0) : 0;
+        if (chunks[g] > 0) lo = std::max(lo, first_query_pos / chunks[g] * chunks[g]);
+        return lo / page_size;
     }
+    bool gives_back(int g) const { return windows[g] > 0 || chunks[g] > 0; }
     void pages_needed(const Request* r, int n_new, int cached, int* out) const {
         const int have_cached = cached >= 0 ? cached : (r ? r->cached : 0);
         for (size_t g = 0; g < pools.size(); ++g) {
@@ -149,6 +151,7 @@ void* li_book_create(int page_size, int max_seqs, int ngroups, const int* window
     if (max_seqs <= 0 || ngroups < 0) { b->error = "cache: max_seqs must be positive"; return b; }
     b->windows.assign(windows, windows + ngroups);
     b->keep_first.assign(ngroups, 0);
+    b->chunks.assign(ngroups, 0);
     b->pools.resize(ngroups);
     size_t at = 0;
     for (int g = 0; g < ngroups; ++g) {
@@ -169,6 +172,15 @@ int li_book_set_keep_first(void* vb, int g, int n) {
     if (g < 0 || g >= (int)b->pools.size() || n < 0) return b->fail(ERR_ARG, "cache: keep_first of an unknown group");
     if (!b->requests.empty()) return b->fail(ERR_LIVE, "cache: keep_first is set before any request is admitted");
     b->keep_first[g] = n;
+    return 0;
+}
+// A group whose queries see only their own run of n positions, counted from the request's position 0: the pages of a
+// run go back when the next one begins.
+int li_book_set_chunk(void* vb, int g, int n) {
+    Book* b = (Book*)vb;
+    if (g < 0 || g >= (int)b->pools.size() || n < 0) return b->fail(ERR_ARG, "cache: chunk of an unknown group");
+    if (!b->requests.empty()) return b->fail(ERR_LIVE, "cache: a group's chunk is set before any request is admitted");
+    b->chunks[g] = n;
     return 0;
 }
 void li_book_destroy(void* b) { delete (Book*)b; }
@@ -320,7 +332,7 @@ int li_book_commit(void* vb, int64_t h, int n_new) {
     if (!r) return b->fail(ERR_UNKNOWN, "cache: unknown request");
     r->cached += n_new;
     for (size_t g = 0; g < b->pools.size(); ++g) {
-        if (b->windows[g] <= 0) continue;
+        if (!b->gives_back((int)g)) continue;
         const int keep_from = std::min(b->first_needed_block((int)g, r->cached), (int)r->tables[g].size());
         const int kept = (b->keep_first[g] + b->page_size - 1) / b->page_size;     // blocks that every later query still sees
         for (int blk = std::max(r->first_live[g], kept); blk < keep_from; ++blk)

@@ -180,10 +180,11 @@ extern "C" int li_moe_route(const void* x, int x_dtype, long x_stride, const voi
 // -------------------------------------------------------------------------------------------------- plan
 // One block.  counts per expert, their running sum, every pair's row among its expert's rows (rows of an expert lie
 // together), and the tiles: (expert, first row, rows).  plan = [n_tiles, 0, 0, 0 | tiles x 4 | ...]; row_token[row] is
-// the token of a sorted row, pair_row[pair] the row of pair = token * top + choice.
+// the token of a sorted row, pair_row[pair] the row of pair = token * top + choice; row_wt[row] (where given) the weight
+// wt[pair] of the row's pair.
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ idx, int pairs, int top, int E, int* __restrict__ plan,
                                                         int max_tiles, int* __restrict__ row_token, int* __restrict__ pair_row,
-                                                        int tile_rows) {
+                                                        int tile_rows, const float* __restrict__ wt, float* __restrict__ row_wt) {
     extern __shared__ int si[];                         // [E] counts, then cursors; [E + 1] starts
     int* cnt = si;
     int* start = si + E;
@@ -218,6 +219,7 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
             const int row = start[e] + atomicAdd(&cnt[e], 1);
             pair_row[i] = row;
             row_token[row] = i / top;
+            if (row_wt) row_wt[row] = wt[i];
         } else {
             pair_row[i] = -1;
         }
@@ -225,15 +227,25 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
 }
 
 extern "C" int li_moe_plan(const int* idx, int T, int top, int E, int* plan, int max_tiles, int* row_token, int* pair_row,
-                           int tile_rows, hipStream_t stream) {
-    if (T <= 0 || top <= 0 || E <= 0 || E > 8000 || max_tiles <= 0 || (tile_rows != MOE_TILE && tile_rows != MOE_BIG_TILE && tile_rows != MOE_HUGE_TILE)) return LI_ERR_SIZE;
-    moe_plan_kernel<<<1, 1024, (size_t)(2 * E + 1) * 4, stream>>>(idx, T * top, top, E, plan, max_tiles, row_token, pair_row, tile_rows);
+                           int tile_rows, const float* wt, float* row_wt, hipStream_t stream) {
+    if (T <= 0 || top <= 0 || E <= 0 || E > 8000 || max_tiles <= 0 || (tile_rows != MOE_TILE && tile_rows != MOE_BIG_TILE && tile_rows != MOE_HUGE_TILE) || (row_wt && !wt)) return LI_ERR_SIZE;
+    moe_plan_kernel<<<1, 1024, (size_t)(2 * E + 1) * 4, stream>>>(idx, T * top, top, E, plan, max_tiles, row_token, pair_row, tile_rows, wt, row_wt);
     return li_launch_status();
 }
 
-// Four consecutive outputs of one row, from column `col` (a multiple of 4) on, with the activation: 0 none, 1 max(., 0)^2,
-// 2 the columns are (gate, up) pairs and the two results silu(gate) * up go to columns col / 2 and col / 2 + 1;
-// 3 the same pairs with g = min(gate, limit), u = clamp(up, -limit, limit) and the result g sigmoid(1.702 g) (u + 1).
+// What follows a product: the activation (0 none, 1 max(., 0)^2, 4 gelu(.) with the error function; 2 and 3: the columns
+// are (gate, up) pairs, 2 gives silu(gate) * up, 3 gives g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u =
+// clamp(up, -limit, limit)), and, where the weight of a choice multiplies the expert's INPUT, the weights of the sorted
+// rows (the product is linear, so the row's sums take the factor, in float32).
+struct MoeEpilogue { int act; float limit; const float* row_wt; };
+
+__device__ __forceinline__ bool moe_is_gated(int act) { return act == 2 || act == 3; }
+__device__ __forceinline__ float moe_row_factor(const MoeEpilogue& ep, int row) { return ep.row_wt ? ep.row_wt[row] : 1.0f; }
+__device__ __forceinline__ float moe_act1(float v, int act) {
+    if (act == 1) { v = fmaxf(v, 0.f); return v * v; }
+    return act == 4 ? gelu_erf(v) : v;
+}
+
 __device__ __forceinline__ float moe_gated(float g, float u, int act, float limit) {
     if (act == 3) {
         g = fminf(g, limit);
@@ -243,19 +255,21 @@ __device__ __forceinline__ float moe_gated(float g, float u, int act, float limi
     return u * (g / (1.0f + expf(-g)));
 }
 
+// Four consecutive outputs of one row, from column `col` (a multiple of 4) on; of (gate, up) pairs the two results go to
+// columns col / 2 and col / 2 + 1.
 template <typename TO>
-__device__ __forceinline__ void moe_store4(TO* __restrict__ row, int col, float v0, float v1, float v2, float v3, int act, float limit) {
-    if (act >= 2) {
+__device__ __forceinline__ void moe_store4(TO* __restrict__ row, int col, float v0, float v1, float v2, float v3, const MoeEpilogue& ep, float factor) {
+    const int act = ep.act;
+    const float limit = ep.limit;
+    v0 *= factor; v1 *= factor; v2 *= factor; v3 *= factor;
+    if (moe_is_gated(act)) {
         const float o0 = moe_gated(v0, v1, act, limit), o1 = moe_gated(v2, v3, act, limit);
         TO* dst = row + (col >> 1);
         if constexpr (sizeof(TO) == 2) *reinterpret_cast<uint32_t*>(dst) = pack2_bf16(o0, o1);
         else *reinterpret_cast<float2*>(dst) = float2{o0, o1};
         return;
     }
-    if (act == 1) {
-        v0 = fmaxf(v0, 0.f); v1 = fmaxf(v1, 0.f); v2 = fmaxf(v2, 0.f); v3 = fmaxf(v3, 0.f);
-        v0 *= v0; v1 *= v1; v2 *= v2; v3 *= v3;
-    }
+    if (act) { v0 = moe_act1(v0, act); v1 = moe_act1(v1, act); v2 = moe_act1(v2, act); v3 = moe_act1(v3, act); }
     TO* dst = row + col;
     if constexpr (sizeof(TO) == 2) {
         uint32_t* d2 = reinterpret_cast<uint32_t*>(dst);
@@ -275,7 +289,7 @@ __device__ __forceinline__ void moe_store4(TO* __restrict__ row, int col, float 
 template <typename TA, typename TW, typename TO>
 __global__ __launch_bounds__(256) void moe_linear_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                          const TW* __restrict__ w, const int* __restrict__ plan,
-                                                         TO* __restrict__ out, long out_stride, int n_out, int K, int act, float limit) {
+                                                         TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
     const int tile = blockIdx.x;
     if (tile >= plan[0]) return;
     const int e = plan[4 + 4 * tile], r0 = plan[5 + 4 * tile], nr = plan[6 + 4 * tile];
@@ -316,18 +330,18 @@ __global__ __launch_bounds__(256) void moe_linear_kernel(const TA* __restrict__ 
     for (int rr = 0; rr < 2; ++rr) {
         const int r = 2 * tr + rr;
         if (r >= nr) continue;
+        const float factor = moe_row_factor(ep, r0 + r);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int j = j0 + 2 * tc + (i & 1) + 32 * (i >> 1);
             if (j >= n_out) continue;
-            float v = acc[rr][i];
-            if (act >= 2) {                            // (gate, up) pairs: i even holds the gate, i + 1 the up value
+            const float v = acc[rr][i] * factor;
+            if (moe_is_gated(ep.act)) {                // (gate, up) pairs: i even holds the gate, i + 1 the up value
                 if (i & 1) continue;
-                store_from_float(out + (size_t)(r0 + r) * out_stride + (j >> 1), moe_gated(v, acc[rr][i + 1], act, limit));
+                store_from_float(out + (size_t)(r0 + r) * out_stride + (j >> 1), moe_gated(v, acc[rr][i + 1] * factor, ep.act, ep.limit));
                 continue;
             }
-            if (act == 1) { v = fmaxf(v, 0.f); v = v * v; }
-            store_from_float(out + (size_t)(r0 + r) * out_stride + j, v);
+            store_from_float(out + (size_t)(r0 + r) * out_stride + j, moe_act1(v, ep.act));
         }
     }
 }
@@ -342,7 +356,7 @@ union moe_frag8 { uint4 raw; uint32_t w[4]; moe_bf16x8 v; };
 template <typename TA, typename TO>
 __global__ __launch_bounds__(256) void moe_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
-                                                              TO* __restrict__ out, long out_stride, int n_out, int K, int act, float limit) {
+                                                              TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
     const int tile = blockIdx.x;
     if (tile >= plan[0]) return;
     const int e = plan[4 + 4 * tile], r0 = plan[5 + 4 * tile], nr = plan[6 + 4 * tile];
@@ -371,9 +385,10 @@ __global__ __launch_bounds__(256) void moe_linear_mfma_kernel(const TA* __restri
     }
     if (ql >= nr) return;
     TO* orow = out + (size_t)(r0 + ql) * out_stride;
+    const float factor = moe_row_factor(ep, r0 + ql);
 #pragma unroll
     for (int rg = 0; rg < 4; ++rg)                     // registers 4 rg .. 4 rg + 3: outputs 8 rg + 4 h2 ..
-        moe_store4(orow, j0 + 8 * rg + 4 * h2, acc[4 * rg], acc[4 * rg + 1], acc[4 * rg + 2], acc[4 * rg + 3], act, limit);
+        moe_store4(orow, j0 + 8 * rg + 4 * h2, acc[4 * rg], acc[4 * rg + 1], acc[4 * rg + 2], acc[4 * rg + 3], ep, factor);
 }
 
 // The wider form, for K a multiple of 32: a wave takes the tile's 32 rows and 128 outputs (four accumulators that
@@ -396,7 +411,7 @@ __device__ __forceinline__ void moe_load_rows(moe_frag8& f, const TA* p) {
 template <typename TA, typename TO, int KSPLIT>
 __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
-                                                              TO* __restrict__ out, long out_stride, int n_out, int K, int act, float limit,
+                                                              TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep,
                                                               int max_tiles) {
     int tile = blockIdx.x, cb = blockIdx.y;
     if (KSPLIT == 1) {
@@ -482,11 +497,12 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
     }
     if (ql >= nr) return;
     TO* orow = out + (size_t)(r0 + ql) * out_stride;
+    const float factor = moe_row_factor(ep, r0 + ql);
     for (int f = f_lo; f < f_hi; ++f) {
         const moe_f32x16 c = KSPLIT > 1 ? acc[0] : (f == 0 ? acc[0] : f == 1 ? acc[1] : f == 2 ? acc[2] : acc[3]);
 #pragma unroll
         for (int rg = 0; rg < 4; ++rg)                 // registers 4 rg .. 4 rg + 3: outputs 32 f + 8 rg + 4 h2 ..
-            moe_store4(orow, j0 + 32 * f + 8 * rg + 4 * h2, c[4 * rg], c[4 * rg + 1], c[4 * rg + 2], c[4 * rg + 3], act, limit);
+            moe_store4(orow, j0 + 32 * f + 8 * rg + 4 * h2, c[4 * rg], c[4 * rg + 1], c[4 * rg + 2], c[4 * rg + 3], ep, factor);
     }
 }
 
@@ -500,7 +516,7 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
 template <typename TO>
 __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
-                                                              TO* __restrict__ out, long out_stride, int n_out, int K, int act, float limit) {
+                                                              TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
     const int tile = blockIdx.x;
     if (tile >= plan[0]) return;
     const int e = plan[4 + 4 * tile], r0 = plan[5 + 4 * tile], nr = plan[6 + 4 * tile];
@@ -555,18 +571,17 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
             for (int r = 0; r < MR_ROWS; ++r) {
                 if (rc + r >= nr) continue;
                 TO* orow = out + (size_t)(r0 + rc + r) * out_stride;
-                if (act >= 2) {                        // (gate, up) pairs: n_out is even and j0 a multiple of 4
+                const float factor = moe_row_factor(ep, r0 + rc + r);
+                if (moe_is_gated(ep.act)) {            // (gate, up) pairs: n_out is even and j0 a multiple of 4
 #pragma unroll
                     for (int j = 0; j < MR_OUT; j += 2)
-                        if (j0 + j < n_out) store_from_float(orow + ((j0 + j) >> 1), moe_gated(acc[j][r], acc[j + 1][r], act, limit));
+                        if (j0 + j < n_out) store_from_float(orow + ((j0 + j) >> 1), moe_gated(acc[j][r] * factor, acc[j + 1][r] * factor, ep.act, ep.limit));
                     continue;
                 }
 #pragma unroll
                 for (int j = 0; j < MR_OUT; ++j) {
                     if (j0 + j >= n_out) continue;
-                    float v = acc[j][r];
-                    if (act == 1) { v = fmaxf(v, 0.f); v = v * v; }
-                    store_from_float(orow + j0 + j, v);
+                    store_from_float(orow + j0 + j, moe_act1(acc[j][r] * factor, ep.act));
                 }
             }
         }
@@ -586,7 +601,7 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
 template <typename TO, int RF>      // RF: row fragments of 32 a wave (1: tiles of 64 rows, 2: of 128)
 __global__ __launch_bounds__(256) void moe_linear_lds_kernel(const bf16_t* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                              const bf16_t* __restrict__ w, const int* __restrict__ plan,
-                                                             TO* __restrict__ out, long out_stride, int n_out, int K, int act, float limit,
+                                                             TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep,
                                                              int max_tiles) {
     constexpr int MB_ROWS = 64 * RF;
     __shared__ __align__(16) uint16_t As[MB_ROWS * MB_LD];
@@ -684,13 +699,14 @@ __global__ __launch_bounds__(256) void moe_linear_lds_kernel(const bf16_t* __res
         const int row = 32 * RF * wr + 32 * rf + ql;
         if (row >= nr) continue;
         TO* orow = out + (size_t)(r0 + row) * out_stride;
+        const float factor = moe_row_factor(ep, r0 + row);
 #pragma unroll
         for (int cf = 0; cf < 2; ++cf) {
             if (j0 + 64 * wc + 32 * cf >= n_out) continue;
 #pragma unroll
             for (int rg = 0; rg < 4; ++rg)             // registers 4 rg .. 4 rg + 3: outputs 32 cf + 8 rg + 4 h2 ..
                 moe_store4(orow, j0 + 64 * wc + 32 * cf + 8 * rg + 4 * h2, acc[rf][cf][4 * rg], acc[rf][cf][4 * rg + 1],
-                           acc[rf][cf][4 * rg + 2], acc[rf][cf][4 * rg + 3], act, limit);
+                           acc[rf][cf][4 * rg + 2], acc[rf][cf][4 * rg + 3], ep, factor);
         }
     }
 }
@@ -702,16 +718,18 @@ extern "C" int li_moe_linear_big_takes(int a_dtype, int w_dtype, int n_out, int 
 
 extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const int* row_token, const void* w, int w_dtype,
                              const int* plan, int max_tiles, void* out, int out_dtype, long out_stride, int n_out, int K, int act, float limit,
-                             int tile_rows, int rows, hipStream_t stream) {
-    if (max_tiles <= 0 || n_out <= 0 || K <= 0 || a_stride < K || act < 0 || act > 3 || out_stride < (act >= 2 ? n_out / 2 : n_out) ||
-        (act >= 2 && (n_out & 1)))
+                             int tile_rows, int rows, const float* row_wt, hipStream_t stream) {
+    const bool gated = act == 2 || act == 3;
+    if (max_tiles <= 0 || n_out <= 0 || K <= 0 || a_stride < K || act < 0 || act > 4 || out_stride < (gated ? n_out / 2 : n_out) ||
+        (gated && (n_out & 1)))
         return LI_ERR_SIZE;
+    const MoeEpilogue ep{act, limit, row_wt};
     if (tile_rows == MOE_BIG_TILE || tile_rows == MOE_HUGE_TILE) {
         if (!li_moe_linear_big_takes(a_dtype, w_dtype, n_out, K) || a_stride % 8 || out_stride % 4 ||
             ((uintptr_t)a | (uintptr_t)w | (uintptr_t)out) % 16)
             return LI_ERR_SIZE;
         const dim3 line((unsigned)((((long)max_tiles * ((n_out + MB_COLS - 1) / MB_COLS) + 63) / 64) * 64));
-#define ML(TO, RF) moe_linear_lds_kernel<TO, RF><<<line, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, act, limit, max_tiles)
+#define ML(TO, RF) moe_linear_lds_kernel<TO, RF><<<line, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles)
         const bool huge = tile_rows == MOE_HUGE_TILE;
         if (out_dtype == LI_BF16) { if (huge) ML(bf16_t, 2); else ML(bf16_t, 1); }
         else if (out_dtype == LI_F32) { if (huge) ML(float, 2); else ML(float, 1); }
@@ -725,9 +743,9 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
         ((uintptr_t)a | (uintptr_t)w) % 16 == 0 && (out_dtype == LI_BF16 || out_dtype == LI_F32)) {
         const dim3 grid(max_tiles, (n_out + 4 * MR_OUT - 1) / (4 * MR_OUT));
         if (out_dtype == LI_BF16)
-            moe_linear_rows_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (bf16_t*)out, out_stride, n_out, K, act, limit);
+            moe_linear_rows_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (bf16_t*)out, out_stride, n_out, K, ep);
         else
-            moe_linear_rows_kernel<float><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (float*)out, out_stride, n_out, K, act, limit);
+            moe_linear_rows_kernel<float><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (float*)out, out_stride, n_out, K, ep);
         return li_launch_status();
     }
     if (w_dtype == LI_BF16 && K % 16 == 0 && n_out % 32 == 0 && a_stride % 8 == 0 && out_stride % 4 == 0 &&
@@ -738,9 +756,9 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
         const dim3 line((unsigned)((((long)max_tiles * ((n_out + 511) / 512) + 63) / 64) * 64));       // whole rounds of eight tiles over eight XCDs
 #define MM(TA, TO)                                                                                                                 \
     {                                                                                                                              \
-        if (split) moe_linear_wide_kernel<TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, act, limit, max_tiles); \
-        else if (wide) moe_linear_wide_kernel<TA, TO, 1><<<line, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, act, limit, max_tiles); \
-        else moe_linear_mfma_kernel<TA, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, act, limit); \
+        if (split) moe_linear_wide_kernel<TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        else if (wide) moe_linear_wide_kernel<TA, TO, 1><<<line, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        else moe_linear_mfma_kernel<TA, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep); \
     }
         if (a_dtype == LI_BF16 && out_dtype == LI_BF16) MM(bf16_t, bf16_t)
         else if (a_dtype == LI_BF16 && out_dtype == LI_F32) MM(bf16_t, float)
@@ -751,7 +769,7 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
         return li_launch_status();
     }
     const dim3 grid(max_tiles, (n_out + 63) / 64);
-#define ML(TA, TW, TO) moe_linear_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const TW*)w, plan, (TO*)out, out_stride, n_out, K, act, limit)
+#define ML(TA, TW, TO) moe_linear_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const TW*)w, plan, (TO*)out, out_stride, n_out, K, ep)
     if (a_dtype == LI_F32 && w_dtype == LI_F32 && out_dtype == LI_F32) ML(float, float, float);
     else if (a_dtype == LI_BF16 && w_dtype == LI_BF16 && out_dtype == LI_BF16) ML(bf16_t, bf16_t, bf16_t);
     else if (a_dtype == LI_BF16 && w_dtype == LI_BF16 && out_dtype == LI_F32) ML(bf16_t, bf16_t, float);
@@ -763,42 +781,52 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
 }
 
 // ----------------------------------------------------------------------------------------------- the sum
-// x[t, :] += sum_c wt[t, c] * yrow[pair_row[t * top + c], :] (in the order of c) + gate[t] * shared[t, :].  A choice
+// x[t, :] += factor * (the sum of what follows); with a tanh norm behind it (xn given), xn[t, :] = tanh(alpha * x[t, :]) *
+// gamma + beta of the new x.  The sum: sum_c wt[t, c] (wt null: 1) * yrow[pair_row[t * top + c], :] (in the order of c) + gate[t] * shared[t, :].  A choice
 // idx[t, c] >= experts (where `ident` is given) is an IDENTITY expert: its output is the token's input row ident[t, :].
 template <typename TI>
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x, long x_stride, const float* __restrict__ yrows,
                                                           long y_stride, const int* __restrict__ pair_row, const float* __restrict__ wt,
                                                           const float* __restrict__ gate, const float* __restrict__ shared_out,
                                                           long s_stride, int H, int top, const int* __restrict__ idx, int experts,
-                                                          const TI* __restrict__ ident, long i_stride) {
+                                                          const TI* __restrict__ ident, long i_stride, float factor,
+                                                          float alpha, const float* __restrict__ gamma, const float* __restrict__ beta,
+                                                          void* __restrict__ xn, int xn_bf16) {
     const int t = blockIdx.x;
     for (int j = blockIdx.y * 256 + threadIdx.x; j < H; j += gridDim.y * 256) {
         float s = 0.f;
         for (int c = 0; c < top; ++c) {
             const int row = pair_row[(size_t)t * top + c];
-            if (row >= 0) s = fmaf(wt[(size_t)t * top + c], yrows[(size_t)row * y_stride + j], s);
+            if (row >= 0) s = fmaf(wt ? wt[(size_t)t * top + c] : 1.0f, yrows[(size_t)row * y_stride + j], s);
             else if (ident && idx[(size_t)t * top + c] >= experts)
-                s = fmaf(wt[(size_t)t * top + c], load_as_float(ident + (size_t)t * i_stride + j), s);
+                s = fmaf(wt ? wt[(size_t)t * top + c] : 1.0f, load_as_float(ident + (size_t)t * i_stride + j), s);
         }
         if (shared_out) s = fmaf(gate ? gate[t] : 1.f, shared_out[(size_t)t * s_stride + j], s);
-        x[(size_t)t * x_stride + j] += s;
+        const float v = fmaf(factor, s, x[(size_t)t * x_stride + j]);
+        x[(size_t)t * x_stride + j] = v;
+        if (xn) {
+            const float r = fmaf(tanhf(alpha * v), gamma[j], beta[j]);
+            if (xn_bf16) reinterpret_cast<bf16_t*>(xn)[(size_t)t * H + j].bits = float_to_bf16(r);
+            else reinterpret_cast<float*>(xn)[(size_t)t * H + j] = r;
+        }
     }
 }
 
 extern "C" int li_moe_combine(float* x, long x_stride, const float* yrows, long y_stride, const int* pair_row, const float* wt,
                               const float* gate, const float* shared_out, long s_stride, int T, int H, int top,
-                              const int* idx, int experts, const void* ident, int ident_dtype, long i_stride, hipStream_t stream) {
+                              const int* idx, int experts, const void* ident, int ident_dtype, long i_stride, float factor,
+                              float alpha, const float* gamma, const float* beta, void* xn, int xn_dtype, hipStream_t stream) {
     if (T <= 0 || H <= 0 || top <= 0 || x_stride < H || y_stride < H || (shared_out && s_stride < H) ||
-        (ident && (!idx || i_stride < H || experts < 0)))
+        (ident && (!idx || i_stride < H || experts < 0)) || (xn && (!gamma || !beta)))
         return LI_ERR_SIZE;
     int ys = (H + 255) / 256;
     if (ys > 64) ys = 64;
     if (ident && ident_dtype == LI_BF16)
         moe_combine_kernel<bf16_t><<<dim3(T, ys), 256, 0, stream>>>(x, x_stride, yrows, y_stride, pair_row, wt, gate, shared_out, s_stride, H, top,
-                                                                    idx, experts, (const bf16_t*)ident, i_stride);
+                                                                    idx, experts, (const bf16_t*)ident, i_stride, factor, alpha, gamma, beta, xn, xn_dtype == LI_BF16);
     else if (!ident || ident_dtype == LI_F32)
         moe_combine_kernel<float><<<dim3(T, ys), 256, 0, stream>>>(x, x_stride, yrows, y_stride, pair_row, wt, gate, shared_out, s_stride, H, top,
-                                                                   idx, experts, (const float*)ident, i_stride);
+                                                                   idx, experts, (const float*)ident, i_stride, factor, alpha, gamma, beta, xn, xn_dtype == LI_BF16);
     else return LI_ERR_DTYPE;
     return li_launch_status();
 }

@@ -1,7 +1,8 @@
 // Kernels of recurrent mixers whose state has a fixed size per request: a short causal convolution
 // per channel with its tail of past inputs, the selective state-space recurrence
 //   S_t = a_t S_{t-1} + dt_t B_t x_t^T,  y_t = S_t^T C_t + D x_t,  a_t = exp(-exp(A_log) dt_t),
-// (with `fixed_a`: a_t = fixed_a[head] and dt_t = fixed_dt for every token, a retention with a decay a head),
+// (with `fixed_a`: a_t = fixed_a[head] and dt_t = fixed_dt for every token, a retention with a decay a head; with
+// `silu_in` x, B and C pass silu on their way in),
 // the gated delta rule, the delta rule with a decay and a removal rate a channel, and the gated RMS norm in groups of columns behind them.  Everything here is float32: inputs, decays,
 // step sizes, the state and the sums; only the normed output is rounded to the activations' type.
 #include "common.h"
@@ -116,6 +117,7 @@ extern "C" int li_causal_conv_silu(const float* u, long u_stride, int C, int tap
 #define SSM_TB 16
 #define SSM_WAVES 4
 
+__device__ __forceinline__ float silu_if(float z, int on) { return on ? z / (1.0f + expf(-z)) : z; }
 __device__ __forceinline__ float softplus_f32(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
 template <int NR, int NS, int MODE>
@@ -124,7 +126,7 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_kernel(
     const float* __restrict__ dt_bias, const float* __restrict__ A_log, const float* __restrict__ Dw,
     float* __restrict__ state, const int* __restrict__ slots, const int* __restrict__ q_start, const int* __restrict__ q_len,
     const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, float* __restrict__ decay,
-    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt) {
+    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt, int silu_in) {
     constexpr int NP = NR * NS, PW = 64 / NS;
     extern __shared__ __align__(16) float lds[];
     float* sB = lds;                                   // [SSM_TB][NP]
@@ -172,14 +174,14 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_kernel(
             const int tt = i / NP, n = i % NP;
             const bool ok = b0 + tt < ntok && n < N;
             const float* row = xbc + (size_t)(t0 + b0 + tt) * xbc_stride + inner + (size_t)g * N + n;
-            sB[i] = ok ? row[0] : 0.f;
-            sC[i] = ok ? row[(size_t)G * N] : 0.f;
+            sB[i] = ok ? silu_if(row[0], silu_in) : 0.f;
+            sC[i] = ok ? silu_if(row[(size_t)G * N], silu_in) : 0.f;
         }
         if (active) {
             for (int i = lane; i < SSM_TB * PW; i += 64) {
                 const int tt = i / PW, pp = pbase + i % PW;
                 const bool ok = b0 + tt < ntok && pp < vdim;
-                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp] : 0.f;
+                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? silu_if(xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp], silu_in) : 0.f;
             }
             if (lane < SSM_TB) {
                 const bool ok = b0 + lane < ntok;
@@ -251,7 +253,7 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_quad_kernel(
     const float* __restrict__ dt_bias, const float* __restrict__ A_log, const float* __restrict__ Dw,
     float* __restrict__ state, const int* __restrict__ slots, const int* __restrict__ q_start, const int* __restrict__ q_len,
     const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, float* __restrict__ decay,
-    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt) {
+    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt, int silu_in) {
     constexpr int NP = NR * NS, PW = 256 / NS;
     extern __shared__ __align__(16) float lds[];
     float* sB = lds;                                   // [SSM_TB][NP]
@@ -300,14 +302,14 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_quad_kernel(
             const int tt = i / NP, n = i % NP;
             const bool ok = b0 + tt < ntok && n < N;
             const float* row = xbc + (size_t)(t0 + b0 + tt) * xbc_stride + inner + (size_t)g * N + n;
-            sB[i] = ok ? row[0] : 0.f;
-            sC[i] = ok ? row[(size_t)G * N] : 0.f;
+            sB[i] = ok ? silu_if(row[0], silu_in) : 0.f;
+            sC[i] = ok ? silu_if(row[(size_t)G * N], silu_in) : 0.f;
         }
         if (active) {
             for (int i = lane; i < SSM_TB * PW; i += 64) {
                 const int tt = i / PW, pp = pbase + i % PW;
                 const bool ok = b0 + tt < ntok && pp < vdim;
-                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp] : 0.f;
+                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? silu_if(xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp], silu_in) : 0.f;
             }
             if (lane < SSM_TB) {
                 const bool ok = b0 + lane < ntok;
@@ -427,7 +429,7 @@ template <int NR, int NS, bool QUAD>
 static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, long dt_stride, const float* dt_bias,
                       const float* A_log, const float* Dw, float* state, const int* slots, const int* q_start, const int* q_len,
                       int* chunk_tab, float* carry, float* decay, float* y, long y_stride, int heads, int vdim, int N, int G,
-                      int Q, int segs, int max_chunks, bool chunked, const float* fixed_a, float fixed_dt, hipStream_t stream) {
+                      int Q, int segs, int max_chunks, bool chunked, const float* fixed_a, float fixed_dt, int silu_in, hipStream_t stream) {
     constexpr int NP = NR * NS, PW = (QUAD ? 256 : 64) / NS;
     const size_t lds = (size_t)(2 * SSM_TB * NP + SSM_WAVES * SSM_TB * PW + 2 * SSM_WAVES * SSM_TB) * sizeof(float);
 #define SSM_KERNEL(MODE_) (QUAD ? ssm_scan_quad_kernel<(QUAD ? NR : 4), (QUAD ? NS : 2), MODE_> : ssm_scan_kernel<(QUAD ? 16 : NR), (QUAD ? 1 : NS), MODE_>)
@@ -435,7 +437,7 @@ static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, lo
     if (!chunked) {
         const dim3 grid(segs, G * ublocks);
         SSM_KERNEL(0)<<<grid, 64 * SSM_WAVES, lds, stream>>>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw,
-            state, slots, q_start, q_len, nullptr, nullptr, nullptr, nullptr, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt);
+            state, slots, q_start, q_len, nullptr, nullptr, nullptr, nullptr, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt, silu_in);
         return li_launch_status();
     }
     int* chunk_seg = chunk_tab;
@@ -444,13 +446,13 @@ static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, lo
     ssm_chunk_index_kernel<<<1, 256, 0, stream>>>(q_len, segs, Q, max_chunks, chunk_seg, chunk_idx, chunk_first);
     const dim3 grid(max_chunks, G * ublocks);
     SSM_KERNEL(1)<<<grid, 64 * SSM_WAVES, lds, stream>>>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw,
-        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt);
+        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt, silu_in);
     const int NV = N * vdim;
     int zs = (NV + 255) / 256;
     if (zs > 16) zs = 16;
     ssm_carry_kernel<<<dim3(segs, heads, zs), 256, 0, stream>>>(carry, decay, state, slots, q_len, chunk_first, heads, NV, Q);
     SSM_KERNEL(0)<<<grid, 64 * SSM_WAVES, lds, stream>>>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw,
-        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt);
+        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt, silu_in);
     return li_launch_status();
 #undef SSM_KERNEL
 }
@@ -502,7 +504,7 @@ extern "C" long li_ssm_scan_work_bytes(int T, int segs, int heads, int vdim, int
 extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_raw, long dt_stride, const float* dt_bias,
                            const float* A_log, const float* Dw, float* state, const int* slots, const int* q_start,
                            const int* q_len, float* y, long y_stride, int heads, int vdim, int N, int G, int Q, int T,
-                           int segs, int max_q_len, void* work, long work_bytes, const float* fixed_a, float fixed_dt, hipStream_t stream) {
+                           int segs, int max_q_len, void* work, long work_bytes, const float* fixed_a, float fixed_dt, int silu_in, hipStream_t stream) {
     if (T <= 0 || segs <= 0 || heads <= 0 || G <= 0 || heads % G || vdim <= 0 || N <= 0 || Q <= 0 || max_q_len <= 0 ||
         xbc_stride < (long)heads * vdim + 2L * G * N || (!fixed_a && (dt_stride < heads || !dt_raw || !dt_bias || !A_log)) || y_stride < (long)heads * vdim)
         return LI_ERR_SIZE;
@@ -526,7 +528,7 @@ extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_ra
 #define SSM_QUAD(NR_, NS_)                                                                                                \
     if (qr == NR_ && qs == NS_)                                                                                           \
         return ssm_launch<NR_, NS_, true>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len, \
-                                          chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, stream);
+                                          chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, silu_in, stream);
         SSM_QUAD(4, 2) SSM_QUAD(8, 2) SSM_QUAD(16, 2) SSM_QUAD(32, 2)
         SSM_QUAD(4, 4) SSM_QUAD(8, 4) SSM_QUAD(16, 4) SSM_QUAD(32, 4)
         SSM_QUAD(4, 8) SSM_QUAD(8, 8) SSM_QUAD(16, 8) SSM_QUAD(32, 8)
@@ -536,7 +538,7 @@ extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_ra
 #define SSM_GO(NR_, NS_)                                                                                                  \
     if (nr == NR_ && ns == NS_)                                                                                           \
         return ssm_launch<NR_, NS_, false>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len,    \
-                                    chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, stream);
+                                    chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, silu_in, stream);
     SSM_GO(16, 1) SSM_GO(32, 1) SSM_GO(64, 1) SSM_GO(128, 1)
     SSM_GO(16, 2) SSM_GO(32, 2) SSM_GO(64, 2) SSM_GO(128, 2)
     SSM_GO(16, 4) SSM_GO(32, 4) SSM_GO(64, 4)

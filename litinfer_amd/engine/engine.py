@@ -173,21 +173,21 @@ class Engine:
             P = self.page_size
             per_seq = -(-self.spec.max_positions // P)
             full = per_seq * self.max_seqs
-            pages = [full if g.window <= 0 else
-                     min(full, self.max_seqs * (-(-g.window // P) + 2 + -(-g.keep_first // P)) + -(-self.step_tokens // P))
+            pages = [full if g.reach <= 0 else
+                     min(full, self.max_seqs * (-(-g.reach // P) + 2 + -(-g.keep_first // P)) + -(-self.step_tokens // P))
                      for g in groups]
             if self.rt.device.type == "cuda" and groups:
                 free, _ = torch.cuda.mem_get_info(self.rt.device)
                 bpp = [max(1, b) for b in self._group_page_bytes()]
                 budget = int(free * 0.85)
-                windowed = sum(n * b for n, b, g in zip(pages, bpp, groups) if g.window > 0)
+                windowed = sum(n * b for n, b, g in zip(pages, bpp, groups) if g.reach > 0)
                 if windowed > budget // 2:                # (windows as long as the contexts: no group is small)
                     share = max(1, budget // sum(bpp))
                     pages = [min(n, share) for n in pages]
                 else:
-                    rest = sum(b for b, g in zip(bpp, groups) if g.window <= 0)
+                    rest = sum(b for b, g in zip(bpp, groups) if g.reach <= 0)
                     share = max(1, (budget - windowed) // max(1, rest))
-                    pages = [n if g.window > 0 else min(n, share) for n, g in zip(pages, groups)]
+                    pages = [n if g.reach > 0 else min(n, share) for n, g in zip(pages, groups)]
         self.cache = CacheManager(needs, sources, page_size=self.page_size, num_pages=pages,
                                   max_seqs=self.max_seqs, dtype=self.rt.dtype, device=self.rt.device,
                                   page_order_seed=self._page_order_seed)

@@ -8,7 +8,7 @@ import torch
 
 from ..config.spec import ModelSpec, PartSpec
 from ..kernels import ops
-from ..parts.base import Runtime, build_part
+from ..parts.base import PagedNeed, Runtime, build_part
 from ..parts.stream import HyperStream, ResidualStream
 from ..weights.loader import ParamSpec
 
@@ -75,9 +75,13 @@ class Model:
     # ---- cache ------------------------------------------------------------
     def cache_needs(self) -> Tuple[List[object], List[Optional[int]]]:
         """What every entry of the execution order keeps, and, as one more entry behind them, what the
-        embedding keeps (per-request state of its own, if any): `cache.view(len(order))` is its view."""
+        embedding keeps (per-request state of its own, if any): `cache.view(len(order))` is its view.
+        An entry whose pages another one reads keeps them as long as either still sees them."""
         needs = [self.layers[e.layer].cache_need() for e in self.order]
         sources = [e.cache_from for e in self.order]
+        for i, src in enumerate(sources):
+            if src is not None and isinstance(needs[i], PagedNeed) and isinstance(needs[src], PagedNeed):
+                needs[src] = needs[src].covering(needs[i])
         own = self.embedding.cache_need() if hasattr(self.embedding, "cache_need") else None
         if own is not None:
             needs.append(own)
@@ -98,7 +102,7 @@ class Model:
             # an injection reads the embedding output again later: a copy beside the stream
             ctx.embedding_out = ctx.ws.buffer("model.embedding_out", (ctx.num_tokens, h), torch.float32)
             ops.cast(x, ctx.embedding_out)
-        stream = HyperStream(x, ctx.ws, self.spec.streams) if self.spec.streams else ResidualStream(x, ctx.ws)
+        stream = HyperStream(x, ctx.ws, self.spec.streams) if self.spec.streams else ResidualStream(x, ctx.ws, self.spec.residual_scale)
         stream.ws_dtype = self.rt.dtype
         for i, e in enumerate(self.order):
             if e.inject is not None:

@@ -38,7 +38,7 @@ _SIGNATURES = {
         "li_rope_kv_store": [P, I, I, I, I, I, I, P, P, P, P, P, I, I, I],
         "li_embedding_add": [P, P, P, P, I, P, P, I, I, I],
         "li_rmsnorm_add": [P, P, F, F, P, F, P, P, F, P, I, I, I, I],
-        "li_gated_act": [P, I, P, I, I, I, I],
+        "li_gated_act": [P, I, P, I, I, I, I, F],
         "li_relu_squared": [P, I, P, I, L],
         "li_gelu_gate_rows": [P, P, P, P, P, I, I, I, I, P, I, I, I],
         "li_rope_freq_table": [P, P, I, F, P, P, I],
@@ -52,6 +52,8 @@ _SIGNATURES = {
         "li_latent_norm_pairs_store": [P, L, I, I, I, P, L, I, P, F, P, P, P, P, I, P, I, I, P, L, I, P, P, I, I],
         "li_pair_embedding": [P, P, P, P, P, P, P, P, P, P, P, I, P, I, I, I, I, L, L],
         "li_layernorm": [P, P, P, F, P, I, I, I],
+        "li_tanh_norm": [P, F, P, P, P, I, I, I],
+        "li_gelu_erf": [P, I, P, I, L],
         "li_gelu_tanh": [P, I, P, I, L],
         "li_concat_rows": [P, P, P, I, I, I],
         "li_sinusoid_add": [P, P, P, I, I],
@@ -61,31 +63,32 @@ _SIGNATURES = {
     },
     "recurrent": {
         "li_causal_conv_silu": [P, L, I, I, P, P, P, P, P, P, P, P, L, I, I, I],
-        "li_ssm_scan": [P, L, P, L, P, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, I, P, L, P, F],
+        "li_ssm_scan": [P, L, P, L, P, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, I, P, L, P, F, I],
         "li_delta_scan": [P, L, P, L, P, P, P, P, P, P, P, L, I, I, I, I, F, I, I, I, I, P, L],
         "li_channel_delta": [P, L, P, L, P, P, P, P, P, L, I, I, I, I, I, I, I, P, L],
         "li_gated_group_norm": [P, L, P, L, P, F, P, I, L, I, I, I, I],
     },
     "moe": {
         "li_moe_route": [P, I, L, P, I, P, P, P, P, P, I, I, I, I, I, P, I, I],
-        "li_moe_plan": [P, I, I, I, P, I, P, P, I],
-        "li_moe_linear": [P, I, L, P, P, I, P, I, P, I, L, I, I, I, F, I, I],
-        "li_moe_combine": [P, L, P, L, P, P, P, P, L, I, I, I, P, I, P, I, L],
+        "li_moe_plan": [P, I, I, I, P, I, P, P, I, P, P],
+        "li_moe_linear": [P, I, L, P, P, I, P, I, P, I, L, I, I, I, F, I, I, P],
+        "li_moe_combine": [P, L, P, L, P, P, P, P, L, I, I, I, P, I, P, I, L, F, F, P, P, P, I],
     },
     "attention_masked": {
-        "li_masked_attention": [P, I, I, P, I, P, P, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I],
-        "li_masked_attention_single": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, P, L],
-        "li_masked_attention_heads": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, P, L],
-        "li_masked_attention_tiles": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, P, L, P, I, I],
+        "li_masked_attention": [P, I, I, P, I, P, P, I, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, I],
+        "li_masked_attention_single": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, I, P, L],
+        "li_masked_attention_heads": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, I, P, L],
+        "li_masked_attention_tiles": [P, I, I, P, P, P, I, I, P, I, P, I, P, P, P, I, I, I, I, I, I, I, I, F, F, P, P, L, I, P, I, I, P, L, P, I, I],
         "li_headwise_linear": [P, I, L, I, P, I, P, I, L, I, I, I, I, I, P, L, I, I, I, P, P],
     },
     "gemm": {
-        "li_linear": [P, P, P, P, I, I, I, I, I, I, P, L],
-        "li_linear_skinny": [P, P, P, P, I, I, I, I, I, I],
-        "li_linear_swiglu": [P, P, P, I, I, I, P, I, F],
-        "li_linear_swiglu_f32": [P, P, P, I, I, I],
-        "li_linear_residual_norm": [P, P, P, P, I, I, I, P, P, P],
-        "li_linear_then_norm": [P, P, P, P, I, I, I, P, L, P, F, P, I],
+        "li_linear": [P, P, P, P, I, I, I, I, I, F, P, L],
+        "li_linear_skinny": [P, P, P, P, I, I, I, I, F, I],
+        "li_linear_swiglu": [P, P, P, I, I, I, P, I, F, F],
+        "li_linear_swiglu_f32": [P, P, P, I, I, I, F],
+        "li_linear_residual_norm": [P, P, P, P, I, I, I, F, P, P, P],
+        "li_linear_then_norm": [P, P, P, P, I, I, I, P, L, F, P, F, P, I],
+        "li_linear_tanh_norm": [P, P, P, P, I, I, I, P, L, F, F, P, P, P, I],
         "li_linear_rope_store": [P, P, P, P, I, I, P, P, P, P, P, I, I, I, I, I, P, I, F],
         "li_linear_rope_store_parts": [P, P, P, P, I, I, P, P, P, P, P, I, I, I, I, I, P, L],
     },
@@ -404,17 +407,18 @@ def rmsnorm_add(y: torch.Tensor, weight: torch.Tensor, eps: float, x: torch.Tens
              0 if next_out is None else next_out.data_ptr(), _DT[next_out.dtype] if next_out is not None else 0, nxt, x.shape[0], h)
 
 
-def gated_act(gate_up: torch.Tensor, out: torch.Tensor, act: str) -> None:
-    """out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]; act "silu" or "gelu_tanh"; float32 arithmetic; gate_up in
+def gated_act(gate_up: torch.Tensor, out: torch.Tensor, act: str, limit: float = 0.0) -> None:
+    """out[t, i] = act(gate_up[t, i]) * gate_up[t, I + i]; act "silu" or "gelu_tanh", or "clamped": g sigmoid(1.702 g) (u + 1)
+    with g = min(gate, limit) and u = clamp(up, -limit, limit); float32 arithmetic; gate_up in
     float32 or the engine's dtype, out in the engine's."""
     _gpu(gate_up, out)
     t, i = out.shape
-    _chk(act in ("silu", "gelu_tanh"), "gated_act: act")
+    _chk(act in ("silu", "gelu_tanh") or (act == "clamped" and limit > 0), "gated_act: act")
     _chk(gate_up.shape == (t, 2 * i) and gate_up.is_contiguous() and out.is_contiguous() and gate_up.dtype in _DT and out.dtype in _DT
          and (gate_up.dtype is torch.float32 or out.dtype is torch.bfloat16), "gated_act: gate_up [T, 2 I], out [T, I]")
     if t:
         _run("elementwise", "li_gated_act", gate_up.data_ptr(), _DT[gate_up.dtype], out.data_ptr(), _DT[out.dtype], t, i,
-             1 if act == "gelu_tanh" else 0)
+             {"silu": 0, "gelu_tanh": 1, "clamped": 2}[act], float(limit))
 
 
 def relu_squared(x: torch.Tensor, out: torch.Tensor) -> None:
@@ -481,10 +485,11 @@ def qk_norm_pairs_store(qkv: torch.Tensor, nh: int, nkv: int, dk: int, dv: int, 
                         v: Optional[torch.Tensor], page_size: int, half_split: bool = False) -> None:
     """qkv float32 rows [q (nh*dk) | k (nkv*dk) | v (nkv*dv)].  q and k are RMS-normed over their WHOLE
     width (weights wq, wk; None: no norm), their heads' first `rotary_dim` columns rotated in neighbouring
-    pairs (`half_split`: column i with column i + rotary_dim / 2); q stays in place, k and v go to their page slots (k None: only q is prepared)."""
+    pairs (`half_split`: column i with column i + rotary_dim / 2); q stays in place, k and v go to their page slots (k None: only q is prepared, and
+    the rows may end behind it)."""
     _gpu(qkv, wq, wk, cos, sin, slot_map, k, v)
     t = qkv.shape[0]
-    _chk(_rows_ok(qkv) and qkv.dtype is torch.float32 and qkv.shape[1] >= nh * dk + nkv * (dk + dv),
+    _chk(_rows_ok(qkv) and qkv.dtype is torch.float32 and qkv.shape[1] >= nh * dk + (nkv * (dk + dv) if k is not None else 0),
          "qk_norm_pairs_store: qkv must be float32 rows of q, k and v")
     _chk(rotary_dim % 2 == 0 and 0 <= rotary_dim <= dk, "qk_norm_pairs_store: rotary_dim")
     _check_tables("qk_norm_pairs_store", t, rotary_dim, cos, sin, slot_map if k is not None else None)
@@ -688,6 +693,27 @@ def layernorm(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor
              out.data_ptr(), _DT[out.dtype], x.shape[0], x.shape[1])
 
 
+def tanh_norm(x: torch.Tensor, alpha: float, weight: torch.Tensor, bias: torch.Tensor, out: torch.Tensor) -> None:
+    """out = tanh(alpha * x) * weight + bias, element by element, in float32."""
+    _gpu(x, weight, bias, out)
+    _chk(x.dim() == 2 and x.shape == out.shape and x.is_contiguous() and out.is_contiguous() and x.dtype is torch.float32
+         and out.dtype in _DT, "tanh_norm: x float32 and out must be contiguous [T, H] of one shape")
+    _chk(all(w.dtype is torch.float32 and w.numel() == x.shape[1] and w.is_contiguous() for w in (weight, bias)),
+         "tanh_norm: weight and bias must be float32 [H]")
+    if x.shape[0]:
+        _run("elementwise", "li_tanh_norm", x.data_ptr(), float(alpha), weight.data_ptr(), bias.data_ptr(), out.data_ptr(),
+             _DT[out.dtype], x.shape[0], x.shape[1])
+
+
+def gelu_erf(x: torch.Tensor, out: torch.Tensor) -> None:
+    """out = 0.5 x (1 + erf(x / sqrt(2)))."""
+    _gpu(x, out)
+    _chk(x.shape == out.shape and x.is_contiguous() and out.is_contiguous() and x.dtype in _DT and out.dtype in _DT
+         and (x.dtype is torch.float32 or out.dtype is x.dtype), "gelu_erf: x, out")
+    if x.numel():
+        _run("elementwise", "li_gelu_erf", x.data_ptr(), _DT[x.dtype], out.data_ptr(), _DT[out.dtype], x.numel())
+
+
 def gelu_tanh(x: torch.Tensor, out: torch.Tensor) -> None:
     """out = 0.5 x (1 + tanh(sqrt(2/pi) (x + 0.044715 x^3)))."""
     _gpu(x, out)
@@ -731,7 +757,7 @@ def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, o
                      v: torch.Tensor, meta, nh: int, nkv: int, dk: int, dv: int, page_size: int, window: int,
                      keep_first: int, softcap: float, scale: float, ws=None, sink: Optional[torch.Tensor] = None,
                      head_gate: Optional[torch.Tensor] = None, column_gate: Optional[torch.Tensor] = None,
-                     slopes: Optional[torch.Tensor] = None) -> None:
+                     slopes: Optional[torch.Tensor] = None, chunk: int = 0) -> None:
     """Attention of every token of the step over its request's cached keys: position p sees j <= p with
     p - j < window (0: all) or j < keep_first; scores (q . k) * scale, then softcap * tanh(score / softcap)
     where softcap > 0; softmax and sums in float32.  q: a float32 tensor in which head h of token t starts at
@@ -740,7 +766,8 @@ def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, o
     `sink` (float32 [nh]): the softmax's denominator also holds exp(sink[head]), a term without key or value.
     `head_gate` (float32 rows [T, nh], a view of columns is fine): head h's output of token t is multiplied by
     sigmoid(head_gate[t, h]).  `column_gate` (float32 rows [T, nh * dv], a view is fine) does that with a number for every
-    head and value column.  `slopes` (float32 [nh]): a key's score loses slopes[head] * (p - j)."""
+    head and value column.  `slopes` (float32 [nh]): a key's score loses slopes[head] * (p - j).  `chunk` > 0: only keys
+    with j // chunk == p // chunk are seen (positions counted from the request's start); not together with keep_first."""
     _gpu(q, out, k, v, meta.block_table, sink, head_gate, column_gate, slopes)
     t = out.shape[0]
     _chk(q.dtype is torch.float32 and q.is_contiguous() and q.numel() >= (t - 1) * q_token_stride + (nh - 1) * q_head_stride + dk,
@@ -759,12 +786,14 @@ def masked_attention(q: torch.Tensor, q_token_stride: int, q_head_stride: int, o
     _chk(slopes is None or (slopes.dtype is torch.float32 and slopes.numel() == nh and slopes.is_contiguous()), "masked_attention: slopes")
     gate = head_gate if column_gate is None else column_gate
     fin = (0 if sink is None else sink.data_ptr(), 0 if gate is None else gate.data_ptr(), 0 if gate is None else gate.stride(0),
-           int(column_gate is not None), 0 if slopes is None else slopes.data_ptr())
+           int(column_gate is not None), 0 if slopes is None else slopes.data_ptr(), int(chunk))
+    _chk(chunk >= 0 and not (chunk and keep_first), "masked_attention: chunk")
     if not t:
         return
     # keys that one query may see, as far as the host knows without looking at the contexts (a recorded step
     # must not depend on them): decides how many waves share a (token, head)'s keys in the general kernel
     bound = window + keep_first if window else meta.max_blocks * page_size
+    bound = min(bound, chunk) if chunk else bound
     waves = 8 if bound >= 512 else 4 if bound >= 128 else 1
 
     def general(token_list, n):
@@ -924,8 +953,8 @@ SPLITK_MAX_PARTS = 8
 
 
 def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor,
-           accumulate: bool = False, ws=None) -> None:
-    """out = x w^T + bias, or out += x w^T + bias when `accumulate`.
+           accumulate: bool = False, ws=None, factor: float = 1.0) -> None:
+    """out = x w^T + bias, or out += factor * (x w^T + bias) when `accumulate`.
     x [M, K] and w [N, K] of one dtype (float32 or bfloat16); out [M, N] of that
     dtype or float32; accumulation of the product is float32.  `ws` lends the
     memory for partial sums where the kernel cuts K into parts (17 rows and more
@@ -942,6 +971,7 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: 
         _chk(False, f"linear: x is {x.dtype}, w is {w.dtype}")
     _chk(out.dtype is x.dtype or out.dtype is torch.float32, "linear: out dtype")
     _chk(not accumulate or out.dtype is torch.float32, "linear: accumulation needs a float32 out")
+    _chk(factor == 1.0 or (accumulate and factor != 0.0), "linear: a factor goes with accumulation and is not zero")
     _chk(bias is None or (bias.dtype is torch.float32 and bias.numel() == n and bias.is_contiguous()),
          "linear: bias must be float32 [N]")
     if m:
@@ -955,7 +985,7 @@ def linear(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: 
                 buf = ws.buffer("gemm.parts", (need // 4,), torch.float32)
                 work, work_bytes = buf.data_ptr(), buf.numel() * 4
         _run("gemm", "li_linear", x.data_ptr(), w.data_ptr(), 0 if bias is None else bias.data_ptr(),
-             out.data_ptr(), m, n, k, _DT[x.dtype], _DT[out.dtype], int(bool(accumulate)), work, work_bytes)
+             out.data_ptr(), m, n, k, _DT[x.dtype], _DT[out.dtype], float(factor) if accumulate else 0.0, work, work_bytes)
 
 
 
@@ -993,7 +1023,7 @@ def linear_skinny(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor]
     _chk(bias is None or (bias.dtype is torch.float32 and bias.numel() == n and bias.is_contiguous()),
          "linear_skinny: bias must be float32 [N]")
     _run("gemm", "li_linear_skinny", x.data_ptr(), w.data_ptr(), 0 if bias is None else bias.data_ptr(),
-         out.data_ptr(), m, n, k, _DT[out.dtype], int(bool(accumulate)), int(bool(swiglu)))
+         out.data_ptr(), m, n, k, _DT[out.dtype], float(bool(accumulate)), int(bool(swiglu)))
 
 
 def swiglu_takes(m: int, k: int, w_dtype: torch.dtype) -> bool:
@@ -1058,8 +1088,8 @@ def row_scale_rows(m: int) -> int:
 
 
 def linear_residual_norm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor,
-                         gamma: torch.Tensor, xg: torch.Tensor, sq_parts: torch.Tensor) -> int:
-    """out += x w^T + bias (float32); xg = bfloat16(gamma * out); sq_parts[p * R + m] = block p's
+                         gamma: torch.Tensor, xg: torch.Tensor, sq_parts: torch.Tensor, factor: float = 1.0) -> int:
+    """out += factor * (x w^T + bias) (float32); xg = bfloat16(gamma * out); sq_parts[p * R + m] = block p's
     share of sum_n out[m, n]^2 (R = `row_scale_rows(m)`).  Returns the number of blocks p."""
     _gpu(x, w, bias, out, gamma, xg, sq_parts)
     m, k = x.shape
@@ -1076,13 +1106,13 @@ def linear_residual_norm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.
     _chk(sq_parts.dtype is torch.float32 and sq_parts.is_contiguous() and sq_parts.numel() >= parts * row_scale_rows(m),
          "linear_residual_norm: sq_parts must be float32 with 16 places a block (32 above 16 rows)")
     _run("gemm", "li_linear_residual_norm", x.data_ptr(), w.data_ptr(), 0 if bias is None else bias.data_ptr(),
-         out.data_ptr(), m, n, k, gamma.data_ptr(), xg.data_ptr(), sq_parts.data_ptr())
+         out.data_ptr(), m, n, k, float(factor), gamma.data_ptr(), xg.data_ptr(), sq_parts.data_ptr())
     return parts
 
 
 def linear_then_norm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor,
-                     gamma: torch.Tensor, eps: float, xn: torch.Tensor, ws) -> bool:
-    """out += x w^T + bias (float32) and xn = gamma * out / sqrt(mean(out^2) + eps), in the kernel
+                     gamma: torch.Tensor, eps: float, xn: torch.Tensor, ws, factor: float = 1.0) -> bool:
+    """out += factor * (x w^T + bias) (float32) and xn = gamma * out / sqrt(mean(out^2) + eps), in the kernel
     that adds up the parts of a product cut along K.  Returns False, having done nothing, where
     `linear` would not cut this product (then multiply and norm in two calls)."""
     _gpu(x, w, bias, out, gamma, xn)
@@ -1105,12 +1135,49 @@ def linear_then_norm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tens
         need = max(need, SPLITK_MAX_PARTS * SKINNY_MAX_ROWS * n * 4)
     buf = ws.buffer("gemm.parts", (need // 4,), torch.float32)
     rc = _fn("gemm", "li_linear_then_norm")(x.data_ptr(), w.data_ptr(), 0 if bias is None else bias.data_ptr(),
-                                             out.data_ptr(), m, n, k, buf.data_ptr(), buf.numel() * 4, gamma.data_ptr(),
+                                             out.data_ptr(), m, n, k, buf.data_ptr(), buf.numel() * 4, float(factor), gamma.data_ptr(),
                                              float(eps), xn.data_ptr(), _DT[xn.dtype], _stream())
     if rc == -1:
         return False
     if rc != 0:
         raise RuntimeError(f"li_linear_then_norm: the kernel library refused the call (code {rc}): {_ERRORS.get(rc, 'unknown')}")
+    return True
+
+
+def linear_tanh_norm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, alpha: float,
+                     gamma: torch.Tensor, beta: torch.Tensor, xn: torch.Tensor, ws, factor: float = 1.0) -> bool:
+    """out += factor * (x w^T + bias) (float32) and xn = tanh(alpha * out) * gamma + beta in one go: in the product's
+    epilogue where the rows are few, or in the kernel that adds up the parts of a product cut along K.  Returns False,
+    having done nothing, where the product takes neither form (then multiply and norm in two calls)."""
+    _gpu(x, w, bias, out, gamma, beta, xn)
+    if x.dtype is not torch.bfloat16 or w.dtype is not torch.bfloat16:
+        return False
+    _chk(x.dim() == 2 and w.dim() == 2, "linear_tanh_norm: needs matrices")
+    m, k = x.shape
+    n = w.shape[0]
+    if not m:
+        return False
+    work, work_bytes = 0, 0
+    if not (m <= RESIDUAL_NORM_MAX_ROWS and few_rows_preferred(m, n, k) and xn.dtype is torch.bfloat16):
+        need = _work_bytes(m, n, k, _DT[x.dtype]) if ws is not None else 0
+        if not need:
+            return False
+        if m <= SKINNY_MAX_ROWS:            # one size for all row counts of a decode batch: the buffer does not move
+            need = max(need, SPLITK_MAX_PARTS * SKINNY_MAX_ROWS * n * 4)
+        buf = ws.buffer("gemm.parts", (need // 4,), torch.float32)
+        work, work_bytes = buf.data_ptr(), buf.numel() * 4
+    _chk(w.shape == (n, k) and x.is_contiguous() and w.is_contiguous(), "linear_tanh_norm: contiguous [M, K] and [N, K]")
+    _chk(out.dtype is torch.float32 and out.shape == (m, n) and out.is_contiguous(), "linear_tanh_norm: out must be float32 [M, N]")
+    _chk(xn.dtype in _DT and xn.shape == (m, n) and xn.is_contiguous(), "linear_tanh_norm: xn must be [M, N]")
+    _chk(all(v is None or (v.dtype is torch.float32 and v.numel() == n and v.is_contiguous()) for v in (bias, gamma, beta))
+         and factor != 0.0, "linear_tanh_norm: bias, gamma and beta must be float32 [N], the factor not zero")
+    rc = _fn("gemm", "li_linear_tanh_norm")(x.data_ptr(), w.data_ptr(), 0 if bias is None else bias.data_ptr(), out.data_ptr(),
+                                             m, n, k, work, work_bytes, float(factor), float(alpha), gamma.data_ptr(),
+                                             beta.data_ptr(), xn.data_ptr(), _DT[xn.dtype], _stream())
+    if rc == -1:
+        return False
+    if rc != 0:
+        raise RuntimeError(f"li_linear_tanh_norm: the kernel library refused the call (code {rc}): {_ERRORS.get(rc, 'unknown')}")
     return True
 
 
@@ -1126,10 +1193,12 @@ def _check_row_scale(what: str, m: int, row_scale: Optional[RowScale]):
     return row_scale.sq_parts.data_ptr(), row_scale.nparts, row_scale.eps
 
 
-def linear_swiglu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, row_scale: Optional[RowScale] = None) -> None:
+def linear_swiglu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, row_scale: Optional[RowScale] = None,
+                  limit: float = 0.0) -> None:
     """out[m, n] = up * gate / (1 + exp(-gate)) with [gate, up] = x w^T, w = [gate; up]
     (2 N rows): the activation in the product's epilogue, from the product's float32 sums.
-    With `row_scale`, x is the xg of `linear_residual_norm` and the result is that of the norm."""
+    With `row_scale`, x is the xg of `linear_residual_norm` and the result is that of the norm.  With `limit` > 0 the
+    clamped form: g sigmoid(1.702 g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit)."""
     _gpu(x, w, out)
     _chk(x.dim() == 2 and w.dim() == 2 and out.dim() == 2, "linear_swiglu: needs matrices")
     m, k = x.shape
@@ -1142,11 +1211,11 @@ def linear_swiglu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, row_scale
         _chk(x.dtype is torch.float32 and out.dtype is torch.float32 and row_scale is None,
              "linear_swiglu: float32 w goes with float32 x and out, and no row scale")
         _chk(x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0, "linear_swiglu: operands must start on 16 bytes")
-        _run("gemm", "li_linear_swiglu_f32", x.data_ptr(), w.data_ptr(), out.data_ptr(), m, n, k)
+        _run("gemm", "li_linear_swiglu_f32", x.data_ptr(), w.data_ptr(), out.data_ptr(), m, n, k, float(limit))
         return
     _chk(x.dtype is torch.bfloat16 and out.dtype is torch.bfloat16, "linear_swiglu: x and out must be bfloat16")
     _run("gemm", "li_linear_swiglu", x.data_ptr(), w.data_ptr(), out.data_ptr(), m, n, k,
-         *_check_row_scale("linear_swiglu", m, row_scale))
+         *_check_row_scale("linear_swiglu", m, row_scale), float(limit))
 
 
 ROPE_STORE_MAX_ROWS = 32
@@ -1630,11 +1699,11 @@ def causal_conv_silu(u: torch.Tensor, w: torch.Tensor, b: Optional[torch.Tensor]
 
 def ssm_scan(xbc: torch.Tensor, dt: Optional[torch.Tensor], dt_bias: Optional[torch.Tensor], a_log: Optional[torch.Tensor],
              d: Optional[torch.Tensor], state: torch.Tensor, ctx, y: torch.Tensor, heads: int, vdim: int, n_state: int,
-             groups: int, ws, fixed_decay: Optional[torch.Tensor] = None, fixed_step: float = 1.0) -> None:
+             groups: int, ws, fixed_decay: Optional[torch.Tensor] = None, fixed_step: float = 1.0, silu_in: bool = False) -> None:
     """The state-space recurrence over each request's tokens of the step, from and into `state`
     [slots, heads, n_state, vdim] (float32):  S <- a S + dt B x^T,  y = S^T C + d_h x,  with a = exp(-exp(a_log_h) dt) and
     dt = softplus(dt_raw + dt_bias_h), or, with `fixed_decay` (float32 [heads]), a = fixed_decay[h] and dt = fixed_step
-    for every token (dt, dt_bias and a_log are then not read; d None: no x term).
+    for every token (dt, dt_bias and a_log are then not read; d None: no x term).  `silu_in`: x, B and C pass silu first.
     xbc: float32 rows [x: heads * vdim | B: groups * n_state | C: groups * n_state];
     dt: float32 rows [heads] (raw); y: float32 rows [heads * vdim].  All float32."""
     fixed = fixed_decay is not None
@@ -1664,7 +1733,7 @@ def ssm_scan(xbc: torch.Tensor, dt: Optional[torch.Tensor], dt_bias: Optional[to
     _run("recurrent", "li_ssm_scan", xbc.data_ptr(), xbc.stride(0), ptr(dt), 0 if dt is None else dt.stride(0), ptr(dt_bias), ptr(a_log),
          ptr(d), state.data_ptr(), ctx.state_slots.data_ptr(), ctx.q_start.data_ptr(), ctx.q_len.data_ptr(), y.data_ptr(),
          y.stride(0), heads, vdim, n_state, groups, SSM_CHUNK, t, ctx.num_segments, int(ctx.max_q_len), work, work_bytes,
-         ptr(fixed_decay), float(fixed_step))
+         ptr(fixed_decay), float(fixed_step), int(bool(silu_in)))
 
 
 # Portions of more than SSM_CHUNK tokens run through the delta rule as chunks side by side (their own states and transition
@@ -1824,11 +1893,13 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
 
 
 def moe_plan(idx: torch.Tensor, experts: int, plan: torch.Tensor, row_token: torch.Tensor, pair_row: torch.Tensor,
-             tile_rows: int = MOE_TILE_ROWS) -> int:
+             tile_rows: int = MOE_TILE_ROWS, wt: Optional[torch.Tensor] = None, row_wt: Optional[torch.Tensor] = None) -> int:
     """Sorts the (token, choice) pairs by expert.  plan int32 [4 + 4 * max_tiles]: the number of tiles, then (expert,
-    first row, rows, 0) a tile; row_token [pairs]: the token of a sorted row; pair_row [pairs]: the row of a pair.
-    Returns max_tiles."""
-    _gpu(idx, plan, row_token, pair_row)
+    first row, rows, 0) a tile; row_token [pairs]: the token of a sorted row; pair_row [pairs]: the row of a pair;
+    row_wt [pairs] float32 (with wt [T, top]): the weight of a sorted row's pair.  Returns max_tiles."""
+    _gpu(idx, plan, row_token, pair_row, wt, row_wt)
+    _chk(row_wt is None or (wt is not None and all(v.dtype is torch.float32 and v.is_contiguous() and v.numel() >= idx.numel()
+                                                   for v in (wt, row_wt))), "moe_plan: wt, row_wt")
     t, top = idx.shape
     max_tiles = moe_max_tiles(t, top, experts, tile_rows)
     _chk(tile_rows in (MOE_TILE_ROWS, MOE_BIG_TILE_ROWS, MOE_HUGE_TILE_ROWS), "moe_plan: tiles of 32, 64 or 128 rows")
@@ -1837,21 +1908,25 @@ def moe_plan(idx: torch.Tensor, experts: int, plan: torch.Tensor, row_token: tor
          "moe_plan: int32 arrays of the step's sizes")
     if t:
         _run("moe", "li_moe_plan", idx.data_ptr(), t, top, experts, plan.data_ptr(), max_tiles, row_token.data_ptr(), pair_row.data_ptr(),
-             int(tile_rows))
+             int(tile_rows), 0 if wt is None else wt.data_ptr(), 0 if row_wt is None else row_wt.data_ptr())
     return max_tiles
 
 
 def moe_linear(a: torch.Tensor, row_token: Optional[torch.Tensor], w: torch.Tensor, plan: torch.Tensor, max_tiles: int,
-               out: torch.Tensor, rows: int, act: int = 0, tile_rows: int = MOE_TILE_ROWS, limit: float = 0.0) -> None:
+               out: torch.Tensor, rows: int, act: int = 0, tile_rows: int = MOE_TILE_ROWS, limit: float = 0.0,
+               row_wt: Optional[torch.Tensor] = None) -> None:
     """out[row] = act(W[expert of the row's tile] a[src(row)]) for the sorted rows of the plan; src(row) = row_token[row]
     where given (rows gathered from tokens), else the row.  w [experts, n_out, K]; act 1: max(., 0)^2; act 2: the
     matrix rows are (gate, up) pairs, out[row, j] = silu(W[2j] a) * (W[2j + 1] a) and out has n_out / 2 columns; act 3:
-    the same pairs with g = min(gate, limit), u = clamp(up, -limit, limit) and out = g sigmoid(1.702 g) (u + 1)."""
-    _gpu(a, row_token, w, plan, out)
+    the same pairs with g = min(gate, limit), u = clamp(up, -limit, limit) and out = g sigmoid(1.702 g) (u + 1);
+    act 4: gelu (with the error function).  `row_wt` (float32, a number a sorted row) multiplies the row of a."""
+    _gpu(a, row_token, w, plan, out, row_wt)
     e, n_out, k = w.shape
-    _chk(act in (0, 1, 2, 3) and (act < 2 or n_out % 2 == 0) and (act != 3 or limit > 0), "moe_linear: act")
+    gated = act in (2, 3)
+    _chk(act in (0, 1, 2, 3, 4) and (not gated or n_out % 2 == 0) and (act != 3 or limit > 0), "moe_linear: act")
+    _chk(row_wt is None or (row_wt.dtype is torch.float32 and row_wt.is_contiguous() and row_wt.numel() >= rows), "moe_linear: row_wt")
     _chk(a.dtype in _DT and _rows_ok(a) and a.shape[1] == k and w.dtype in _DT and w.is_contiguous() and out.dtype in _DT and _rows_ok(out)
-         and out.shape == (rows, n_out // 2 if act >= 2 else n_out)
+         and out.shape == (rows, n_out // 2 if gated else n_out)
          and (w.dtype is torch.bfloat16 or (a.dtype is torch.float32 and out.dtype is torch.float32)),
          "moe_linear: a [*, K], w [E, n_out, K], out [rows, n_out]")
     _chk(plan.dtype is torch.int32 and plan.numel() >= 4 + 4 * max_tiles and (row_token is not None or a.shape[0] >= rows)
@@ -1859,29 +1934,38 @@ def moe_linear(a: torch.Tensor, row_token: Optional[torch.Tensor], w: torch.Tens
     if rows:
         _run("moe", "li_moe_linear", a.data_ptr(), _DT[a.dtype], a.stride(0), 0 if row_token is None else row_token.data_ptr(),
              w.data_ptr(), _DT[w.dtype], plan.data_ptr(), int(max_tiles), out.data_ptr(), _DT[out.dtype], out.stride(0), n_out, k, int(act),
-             float(limit), int(tile_rows), int(rows))
+             float(limit), int(tile_rows), int(rows), 0 if row_wt is None else row_wt.data_ptr())
 
 
-def moe_combine(x: torch.Tensor, yrows: torch.Tensor, pair_row: torch.Tensor, wt: torch.Tensor, gate: Optional[torch.Tensor],
+def moe_combine(x: torch.Tensor, yrows: torch.Tensor, pair_row: torch.Tensor, wt: Optional[torch.Tensor], gate: Optional[torch.Tensor],
                 shared_out: Optional[torch.Tensor], idx: Optional[torch.Tensor] = None, experts: int = 0,
-                identity_rows: Optional[torch.Tensor] = None) -> None:
-    """x[t] += sum_c wt[t, c] * yrows[pair_row[t * top + c]] (in the order of c) + gate[t] * shared_out[t]; float32.
+                identity_rows: Optional[torch.Tensor] = None, top: int = 0, factor: float = 1.0, tanh_norm=None) -> None:
+    """x[t] += factor * (sum_c wt[t, c] * yrows[pair_row[t * top + c]] (in the order of c) + gate[t] * shared_out[t]); float32.
+    wt None: every choice counts once (`top` says how many there are).  `tanh_norm` = (alpha, weight, bias, xn): xn [T, H] =
+    tanh(alpha * x) * weight + bias of the new x.
     With `identity_rows` [T, H] (the feed-forward's input), a choice idx[t, c] >= experts is an identity expert whose
     output is identity_rows[t]."""
     _gpu(x, yrows, pair_row, wt, gate, shared_out, idx, identity_rows)
     t, h = x.shape
-    top = wt.shape[1]
+    top = wt.shape[1] if wt is not None else int(top)
+    alpha, gamma, beta, xn = tanh_norm if tanh_norm is not None else (0.0, None, None, None)
+    _gpu(gamma, beta, xn)
+    _chk(xn is None or (xn.dtype in _DT and xn.shape == (t, h) and xn.is_contiguous()
+                        and all(v.dtype is torch.float32 and v.numel() == h and v.is_contiguous() for v in (gamma, beta))),
+         "moe_combine: tanh_norm")
     _chk(x.dtype is torch.float32 and _rows_ok(x) and yrows.dtype is torch.float32 and _rows_ok(yrows) and yrows.shape == (t * top, h)
-         and pair_row.dtype is torch.int32 and pair_row.numel() >= t * top and wt.dtype is torch.float32 and wt.is_contiguous()
-         and wt.shape[0] == t, "moe_combine: x [T, H], yrows [T * top, H], pair_row, wt")
+         and pair_row.dtype is torch.int32 and pair_row.numel() >= t * top and top > 0
+         and (wt is None or (wt.dtype is torch.float32 and wt.is_contiguous() and wt.shape[0] == t)), "moe_combine: x [T, H], yrows [T * top, H], pair_row, wt")
     _chk(shared_out is None or (shared_out.dtype is torch.float32 and _rows_ok(shared_out) and shared_out.shape == (t, h)
                                 and (gate is None or (gate.dtype is torch.float32 and gate.numel() == t))), "moe_combine: shared")
     _chk(identity_rows is None or (idx is not None and idx.dtype is torch.int32 and idx.is_contiguous() and idx.shape == (t, top)
                                    and identity_rows.dtype in _DT and _rows_ok(identity_rows) and identity_rows.shape == (t, h)
                                    and experts >= 0), "moe_combine: identity experts")
     if t:
-        _run("moe", "li_moe_combine", x.data_ptr(), x.stride(0), yrows.data_ptr(), yrows.stride(0), pair_row.data_ptr(), wt.data_ptr(),
+        _run("moe", "li_moe_combine", x.data_ptr(), x.stride(0), yrows.data_ptr(), yrows.stride(0), pair_row.data_ptr(), 0 if wt is None else wt.data_ptr(),
              0 if gate is None else gate.data_ptr(), 0 if shared_out is None else shared_out.data_ptr(),
              0 if shared_out is None else shared_out.stride(0), t, h, top,
              0 if identity_rows is None else idx.data_ptr(), int(experts), 0 if identity_rows is None else identity_rows.data_ptr(),
-             _DT[identity_rows.dtype] if identity_rows is not None else 0, 0 if identity_rows is None else identity_rows.stride(0))
+             _DT[identity_rows.dtype] if identity_rows is not None else 0, 0 if identity_rows is None else identity_rows.stride(0),
+             float(factor), float(alpha), 0 if gamma is None else gamma.data_ptr(), 0 if beta is None else beta.data_ptr(),
+             0 if xn is None else xn.data_ptr(), 0 if xn is None else _DT[xn.dtype])

@@ -95,11 +95,34 @@ class PagedNeed:
     """What a mixer keeps per token in pages: any number of named tensors of any shapes;
     `window` > 0 keeps only the last `window` positions visible (older pages are given
     back); with `keep_first` > 0 the first so many positions of a request stay visible
-    beside the window, and their pages stay.  Entries of the execution order with equal
+    beside the window, and their pages stay; `chunk` > 0: a query sees only its own run of `chunk`
+    positions, counted from the request's start (older pages are given back).  Entries of the execution order with equal
     needs share a page group: one page id and one block table per request serve all of them."""
     tensors: Tuple[PagedTensor, ...]
     window: int = 0
     keep_first: int = 0
+    chunk: int = 0
+
+    @property
+    def reach(self) -> int:
+        """The most positions, its own included, that a query sees beside the kept first ones (0: all before it)."""
+        bounds = [n for n in (self.window, self.chunk) if n > 0]
+        return min(bounds) if bounds else 0
+
+    def covering(self, other: "PagedNeed") -> "PagedNeed":
+        """The need whose pages stay as long as either of the two wants them: what an owner keeps whose tensors
+        another entry of the execution order reads with a visibility of its own."""
+        if self.tensors != other.tensors:
+            raise ValueError(f"cache: an entry that keeps {self.tensors!r} is read by one that asks for {other.tensors!r}")
+        if self == other:
+            return self
+        if not self.reach or not other.reach:
+            return PagedNeed(self.tensors)
+        keep = max(self.keep_first, other.keep_first)
+        if not keep and not self.window and not other.window and max(self.chunk, other.chunk) % min(self.chunk, other.chunk) == 0:
+            return PagedNeed(self.tensors, chunk=max(self.chunk, other.chunk))       # (runs of the one are made of whole runs of the other)
+        # a key that is seen lies fewer than `reach` positions back
+        return PagedNeed(self.tensors, max(self.reach, other.reach), keep)
 
     def bytes_per_token(self, default_dtype: torch.dtype) -> int:
         total = 0
@@ -210,6 +233,14 @@ class ScaledRows:
     scale: Any
 
 
+@dataclass(frozen=True)
+class TanhScaling:
+    """A norm without statistics, y = tanh(alpha * x) * weight + bias: whoever writes x can write y beside it."""
+    alpha: float
+    weight: torch.Tensor          # float32 [size]
+    bias: torch.Tensor            # float32 [size]
+
+
 class Norm(Part):
     category = "norm"
 
@@ -219,6 +250,11 @@ class Norm(Part):
     def as_scaling(self) -> Optional[RmsScaling]:
         """How the products on the two sides of this norm can share it between them
         (an RmsScaling), or None: then the norm is always a pass of its own."""
+        return None
+
+    def as_tanh(self) -> Optional[TanhScaling]:
+        """The norm as an elementwise function of the sum that it reads (a TanhScaling), which the kernel that writes
+        the sum can leave beside it; None where it needs a row's statistics."""
         return None
 
 

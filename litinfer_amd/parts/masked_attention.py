@@ -13,7 +13,9 @@ gate a head (`head_gate`): head h's output is multiplied by sigmoid(Wg xn)_h bef
 column (`column_gate`: the heads side by side times sigmoid(Wg xn), element by element); `qk_norm` "heads" norms every
 query and key head by itself, with one weight vector of the head size for all query heads and one for all key heads;
 `keys_are_values`: there is no Wv, a token's value is its key as projected (before norm and rotation); `slopes`: the
-scores lose slopes[h] times the distance between query and key (and there may be no position part); the position part says how
+scores lose slopes[h] times the distance between query and key (and there may be no position part); `chunk`: position p sees
+the keys j <= p of its own run of `chunk` positions, counted from the request's start; `shared_keys`: the mixer has no Wk and
+Wv of its own and reads what another entry of the execution order keeps (keys after their rotation); the position part says how
 it pairs columns (`layout`: neighbouring ones, or column i with column i + rotary_dim/2).
 
 `LatentAttention`: keys and values are expanded from one latent vector c per token, c = the RMS
@@ -27,7 +29,7 @@ rank + rot_dim key columns whose first `rank` are also the value, with a per-hea
 Options: the queries may go through a latent of their own (`q_rank` > 0: c_q = RMS norm of Wdq xn with weights
 `q_down_norm`, q = Wuq c_q); every head's output may be multiplied by a sigmoid gate of the mixer's input
 (`head_gate`: sigmoid(Wg xn)_h, one row of Wg a head) or element by element (`column_gate`: the heads side by side
-times sigmoid(Wg xn)); with `rot_dim` 0 there is no rotated part and no position part; the position part says how it pairs columns (`layout`:
+times sigmoid(Wg xn)); a SINK a head (`sink`), as above; with `rot_dim` 0 there is no rotated part and no position part; the position part says how it pairs columns (`layout`:
 neighbouring ones, or column i with column i + rot_dim/2).
 """
 from __future__ import annotations
@@ -52,6 +54,8 @@ class MaskedAttention(Mixer):
         self.dv = int(a.get("value_dim") or self.dk)
         self.window = int(a.get("window") or 0)
         self.keep_first = int(a.get("keep_first") or 0) if self.window else 0
+        self.chunk = int(a.get("chunk") or 0)
+        self.shared_keys = bool(a.get("shared_keys", False))
         self.softcap = float(a.get("softcap") or 0.0)
         self.scale = float(a["scale"]) if a.get("scale") is not None else self.dk ** -0.5
         self.qk_norm = bool(a.get("qk_norm", False))
@@ -67,6 +71,8 @@ class MaskedAttention(Mixer):
         self.gate_cols = -(-self.n_gate // 4) * 4
         if self.nh <= 0 or self.nkv <= 0 or self.nh % self.nkv:
             raise ValueError(f"attention: {self.nh} heads are not a multiple of {self.nkv} kv heads")
+        if self.chunk < 0 or (self.chunk and self.window) or (self.shared_keys and (self.qk_norm or self.keys_are_values)):
+            raise ValueError("attention: chunks go without a window, shared keys without norms of their own")
         if self.softcap < 0 or self.window < 0 or self.keep_first < 0:
             raise ValueError("attention: the cap, the window and the kept first positions must not be negative")
         if self.head_gate and self.column_gate:
@@ -81,7 +87,9 @@ class MaskedAttention(Mixer):
         self.names = {"q": "q", "k": "k", "v": "v", "o": "o", "q_norm": "q.norm", "k_norm": "k.norm", "bias_suffix": ".b",
                       "sink": "sink", "gate": "g", **(a.get("names") or {})}
         self.n_q, self.n_k, self.n_v = self.nh * self.dk, self.nkv * self.dk, 0 if self.keys_are_values else self.nkv * self.dv
-        self.projected = (("q", self.n_q), ("k", self.n_k)) + (() if self.keys_are_values else (("v", self.n_v),))
+        if self.shared_keys:
+            self.n_k = self.n_v = 0
+        self.projected = (("q", self.n_q),) if self.shared_keys else (("q", self.n_q), ("k", self.n_k)) + (() if self.keys_are_values else (("v", self.n_v),))
         self.qkv = self.out = self.wq = self.wk = self.sink = self.slopes_dev = None
 
     @property
@@ -90,7 +98,7 @@ class MaskedAttention(Mixer):
 
     def cache_need(self):
         return PagedNeed((PagedTensor("k", (self.nkv, self.dk)), PagedTensor("v", (self.nkv, self.dv))),
-                         self.window, self.keep_first)
+                         self.window, self.keep_first, self.chunk)
 
     def batch_needs(self):
         # the kernels take single-token segments and the others (tiles of queries) apart
@@ -134,6 +142,8 @@ class MaskedAttention(Mixer):
             self.wq, self.wk = self.rt.vector(get(p + n["q_norm"])), self.rt.vector(get(p + n["k_norm"]))
 
     def forward(self, xn, residual, ctx, cache):
+        if self.shared_keys and cache.owned:
+            raise ValueError("attention: a mixer without keys of its own reads another entry's cache")
         t = xn.shape[0]
         n_qkv = self.n_q + self.n_k + self.n_v
         qkv = ctx.ws.buffer("attn.qkv32", (t, n_qkv + self.gate_cols), torch.float32)
@@ -157,7 +167,7 @@ class MaskedAttention(Mixer):
                              self.nh, self.nkv, self.dk, self.dv, cache.page_size, self.window, self.keep_first,
                              self.softcap, self.scale, ws=ctx.ws, sink=self.sink,
                              head_gate=gate if self.head_gate else None, column_gate=gate if self.column_gate else None,
-                             slopes=self.slopes_dev)
+                             slopes=self.slopes_dev, chunk=self.chunk)
         residual.add_linear(self.out, attn)
 
 
@@ -173,6 +183,7 @@ class LatentAttention(Mixer):
         self.dv = int(a.get("value_dim") or self.dn)
         self.rank = int(a["kv_rank"])
         self.q_rank = int(a.get("q_rank") or 0)      # 0: the queries are one product of the input
+        self.has_sink = bool(a.get("sink", False))
         self.head_gate = bool(a.get("head_gate", False))
         self.column_gate = bool(a.get("column_gate", False))
         self.n_gate = self.nh * self.dv if self.column_gate else self.nh if self.head_gate else 0
@@ -192,9 +203,9 @@ class LatentAttention(Mixer):
             raise ValueError("latent attention: the position encoding must rotate the whole rotated part")
         self.half_split = getattr(self.position, "layout", "pairs") == "half"
         self.names = {"q": "q", "q_down": "dq", "q_down_norm": "dq.norm", "q_up": "uq", "down": "dkv", "down_norm": "dkv.norm",
-                      "up_k": "uk", "up_v": "uv", "gate": "g", "o": "o", **(a.get("names") or {})}
+                      "up_k": "uk", "up_v": "uv", "gate": "g", "o": "o", "sink": "sink", **(a.get("names") or {})}
         self.n_q = self.nh * (self.dn + self.dr)
-        self.q_down = self.q_up = self.out = self.wc = self.wq = self.to_latent = self.from_latent = None
+        self.q_down = self.q_up = self.out = self.wc = self.wq = self.to_latent = self.from_latent = self.sink = None
 
     @property
     def graph_safe(self):
@@ -223,10 +234,14 @@ class LatentAttention(Mixer):
             e[p + n["q"]] = ParamSpec((self.n_q, self.hidden))
         if self.n_gate:
             e[p + n["gate"]] = ParamSpec((self.n_gate, self.hidden))
+        if self.has_sink:
+            e[p + n["sink"]] = ParamSpec((self.nh,), init="normal")
         return e
 
     def load_params(self, get):
         p, n = self.prefix, self.names
+        if self.has_sink:
+            self.sink = self.rt.vector(get(p + n["sink"]))
         # ONE product of the mixer's input: [queries, or their latent | latent and shared key part | gates]
         first = [get(p + n["q_down"] if self.q_rank else p + n["q"]), get(p + n["down"])]
         if self.n_gate:
@@ -273,7 +288,7 @@ class LatentAttention(Mixer):
         summed = ctx.ws.buffer("latent.summed", (t, nh * rank), self.rt.dtype)
         ops.masked_attention(qfull, nh * (rank + dr), rank + dr, summed, rows, rows, ctx.attention_meta(cache.group),
                              nh, 1, rank + dr, rank, cache.page_size, self.window, self.keep_first, self.softcap, self.scale,
-                             ws=ctx.ws)
+                             ws=ctx.ws, sink=self.sink)
         heads = ctx.ws.buffer("attn.out", (t, nh * self.dv), self.rt.dtype)
         gate = qd[:, n_first + rank + dr:n_first + rank + dr + self.n_gate] if self.n_gate else None
         ops.headwise_linear(summed, nh * rank, rank, self.from_latent, heads, nh * self.dv, self.dv, t, gate=gate,

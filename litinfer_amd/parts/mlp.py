@@ -2,8 +2,8 @@
 gate = xn Wg^T, up = xn Wu^T, no biases (src/llaisys/models/qwen2.cpp:744-759,
 src/ops/swiglu/op.cpp:19-22).  Gate and up are one product with the packed
 matrix [Wg; Wu]; the result is added to the residual stream.  With `activation` = "gelu_tanh" the gate passes the
-tanh form of GELU instead: y = (up * gelu_tanh(gate)) Wd^T; the tensors' names behind the prefix are parameters
-(`names`)."""
+tanh form of GELU instead: y = (up * gelu_tanh(gate)) Wd^T; with "clamped" and `limit` y = (g sigmoid(1.702 g) (u + 1)) Wd^T,
+g = min(gate, limit), u = clamp(up, -limit, limit); the tensors' names behind the prefix are parameters (`names`)."""
 from __future__ import annotations
 
 import torch
@@ -22,8 +22,12 @@ class SwiGLUMLP(FeedForward):
         self.hidden = int(spec.args["hidden_size"])
         self.inter = int(spec.args["intermediate_size"])
         self.activation = str(spec.args.get("activation") or "silu")
-        if self.activation not in ("silu", "gelu_tanh"):
-            raise ValueError(f"gated feed-forward: activation {self.activation!r} (silu or gelu_tanh)")
+        self.limit = float(spec.args.get("limit") or 0.0)
+        if self.activation not in ("silu", "gelu_tanh", "clamped"):
+            raise ValueError(f"gated feed-forward: activation {self.activation!r} (silu, gelu_tanh or clamped)")
+        if (self.activation == "clamped") != (self.limit > 0):
+            raise ValueError("gated feed-forward: the clamped activation takes a positive limit, the others none")
+        self.fused = self.activation in ("silu", "clamped")         # the activations that the products have as an epilogue
         self.names = {"gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight", **(spec.args.get("names") or {})}
         self.gate_up = None
         self.down = None
@@ -47,18 +51,18 @@ class SwiGLUMLP(FeedForward):
     def forward_prenorm(self, norm, residual, xn, ctx):
         # few rows (decoding): the product before the norm may have left its rows scaled by the
         # norm's weights; the gate/up product then applies the rows' factors with its activation
-        sc = residual.scaled_rows(norm) if self.activation == "silu" else None
+        sc = residual.scaled_rows(norm) if self.fused else None
         if sc is not None and self.gate_up.takes_swiglu(sc.rows):
             h = ctx.ws.buffer("mlp.h", (sc.rows.shape[0], self.inter), self.rt.dtype)
-            self.gate_up(sc.rows, h, ws=ctx.ws, swiglu=True, row_scale=sc.scale)
+            self.gate_up(sc.rows, h, ws=ctx.ws, swiglu=True, row_scale=sc.scale, limit=self.limit)
             return residual.add_linear(self.down, h)
         self.forward(residual.normed(norm, xn), residual, ctx)
 
     def forward(self, xn, residual, ctx):
         t = xn.shape[0]
         h = ctx.ws.buffer("mlp.h", (t, self.inter), self.rt.dtype)
-        if self.activation == "silu" and self.gate_up.takes_swiglu(xn):
-            self.gate_up(xn, h, ws=ctx.ws, swiglu=True)        # few rows: the activation is the epilogue
+        if self.fused and self.gate_up.takes_swiglu(xn):
+            self.gate_up(xn, h, ws=ctx.ws, swiglu=True, limit=self.limit)        # few rows: the activation is the epilogue
         else:
             if self.activation == "silu":
                 gu = ctx.ws.buffer("mlp.gate_up", (t, 2 * self.inter), self.rt.dtype)
@@ -67,7 +71,7 @@ class SwiGLUMLP(FeedForward):
             else:                                              # the product is left in float32 and the activation rounds once
                 gu = ctx.ws.buffer("mlp.gate_up32", (t, 2 * self.inter), torch.float32)
                 self.gate_up(xn, gu, ws=ctx.ws)
-                ops.gated_act(gu, h, self.activation)
+                ops.gated_act(gu, h, self.activation, self.limit)
         residual.add_linear(self.down, h)
 
 

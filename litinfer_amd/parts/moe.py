@@ -12,8 +12,10 @@ divided by their sum.  `scores` = "softmax": the same with an expert's score = t
 more than there are experts; the last `identity` of them are identity experts, which have no tensors and whose output
 is the feed-forward's input itself (times the weight); groups are formed over all router outputs.
 An expert (`activation`): "relu2" is Wdown max(Wup xn, 0)^2; "swiglu" is Wdown (silu(Wgate xn) * (Wup xn));
-"clamped_swiglu" is Wdown (g sigmoid(1.702 g) (u + 1)) with g = min(Wgate xn, limit), u = clamp(Wup xn, -limit, limit).  No
-biases.  The shared expert (relu2 only) has a width of its own; its output is multiplied by sigmoid(wg . xn), one
+"clamped_swiglu" is Wdown (g sigmoid(1.702 g) (u + 1)) with g = min(Wgate xn, limit), u = clamp(Wup xn, -limit, limit);
+"gelu" is Wdown gelu(Wup xn) with the error function.  No biases.  `weigh_input`: a choice's weight multiplies the
+expert's input instead of its output (the first product is linear, so its float32 sums take the factor).  The shared
+expert (relu2 and gelu) has a width of its own; its output is multiplied by sigmoid(wg . xn), one
 number a token, where a gate row is given.  The output is the weighted sum, added to the stream in float32.
 
 On the device: one kernel routes (logits, choice, weights and the shared gate), one sorts the step's (token,
@@ -32,6 +34,10 @@ from ..kernels import ops
 from ..weights.loader import ParamSpec
 from .base import BatchNeeds, FeedForward, register_part
 from .linear import Linear
+
+
+ACTIVATIONS = {"relu2": 1, "swiglu": 2, "clamped_swiglu": 3, "gelu": 4}        # the kernels' numbers
+SHARED_ACTIVATIONS = {"relu2": ops.relu_squared, "gelu": ops.gelu_erf}
 
 
 class RoutedMLP(FeedForward):
@@ -62,7 +68,10 @@ class RoutedMLP(FeedForward):
             raise ValueError(f"routed feed-forward: {self.top} of {self.experts} experts of width {self.inter}")
         if self.top > 64:
             raise ValueError("routed feed-forward: the router kernel picks at most 64 experts a token")
-        if (self.activation not in ("relu2", "swiglu", "clamped_swiglu") or self.scores not in ("softmax_chosen", "sigmoid", "softmax")
+        self.weigh_input = bool(a.get("weigh_input", False))
+        if self.weigh_input and self.identity:
+            raise ValueError("routed feed-forward: identity experts take their weight on the output")
+        if (self.activation not in ACTIVATIONS or self.scores not in ("softmax_chosen", "sigmoid", "softmax")
                 or self.group_score not in ("top2_sum", "max")):
             raise ValueError(f"routed feed-forward: activation {self.activation!r}, scores {self.scores!r}, group score {self.group_score!r}")
         if self.activation == "clamped_swiglu" and self.limit <= 0:
@@ -75,8 +84,8 @@ class RoutedMLP(FeedForward):
         if self.top > self.keep_groups * (self.n_router // self.groups):
             raise ValueError(f"routed feed-forward: {self.top} choices, but the kept groups hold "
                              f"{self.keep_groups * (self.n_router // self.groups)} experts")
-        if self.shared_inter and self.activation != "relu2":
-            raise ValueError("routed feed-forward: the shared expert is a squared-ReLU one")
+        if self.shared_inter and self.activation not in SHARED_ACTIVATIONS:
+            raise ValueError(f"routed feed-forward: no shared expert with activation {self.activation!r}")
         self.names = {"expert": "e{}.", "up": "up", "gate": "gate", "down": "down", "router": "router", "router_bias": "router.b",
                       "correction": "correction", "shared": "shared.", "shared_gate": "sg", **(a.get("names") or {})}
         self.gated = self.activation in ("swiglu", "clamped_swiglu")
@@ -145,10 +154,11 @@ class RoutedMLP(FeedForward):
         plan = ws.buffer("moe.plan", (4 + 4 * max_tiles,), torch.int32)
         row_token = ws.buffer("moe.row_token", (pairs,), torch.int32)
         pair_row = ws.buffer("moe.pair_row", (pairs,), torch.int32)
-        ops.moe_plan(idx, self.experts, plan, row_token, pair_row, rows_a_tile)
+        row_wt = ws.buffer("moe.row_wt", (pairs,), torch.float32) if self.weigh_input else None
+        ops.moe_plan(idx, self.experts, plan, row_token, pair_row, rows_a_tile, wt=wt if self.weigh_input else None, row_wt=row_wt)
         h = ws.buffer("moe.h", (pairs, self.inter), self.rt.dtype)
-        ops.moe_linear(xn, row_token, self.w_up, plan, max_tiles, h, pairs, act={"relu2": 1, "swiglu": 2, "clamped_swiglu": 3}[self.activation],
-                       tile_rows=rows_a_tile, limit=self.limit)
+        ops.moe_linear(xn, row_token, self.w_up, plan, max_tiles, h, pairs, act=ACTIVATIONS[self.activation],
+                       tile_rows=rows_a_tile, limit=self.limit, row_wt=row_wt)
         yrows = ws.buffer("moe.y", (pairs, self.hidden), torch.float32)
         ops.moe_linear(h, None, self.w_down, plan, max_tiles, yrows, pairs, tile_rows=rows_a_tile)
         shared = None
@@ -156,12 +166,13 @@ class RoutedMLP(FeedForward):
             u = ws.buffer("mlp.up32", (t, self.shared_inter), torch.float32)
             self.shared_up(xn, u, ws=ws)
             hs = ws.buffer("mlp.h", (t, self.shared_inter), self.rt.dtype)
-            ops.relu_squared(u, hs)
+            SHARED_ACTIVATIONS[self.activation](u, hs)
             shared = ws.buffer("moe.shared", (t, self.hidden), torch.float32)
             self.shared_down(hs, shared, ws=ws)
         # (a pair whose choice is an identity expert has no row in the plan: the sum takes the token's input for it)
-        ops.moe_combine(residual.tensor(), yrows, pair_row, wt, gate, shared, idx=idx if self.identity else None,
-                        experts=self.experts, identity_rows=xn if self.identity else None)
+        residual.add_by(lambda x, factor, tanh_norm: ops.moe_combine(
+            x, yrows, pair_row, None if self.weigh_input else wt, gate, shared, idx=idx if self.identity else None,
+            experts=self.experts, identity_rows=xn if self.identity else None, top=top, factor=factor, tanh_norm=tanh_norm))
 
 
 class RoutedReluSquaredMLP(RoutedMLP):

@@ -7,9 +7,11 @@ zero and the weight is offset + stored: y = (offset + w) * x / sqrt(...); the su
 is made once, in float32, when the tensor is bound."""
 from __future__ import annotations
 
+import torch
+
 from ..kernels import ops
 from ..weights.loader import ParamSpec
-from .base import Norm, RmsScaling, register_part
+from .base import Norm, RmsScaling, TanhScaling, register_part
 
 
 class RMSNorm(Norm):
@@ -73,5 +75,36 @@ class LayerNorm(Norm):
         return out
 
 
+class DynamicTanhNorm(Norm):
+    """A norm that computes no mean or variance: y = tanh(alpha * x) * w + b, element by element in 32-bit, with a scalar
+    alpha (the tensor named like the weight with `alpha_suffix`, default ".alpha", added; stored without dimensions) and
+    a bias vector (`bias_suffix`, default ".b")."""
+    graph_safe = True
+
+    def __init__(self, spec, rt):
+        super().__init__(spec, rt)
+        self.size = int(spec.args["size"])
+        self.param = self.prefix + str(spec.args.get("param", "weight"))
+        self.alpha_param = self.param + str(spec.args.get("alpha_suffix", ".alpha"))
+        self.bias_param = self.param + str(spec.args.get("bias_suffix", ".b"))
+        self.alpha, self.weight, self.bias = 0.0, None, None
+
+    def expected_params(self):
+        return {self.param: ParamSpec((self.size,), init="one_plus_normal"), self.alpha_param: ParamSpec((), init="one_plus_normal"),
+                self.bias_param: ParamSpec((self.size,), init="normal")}
+
+    def load_params(self, get):
+        self.alpha = float(get(self.alpha_param).to(torch.float32).reshape(()).item())
+        self.weight, self.bias = self.rt.vector(get(self.param)), self.rt.vector(get(self.bias_param))
+
+    def forward(self, x, out):
+        ops.tanh_norm(x, self.alpha, self.weight, self.bias, out)
+        return out
+
+    def as_tanh(self):
+        return TanhScaling(self.alpha, self.weight, self.bias)
+
+
 register_part("norm", "rmsnorm", RMSNorm)
+register_part("norm", "dynamic_tanh", DynamicTanhNorm)
 register_part("norm", "layernorm", LayerNorm)

@@ -11,7 +11,10 @@ Whoever knows which norm reads the stream next says so in `next_norm`.  Then
 `add_linear` may, for the few rows of a decoding step, have its kernel leave the
 sum times that norm's weights and the rows' sums of squares beside the sum
 itself, and the part behind the norm finds them under `scaled_rows(norm)`: the
-norm costs no pass of its own.  Any other write to the stream forgets them.
+norm costs no pass of its own.  A norm that is an elementwise function of the sum
+(`Norm.as_tanh`) is left beside the sum whole.  Any other write to the stream forgets them.
+
+A stream may have a `factor`: everything that a sublayer adds is multiplied by it.
 """
 from __future__ import annotations
 
@@ -26,9 +29,10 @@ _PLAIN = object()         # in place of a norm: "the sum itself, in the parts' d
 
 
 class ResidualStream:
-    def __init__(self, x: torch.Tensor, ws):
+    def __init__(self, x: torch.Tensor, ws, factor: float = 1.0):
         self.x = x
         self.ws = ws
+        self.factor = float(factor)           # what a sublayer's output is multiplied by when it joins
         self.next_norm = None                 # the norm through which the stream is read next, if known
         self.next_plain = False               # the next reader takes the sum itself, without a norm (known like next_norm)
         self._scaled = None                   # (norm, ScaledRows) left by the last add_linear
@@ -40,7 +44,7 @@ class ResidualStream:
         return self.x.shape
 
     def tensor(self) -> torch.Tensor:
-        """The sum so far (whoever takes it may write to it)."""
+        """The sum so far (whoever takes it may write to it, and applies the stream's factor to what it adds)."""
         self._scaled = self._normed = None
         return self.x
 
@@ -54,20 +58,38 @@ class ResidualStream:
         ops.gather_rows(self.x, rows, out)
 
     def add_linear(self, linear, h: torch.Tensor) -> None:
-        """x += h W^T + b."""
+        """x += factor * (h W^T + b)."""
         norm, self._scaled, self._normed = self.next_norm, None, None
         scaling = norm.as_scaling() if norm is not None else None
         if scaling is not None and linear.takes_scaling(h, self.x):
             rows = self.ws.buffer("stream.scaled_rows", self.x.shape, h.dtype)
-            self._scaled = (norm, ScaledRows(rows, linear.add_with_scaling(h, self.x, scaling, rows, self.ws)))
+            self._scaled = (norm, ScaledRows(rows, linear.add_with_scaling(h, self.x, scaling, rows, self.ws, factor=self.factor)))
             return
         if scaling is not None:
             # some more rows: where the product is cut along K, the kernel that adds the parts up norms as well
             rows = self.ws.buffer("stream.normed_rows", self.x.shape, h.dtype)
-            if linear.add_then_norm(h, self.x, scaling, rows, self.ws):
+            if linear.add_then_norm(h, self.x, scaling, rows, self.ws, factor=self.factor):
                 self._normed = (norm, rows)
                 return
-        linear(h, self.x, accumulate=True, ws=self.ws)
+        tanh = norm.as_tanh() if norm is not None else None
+        if tanh is not None:
+            rows = self.ws.buffer("stream.normed_rows", self.x.shape, self.ws_dtype)
+            if linear.add_then_tanh(h, self.x, tanh, rows, self.ws, factor=self.factor):
+                self._normed = (norm, rows)
+                return
+        linear(h, self.x, accumulate=True, ws=self.ws, factor=self.factor)
+
+    def add_by(self, add) -> None:
+        """For a sublayer whose own kernel adds into the stream: `add(x, factor, tanh_norm)` adds factor * (its output) to
+        the float32 sum x and, where `tanh_norm` = (alpha, weight, bias, rows) is given, leaves that norm of the new sum in
+        rows (the norm through which the stream is read next, if it is an elementwise one)."""
+        norm, self._scaled, self._normed = self.next_norm, None, None
+        tanh = norm.as_tanh() if norm is not None else None
+        if tanh is None:
+            return add(self.x, self.factor, None)
+        rows = self.ws.buffer("stream.normed_rows", self.x.shape, self.ws_dtype)
+        add(self.x, self.factor, (tanh.alpha, tanh.weight, tanh.bias, rows))
+        self._normed = (norm, rows)
 
     def scaled_rows(self, norm) -> Optional[ScaledRows]:
         """What the last addition left for this norm's reader, if it did."""
@@ -104,6 +126,8 @@ class ResidualStream:
         scaling = norm.as_scaling()
         if scaling is None:
             raise NotImplementedError("add_normed: the norm behind a sublayer must be an RMS norm with weights")
+        if self.factor != 1.0:
+            raise NotImplementedError("add_normed: a factor on the sublayers' outputs goes with the pre-norm arrangements")
         y2, factors = None, (1.0, 1.0)
         if isinstance(y, BranchStream):
             y, y2, factors = y.outputs()
@@ -129,7 +153,6 @@ class BranchStream(ResidualStream):
     def __init__(self, y: torch.Tensor, ws):
         super().__init__(y, ws)
         self._fresh = True
-        self.factor = 1.0                    # what this output is multiplied by when it joins
         self.second = None                   # a second output beside this one (a BranchStream with a factor of its own)
 
     def fork(self, name: str) -> "BranchStream":
@@ -156,6 +179,9 @@ class BranchStream(ResidualStream):
     def add_linear(self, linear, h: torch.Tensor) -> None:
         linear(h, self.x, accumulate=not self._fresh, ws=self.ws)
         self._fresh = False
+
+    def add_by(self, add) -> None:
+        add(self.tensor(), 1.0, None)        # (a branch's factor is applied when it joins)
 
     def result(self) -> torch.Tensor:
         return self.tensor()

@@ -76,12 +76,12 @@ def rope_kv_store(qkv, nh, nkv, dh, rotary_dim, cos, sin, slot_map, k, v, page_s
     kv_store(qkv, nh, nkv, dh, slot_map, k, v, page_size)
 
 
-def linear(x, w, bias, out, accumulate=False, ws=None):
+def linear(x, w, bias, out, accumulate=False, ws=None, factor=1.0):
     y = x.float() @ w.float().T
     if bias is not None:
         y = y + bias
     if accumulate:
-        out += y
+        out += factor * y
     else:
         out.copy_(y.to(out.dtype))
 
@@ -153,8 +153,8 @@ def residual_norm_takes(m, n, k, w_dtype):
     return w_dtype is torch.bfloat16 and 0 < m <= 32 and k % 8 == 0 and residual_norm_parts(n) <= RESIDUAL_NORM_MAX_PARTS
 
 
-def linear_residual_norm(x, w, bias, out, gamma, xg, sq_parts):
-    linear(x, w, bias, out, True)
+def linear_residual_norm(x, w, bias, out, gamma, xg, sq_parts, factor=1.0):
+    linear(x, w, bias, out, True, factor=factor)
     xg.copy_((gamma * out).to(xg.dtype))
     per = 32 if out.shape[1] >= 8192 else 16
     parts = residual_norm_parts(out.shape[1])
@@ -164,7 +164,7 @@ def linear_residual_norm(x, w, bias, out, gamma, xg, sq_parts):
     return parts
 
 
-def linear_then_norm(x, w, bias, out, gamma, eps, xn, ws):
+def linear_then_norm(x, w, bias, out, gamma, eps, xn, ws, factor=1.0):
     return False                                         # the stand-ins cut no product along K
 
 
@@ -174,7 +174,8 @@ def _row_factors(row_scale, m, k):
     return (1.0 / torch.sqrt(sq / k + row_scale.eps))[:, None]
 
 
-def linear_swiglu(x, w, out, row_scale=None):
+def linear_swiglu(x, w, out, row_scale=None, limit=0.0):
+    assert limit == 0.0, "the stand-ins have the plain activation"
     if row_scale is None:
         return linear_skinny(x, w, None, out, False, swiglu=True)
     y = (x.float() @ w.float().T) * _row_factors(row_scale, x.shape[0], x.shape[1])
