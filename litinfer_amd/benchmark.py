@@ -859,9 +859,37 @@ def tovasun_beside_dimelix_config(size: str, layers: int, vocab: int = 32000) ->
             "loop": {"start": 1, "stop": 3, "times": 2} if layers >= 4 else None}
 
 
+BESORAX_SIZES = {         # lightning heads, their key and value size; queries' latent; experts, chosen, expert width, shared width: the
+    # chosen experts and the shared one together are as wide as the dense feed-forward
+    "1.5b": (12, 128, 768, 16, 2, 2240, 4480),
+    "7b": (28, 128, 1536, 16, 2, 4736, 9472),
+}
+
+
+def besorax_config(size: str, layers: int, vocab: int = 32000) -> Dict[str, object]:
+    """A Besorax model at the layer sizes of a Qwen2 family member: lightning attention, chunk-masked attention (every
+    second one reads the keys of the first) and latent attention in turn, routed feed-forwards and in the first layer a dense one."""
+    width, heads, kv, dim, ff, rank, rot, _ = DESIGN_SIZES[size]
+    lh, ldim, q_rank, ne, top, eff, sff = BESORAX_SIZES[size]
+    moe = {"kind": "moe", "expert": {"ff": eff}, "router": {"experts": ne, "top": top}, "shared": {"ff": sff}}
+    light = {"heads": lh, "dim": ldim, "vdim": ldim, "decay": [1.0 - 2.0 ** -(4 + i % 7) for i in range(lh)]}
+    attn = {"heads": heads, "kv_heads": kv, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": DESIGN_WINDOW},
+            "rot": {"base": 10000.0, "dims": dim // 2}}
+    latent = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": dim, "kv_rank": rank, "q_rank": q_rank,
+              "scale": (dim + rot) ** -0.5, "rot": {"base": 10000.0, "dims": rot}}
+    out = []
+    for i in range(layers):
+        kind, mixer = (("lightning", light), ("attention", attn), ("latent_attention", latent))[i % 3]
+        if i % 6 == 4:
+            mixer = {**mixer, "kv_from": i - 3}
+        out.append({"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": ff, "limit": 7.0} if i == 0 else moe})
+    return {"architecture": "Besorax", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "residual_mult": 0.4,
+            "embedding": {"scale": float(width) ** 0.5}, "layers": out}
+
+
 def compare_designs(a) -> Dict[str, object]:
     """Prefill and decode throughput of a second design (`--design`) beside Qwen2 or, where another model is closer
-    (Nusuvik, Kufolorn, Dimelix), beside that one, at the same width, heads, (active) feed-forward width,
+    (Nusuvik, Kufolorn, Dimelix, Besorax), beside that one, at the same width, heads, (active) feed-forward width,
     window and number of layer runs (random weights, random cache content)."""
     import numpy as np
     import torch
@@ -873,14 +901,15 @@ def compare_designs(a) -> Dict[str, object]:
     for size in sizes:
         layers = a.layers or 6
         design = getattr(a, "design", None) or "tovasun"
-        tcfg = {"sogenex": sogenex_config, "nusuvik": nusuvik_config, "kufolorn": kufolorn_config, "dimelix": dimelix_config}.get(design, tovasun_config)(size, layers)
+        tcfg = {"sogenex": sogenex_config, "nusuvik": nusuvik_config, "kufolorn": kufolorn_config, "dimelix": dimelix_config,
+                "besorax": besorax_config}.get(design, tovasun_config)(size, layers)
         runs = layers + (2 if tcfg.get("loop") else 0)
         width, heads, kv, dim, ff = DESIGN_SIZES[size][:5]
         if design == "nusuvik":
             beside, qcfg = "tovasun", tovasun_latent_config(size, layers)
         elif design == "dimelix":
             beside, qcfg = "tovasun", tovasun_beside_dimelix_config(size, layers)
-        elif design == "kufolorn":                   # its closest relative: recurrent layers, every third one attention, routed feed-forwards
+        elif design in ("kufolorn", "besorax"):      # its closest relative: recurrent layers, every third one attention, routed feed-forwards
             beside, qcfg = "sogenex", sogenex_config(size, layers)
         else:
             beside = "qwen2"
@@ -891,7 +920,7 @@ def compare_designs(a) -> Dict[str, object]:
             if a.only and name != a.only:
                 continue
             eng = Engine.from_random(cfg, seed=0, dtype=ENGINE_DTYPE[a.dtype], device=dev, page_size=PAGE,
-                                     num_pages=(64 * ((2 if design in ("nusuvik", "kufolorn", "dimelix") else 1) * DESIGN_WINDOW + 64) + 2 * PREFILL_TOKENS) // PAGE,
+                                     num_pages=(64 * ((2 if design in ("nusuvik", "kufolorn", "dimelix", "besorax") else 1) * DESIGN_WINDOW + 64) + 2 * PREFILL_TOKENS) // PAGE,
                                      max_seqs=65)
             for g in eng.cache.groups:
                 for data in g.data.values():
@@ -910,12 +939,14 @@ def compare_designs(a) -> Dict[str, object]:
                 raise RuntimeError(f"bench: non-finite logits after the prompt ({name})")
             r["prefill_tok_s"] = round(PREFILL_TOKENS / min(times[1:]), 1)
             r["prefill_ms"] = round(min(times[1:]) * 1e3, 3)
+            # the cache "holds" a context longer than the window (beside chunks: one whose last chunk is nearly full)
+            held = 2 * DESIGN_WINDOW - (a.steps + a.warmup if design == "besorax" else 0)
             for b in batches:
                 rids = [f"d{b}_{i}" for i in range(b)]
-                for rid in rids:                     # the cache "holds" a context longer than the window
+                for rid in rids:
                     eng.cache.admit(rid)
-                    eng.cache.reserve(rid, 2 * DESIGN_WINDOW)
-                    eng.cache.commit(rid, 2 * DESIGN_WINDOW)
+                    eng.cache.reserve(rid, held)
+                    eng.cache.commit(rid, held)
                 toks = rng.integers(0, vocab, b).tolist()
 
                 def one():
@@ -945,13 +976,14 @@ def compare_designs(a) -> Dict[str, object]:
     first = out[sizes[0]]
     title = design.capitalize()
     return {"metric": f"decode tok/s ({title} at the Qwen2-{sizes[0]} layer sizes, batch {a.batch}, "
-                      + ("no window)" if design in ("nusuvik", "kufolorn") else f"window {DESIGN_WINDOW} in every third layer)" if design == "dimelix" else f"window {DESIGN_WINDOW})"),
+                      + ("no window)" if design in ("nusuvik", "kufolorn") else f"window {DESIGN_WINDOW} in every third layer)" if design == "dimelix" else
+                         f"chunks of {DESIGN_WINDOW} in every third layer)" if design == "besorax" else f"window {DESIGN_WINDOW})"),
             "value": first[a.only or design][f"decode_b{a.batch}_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": a.steps,
             "warmup": a.warmup, "ms_per_step": first[a.only or design][f"decode_b{a.batch}_ms"], "higher_is_better": True,
             "scaling": "weak", "vs_baseline": None, "dtype": a.dtype,
             "data": "synthetic: seeded random token ids, random weights N(0, 0.02), random cache content",
             "config": {"model": f"{title} beside {beside.capitalize()} at equal layer sizes", "global_batch": a.batch,
-                       "seq_len": 2 * DESIGN_WINDOW, "prefill_tokens": PREFILL_TOKENS, "page_size": PAGE,
+                       "seq_len": held, "prefill_tokens": PREFILL_TOKENS, "page_size": PAGE,
                        "parallelism": "none (1 GPU)"},
             "designs": out}
 
@@ -967,8 +999,8 @@ def main(argv: Optional[List[str]] = None) -> int:
     ap.add_argument("--mode", default="headline", choices=["headline", "serving", "long", "sweep", "designs"])
     ap.add_argument("--shape", default=None, choices=sorted(SHAPES),
                     help="sweep: the member of the family whose layer sizes are taken (7b); designs: 1.5b or 7b (both)")
-    ap.add_argument("--design", default="tovasun", choices=["tovasun", "sogenex", "nusuvik", "kufolorn", "dimelix"],
-                    help="designs: the design that is set beside Qwen2 (Nusuvik: beside an all-latent Tovasun; Kufolorn: beside Sogenex; Dimelix: beside a Tovasun of the same layer order)")
+    ap.add_argument("--design", default="tovasun", choices=["tovasun", "sogenex", "nusuvik", "kufolorn", "dimelix", "besorax"],
+                    help="designs: the design that is set beside Qwen2 (Nusuvik: beside an all-latent Tovasun; Kufolorn and Besorax: beside Sogenex; Dimelix: beside a Tovasun of the same layer order)")
     ap.add_argument("--only", default=None, help="designs: run one of the two models only (its name)")
     ap.add_argument("--page-order-seed", type=int, default=0,
                     help="headline: the cache's pages are handed out in a shuffled order, as a pool that has served requests "

@@ -457,6 +457,276 @@ static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, lo
 #undef SSM_KERNEL
 }
 
+// ------------------------------------------------------------------------------- retention of long portions, as products
+// With the same decay a for every token of a head the recurrence S_t = a S_(t-1) + f k_t v_t^T, y_t = S_t^T q_t over a chunk
+// of n <= 64 tokens (numbered from 0) that begins with the state S is
+//     y_i = a^(i+1) q_i S + sum_(j<=i) a^(i-j) f (q_i . k_j) v_j,      S' = a^n S + sum_j a^(n-1-j) f k_j v_j^T,
+// three matrix products, on the float32 matrix cores (v_mfma_f32_32x32x2_f32: float32 operands, products and sums; lane l of
+// the row operand holds row l % 32 and k-value l / 32, of the column operand column l % 32 and k-value l / 32, of the result
+// column l % 32 and, in register r, row 8 (r / 4) + 4 (l / 32) + r % 4).  A decay is only ever raised to powers >= 0.
+//   retention_states_kernel: the second term of S' of every chunk;
+//   retention_carry_kernel: the state with which every chunk begins, chunk after chunk, and the request's state at the end;
+//   retention_outputs_kernel: the outputs.
+// Which k-value a step of the matrix cores takes is free as long as both operands agree: the scores K Q^T take the four
+// k-values 8 t + 4 (l / 32) .. + 3 of a 16-byte piece in four steps, and their result, keys as rows, is the row operand of
+// the product with V as it is (register r holds the key whose number the column operand then reads).
+#define RET_Q 64               // tokens of a chunk (SSM chunks of the same length are what the host numbers)
+typedef float ret_f32x16 __attribute__((ext_vector_type(16)));
+
+__device__ __forceinline__ float4 silu_if4(float4 v, int on) { return float4{silu_if(v.x, on), silu_if(v.y, on), silu_if(v.z, on), silu_if(v.w, on)}; }
+
+// WT: fragments of 32 rows (state values) and of 32 columns a wave; the four waves are two by two, a block takes 64 WT of both.
+template <int WT>
+__global__ __launch_bounds__(256) void retention_states_kernel(
+    const float* __restrict__ xbc, long xbc_stride, const int* __restrict__ q_start, const int* __restrict__ q_len,
+    const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, int heads, int vdim, int N,
+    const float* __restrict__ fixed_a, float step, int silu_in) {
+    constexpr int B = 64 * WT;
+    extern __shared__ __align__(16) float lds[];
+    float* sK = lds;                                   // [RET_Q][B]
+    float* sV = lds + RET_Q * B;                       // [RET_Q][B], times a^(n-1-j) f
+    const int bx = blockIdx.x, seg = chunk_seg[bx];
+    if (seg < 0) return;
+    const int first = chunk_idx[bx] * RET_Q, L = q_len[seg];
+    const int ntok = L - first < RET_Q ? L - first : RET_Q, t0 = q_start[seg] + first, head = blockIdx.y;
+    const int vb = (vdim + B - 1) / B, n0 = (blockIdx.z / vb) * B, p0 = (blockIdx.z % vb) * B;
+    const float a = fixed_a[head];
+    const int inner = heads * vdim;
+    const int rows = (ntok + 1) & ~1;                  // (whole pairs of tokens: the row behind an odd last one is zero)
+    for (int i = threadIdx.x; i < rows * (B / 4); i += 256) {
+        const int j = i / (B / 4), c = 4 * (i % (B / 4));
+        const float* row = xbc + (size_t)(t0 + j) * xbc_stride;
+        float4 k = float4{0.f, 0.f, 0.f, 0.f}, v = k;
+        if (j < ntok && n0 + c < N) k = silu_if4(*reinterpret_cast<const float4*>(row + inner + (size_t)head * N + n0 + c), silu_in);
+        if (j < ntok && p0 + c < vdim) {
+            v = silu_if4(*reinterpret_cast<const float4*>(row + (size_t)head * vdim + p0 + c), silu_in);
+            const float f = powf(a, (float)(ntok - 1 - j)) * step;
+            v = float4{v.x * f, v.y * f, v.z * f, v.w * f};
+        }
+        *reinterpret_cast<float4*>(sK + j * B + c) = k;
+        *reinterpret_cast<float4*>(sV + j * B + c) = v;
+    }
+    __syncthreads();
+    const int w = threadIdx.x >> 6, lane = threadIdx.x & 63, ql = lane & 31, h = lane >> 5;
+    const int wn = (w >> 1) * 32 * WT, wp = (w & 1) * 32 * WT;
+    if (n0 + wn >= N || p0 + wp >= vdim) return;
+    ret_f32x16 acc[WT][WT];
+#pragma unroll
+    for (int x = 0; x < WT; ++x)
+#pragma unroll
+        for (int y = 0; y < WT; ++y)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) acc[x][y][r] = 0.f;
+#pragma unroll 4
+    for (int j = 0; j < rows; j += 2) {
+        float kf[WT], vf[WT];
+#pragma unroll
+        for (int x = 0; x < WT; ++x) { kf[x] = sK[(j + h) * B + wn + 32 * x + ql]; vf[x] = sV[(j + h) * B + wp + 32 * x + ql]; }
+#pragma unroll
+        for (int x = 0; x < WT; ++x)
+#pragma unroll
+            for (int y = 0; y < WT; ++y) acc[x][y] = __builtin_amdgcn_mfma_f32_32x32x2f32(kf[x], vf[y], acc[x][y], 0, 0, 0);
+    }
+    float* dst = carry + ((size_t)bx * heads + head) * N * vdim;
+#pragma unroll
+    for (int x = 0; x < WT; ++x)
+#pragma unroll
+        for (int y = 0; y < WT; ++y)
+#pragma unroll
+            for (int r = 0; r < 16; ++r) {
+                const int n = n0 + wn + 32 * x + 8 * (r >> 2) + 4 * h + (r & 3), p = p0 + wp + 32 * y + ql;
+                if (n < N && p < vdim) dst[(size_t)n * vdim + p] = acc[x][y][r];
+            }
+}
+
+// carry[chunk]: in: what the chunk alone adds; out: the state with which it begins.  The next eight chunks' values are on
+// their way while a chunk is worked on.  NV4: a head's state in 16-byte pieces.
+#define RET_AHEAD 8
+__global__ __launch_bounds__(64) void retention_carry_kernel(float4* __restrict__ carry, float4* __restrict__ state,
+                                                             const int* __restrict__ slots, const int* __restrict__ q_len,
+                                                             const int* __restrict__ chunk_first, int heads, int NV4,
+                                                             const float* __restrict__ fixed_a) {
+    const int seg = blockIdx.x, head = blockIdx.y, e = blockIdx.z * 64 + threadIdx.x;
+    if (e >= NV4) return;
+    const int L = q_len[seg], nch = (L + RET_Q - 1) / RET_Q;
+    const float a = fixed_a[head], whole = powf(a, (float)RET_Q), tail = powf(a, (float)(L - (nch - 1) * RET_Q));
+    float4* at = carry + ((size_t)chunk_first[seg] * heads + head) * NV4 + e;
+    const size_t next = (size_t)heads * NV4;
+    float4* st = state + ((size_t)slots[seg] * heads + head) * NV4 + e;
+    float4 run = *st, own[RET_AHEAD];
+#pragma unroll
+    for (int u = 0; u < RET_AHEAD; ++u) own[u] = at[(size_t)(u < nch ? u : nch - 1) * next];
+    for (int c0 = 0; c0 < nch; c0 += RET_AHEAD) {
+        float4 ahead[RET_AHEAD];
+#pragma unroll
+        for (int u = 0; u < RET_AHEAD; ++u) {
+            const int c = c0 + RET_AHEAD + u;
+            ahead[u] = at[(size_t)(c < nch ? c : nch - 1) * next];      // (past the end: the last chunk's again, not used)
+        }
+#pragma unroll
+        for (int u = 0; u < RET_AHEAD; ++u) {
+            const int c = c0 + u;
+            if (c < nch) {
+                const float f = c + 1 < nch ? whole : tail;
+                at[(size_t)c * next] = run;
+                run = float4{fmaf(f, run.x, own[u].x), fmaf(f, run.y, own[u].y), fmaf(f, run.z, own[u].z), fmaf(f, run.w, own[u].w)};
+            }
+        }
+#pragma unroll
+        for (int u = 0; u < RET_AHEAD; ++u) own[u] = ahead[u];
+    }
+    *st = run;
+}
+
+// NQ: 8-value pieces of a query (N <= 8 NQ); PT: fragments of 32 columns a wave.  The four waves are two query tiles of 32 by two
+// column ranges; a query lies in registers (16-byte pieces 2 t + l / 32 of row l % 32), keys and values in LDS.
+template <int NQ, int PT>
+__global__ __launch_bounds__(256) void retention_outputs_kernel(
+    const float* __restrict__ xbc, long xbc_stride, const int* __restrict__ q_start, const int* __restrict__ q_len,
+    const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, const float* __restrict__ carry, float* __restrict__ y,
+    long y_stride, int heads, int vdim, int N, const float* __restrict__ fixed_a, float step, int silu_in) {
+    constexpr int NP = 8 * NQ, KS = NP + 4, VB = 64 * PT;
+    extern __shared__ __align__(16) float lds[];
+    float* sK = lds;                                   // [RET_Q][KS]: four floats of padding spread the 16-byte reads over the banks
+    float* sV = sK + RET_Q * KS;                       // [RET_Q][VB]
+    float* pw = sV + RET_Q * VB;                       // [RET_Q + 1]: the powers of the decay
+    const int bx = blockIdx.x, seg = chunk_seg[bx];
+    if (seg < 0) return;
+    const int first = chunk_idx[bx] * RET_Q, L = q_len[seg];
+    const int ntok = L - first < RET_Q ? L - first : RET_Q, t0 = q_start[seg] + first, head = blockIdx.y, p0 = blockIdx.z * VB;
+    const int inner = heads * vdim;
+    const int w = threadIdx.x >> 6, lane = threadIdx.x & 63, ql = lane & 31, h = lane >> 5;
+    const int it = w >> 1, pc = p0 + (w & 1) * 32 * PT, i = it * 32 + ql;
+    // the wave's queries, asked for before keys and values are staged
+    float4 q[NQ];
+    {
+        const float* row = xbc + (size_t)(t0 + (i < ntok ? i : ntok - 1)) * xbc_stride + inner + (size_t)(heads + head) * N;
+#pragma unroll
+        for (int t = 0; t < NQ; ++t) {
+            const int n = 8 * t + 4 * h;
+            q[t] = n < N ? *reinterpret_cast<const float4*>(row + n) : float4{0.f, 0.f, 0.f, 0.f};
+        }
+    }
+    if (threadIdx.x <= RET_Q) pw[threadIdx.x] = powf(fixed_a[head], (float)threadIdx.x);
+    for (int x = threadIdx.x; x < RET_Q * (NP / 4); x += 256) {
+        const int j = x / (NP / 4), c = 4 * (x % (NP / 4));
+        float4 k = float4{0.f, 0.f, 0.f, 0.f};
+        if (j < ntok && c < N) k = silu_if4(*reinterpret_cast<const float4*>(xbc + (size_t)(t0 + j) * xbc_stride + inner + (size_t)head * N + c), silu_in);
+        *reinterpret_cast<float4*>(sK + j * KS + c) = k;
+    }
+    for (int x = threadIdx.x; x < RET_Q * (VB / 4); x += 256) {
+        const int j = x / (VB / 4), c = 4 * (x % (VB / 4));
+        float4 v = float4{0.f, 0.f, 0.f, 0.f};
+        if (j < ntok && p0 + c < vdim) v = silu_if4(*reinterpret_cast<const float4*>(xbc + (size_t)(t0 + j) * xbc_stride + (size_t)head * vdim + p0 + c), silu_in);
+        *reinterpret_cast<float4*>(sV + j * VB + c) = v;
+    }
+#pragma unroll
+    for (int t = 0; t < NQ; ++t) q[t] = silu_if4(q[t], silu_in);        // (silu(0) = 0)
+    __syncthreads();
+    if (it * 32 >= ntok || pc >= vdim) return;
+    ret_f32x16 out[PT];
+#pragma unroll
+    for (int pt = 0; pt < PT; ++pt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) out[pt][r] = 0.f;
+    for (int jt = 0; jt <= it; ++jt) {
+        ret_f32x16 sc;                                 // keys as rows, the wave's queries as columns
+#pragma unroll
+        for (int r = 0; r < 16; ++r) sc[r] = 0.f;
+        const float* krow = sK + (jt * 32 + ql) * KS + 4 * h;
+#pragma unroll
+        for (int t = 0; t < NQ; ++t) {
+            const float4 k = *reinterpret_cast<const float4*>(krow + 8 * t);
+            sc = __builtin_amdgcn_mfma_f32_32x32x2f32(k.x, q[t].x, sc, 0, 0, 0);
+            sc = __builtin_amdgcn_mfma_f32_32x32x2f32(k.y, q[t].y, sc, 0, 0, 0);
+            sc = __builtin_amdgcn_mfma_f32_32x32x2f32(k.z, q[t].z, sc, 0, 0, 0);
+            sc = __builtin_amdgcn_mfma_f32_32x32x2f32(k.w, q[t].w, sc, 0, 0, 0);
+        }
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            const int d = i - (jt * 32 + 8 * (r >> 2) + 4 * h + (r & 3));
+            sc[r] = d >= 0 ? sc[r] * (pw[d >= 0 ? d : 0] * step) : 0.f;
+        }
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            const float* vrow = sV + (jt * 32 + 8 * (r >> 2) + 4 * h + (r & 3)) * VB + (pc - p0) + ql;
+#pragma unroll
+            for (int pt = 0; pt < PT; ++pt) out[pt] = __builtin_amdgcn_mfma_f32_32x32x2f32(sc[r], vrow[32 * pt], out[pt], 0, 0, 0);
+        }
+    }
+    // what the state at the chunk's beginning adds
+    const float* S = carry + ((size_t)bx * heads + head) * N * vdim;
+    const float f = pw[i + 1];
+    int col[PT];
+#pragma unroll
+    for (int pt = 0; pt < PT; ++pt) col[pt] = pc + 32 * pt + ql < vdim ? pc + 32 * pt + ql : vdim - 1;     // (a column past the last is not written)
+#pragma unroll
+    for (int t = 0; t < NQ; ++t) {
+        const float qs[4] = {q[t].x * f, q[t].y * f, q[t].z * f, q[t].w * f};
+        float sv[4][PT];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int n = 8 * t + 4 * h + e;
+            const float* row = S + (size_t)(n < N ? n : N - 1) * vdim;          // (a value past the last meets a zero of q)
+#pragma unroll
+            for (int pt = 0; pt < PT; ++pt) sv[e][pt] = row[col[pt]];
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+            for (int pt = 0; pt < PT; ++pt) out[pt] = __builtin_amdgcn_mfma_f32_32x32x2f32(qs[e], sv[e][pt], out[pt], 0, 0, 0);
+    }
+#pragma unroll
+    for (int pt = 0; pt < PT; ++pt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+            const int row = it * 32 + 8 * (r >> 2) + 4 * h + (r & 3), p = pc + 32 * pt + ql;
+            if (row < ntok && p < vdim) y[(size_t)(t0 + row) * y_stride + (size_t)head * vdim + p] = out[pt][r];
+        }
+}
+
+template <int NQ, int PT>
+static int retention_outputs_launch(const dim3& grid, const float* xbc, long xbc_stride, const int* q_start, const int* q_len,
+                                    const int* chunk_seg, const int* chunk_idx, const float* carry, float* y, long y_stride,
+                                    int heads, int vdim, int N, const float* fixed_a, float step, int silu_in, hipStream_t stream) {
+    constexpr int bytes = (RET_Q * (8 * NQ + 4) + RET_Q * 64 * PT + RET_Q + 4) * 4;
+    static bool configured = false;
+    if (!configured) {
+        if (hipFuncSetAttribute((const void*)retention_outputs_kernel<NQ, PT>, hipFuncAttributeMaxDynamicSharedMemorySize, bytes) != hipSuccess)
+            return LI_ERR_LAUNCH;
+        configured = true;
+    }
+    retention_outputs_kernel<NQ, PT><<<grid, 256, bytes, stream>>>(xbc, xbc_stride, q_start, q_len, chunk_seg, chunk_idx, carry, y, y_stride,
+                                                                   heads, vdim, N, fixed_a, step, silu_in);
+    return li_launch_status();
+}
+
+// The chunked form of a retention (every head with keys of its own); operands in 16-byte pieces, N and vdim multiples of four.
+static int retention_launch(const float* xbc, long xbc_stride, float* state, const int* slots, const int* q_start, const int* q_len,
+                            int* chunk_tab, float* carry, float* y, long y_stride, int heads, int vdim, int N, int segs, int max_chunks,
+                            const float* fixed_a, float step, int silu_in, hipStream_t stream) {
+    int* chunk_seg = chunk_tab;
+    int* chunk_idx = chunk_tab + max_chunks;
+    int* chunk_first = chunk_tab + 2 * max_chunks;
+    ssm_chunk_index_kernel<<<1, 256, 0, stream>>>(q_len, segs, RET_Q, max_chunks, chunk_seg, chunk_idx, chunk_first);
+    const int wt = (N > 64 || vdim > 64) ? 2 : 1, b = 64 * wt;
+    const dim3 gs(max_chunks, heads, ((N + b - 1) / b) * ((vdim + b - 1) / b));
+    if (wt == 2) retention_states_kernel<2><<<gs, 256, 2 * RET_Q * 128 * 4, stream>>>(xbc, xbc_stride, q_start, q_len, chunk_seg, chunk_idx, carry, heads, vdim, N, fixed_a, step, silu_in);
+    else retention_states_kernel<1><<<gs, 256, 2 * RET_Q * 64 * 4, stream>>>(xbc, xbc_stride, q_start, q_len, chunk_seg, chunk_idx, carry, heads, vdim, N, fixed_a, step, silu_in);
+    const int NV4 = N * vdim / 4;
+    retention_carry_kernel<<<dim3(segs, heads, (NV4 + 63) / 64), 64, 0, stream>>>((float4*)carry, (float4*)state, slots, q_len, chunk_first, heads, NV4, fixed_a);
+    const int pt = vdim > 64 ? 2 : 1;
+    const dim3 go(max_chunks, heads, (vdim + 64 * pt - 1) / (64 * pt));
+#define RET_GO(NQ_)                                                                                                                  \
+    return pt == 2 ? retention_outputs_launch<NQ_, 2>(go, xbc, xbc_stride, q_start, q_len, chunk_seg, chunk_idx, carry, y, y_stride, heads, vdim, N, fixed_a, step, silu_in, stream) \
+                   : retention_outputs_launch<NQ_, 1>(go, xbc, xbc_stride, q_start, q_len, chunk_seg, chunk_idx, carry, y, y_stride, heads, vdim, N, fixed_a, step, silu_in, stream)
+    if (N <= 32) RET_GO(4);
+    if (N <= 64) RET_GO(8);
+    if (N <= 128) RET_GO(16);
+    RET_GO(32);
+#undef RET_GO
+}
+
 // The four-columns-a-lane layout for a state of N values a column and heads of vdim columns (a multiple of 4): lanes
 // a quad of columns (2 to 16) and values a lane and column (4 to 32); 0 if it has none.
 static int ssm_quad_layout(int N, int vdim, int* slices, int* per_lane) {
@@ -523,8 +793,13 @@ extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_ra
         decay = carry + (size_t)max_chunks * heads * N * vdim;
     }
     const bool aligned = ((uintptr_t)state | (uintptr_t)y | (uintptr_t)carry) % 16 == 0 && y_stride % 4 == 0;
+    if (chunked && fixed_a && G == heads && !Dw && aligned && Q == RET_Q && N % 4 == 0 && vdim % 4 == 0 && xbc_stride % 4 == 0 && ((uintptr_t)xbc % 16) == 0)
+        return retention_launch(xbc, xbc_stride, state, slots, q_start, q_len, chunk_tab, carry, y, y_stride, heads, vdim, N, segs,
+                                max_chunks, fixed_a, fixed_dt, silu_in, stream);
     int qs = 0, qr = 0;
     if (aligned && ssm_quad_layout(N, vdim, &qs, &qr)) {
+        // heads that share no B and C have a block of four waves each: columns are spread over more lanes until all four work
+        while (!chunked && G == heads && qs < 16 && qr > 4 && vdim <= 2 * (256 / qs)) { qs *= 2; qr /= 2; }
 #define SSM_QUAD(NR_, NS_)                                                                                                \
     if (qr == NR_ && qs == NS_)                                                                                           \
         return ssm_launch<NR_, NS_, true>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len, \
