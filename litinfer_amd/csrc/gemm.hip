@@ -814,9 +814,10 @@ __device__ __forceinline__ float swiglu_bf16(float gate, float up) {
     return up * (gate * __builtin_amdgcn_rcpf(1.0f + e));
 }
 
-// With limit > 0 the clamped form: g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+// CLAMP: the clamped form, g = min(gate, limit), u = clamp(up, -limit, limit), g sigmoid(1.702 g) (u + 1).
+template <bool CLAMP>
 __device__ __forceinline__ float gated_bf16(float gate, float up, float limit) {
-    if (!(limit > 0.f)) return swiglu_bf16(gate, up);
+    if constexpr (!CLAMP) return swiglu_bf16(gate, up);
     const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
     const float e = __builtin_amdgcn_exp2f(-1.702f * 1.44269504088896341f * g);
     return (u + 1.0f) * (g * __builtin_amdgcn_rcpf(1.0f + e));
@@ -838,7 +839,7 @@ __device__ __forceinline__ void static_for(F&& f) {
     asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2"                          \
                  :: "s"((uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)(lptr)), "v"(voff), "s"(base) : "memory", "m0")
 
-template <int BM, int BN, int BK, int NSTAGE, bool SWIGLU, typename TO, int WLM = 2>
+template <int BM, int BN, int BK, int NSTAGE, bool SWIGLU, typename TO, int WLM = 2, bool CLAMP = false>
 __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __restrict__ x,
                                                              const bf16_t* __restrict__ w,
                                                              const float* __restrict__ bias,
@@ -1107,7 +1108,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
                 float f = 1.0f;
                 if constexpr (ROWSCALE) f = row_parts ? row_inv[row & 31] : 1.0f;      // (row_parts: M <= 32, so row < 32 here)
 #pragma unroll
-                for (int e = 0; e < 8; ++e) v[e] = gated_bf16(gs[e] * f, us[e] * f, limit);
+                for (int e = 0; e < 8; ++e) v[e] = gated_bf16<CLAMP>(gs[e] * f, us[e] * f, limit);
                 const size_t o_idx = (size_t)row * NO + col;
                 if (col + 8 <= NO && (NO % 8) == 0) {
                     chunk16 o;
@@ -1148,7 +1149,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
                             uv *= f;
                         }
                     }
-                    band[(8 * (r >> 2) + crow + (r & 3)) * ESTRIDE + 16 * j + ccol] = gated_bf16(gv, uv, limit);
+                    band[(8 * (r >> 2) + crow + (r & 3)) * ESTRIDE + 16 * j + ccol] = gated_bf16<CLAMP>(gv, uv, limit);
                 }
         } else {
 #pragma unroll
@@ -1197,7 +1198,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_dma_kernel(const bf16_t* __rest
     }
 }
 
-template <int BM, int BN, int BK, int NSTAGE, bool SWIGLU, typename TO, int WLM = 2>
+template <int BM, int BN, int BK, int NSTAGE, bool SWIGLU, typename TO, int WLM = 2, bool CLAMP = false>
 static int launch_dma(const bf16_t* x, const bf16_t* w, const float* bias, TO* out, int M, int N, int K,
                       float accumulate, hipStream_t stream, int nsplit = 1, const float* row_parts = nullptr,
                       int nparts = 0, float eps = 0.f, float limit = 0.f) {
@@ -1213,12 +1214,12 @@ static int launch_dma(const bf16_t* x, const bf16_t* w, const float* bias, TO* o
     constexpr int lds_bytes = NSTAGE * (BM + BN) * BK * 2;
     static bool configured = false;
     if (!configured) {
-        if (hipFuncSetAttribute((const void*)gemm_bf16_dma_kernel<BM, BN, BK, NSTAGE, SWIGLU, TO, WLM>,
+        if (hipFuncSetAttribute((const void*)gemm_bf16_dma_kernel<BM, BN, BK, NSTAGE, SWIGLU, TO, WLM, CLAMP>,
                                 hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes) != hipSuccess)
             return LI_ERR_LAUNCH;
         configured = true;
     }
-    gemm_bf16_dma_kernel<BM, BN, BK, NSTAGE, SWIGLU, TO, WLM><<<(unsigned)blocks, 256, lds_bytes, stream>>>(x, w, bias, out, M, N, K, accumulate, nsplit, row_parts, nparts, eps, limit);
+    gemm_bf16_dma_kernel<BM, BN, BK, NSTAGE, SWIGLU, TO, WLM, CLAMP><<<(unsigned)blocks, 256, lds_bytes, stream>>>(x, w, bias, out, M, N, K, accumulate, nsplit, row_parts, nparts, eps, limit);
     return li_launch_status();
 }
 
@@ -1375,7 +1376,7 @@ struct SkinnyArgs {
     // Columns a block takes (with ROPE: rotation pairs a block takes); 0: as many as its tiles hold.
     // Fewer than the tiles hold where that spreads a matrix of few columns evenly over the compute units.
     int cols;
-    // A tanh norm behind the sum (beta given): xg[m, n] = bf16(tanh(alpha * out[m, n]) * gamma[n] + beta[n]).  It takes
+    // A tanh norm behind the sum (EPI 1 of the kernel): xg[m, n] = bf16(tanh(alpha * out[m, n]) * gamma[n] + beta[n]).  It takes
     // no statistics of a row, so it is done here and sq_parts stays as it is.
     const float* beta;
     float alpha;
@@ -1384,7 +1385,8 @@ struct SkinnyArgs {
 };
 #define SK_MAX_PARTS 512            // blocks of a producing product whose sums one consumer adds up
 
-template <int MT, int NT, int WAVES, bool SWIGLU, typename TO, bool ROPE = false>
+// EPI 1: with SWIGLU the clamped activation, else (float out) the tanh norm of the new sum beside it (SkinnyArgs: beta).
+template <int MT, int NT, int WAVES, bool SWIGLU, typename TO, bool ROPE = false, int EPI = 0>
 __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs a) {
     static_assert(!ROPE || (MT <= 2 && !SWIGLU), "the rotary epilogue takes one or two tiles of rows");
     static_assert(MT <= WAVES, "wave mt writes the results of row tile mt");
@@ -1467,7 +1469,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                         const int nc = n < nend ? n : nend - 1;
                         pre_bias[nt][r] = a.bias ? a.bias[nc] : 0.f;
                         pre_gamma[nt][r] = a.gamma ? a.gamma[nc] : 0.f;
-                        pre_beta[nt][r] = a.beta ? a.beta[nc] : 0.f;
+                        if constexpr (EPI == 1) pre_beta[nt][r] = a.beta[nc];
                         if constexpr (sizeof(TO) == 4)
                             pre_res[nt][r] = a.accumulate != 0.f ? reinterpret_cast<const float*>(a.out)[(size_t)m * N + nc] : 0.f;
                         else pre_res[nt][r] = 0.f;
@@ -1663,7 +1665,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                 const int n = n0 + 4 * (l >> 4) + r;
                 if (n < nend) {
                     const float gv = s[0][r], uv = s[NT - 1][r];
-                    store_from_float(out + (size_t)m * N + n, gated_bf16(gv, uv, a.limit));
+                    store_from_float(out + (size_t)m * N + n, gated_bf16<EPI == 1>(gv, uv, a.limit));
                 }
             }
         } else {
@@ -1680,12 +1682,12 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_bf16_skinny_kernel(SkinnyArgs
                                 const size_t idx = (size_t)m * N + n;
                                 const float v = fmaf(factor, s[nt][r] + pre_bias[nt][r], pre_res[nt][r]);
                                 reinterpret_cast<float*>(out)[idx] = v;
-                                a.xg[idx].bits = float_to_bf16(a.beta ? fmaf(tanhf(a.alpha * v), pre_gamma[nt][r], pre_beta[nt][r])
-                                                                      : pre_gamma[nt][r] * v);
+                                a.xg[idx].bits = float_to_bf16(EPI == 1 ? fmaf(tanhf(a.alpha * v), pre_gamma[nt][r], pre_beta[nt][r])
+                                                                        : pre_gamma[nt][r] * v);
                                 sq += v * v;
                             }
                         }
-                    if (a.beta) continue;            // (nobody asks for sums of squares)
+                    if constexpr (EPI == 1) continue;      // (nobody asks for sums of squares)
                     // the four lanes of a row (l, l ^ 16, l ^ 32, l ^ 48: all of them are here, or none)
                     sq += __shfl_xor(sq, 16, 64);
                     sq += __shfl_xor(sq, 32, 64);
@@ -1743,28 +1745,28 @@ static int balanced_round_cols(int total, int unit) {
     return (int)(per > unit ? unit : per);
 }
 
-template <bool SWIGLU, typename TO>
+template <bool SWIGLU, typename TO, int EPI = 0>
 static void launch_skinny(SkinnyArgs a, hipStream_t stream) {
     const int M = a.M, N = a.N;
-#define LI_SK(MT, NT, WV) gemm_bf16_skinny_kernel<MT, NT, WV, SWIGLU, TO><<<(N + 16 * (SWIGLU ? 1 : NT) - 1) / (16 * (SWIGLU ? 1 : NT)), WV * 64, 0, stream>>>(a)
+#define LI_SK(MT, NT, WV) gemm_bf16_skinny_kernel<MT, NT, WV, SWIGLU, TO, false, EPI><<<(N + 16 * (SWIGLU ? 1 : NT) - 1) / (16 * (SWIGLU ? 1 : NT)), WV * 64, 0, stream>>>(a)
     if constexpr (SWIGLU) {
         a.cols = balanced_round_cols(N, 16);
         const int blocks = (N + a.cols - 1) / a.cols;
-        if (M <= 16) gemm_bf16_skinny_kernel<1, 2, 4, true, TO><<<blocks, 4 * 64, 0, stream>>>(a);
-        else if (M <= 32) gemm_bf16_skinny_kernel<2, 2, 4, true, TO><<<blocks, 4 * 64, 0, stream>>>(a);
-        else gemm_bf16_skinny_kernel<4, 2, 8, true, TO><<<blocks, 8 * 64, 0, stream>>>(a);
+        if (M <= 16) gemm_bf16_skinny_kernel<1, 2, 4, true, TO, false, EPI><<<blocks, 4 * 64, 0, stream>>>(a);
+        else if (M <= 32) gemm_bf16_skinny_kernel<2, 2, 4, true, TO, false, EPI><<<blocks, 4 * 64, 0, stream>>>(a);
+        else gemm_bf16_skinny_kernel<4, 2, 8, true, TO, false, EPI><<<blocks, 8 * 64, 0, stream>>>(a);
     } else if (N >= 8192) {                                 // many columns: many blocks, two tiles share each piece of x
         if (M <= 16) LI_SK(1, 2, 4); else if (M <= 32) LI_SK(2, 2, 4); else LI_SK(4, 2, 8);
     } else if (M <= 16) {                                   // few columns: a block a compute unit, eight waves split K
         a.cols = balanced_per_block(N, 16);
         const int per = a.cols ? a.cols : 16, blocks = (N + per - 1) / per;
-        if (per > 16) gemm_bf16_skinny_kernel<1, 2, 8, false, TO><<<blocks, 8 * 64, 0, stream>>>(a);
-        else gemm_bf16_skinny_kernel<1, 1, 8, false, TO><<<blocks, 8 * 64, 0, stream>>>(a);
+        if (per > 16) gemm_bf16_skinny_kernel<1, 2, 8, false, TO, false, EPI><<<blocks, 8 * 64, 0, stream>>>(a);
+        else gemm_bf16_skinny_kernel<1, 1, 8, false, TO, false, EPI><<<blocks, 8 * 64, 0, stream>>>(a);
     } else if (M <= 32) {
         a.cols = balanced_per_block(N, 16);
         const int per = a.cols ? a.cols : 16, blocks = (N + per - 1) / per;
-        if (per > 16) gemm_bf16_skinny_kernel<2, 2, 4, false, TO><<<blocks, 4 * 64, 0, stream>>>(a);
-        else gemm_bf16_skinny_kernel<2, 1, 4, false, TO><<<blocks, 4 * 64, 0, stream>>>(a);
+        if (per > 16) gemm_bf16_skinny_kernel<2, 2, 4, false, TO, false, EPI><<<blocks, 4 * 64, 0, stream>>>(a);
+        else gemm_bf16_skinny_kernel<2, 1, 4, false, TO, false, EPI><<<blocks, 4 * 64, 0, stream>>>(a);
     } else {
         LI_SK(4, 2, 8);
     }
@@ -2021,7 +2023,7 @@ extern "C" int li_linear_tanh_norm(const void* x, const void* w, const float* bi
                      nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, gamma, (bf16_t*)xn, nullptr, nullptr, 0, 0.f};
         a.beta = beta;
         a.alpha = alpha;
-        launch_skinny<false, float>(a, stream);
+        launch_skinny<false, float, 1>(a, stream);
         return li_launch_status();
     }
     const long need = li_linear_work_bytes(M, N, K, LI_BF16);
@@ -2187,7 +2189,8 @@ extern "C" int li_linear_swiglu(const void* x, const void* w, void* out, int M, 
             const double c = tile_cost(64, widths[i], 1.0, M, N, K);
             if (pick < 0 || c < best) { best = c; pick = i; }
         }
-#define LI_SW64(BN, NS) launch_dma<64, BN, 64, NS, true, bf16_t>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, row_parts, nparts, eps, limit)
+#define LI_SW64(BN, NS) (limit > 0.f ? launch_dma<64, BN, 64, NS, true, bf16_t, 2, true>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, row_parts, nparts, eps, limit) \
+                                     : launch_dma<64, BN, 64, NS, true, bf16_t>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, row_parts, nparts, eps))
         if (pick == 0) return LI_SW64(256, 3);
         if (pick == 1) return LI_SW64(192, 4);
         if (pick == 2) return LI_SW64(128, 4);
@@ -2198,12 +2201,14 @@ extern "C" int li_linear_swiglu(const void* x, const void* w, void* out, int M, 
         SkinnyArgs a{(const bf16_t*)x, (const bf16_t*)w, nullptr, out, M, I, K, 0.f,
                      nullptr, nullptr, nullptr, nullptr, nullptr, 0, 0, 0, 0, 0, nullptr, nullptr, nullptr, row_parts, nparts, eps};
         a.limit = limit;
-        launch_skinny<true, bf16_t>(a, stream);
+        if (limit > 0.f) launch_skinny<true, bf16_t, 1>(a, stream);
+        else launch_skinny<true, bf16_t>(a, stream);
         return li_launch_status();
     }
     if (M <= 64) return li_linear_skinny(x, w, nullptr, out, M, I, K, LI_BF16, 0, 1, stream);
     if (K % 64) return LI_ERR_SIZE;
-#define LI_DMA(BM, BN, BK, NS, WLM) launch_dma<BM, BN, BK, NS, true, bf16_t, WLM>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, nullptr, 0, 0.f, limit)
+#define LI_DMA(BM, BN, BK, NS, WLM) (limit > 0.f ? launch_dma<BM, BN, BK, NS, true, bf16_t, WLM, true>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream, 1, nullptr, 0, 0.f, limit) \
+                                                 : launch_dma<BM, BN, BK, NS, true, bf16_t, WLM>((const bf16_t*)x, (const bf16_t*)w, nullptr, (bf16_t*)out, M, N, K, 0.f, stream))
     // (a tile's columns are gate and up columns in turn, 32 of each: its width is a multiple of 64)
     // (128 x 320: 160 gate columns in one wave, their ups in the wave beside it; for portions of a few hundred rows,
     // where no other width comes near whole rounds of the compute units: 512 rows against the 1.5B's 17,920

@@ -237,13 +237,18 @@ extern "C" int li_moe_plan(const int* idx, int T, int top, int E, int* plan, int
 // are (gate, up) pairs, 2 gives silu(gate) * up, 3 gives g sigmoid(1.702 g) (u + 1) with g = min(gate, limit), u =
 // clamp(up, -limit, limit)), and, where the weight of a choice multiplies the expert's INPUT, the weights of the sorted
 // rows (the product is linear, so the row's sums take the factor, in float32).
+// The kernels have two forms: EXT with row weights and activation 4, and without (0 to 3).
 struct MoeEpilogue { int act; float limit; const float* row_wt; };
 
 __device__ __forceinline__ bool moe_is_gated(int act) { return act == 2 || act == 3; }
-__device__ __forceinline__ float moe_row_factor(const MoeEpilogue& ep, int row) { return ep.row_wt ? ep.row_wt[row] : 1.0f; }
-__device__ __forceinline__ float moe_act1(float v, int act) {
-    if (act == 1) { v = fmaxf(v, 0.f); return v * v; }
-    return act == 4 ? gelu_erf(v) : v;
+template <bool EXT> __device__ __forceinline__ float moe_row_factor(const MoeEpilogue& ep, int row) {
+    if constexpr (EXT) return ep.row_wt ? ep.row_wt[row] : 1.0f;
+    return 1.0f;
+}
+template <bool EXT> __device__ __forceinline__ float moe_act1(float v, int act) {
+    if (EXT && act == 4) return gelu_erf(v);
+    if (act == 1) { v = fmaxf(v, 0.f); v *= v; }
+    return v;
 }
 
 __device__ __forceinline__ float moe_gated(float g, float u, int act, float limit) {
@@ -257,11 +262,11 @@ __device__ __forceinline__ float moe_gated(float g, float u, int act, float limi
 
 // Four consecutive outputs of one row, from column `col` (a multiple of 4) on; of (gate, up) pairs the two results go to
 // columns col / 2 and col / 2 + 1.
-template <typename TO>
+template <bool EXT, typename TO>
 __device__ __forceinline__ void moe_store4(TO* __restrict__ row, int col, float v0, float v1, float v2, float v3, const MoeEpilogue& ep, float factor) {
     const int act = ep.act;
     const float limit = ep.limit;
-    v0 *= factor; v1 *= factor; v2 *= factor; v3 *= factor;
+    if constexpr (EXT) { v0 *= factor; v1 *= factor; v2 *= factor; v3 *= factor; }
     if (moe_is_gated(act)) {
         const float o0 = moe_gated(v0, v1, act, limit), o1 = moe_gated(v2, v3, act, limit);
         TO* dst = row + (col >> 1);
@@ -269,7 +274,7 @@ __device__ __forceinline__ void moe_store4(TO* __restrict__ row, int col, float 
         else *reinterpret_cast<float2*>(dst) = float2{o0, o1};
         return;
     }
-    if (act) { v0 = moe_act1(v0, act); v1 = moe_act1(v1, act); v2 = moe_act1(v2, act); v3 = moe_act1(v3, act); }
+    if (act) { v0 = moe_act1<EXT>(v0, act); v1 = moe_act1<EXT>(v1, act); v2 = moe_act1<EXT>(v2, act); v3 = moe_act1<EXT>(v3, act); }
     TO* dst = row + col;
     if constexpr (sizeof(TO) == 2) {
         uint32_t* d2 = reinterpret_cast<uint32_t*>(dst);
@@ -286,7 +291,7 @@ __device__ __forceinline__ void moe_store4(TO* __restrict__ row, int col, float 
 // matrix rows come in pairs (2 j: gate, 2 j + 1: up) and out[row, j] = silu(gate) * up: half as many columns.
 // General form: a block takes a tile and 64 outputs; rows and matrix rows go through LDS in float32, K in steps
 // of 32; a thread owns 2 rows x 4 outputs.  Sums are float32 in the order of k.
-template <typename TA, typename TW, typename TO>
+template <bool EXT, typename TA, typename TW, typename TO>
 __global__ __launch_bounds__(256) void moe_linear_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                          const TW* __restrict__ w, const int* __restrict__ plan,
                                                          TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
@@ -330,7 +335,7 @@ __global__ __launch_bounds__(256) void moe_linear_kernel(const TA* __restrict__ 
     for (int rr = 0; rr < 2; ++rr) {
         const int r = 2 * tr + rr;
         if (r >= nr) continue;
-        const float factor = moe_row_factor(ep, r0 + r);
+        const float factor = moe_row_factor<EXT>(ep, r0 + r);
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int j = j0 + 2 * tc + (i & 1) + 32 * (i >> 1);
@@ -341,7 +346,7 @@ __global__ __launch_bounds__(256) void moe_linear_kernel(const TA* __restrict__ 
                 store_from_float(out + (size_t)(r0 + r) * out_stride + (j >> 1), moe_gated(v, acc[rr][i + 1] * factor, ep.act, ep.limit));
                 continue;
             }
-            store_from_float(out + (size_t)(r0 + r) * out_stride + j, moe_act1(v, ep.act));
+            store_from_float(out + (size_t)(r0 + r) * out_stride + j, moe_act1<EXT>(v, ep.act));
         }
     }
 }
@@ -353,7 +358,7 @@ typedef __bf16 moe_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float moe_f32x16 __attribute__((ext_vector_type(16)));
 union moe_frag8 { uint4 raw; uint32_t w[4]; moe_bf16x8 v; };
 
-template <typename TA, typename TO>
+template <bool EXT, typename TA, typename TO>
 __global__ __launch_bounds__(256) void moe_linear_mfma_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
                                                               TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
@@ -385,10 +390,10 @@ __global__ __launch_bounds__(256) void moe_linear_mfma_kernel(const TA* __restri
     }
     if (ql >= nr) return;
     TO* orow = out + (size_t)(r0 + ql) * out_stride;
-    const float factor = moe_row_factor(ep, r0 + ql);
+    const float factor = moe_row_factor<EXT>(ep, r0 + ql);
 #pragma unroll
     for (int rg = 0; rg < 4; ++rg)                     // registers 4 rg .. 4 rg + 3: outputs 8 rg + 4 h2 ..
-        moe_store4(orow, j0 + 8 * rg + 4 * h2, acc[4 * rg], acc[4 * rg + 1], acc[4 * rg + 2], acc[4 * rg + 3], ep, factor);
+        moe_store4<EXT>(orow, j0 + 8 * rg + 4 * h2, acc[4 * rg], acc[4 * rg + 1], acc[4 * rg + 2], acc[4 * rg + 3], ep, factor);
 }
 
 // The wider form, for K a multiple of 32: a wave takes the tile's 32 rows and 128 outputs (four accumulators that
@@ -408,7 +413,7 @@ __device__ __forceinline__ void moe_load_rows(moe_frag8& f, const TA* p) {
     }
 }
 
-template <typename TA, typename TO, int KSPLIT>
+template <bool EXT, typename TA, typename TO, int KSPLIT>
 __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
                                                               TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep,
@@ -497,12 +502,12 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
     }
     if (ql >= nr) return;
     TO* orow = out + (size_t)(r0 + ql) * out_stride;
-    const float factor = moe_row_factor(ep, r0 + ql);
+    const float factor = moe_row_factor<EXT>(ep, r0 + ql);
     for (int f = f_lo; f < f_hi; ++f) {
         const moe_f32x16 c = KSPLIT > 1 ? acc[0] : (f == 0 ? acc[0] : f == 1 ? acc[1] : f == 2 ? acc[2] : acc[3]);
 #pragma unroll
         for (int rg = 0; rg < 4; ++rg)                 // registers 4 rg .. 4 rg + 3: outputs 32 f + 8 rg + 4 h2 ..
-            moe_store4(orow, j0 + 32 * f + 8 * rg + 4 * h2, c[4 * rg], c[4 * rg + 1], c[4 * rg + 2], c[4 * rg + 3], ep, factor);
+            moe_store4<EXT>(orow, j0 + 32 * f + 8 * rg + 4 * h2, c[4 * rg], c[4 * rg + 1], c[4 * rg + 2], c[4 * rg + 3], ep, factor);
     }
 }
 
@@ -513,7 +518,7 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
 #define MR_OUT 4
 #define MR_ROWS 4
 
-template <typename TO>
+template <bool EXT, typename TO>
 __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
                                                               TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
@@ -571,7 +576,7 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
             for (int r = 0; r < MR_ROWS; ++r) {
                 if (rc + r >= nr) continue;
                 TO* orow = out + (size_t)(r0 + rc + r) * out_stride;
-                const float factor = moe_row_factor(ep, r0 + rc + r);
+                const float factor = moe_row_factor<EXT>(ep, r0 + rc + r);
                 if (moe_is_gated(ep.act)) {            // (gate, up) pairs: n_out is even and j0 a multiple of 4
 #pragma unroll
                     for (int j = 0; j < MR_OUT; j += 2)
@@ -581,7 +586,7 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
 #pragma unroll
                 for (int j = 0; j < MR_OUT; ++j) {
                     if (j0 + j >= n_out) continue;
-                    store_from_float(orow + j0 + j, moe_act1(acc[j][r] * factor, ep.act));
+                    store_from_float(orow + j0 + j, moe_act1<EXT>(acc[j][r] * factor, ep.act));
                 }
             }
         }
@@ -598,7 +603,7 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
 #define MB_DEPTH 2             // steps whose pieces wait in registers (four: no faster)
 #define MB_LD (MB_K + 8)       // elements of an LDS row: 8 of padding (144 bytes: the 16-byte reads of 16 lanes spread over the banks)
 
-template <typename TO, int RF>      // RF: row fragments of 32 a wave (1: tiles of 64 rows, 2: of 128)
+template <bool EXT, typename TO, int RF>      // RF: row fragments of 32 a wave (1: tiles of 64 rows, 2: of 128)
 __global__ __launch_bounds__(256) void moe_linear_lds_kernel(const bf16_t* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                              const bf16_t* __restrict__ w, const int* __restrict__ plan,
                                                              TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep,
@@ -699,13 +704,13 @@ __global__ __launch_bounds__(256) void moe_linear_lds_kernel(const bf16_t* __res
         const int row = 32 * RF * wr + 32 * rf + ql;
         if (row >= nr) continue;
         TO* orow = out + (size_t)(r0 + row) * out_stride;
-        const float factor = moe_row_factor(ep, r0 + row);
+        const float factor = moe_row_factor<EXT>(ep, r0 + row);
 #pragma unroll
         for (int cf = 0; cf < 2; ++cf) {
             if (j0 + 64 * wc + 32 * cf >= n_out) continue;
 #pragma unroll
             for (int rg = 0; rg < 4; ++rg)             // registers 4 rg .. 4 rg + 3: outputs 32 cf + 8 rg + 4 h2 ..
-                moe_store4(orow, j0 + 64 * wc + 32 * cf + 8 * rg + 4 * h2, acc[rf][cf][4 * rg], acc[rf][cf][4 * rg + 1],
+                moe_store4<EXT>(orow, j0 + 64 * wc + 32 * cf + 8 * rg + 4 * h2, acc[rf][cf][4 * rg], acc[rf][cf][4 * rg + 1],
                            acc[rf][cf][4 * rg + 2], acc[rf][cf][4 * rg + 3], ep, factor);
         }
     }
@@ -716,20 +721,16 @@ extern "C" int li_moe_linear_big_takes(int a_dtype, int w_dtype, int n_out, int 
     return a_dtype == LI_BF16 && w_dtype == LI_BF16 && K % MB_K == 0 && n_out % 32 == 0;
 }
 
-extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const int* row_token, const void* w, int w_dtype,
-                             const int* plan, int max_tiles, void* out, int out_dtype, long out_stride, int n_out, int K, int act, float limit,
-                             int tile_rows, int rows, const float* row_wt, hipStream_t stream) {
-    const bool gated = act == 2 || act == 3;
-    if (max_tiles <= 0 || n_out <= 0 || K <= 0 || a_stride < K || act < 0 || act > 4 || out_stride < (gated ? n_out / 2 : n_out) ||
-        (gated && (n_out & 1)))
-        return LI_ERR_SIZE;
-    const MoeEpilogue ep{act, limit, row_wt};
+template <bool EXT>
+static int moe_linear_launch(const void* a, int a_dtype, long a_stride, const int* row_token, const void* w, int w_dtype,
+                             const int* plan, int max_tiles, void* out, int out_dtype, long out_stride, int n_out, int K, MoeEpilogue ep,
+                             int tile_rows, int rows, hipStream_t stream) {
     if (tile_rows == MOE_BIG_TILE || tile_rows == MOE_HUGE_TILE) {
         if (!li_moe_linear_big_takes(a_dtype, w_dtype, n_out, K) || a_stride % 8 || out_stride % 4 ||
             ((uintptr_t)a | (uintptr_t)w | (uintptr_t)out) % 16)
             return LI_ERR_SIZE;
         const dim3 line((unsigned)((((long)max_tiles * ((n_out + MB_COLS - 1) / MB_COLS) + 63) / 64) * 64));
-#define ML(TO, RF) moe_linear_lds_kernel<TO, RF><<<line, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles)
+#define ML(TO, RF) moe_linear_lds_kernel<EXT, TO, RF><<<line, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles)
         const bool huge = tile_rows == MOE_HUGE_TILE;
         if (out_dtype == LI_BF16) { if (huge) ML(bf16_t, 2); else ML(bf16_t, 1); }
         else if (out_dtype == LI_F32) { if (huge) ML(float, 2); else ML(float, 1); }
@@ -743,9 +744,9 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
         ((uintptr_t)a | (uintptr_t)w) % 16 == 0 && (out_dtype == LI_BF16 || out_dtype == LI_F32)) {
         const dim3 grid(max_tiles, (n_out + 4 * MR_OUT - 1) / (4 * MR_OUT));
         if (out_dtype == LI_BF16)
-            moe_linear_rows_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (bf16_t*)out, out_stride, n_out, K, ep);
+            moe_linear_rows_kernel<EXT, bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (bf16_t*)out, out_stride, n_out, K, ep);
         else
-            moe_linear_rows_kernel<float><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (float*)out, out_stride, n_out, K, ep);
+            moe_linear_rows_kernel<EXT, float><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (float*)out, out_stride, n_out, K, ep);
         return li_launch_status();
     }
     if (w_dtype == LI_BF16 && K % 16 == 0 && n_out % 32 == 0 && a_stride % 8 == 0 && out_stride % 4 == 0 &&
@@ -756,9 +757,9 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
         const dim3 line((unsigned)((((long)max_tiles * ((n_out + 511) / 512) + 63) / 64) * 64));       // whole rounds of eight tiles over eight XCDs
 #define MM(TA, TO)                                                                                                                 \
     {                                                                                                                              \
-        if (split) moe_linear_wide_kernel<TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
-        else if (wide) moe_linear_wide_kernel<TA, TO, 1><<<line, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
-        else moe_linear_mfma_kernel<TA, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep); \
+        if (split) moe_linear_wide_kernel<EXT, TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        else if (wide) moe_linear_wide_kernel<EXT, TA, TO, 1><<<line, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        else moe_linear_mfma_kernel<EXT, TA, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep); \
     }
         if (a_dtype == LI_BF16 && out_dtype == LI_BF16) MM(bf16_t, bf16_t)
         else if (a_dtype == LI_BF16 && out_dtype == LI_F32) MM(bf16_t, float)
@@ -769,7 +770,7 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
         return li_launch_status();
     }
     const dim3 grid(max_tiles, (n_out + 63) / 64);
-#define ML(TA, TW, TO) moe_linear_kernel<TA, TW, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const TW*)w, plan, (TO*)out, out_stride, n_out, K, ep)
+#define ML(TA, TW, TO) moe_linear_kernel<EXT, TA, TW, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const TW*)w, plan, (TO*)out, out_stride, n_out, K, ep)
     if (a_dtype == LI_F32 && w_dtype == LI_F32 && out_dtype == LI_F32) ML(float, float, float);
     else if (a_dtype == LI_BF16 && w_dtype == LI_BF16 && out_dtype == LI_BF16) ML(bf16_t, bf16_t, bf16_t);
     else if (a_dtype == LI_BF16 && w_dtype == LI_BF16 && out_dtype == LI_F32) ML(bf16_t, bf16_t, float);
@@ -780,11 +781,24 @@ extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const in
     return li_launch_status();
 }
 
+extern "C" int li_moe_linear(const void* a, int a_dtype, long a_stride, const int* row_token, const void* w, int w_dtype,
+                             const int* plan, int max_tiles, void* out, int out_dtype, long out_stride, int n_out, int K, int act, float limit,
+                             int tile_rows, int rows, const float* row_wt, hipStream_t stream) {
+    const bool gated = act == 2 || act == 3;
+    if (max_tiles <= 0 || n_out <= 0 || K <= 0 || a_stride < K || act < 0 || act > 4 || out_stride < (gated ? n_out / 2 : n_out) ||
+        (gated && (n_out & 1)))
+        return LI_ERR_SIZE;
+    const MoeEpilogue ep{act, limit, row_wt};
+    if (act == 4 || row_wt)
+        return moe_linear_launch<true>(a, a_dtype, a_stride, row_token, w, w_dtype, plan, max_tiles, out, out_dtype, out_stride, n_out, K, ep, tile_rows, rows, stream);
+    return moe_linear_launch<false>(a, a_dtype, a_stride, row_token, w, w_dtype, plan, max_tiles, out, out_dtype, out_stride, n_out, K, ep, tile_rows, rows, stream);
+}
+
 // ----------------------------------------------------------------------------------------------- the sum
 // x[t, :] += factor * (the sum of what follows); with a tanh norm behind it (xn given), xn[t, :] = tanh(alpha * x[t, :]) *
 // gamma + beta of the new x.  The sum: sum_c wt[t, c] (wt null: 1) * yrow[pair_row[t * top + c], :] (in the order of c) + gate[t] * shared[t, :].  A choice
 // idx[t, c] >= experts (where `ident` is given) is an IDENTITY expert: its output is the token's input row ident[t, :].
-template <typename TI>
+template <typename TI, bool NORM>
 __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x, long x_stride, const float* __restrict__ yrows,
                                                           long y_stride, const int* __restrict__ pair_row, const float* __restrict__ wt,
                                                           const float* __restrict__ gate, const float* __restrict__ shared_out,
@@ -804,7 +818,7 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(float* __restrict__ x,
         if (shared_out) s = fmaf(gate ? gate[t] : 1.f, shared_out[(size_t)t * s_stride + j], s);
         const float v = fmaf(factor, s, x[(size_t)t * x_stride + j]);
         x[(size_t)t * x_stride + j] = v;
-        if (xn) {
+        if constexpr (NORM) {
             const float r = fmaf(tanhf(alpha * v), gamma[j], beta[j]);
             if (xn_bf16) reinterpret_cast<bf16_t*>(xn)[(size_t)t * H + j].bits = float_to_bf16(r);
             else reinterpret_cast<float*>(xn)[(size_t)t * H + j] = r;
@@ -821,12 +835,13 @@ extern "C" int li_moe_combine(float* x, long x_stride, const float* yrows, long 
         return LI_ERR_SIZE;
     int ys = (H + 255) / 256;
     if (ys > 64) ys = 64;
-    if (ident && ident_dtype == LI_BF16)
-        moe_combine_kernel<bf16_t><<<dim3(T, ys), 256, 0, stream>>>(x, x_stride, yrows, y_stride, pair_row, wt, gate, shared_out, s_stride, H, top,
-                                                                    idx, experts, (const bf16_t*)ident, i_stride, factor, alpha, gamma, beta, xn, xn_dtype == LI_BF16);
-    else if (!ident || ident_dtype == LI_F32)
-        moe_combine_kernel<float><<<dim3(T, ys), 256, 0, stream>>>(x, x_stride, yrows, y_stride, pair_row, wt, gate, shared_out, s_stride, H, top,
-                                                                   idx, experts, (const float*)ident, i_stride, factor, alpha, gamma, beta, xn, xn_dtype == LI_BF16);
+#define MC(TI, NORM)                                                                                                              \
+    moe_combine_kernel<TI, NORM><<<dim3(T, ys), 256, 0, stream>>>(x, x_stride, yrows, y_stride, pair_row, wt, gate, shared_out,    \
+                                                                  s_stride, H, top, idx, experts, (const TI*)ident, i_stride, factor, \
+                                                                  alpha, gamma, beta, xn, xn_dtype == LI_BF16)
+    if (ident && ident_dtype == LI_BF16) { if (xn) MC(bf16_t, true); else MC(bf16_t, false); }
+    else if (!ident || ident_dtype == LI_F32) { if (xn) MC(float, true); else MC(float, false); }
     else return LI_ERR_DTYPE;
+#undef MC
     return li_launch_status();
 }

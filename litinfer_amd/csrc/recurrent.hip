@@ -117,16 +117,17 @@ extern "C" int li_causal_conv_silu(const float* u, long u_stride, int C, int tap
 #define SSM_TB 16
 #define SSM_WAVES 4
 
-__device__ __forceinline__ float silu_if(float z, int on) { return on ? z / (1.0f + expf(-z)) : z; }
+__device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
+template <bool ON> __device__ __forceinline__ float silu_if(float z) { if constexpr (ON) return silu_f32(z); return z; }
 __device__ __forceinline__ float softplus_f32(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 
-template <int NR, int NS, int MODE>
+template <int NR, int NS, int MODE, bool SILU>
 __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_kernel(
     const float* __restrict__ xbc, long xbc_stride, const float* __restrict__ dt_raw, long dt_stride,
     const float* __restrict__ dt_bias, const float* __restrict__ A_log, const float* __restrict__ Dw,
     float* __restrict__ state, const int* __restrict__ slots, const int* __restrict__ q_start, const int* __restrict__ q_len,
     const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, float* __restrict__ decay,
-    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt, int silu_in) {
+    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt) {
     constexpr int NP = NR * NS, PW = 64 / NS;
     extern __shared__ __align__(16) float lds[];
     float* sB = lds;                                   // [SSM_TB][NP]
@@ -174,14 +175,14 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_kernel(
             const int tt = i / NP, n = i % NP;
             const bool ok = b0 + tt < ntok && n < N;
             const float* row = xbc + (size_t)(t0 + b0 + tt) * xbc_stride + inner + (size_t)g * N + n;
-            sB[i] = ok ? silu_if(row[0], silu_in) : 0.f;
-            sC[i] = ok ? silu_if(row[(size_t)G * N], silu_in) : 0.f;
+            sB[i] = ok ? silu_if<SILU>(row[0]) : 0.f;
+            sC[i] = ok ? silu_if<SILU>(row[(size_t)G * N]) : 0.f;
         }
         if (active) {
             for (int i = lane; i < SSM_TB * PW; i += 64) {
                 const int tt = i / PW, pp = pbase + i % PW;
                 const bool ok = b0 + tt < ntok && pp < vdim;
-                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? silu_if(xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp], silu_in) : 0.f;
+                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? silu_if<SILU>(xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp]) : 0.f;
             }
             if (lane < SSM_TB) {
                 const bool ok = b0 + lane < ntok;
@@ -247,13 +248,13 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_kernel(
 // slice holds NR state values of each of its four columns.  A value of B_t or C_t read from LDS then serves four
 // state elements instead of one, and the state comes from and goes to memory in 16-byte pieces.  A wave is 256 / NS
 // columns of one head.  Modes, chunks and blocks as above.
-template <int NR, int NS, int MODE>
+template <int NR, int NS, int MODE, bool SILU>
 __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_quad_kernel(
     const float* __restrict__ xbc, long xbc_stride, const float* __restrict__ dt_raw, long dt_stride,
     const float* __restrict__ dt_bias, const float* __restrict__ A_log, const float* __restrict__ Dw,
     float* __restrict__ state, const int* __restrict__ slots, const int* __restrict__ q_start, const int* __restrict__ q_len,
     const int* __restrict__ chunk_seg, const int* __restrict__ chunk_idx, float* __restrict__ carry, float* __restrict__ decay,
-    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt, int silu_in) {
+    float* __restrict__ y, long y_stride, int heads, int vdim, int N, int G, int Q, const float* __restrict__ fixed_a, float fixed_dt) {
     constexpr int NP = NR * NS, PW = 256 / NS;
     extern __shared__ __align__(16) float lds[];
     float* sB = lds;                                   // [SSM_TB][NP]
@@ -302,14 +303,14 @@ __global__ __launch_bounds__(64 * SSM_WAVES) void ssm_scan_quad_kernel(
             const int tt = i / NP, n = i % NP;
             const bool ok = b0 + tt < ntok && n < N;
             const float* row = xbc + (size_t)(t0 + b0 + tt) * xbc_stride + inner + (size_t)g * N + n;
-            sB[i] = ok ? silu_if(row[0], silu_in) : 0.f;
-            sC[i] = ok ? silu_if(row[(size_t)G * N], silu_in) : 0.f;
+            sB[i] = ok ? silu_if<SILU>(row[0]) : 0.f;
+            sC[i] = ok ? silu_if<SILU>(row[(size_t)G * N]) : 0.f;
         }
         if (active) {
             for (int i = lane; i < SSM_TB * PW; i += 64) {
                 const int tt = i / PW, pp = pbase + i % PW;
                 const bool ok = b0 + tt < ntok && pp < vdim;
-                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? silu_if(xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp], silu_in) : 0.f;
+                sX[(w * SSM_TB + tt) * PW + i % PW] = ok ? silu_if<SILU>(xbc[(size_t)(t0 + b0 + tt) * xbc_stride + (size_t)head * vdim + pp]) : 0.f;
             }
             if (lane < SSM_TB) {
                 const bool ok = b0 + lane < ntok;
@@ -425,19 +426,19 @@ __global__ __launch_bounds__(256) void ssm_carry_kernel(float* __restrict__ carr
     }
 }
 
-template <int NR, int NS, bool QUAD>
-static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, long dt_stride, const float* dt_bias,
+template <int NR, int NS, bool QUAD, bool SILU>
+static int ssm_launch_as(const float* xbc, long xbc_stride, const float* dt_raw, long dt_stride, const float* dt_bias,
                       const float* A_log, const float* Dw, float* state, const int* slots, const int* q_start, const int* q_len,
                       int* chunk_tab, float* carry, float* decay, float* y, long y_stride, int heads, int vdim, int N, int G,
-                      int Q, int segs, int max_chunks, bool chunked, const float* fixed_a, float fixed_dt, int silu_in, hipStream_t stream) {
+                      int Q, int segs, int max_chunks, bool chunked, const float* fixed_a, float fixed_dt, hipStream_t stream) {
     constexpr int NP = NR * NS, PW = (QUAD ? 256 : 64) / NS;
     const size_t lds = (size_t)(2 * SSM_TB * NP + SSM_WAVES * SSM_TB * PW + 2 * SSM_WAVES * SSM_TB) * sizeof(float);
-#define SSM_KERNEL(MODE_) (QUAD ? ssm_scan_quad_kernel<(QUAD ? NR : 4), (QUAD ? NS : 2), MODE_> : ssm_scan_kernel<(QUAD ? 16 : NR), (QUAD ? 1 : NS), MODE_>)
+#define SSM_KERNEL(MODE_) (QUAD ? ssm_scan_quad_kernel<(QUAD ? NR : 4), (QUAD ? NS : 2), MODE_, SILU> : ssm_scan_kernel<(QUAD ? 16 : NR), (QUAD ? 1 : NS), MODE_, SILU>)
     const int hpg = heads / G, PS = (vdim + PW - 1) / PW, U = hpg * PS, ublocks = (U + SSM_WAVES - 1) / SSM_WAVES;
     if (!chunked) {
         const dim3 grid(segs, G * ublocks);
         SSM_KERNEL(0)<<<grid, 64 * SSM_WAVES, lds, stream>>>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw,
-            state, slots, q_start, q_len, nullptr, nullptr, nullptr, nullptr, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt, silu_in);
+            state, slots, q_start, q_len, nullptr, nullptr, nullptr, nullptr, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt);
         return li_launch_status();
     }
     int* chunk_seg = chunk_tab;
@@ -446,16 +447,19 @@ static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, lo
     ssm_chunk_index_kernel<<<1, 256, 0, stream>>>(q_len, segs, Q, max_chunks, chunk_seg, chunk_idx, chunk_first);
     const dim3 grid(max_chunks, G * ublocks);
     SSM_KERNEL(1)<<<grid, 64 * SSM_WAVES, lds, stream>>>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw,
-        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt, silu_in);
+        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt);
     const int NV = N * vdim;
     int zs = (NV + 255) / 256;
     if (zs > 16) zs = 16;
     ssm_carry_kernel<<<dim3(segs, heads, zs), 256, 0, stream>>>(carry, decay, state, slots, q_len, chunk_first, heads, NV, Q);
     SSM_KERNEL(0)<<<grid, 64 * SSM_WAVES, lds, stream>>>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw,
-        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt, silu_in);
+        state, slots, q_start, q_len, chunk_seg, chunk_idx, carry, decay, y, y_stride, heads, vdim, N, G, Q, fixed_a, fixed_dt);
     return li_launch_status();
 #undef SSM_KERNEL
 }
+
+template <int NR, int NS, bool QUAD, typename... A>
+static int ssm_launch(int silu_in, A... args) { return silu_in ? ssm_launch_as<NR, NS, QUAD, true>(args...) : ssm_launch_as<NR, NS, QUAD, false>(args...); }
 
 // ------------------------------------------------------------------------------- retention of long portions, as products
 // With the same decay a for every token of a head the recurrence S_t = a S_(t-1) + f k_t v_t^T, y_t = S_t^T q_t over a chunk
@@ -473,7 +477,7 @@ static int ssm_launch(const float* xbc, long xbc_stride, const float* dt_raw, lo
 #define RET_Q 64               // tokens of a chunk (SSM chunks of the same length are what the host numbers)
 typedef float ret_f32x16 __attribute__((ext_vector_type(16)));
 
-__device__ __forceinline__ float4 silu_if4(float4 v, int on) { return float4{silu_if(v.x, on), silu_if(v.y, on), silu_if(v.z, on), silu_if(v.w, on)}; }
+__device__ __forceinline__ float4 silu_if4(float4 v, int on) { return on ? float4{silu_f32(v.x), silu_f32(v.y), silu_f32(v.z), silu_f32(v.w)} : v; }
 
 // WT: fragments of 32 rows (state values) and of 32 columns a wave; the four waves are two by two, a block takes 64 WT of both.
 template <int WT>
@@ -802,8 +806,8 @@ extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_ra
         while (!chunked && G == heads && qs < 16 && qr > 4 && vdim <= 2 * (256 / qs)) { qs *= 2; qr /= 2; }
 #define SSM_QUAD(NR_, NS_)                                                                                                \
     if (qr == NR_ && qs == NS_)                                                                                           \
-        return ssm_launch<NR_, NS_, true>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len, \
-                                          chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, silu_in, stream);
+        return ssm_launch<NR_, NS_, true>(silu_in, xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len, \
+                                          chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, stream);
         SSM_QUAD(4, 2) SSM_QUAD(8, 2) SSM_QUAD(16, 2) SSM_QUAD(32, 2)
         SSM_QUAD(4, 4) SSM_QUAD(8, 4) SSM_QUAD(16, 4) SSM_QUAD(32, 4)
         SSM_QUAD(4, 8) SSM_QUAD(8, 8) SSM_QUAD(16, 8) SSM_QUAD(32, 8)
@@ -812,8 +816,8 @@ extern "C" int li_ssm_scan(const float* xbc, long xbc_stride, const float* dt_ra
     }
 #define SSM_GO(NR_, NS_)                                                                                                  \
     if (nr == NR_ && ns == NS_)                                                                                           \
-        return ssm_launch<NR_, NS_, false>(xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len,    \
-                                    chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, silu_in, stream);
+        return ssm_launch<NR_, NS_, false>(silu_in, xbc, xbc_stride, dt_raw, dt_stride, dt_bias, A_log, Dw, state, slots, q_start, q_len,    \
+                                    chunk_tab, carry, decay, y, y_stride, heads, vdim, N, G, Q, segs, max_chunks, chunked, fixed_a, fixed_dt, stream);
     SSM_GO(16, 1) SSM_GO(32, 1) SSM_GO(64, 1) SSM_GO(128, 1)
     SSM_GO(16, 2) SSM_GO(32, 2) SSM_GO(64, 2) SSM_GO(128, 2)
     SSM_GO(16, 4) SSM_GO(32, 4) SSM_GO(64, 4)
