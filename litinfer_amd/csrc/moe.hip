@@ -8,6 +8,7 @@
 #define MOE_TILE 32            // rows of one expert that a tile holds
 #define MOE_BIG_TILE 64        // ... where experts get hundreds of rows each (a prompt's portion): the tiles of the LDS kernel,
 #define MOE_HUGE_TILE 128      // and twice that where they get still more
+#define MOE_NARROW_BYTES (16l << 20)   // a decoding step's tiles against matrices below this size take 64 columns a block: more blocks, filled more evenly (1.5B sizes 38 -> 32 us; 7B sizes 138 against 155 us)
 #define MOE_FEW_ROWS 32        // rows of a step up to which every row is a matrix-vector product of its own
 
 // ------------------------------------------------------------------------------------------------ router
@@ -396,10 +397,10 @@ __global__ __launch_bounds__(256) void moe_linear_mfma_kernel(const TA* __restri
         moe_store4<EXT>(orow, j0 + 8 * rg + 4 * h2, acc[4 * rg], acc[4 * rg + 1], acc[4 * rg + 2], acc[4 * rg + 3], ep, factor);
 }
 
-// The wider form, for K a multiple of 32: a wave takes the tile's 32 rows and 128 outputs (four accumulators that
-// share the rows' operand), K in steps of 32 with the next step's ten loads asked for before this step's eight
+// The wider form, for K a multiple of 32: a wave takes the tile's 32 rows and 32 NF outputs (NF accumulators that
+// share the rows' operand), K in steps of 32 with the next step's loads asked for before this step's
 // matrix products.  KSPLIT = 1: the four waves of a block take 512 outputs side by side (many rows: a prompt).
-// KSPLIT = 4: they take the same 128 outputs and a quarter of K each and add up through LDS, so that the few tiles
+// KSPLIT = 4: they take the same outputs and a quarter of K each and add up through LDS, so that the few tiles
 // of a decoding step, each of which streams its expert's whole matrix, are spread over four times the waves.
 template <typename TA>
 __device__ __forceinline__ void moe_load_rows(moe_frag8& f, const TA* p) {
@@ -413,12 +414,12 @@ __device__ __forceinline__ void moe_load_rows(moe_frag8& f, const TA* p) {
     }
 }
 
-template <bool EXT, typename TA, typename TO, int KSPLIT>
+template <bool EXT, typename TA, typename TO, int KSPLIT, int NF>
 __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
                                                               TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep,
                                                               int max_tiles) {
-    int tile = blockIdx.x, cb = blockIdx.y;
+    int tile = blockIdx.y, cb = blockIdx.x;            // (columns first, as in the kernel of few rows)
     if (KSPLIT == 1) {
         // Many tiles: the grid is one row of blocks, which the chip deals out to its eight XCDs in turn.  Eight tiles
         // that follow each other (mostly rows of one expert) against the same columns go to ONE XCD, next to each other
@@ -432,10 +433,10 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
     if (tile >= plan[0]) return;
     const int e = plan[4 + 4 * tile], r0 = plan[5 + 4 * tile], nr = plan[6 + 4 * tile];
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6, ql = lane & 31, h2 = lane >> 5;
-    const int j0 = (KSPLIT == 1 ? cb * 4 + wv : cb) * 128;
+    const int j0 = (KSPLIT == 1 ? cb * 4 + wv : cb) * 32 * NF;
     if (KSPLIT == 1 && j0 >= n_out) return;
     int nf = (n_out - j0) / 32;                        // column fragments of 32 that exist (n_out is a multiple of 32)
-    if (nf > 4) nf = 4;
+    if (nf > NF) nf = NF;
     int k0 = 0, k1 = K;
     if (KSPLIT > 1) {
         const int per = ((K / 32 + KSPLIT - 1) / KSPLIT) * 32;
@@ -444,21 +445,21 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
     }
     const int r = r0 + (ql < nr ? ql : 0);
     const TA* arow = a + (size_t)(row_token ? row_token[r] : r) * a_stride + 8 * h2;
-    const bf16_t* mrow[4];
+    const bf16_t* mrow[NF];
 #pragma unroll
-    for (int f = 0; f < 4; ++f) mrow[f] = w + ((size_t)e * n_out + j0 + 32 * (f < nf ? f : 0) + ql) * K + 8 * h2;
-    moe_f32x16 acc[4];
+    for (int f = 0; f < NF; ++f) mrow[f] = w + ((size_t)e * n_out + j0 + 32 * (f < nf ? f : 0) + ql) * K + 8 * h2;
+    moe_f32x16 acc[NF];
 #pragma unroll
-    for (int f = 0; f < 4; ++f)
+    for (int f = 0; f < NF; ++f)
 #pragma unroll
         for (int i = 0; i < 16; ++i) acc[f][i] = 0.f;
-    moe_frag8 ca[2], cw[4][2], na[2], nw[4][2];
+    moe_frag8 ca[2], cw[NF][2], na[2], nw[NF][2];
     if (k0 < k1) {
 #pragma unroll
         for (int s2 = 0; s2 < 2; ++s2) {
             moe_load_rows<TA>(ca[s2], arow + k0 + 16 * s2);
 #pragma unroll
-            for (int f = 0; f < 4; ++f) cw[f][s2].raw = *reinterpret_cast<const uint4*>(mrow[f] + k0 + 16 * s2);
+            for (int f = 0; f < NF; ++f) cw[f][s2].raw = *reinterpret_cast<const uint4*>(mrow[f] + k0 + 16 * s2);
         }
     }
     for (int k = k0; k < k1; k += 32) {
@@ -467,25 +468,28 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
         for (int s2 = 0; s2 < 2; ++s2) {
             moe_load_rows<TA>(na[s2], arow + kn + 16 * s2);
 #pragma unroll
-            for (int f = 0; f < 4; ++f) nw[f][s2].raw = *reinterpret_cast<const uint4*>(mrow[f] + kn + 16 * s2);
+            for (int f = 0; f < NF; ++f) nw[f][s2].raw = *reinterpret_cast<const uint4*>(mrow[f] + kn + 16 * s2);
         }
+        // (the compiler would fold "loaded here or before the loop, used in the next turn" into one load at its use, and
+        // nothing would be on its way while the wave multiplies; a load is not moved past this)
+        asm volatile("" ::: "memory");
 #pragma unroll
         for (int s2 = 0; s2 < 2; ++s2)
 #pragma unroll
-            for (int f = 0; f < 4; ++f) acc[f] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(cw[f][s2].v, ca[s2].v, acc[f], 0, 0, 0);
+            for (int f = 0; f < NF; ++f) acc[f] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(cw[f][s2].v, ca[s2].v, acc[f], 0, 0, 0);
 #pragma unroll
         for (int s2 = 0; s2 < 2; ++s2) {
             ca[s2] = na[s2];
 #pragma unroll
-            for (int f = 0; f < 4; ++f) cw[f][s2] = nw[f][s2];
+            for (int f = 0; f < NF; ++f) cw[f][s2] = nw[f][s2];
         }
     }
     int f_lo = 0, f_hi = nf;
     if (KSPLIT > 1) {
         // the four waves' sums meet in LDS; wave f then owns column fragment f
-        __shared__ float red[KSPLIT][4][16][64];
+        __shared__ float red[KSPLIT][NF][16][64];
 #pragma unroll
-        for (int f = 0; f < 4; ++f)
+        for (int f = 0; f < NF; ++f)
 #pragma unroll
             for (int i = 0; i < 16; ++i) red[wv][f][i][lane] = acc[f][i];
         __syncthreads();
@@ -504,7 +508,7 @@ __global__ __launch_bounds__(256) void moe_linear_wide_kernel(const TA* __restri
     TO* orow = out + (size_t)(r0 + ql) * out_stride;
     const float factor = moe_row_factor<EXT>(ep, r0 + ql);
     for (int f = f_lo; f < f_hi; ++f) {
-        const moe_f32x16 c = KSPLIT > 1 ? acc[0] : (f == 0 ? acc[0] : f == 1 ? acc[1] : f == 2 ? acc[2] : acc[3]);
+        const moe_f32x16 c = KSPLIT > 1 ? acc[0] : (f == 0 ? acc[0] : f == 1 ? acc[1] : f == 2 ? acc[NF > 2 ? 2 : 0] : acc[NF > 2 ? 3 : 0]);
 #pragma unroll
         for (int rg = 0; rg < 4; ++rg)                 // registers 4 rg .. 4 rg + 3: outputs 32 f + 8 rg + 4 h2 ..
             moe_store4<EXT>(orow, j0 + 32 * f + 8 * rg + 4 * h2, c[4 * rg], c[4 * rg + 1], c[4 * rg + 2], c[4 * rg + 3], ep, factor);
@@ -522,11 +526,11 @@ template <bool EXT, typename TO>
 __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __restrict__ a, long a_stride, const int* __restrict__ row_token,
                                                               const bf16_t* __restrict__ w, const int* __restrict__ plan,
                                                               TO* __restrict__ out, long out_stride, int n_out, int K, MoeEpilogue ep) {
-    const int tile = blockIdx.x;
+    const int tile = blockIdx.y;              // (columns first: neighbouring blocks go to different XCDs, and each XCD gets a share of every expert)
     if (tile >= plan[0]) return;
     const int e = plan[4 + 4 * tile], r0 = plan[5 + 4 * tile], nr = plan[6 + 4 * tile];
     const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
-    const int j0 = (blockIdx.y * 4 + wv) * MR_OUT;
+    const int j0 = (blockIdx.x * 4 + wv) * MR_OUT;
     if (j0 >= n_out) return;
     const bf16_t* wrow[MR_OUT];
 #pragma unroll
@@ -543,12 +547,20 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
         for (int j = 0; j < MR_OUT; ++j)
 #pragma unroll
             for (int r = 0; r < MR_ROWS; ++r) acc[j][r] = 0.f;
-        for (int i = lane; i < K / 8; i += 64) {
-            uint4 wp[MR_OUT], xp[MR_ROWS];
+        // the next turn's pieces of the matrix rows are on their way while this one's are multiplied (past the end: the last
+        // turn's again, not used); a load is not moved past the empty statement behind it
+        uint4 wp[MR_OUT], wn[MR_OUT];
+        const int i_last = K / 8 - 1;
 #pragma unroll
-            for (int j = 0; j < MR_OUT; ++j) wp[j] = *reinterpret_cast<const uint4*>(wrow[j] + 8 * i);
+        for (int j = 0; j < MR_OUT; ++j) wp[j] = *reinterpret_cast<const uint4*>(wrow[j] + 8 * (lane < i_last ? lane : i_last));
+        for (int i = lane; i < K / 8; i += 64) {
+            uint4 xp[MR_ROWS];
 #pragma unroll
             for (int r = 0; r < MR_ROWS; ++r) xp[r] = *reinterpret_cast<const uint4*>(xrow[r] + 8 * i);
+            const int in = i + 64 < i_last ? i + 64 : i_last;
+#pragma unroll
+            for (int j = 0; j < MR_OUT; ++j) wn[j] = *reinterpret_cast<const uint4*>(wrow[j] + 8 * in);
+            asm volatile("" ::: "memory");
             float xf[MR_ROWS][8];
 #pragma unroll
             for (int r = 0; r < MR_ROWS; ++r) {
@@ -566,11 +578,14 @@ __global__ __launch_bounds__(256) void moe_linear_rows_kernel(const bf16_t* __re
                     for (int r = 0; r < MR_ROWS; ++r) acc[j][r] = fmaf(hi, xf[r][2 * q + 1], fmaf(lo, xf[r][2 * q], acc[j][r]));
                 }
             }
+#pragma unroll
+            for (int j = 0; j < MR_OUT; ++j) wp[j] = wn[j];
         }
 #pragma unroll
         for (int j = 0; j < MR_OUT; ++j)
 #pragma unroll
-            for (int r = 0; r < MR_ROWS; ++r) acc[j][r] = wave_sum(acc[j][r]);
+            for (int r = 0; r < MR_ROWS; ++r)
+                if (rc + r < nr) acc[j][r] = wave_sum(acc[j][r]);
         if (lane == 0) {
 #pragma unroll
             for (int r = 0; r < MR_ROWS; ++r) {
@@ -742,7 +757,7 @@ static int moe_linear_launch(const void* a, int a_dtype, long a_stride, const in
     // a handful of rows in all: a matrix-vector product a row (each tile streams its expert's matrix anyway)
     if (rows <= MOE_FEW_ROWS && a_dtype == LI_BF16 && w_dtype == LI_BF16 && K % 8 == 0 && a_stride % 8 == 0 &&
         ((uintptr_t)a | (uintptr_t)w) % 16 == 0 && (out_dtype == LI_BF16 || out_dtype == LI_F32)) {
-        const dim3 grid(max_tiles, (n_out + 4 * MR_OUT - 1) / (4 * MR_OUT));
+        const dim3 grid((n_out + 4 * MR_OUT - 1) / (4 * MR_OUT), max_tiles);
         if (out_dtype == LI_BF16)
             moe_linear_rows_kernel<EXT, bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)a, a_stride, row_token, (const bf16_t*)w, plan, (bf16_t*)out, out_stride, n_out, K, ep);
         else
@@ -753,12 +768,14 @@ static int moe_linear_launch(const void* a, int a_dtype, long a_stride, const in
         ((uintptr_t)a | (uintptr_t)w | (uintptr_t)out) % 16 == 0 && (a_dtype == LI_BF16 || a_dtype == LI_F32)) {
         // few tiles (a decoding step: each streams its expert's whole matrix): K in quarters over a block's waves
         const bool wide = K % 32 == 0, split = wide && max_tiles <= 128 && K >= 256;
+        const bool narrow = (long)n_out * K * 2 < MOE_NARROW_BYTES;
         const dim3 grid(max_tiles, (n_out + 127) / 128);
         const dim3 line((unsigned)((((long)max_tiles * ((n_out + 511) / 512) + 63) / 64) * 64));       // whole rounds of eight tiles over eight XCDs
 #define MM(TA, TO)                                                                                                                 \
     {                                                                                                                              \
-        if (split) moe_linear_wide_kernel<EXT, TA, TO, 4><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
-        else if (wide) moe_linear_wide_kernel<EXT, TA, TO, 1><<<line, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        if (split && narrow) moe_linear_wide_kernel<EXT, TA, TO, 4, 2><<<dim3((n_out + 63) / 64, max_tiles), 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        else if (split) moe_linear_wide_kernel<EXT, TA, TO, 4, 4><<<dim3((n_out + 127) / 128, max_tiles), 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
+        else if (wide) moe_linear_wide_kernel<EXT, TA, TO, 1, 4><<<line, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep, max_tiles); \
         else moe_linear_mfma_kernel<EXT, TA, TO><<<grid, 256, 0, stream>>>((const TA*)a, a_stride, row_token, (const bf16_t*)w, plan, (TO*)out, out_stride, n_out, K, ep); \
     }
         if (a_dtype == LI_BF16 && out_dtype == LI_BF16) MM(bf16_t, bf16_t)
